@@ -33,7 +33,7 @@
 extern "C" {
 #endif
 
-#define NVH_VERSION 205          /* major*100 + minor; 201: nvh_allreduce_status; 202: nvh_linear_desc.prefetch; 203: NVH_DECODE_CHUNKED_P256; 204: nvh_qkv_rope_attend; 205: nvh_prefill_varlen_pv16 */
+#define NVH_VERSION 206          /* major*100 + minor; 201: nvh_allreduce_status; 202: nvh_linear_desc.prefetch; 203: NVH_DECODE_CHUNKED_P256; 204: nvh_qkv_rope_attend; 205: nvh_prefill_varlen_pv16; 206: nvh_linear_desc.glu_*, nvh_rglru_*, nvh_latent_* */
 
 /* dtype codes */
 #define NVH_BF16 0
@@ -330,6 +330,8 @@ typedef struct nvh_linear_desc {
        read, NULL / 0 = none; ranges above 4 MiB are ignored (large prefetches cost the launch more than they save). */
     const void* prefetch;
     size_t prefetch_bytes;
+    /* SILU_MUL with glu_alpha != 0: the clamped gated unit of nvh_clamped_glu (limit glu_limit) instead of SiLU(g) * u */
+    float glu_limit, glu_alpha;
 } nvh_linear_desc;
 int nvh_linear_small_m_ex(const nvh_linear_desc* desc, int dtype, void* stream);
 /* residual[n_rows, hidden] += y (bf16, one rounding — the add of add_rms_forward, layers/layernorm.py:35-36) and, if `packed` is
@@ -433,6 +435,133 @@ int nvh_allreduce_status(const void* state, uint32_t* calls_completed, uint32_t*
 int nvh_allreduce_oneshot(void* out, const void* x, void* packed, void* const* stage_ptrs, void* const* flag_ptrs, void* state,
                           int world, int rank, int rows, int hidden, int64_t x_row_stride, int64_t out_row_stride,
                           size_t stage_bytes, int epilogue, int dtype, void* stream);
+
+/* ================================================================================================================================
+ * Layers with their own state: gated linear recurrence and latent attention, and the row ops of models that keep the residual stream in
+ * fp32 and normalise a sublayer's output.  `dtype` is the activation type: NVH_BF16, or NVH_F32 for a true 32-bit model (every activation,
+ * cache row and matrix operand is then float).  Widths ("cols") may be padded with zeros; the counts a mean runs over are given apart.
+ */
+/* x[rows, cols] (fp32) = embed[token] * scale; xb (nullable): the same in the activation type; packed
+ * (nullable, bf16, cols % 32 == 0): in fragment order.  Tokens outside [0, vocab) are clamped. */
+int nvh_embed_rows(float* x, void* xb, void* packed, const int64_t* tokens, const void* embed, float scale, int rows, int cols, int vocab, int dtype, void* stream);
+/* x += rmsnorm(y) * w (y given), or the result = rmsnorm(x) * w with x unchanged (y NULL). */
+typedef struct nvh_norm_residual_desc {
+    float* x;                    /* [rows, cols] fp32 residual stream */
+    void* xb;                    /* nullable: the result in the activation type */
+    void* packed;                /* nullable (bf16): the same rows in MFMA-fragment order */
+    const void* y;               /* sublayer output [rows, cols] (residual form) or null: norm of x itself, x unchanged */
+    const float* w;              /* [cols] multiplicative weight (a zero-centred weight has its one already added) */
+    float eps;
+    int32_t rows, cols, n;           /* n: elements the mean runs over (columns n.. are zero padding) */
+    int64_t y_stride;
+} nvh_norm_residual_desc;
+int nvh_norm_residual(const nvh_norm_residual_desc* d, int dtype, void* stream);
+/* out[rows, inter] = g sigmoid(alpha g) (u + 1), g = min(gate, limit), u = clamp(up, -limit, limit); gate_up rows hold gate | up. */
+int nvh_clamped_glu(void* out, const void* gate_up, int rows, int inter, int64_t gate_up_row_stride, int64_t out_row_stride, float limit, float alpha,
+                    int dtype, void* stream);
+/* Real-gated linear recurrent unit behind a causal depthwise convolution: log a = -rate sigmoid(ra u), S = a S + sqrt(1 - a^2) sigmoid(ri u) u,
+ * out = S gelu(y).  nvh_rglru_chunks: portions of prompts (and single tokens), cut by the caller into chunks of at most nvh_rglru_chunk_tokens()
+ * tokens; chunks of one portion are consecutive.  nvh_rglru_step: row i is one new token of sequence i (bf16; nvh_rglru_step_supported(block)).
+ * generic != 0 forces the plain kernel (tests). */
+typedef struct nvh_rglru_desc {
+    const void* yx;              /* [rows, 2 * width]: gate branch | recurrent branch (biases added), row stride yx_stride */
+    int64_t yx_stride;
+    int32_t width, block, blocks;    /* width == blocks * block, a multiple of 64; block % 32 == 0 */
+    int32_t taps;
+    const float* conv_w;         /* [taps, width], last row = the current token */
+    const float* conv_b;         /* [width] */
+    const void* ra;              /* [blocks, block, block] ([out, in]) */
+    const void* ri;
+    const float* ra_b;           /* [width] */
+    const float* ri_b;
+    const float* rate;           /* [width]: log a = -rate * r */
+    const int32_t* chunks;       /* [n_chunks, 4]: first row, rows (<= nvh_rglru_chunk_tokens()), sequence, index of the chunk in its sequence's portion */
+    int32_t n_chunks;
+    const int64_t* positions;    /* [rows] */
+    const int32_t* state_slots;  /* [sequences]; < 0: nothing is read or kept */
+    float* state;                /* [slots, width] */
+    void* conv_state;            /* [slots, taps, width]: input of position p at ring entry p % taps */
+    float* s_loc;                /* [rows, width] scratch: scan inside the chunk */
+    float* a_cum;                /* [rows, width] scratch: product of the decays since the chunk began */
+    void* out;                   /* [rows, width]: S * gelu(y), row stride out_stride */
+    int64_t out_stride;
+    void* out_packed;            /* nullable (bf16, step form): the result in MFMA-fragment order */
+} nvh_rglru_desc;
+int nvh_rglru_chunk_tokens(void);
+int nvh_rglru_chunks(const nvh_rglru_desc* d, int generic, int dtype, void* stream);
+int nvh_rglru_step(const nvh_rglru_desc* d, int rows, int dtype, void* stream);
+int nvh_rglru_step_supported(int block);
+/* Latent attention, row ops in front: query-latent norm, key-latent norm, rotation of interleaved pairs of the shared key part, cache store. */
+typedef struct nvh_latent_prep_desc {
+    const void* a;               /* [rows, a_stride]: query latent (q_cols) | key latent (kv_cols) | shared key part (rot_cols) */
+    int64_t a_stride;
+    int32_t rows, q_rank, q_cols, kv_rank, kv_cols, rot, rot_cols;   /* *_cols: padded widths; kv_cols == 0: no key latent in `a` */
+    const float* q_w;            /* [q_cols] */
+    const float* kv_w;           /* [kv_cols] */
+    float eps;
+    void* cq;                    /* [rows, q_cols] normed query latent */
+    void* cq_packed;             /* nullable (bf16): in MFMA-fragment order instead */
+    void* cache;                 /* [slots, kv_cols + rot_cols] */
+    const int32_t* slots;        /* [rows]; < 0: not stored */
+    const int64_t* positions;    /* [rows] */
+    const float* cos_sin;        /* [max_position, rot]: cos(0..rot/2) | sin(0..rot/2) */
+    int32_t max_position;
+} nvh_latent_prep_desc;
+int nvh_latent_prep(const nvh_latent_prep_desc* d, int dtype, void* stream);
+/* Latent attention in the cache's own space: queries absorbed through w_uk, attention over the shared rows, values through w_uv.  Three launches;
+ * generic != 0 forces the plain attention kernel (tests).  bf16 and nvh_latent_attend_mfma(kv_cols, rot_cols, block_size) and row_seq == NULL:
+ * MFMA tiles; anything else: the plain kernel (kv_cols <= 2048). */
+typedef struct nvh_latent_attn_desc {
+    /* queries */
+    const void* q;               /* [rows, heads, dim_cols + qrot_cols] (row stride q_stride): unrotated | rotated part, not rotated yet */
+    int64_t q_stride;
+    int32_t rows, heads, dim_cols, qrot_cols;
+    /* cache */
+    const void* cache;           /* pages of block_size rows [kv_cols + rot_cols] */
+    int32_t kv_cols, rot, rot_cols, block_size;
+    const int32_t* block_tables; /* [sequences, bt_stride] */
+    int64_t bt_stride;
+    int32_t max_blocks;
+    const int32_t* row_seq;      /* nullable: sequence of a row (null: row i is sequence i) */
+    const int64_t* positions;    /* [rows]; a row sees positions 0 .. its own */
+    const float* cos_sin;
+    int32_t max_position;
+    const void* w_uk;            /* [heads, kv_cols, dim_cols] */
+    const void* w_uv;            /* [heads, v_cols, kv_cols] */
+    int32_t v_cols;
+    float scale;
+    /* scratch and result */
+    void* qa;                    /* [rows, heads, kv_cols + rot_cols]: queries in the latent space */
+    float* part_o;               /* [rows, splits, heads, kv_cols] un-normalised */
+    float* part_ml;              /* [rows, splits, heads, 2]: running max (log2 domain), sum */
+    int32_t splits;
+    void* out;                   /* [rows, heads * v_cols], row stride out_stride */
+    int64_t out_stride;
+    void* out_packed;            /* nullable (bf16) */
+} nvh_latent_attn_desc;
+int nvh_latent_attention(const nvh_latent_attn_desc* d, int generic, int dtype, void* stream);
+int nvh_latent_attend_mfma(int kv_cols, int rot_cols, int block_size);
+/* out[total, cols] = the cache rows of every key of the sequences, in order (cu_k: [batch + 1] key offsets). */
+int nvh_latent_gather(void* out, const void* cache, const int32_t* cu_k, const int32_t* block_tables, int64_t bt_stride, int batch, int total, int cols,
+                      int block_size, int dtype, void* stream);
+/* Causal attention of prompt portions over expanded keys and values (bf16, bottom-right aligned mask), key width dk != value width dv. */
+typedef struct nvh_latent_prefill_desc {
+    const uint16_t* q;           /* [rows, heads, dk] unrotated | rotated part (not rotated yet), row stride q_stride */
+    const uint16_t* k;           /* [keys, heads, dim_cols], row stride k_stride */
+    const uint16_t* k_rot;       /* [keys, dk - dim_cols] shared rotated part, row stride kr_stride */
+    const uint16_t* v;           /* [keys, heads, dv], row stride v_stride */
+    uint16_t* out;               /* [rows, heads * dv], row stride out_stride */
+    int64_t q_stride, k_stride, kr_stride, v_stride, out_stride;
+    const int32_t* cu_q;         /* [batch + 1] */
+    const int32_t* cu_k;
+    const int64_t* positions;    /* [rows] */
+    const float* cos_sin;
+    int32_t max_position, rot;
+    int32_t batch, heads, dim_cols, dk, dv, max_q;
+    float scale_log2;
+} nvh_latent_prefill_desc;
+int nvh_latent_prefill(const nvh_latent_prefill_desc* d, int dtype, void* stream);
+int nvh_latent_prefill_supported(int dk, int dv);
 
 #ifdef __cplusplus
 }

@@ -18,8 +18,12 @@ CSRC = os.path.join(HERE, "csrc")
 OUT_DIR = os.path.join(HERE, "nanovllm_hip", "lib")
 OBJ_DIR = os.path.join(HERE, "build")
 LIB = os.path.join(OUT_DIR, "libnvh_attn.so")
-SOURCES = ["api.hip", "store_kvcache.hip", "paged_decode.hip", "prefill_mfma.hip", "rope_store.hip", "layer_ops.hip", "skinny_gemm.hip", "linear_stream.hip", "allreduce_oneshot.hip", "qkv_attend.hip"]
-HEADERS = ["common.h", "kernels.h", "decode_chunked.h", os.path.join("..", "..", "include", "nvh_attn.h")]
+LAYERS_LIB = os.path.join(OUT_DIR, "libnvh_layers.so")       # the LAYER_SOURCES subset of the same library
+# the linear layer, row ops, recurrence and latent attention: all that a model without paged K/V attention needs
+LAYER_SOURCES = ["api_layers.hip", "api_hybrid.hip", "layer_ops.hip", "skinny_gemm.hip", "linear_stream.hip", "hybrid_ops.hip", "rglru.hip", "latent_attention.hip",
+                 "latent_prefill.hip"]
+SOURCES = ["api.hip", "store_kvcache.hip", "paged_decode.hip", "prefill_mfma.hip", "rope_store.hip", "allreduce_oneshot.hip", "qkv_attend.hip", *LAYER_SOURCES]
+HEADERS = ["common.h", "kernels.h", "hybrid.h", "api_common.h", "decode_chunked.h", os.path.join("..", "..", "include", "nvh_attn.h")]
 HIPCC = os.environ.get("HIPCC", "/opt/rocm/bin/hipcc")
 # -amdgpu-mfma-vgpr-form: MFMA results stay in the architectural VGPRs.  By default hipcc parks accumulators in the AGPR file
 # and pays a v_accvgpr_read/write per element wherever VALU code touches them (softmax on S, rescale of O): 159 such moves in
@@ -29,16 +33,18 @@ HIPCC = os.environ.get("HIPCC", "/opt/rocm/bin/hipcc")
 # put the operands of their first DMA there (measured: attention call 9.22 -> 9.08 us together with the hoisted table loads).
 FLAGS = ["--offload-arch=gfx950", "-O3", "-std=c++17", "-fPIC", "-ffp-contract=fast", "-mllvm", "-amdgpu-mfma-vgpr-form",
          "-mllvm", "-amdgpu-kernarg-preload-count=14",
+         # no packed fp32 instructions: some of their forms have returned wrong results on these parts
+         "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops",
          "-Wall", "-Wno-unused-function", "-Wno-unused-command-line-argument"]
 # rope_store.hip must round RoPE's products and sums separately (bit parity with the reference's elementwise fp32 ops);
 # HIP's default backend contraction ignores the source pragma, so that file is built with contraction off.
 FILE_FLAGS = {"rope_store.hip": ["-ffp-contract=off"], "skinny_gemm.hip": ["-ffp-contract=off"], "linear_stream.hip": ["-ffp-contract=off"]}   # its RoPE epilogue too
 
 
-def _digest():
+def _digest(sources=SOURCES):
     h = hashlib.sha256()
     h.update((" ".join(FLAGS) + repr(sorted(FILE_FLAGS.items()))).encode())
-    for name in SOURCES + HEADERS:
+    for name in sources + HEADERS:
         with open(os.path.join(CSRC, name), "rb") as f:
             h.update(f.read())
     return h.hexdigest()
@@ -58,26 +64,30 @@ def _compile(src, asm, extra=(), obj_dir=None):
     return obj
 
 
-def build(force=False, asm=False, verbose=True):
-    """Compile every HIP source for gfx950 and link libnvh_attn.so.  Returns the library path."""
+def build(force=False, asm=False, verbose=True, layers_only=False):
+    """Compile every HIP source for gfx950 and link libnvh_attn.so — or, with layers_only, the LAYER_SOURCES subset into
+    libnvh_layers.so.  Returns the library path."""
+    sources, lib = (LAYER_SOURCES, LAYERS_LIB) if layers_only else (SOURCES, LIB)
     os.makedirs(OUT_DIR, exist_ok=True)
     os.makedirs(OBJ_DIR, exist_ok=True)
-    stamp = os.path.join(OBJ_DIR, "digest.txt")
-    digest = _digest()
-    if not force and not asm and os.path.exists(LIB) and os.path.exists(stamp) and open(stamp).read() == digest:
+    stamp = os.path.join(OBJ_DIR, f"digest_{os.path.basename(lib)}.txt")
+    digest = _digest(sources)
+    if not force and not asm and os.path.exists(lib) and os.path.exists(stamp) and open(stamp).read() == digest:
         if verbose:
-            print(f"[nvh build] up to date: {LIB}")
-        return LIB
+            print(f"[nvh build] up to date: {lib}")
+        return lib
     if not os.path.exists(HIPCC):
         raise RuntimeError(f"hipcc not found at {HIPCC}; set HIPCC")
-    with ThreadPoolExecutor(max_workers=4) as ex:
-        objs = list(ex.map(lambda s: _compile(s, asm), SOURCES))
-    subprocess.run([HIPCC, "--offload-arch=gfx950", "-shared", "-fPIC", "-o", LIB, *objs], check=True)
+    with ThreadPoolExecutor(max_workers=8) as ex:
+        objs = list(ex.map(lambda s: _compile(s, asm), sources))
+    part = f"{lib}.{os.getpid()}"                            # linked beside its final name: a reader never sees half a library
+    subprocess.run([HIPCC, "--offload-arch=gfx950", "-shared", "-fPIC", "-o", part, *objs], check=True)
+    os.replace(part, lib)
     with open(stamp, "w") as f:
         f.write(digest)
     if verbose:
-        print(f"[nvh build] built {LIB}")
-    return LIB
+        print(f"[nvh build] built {lib}")
+    return lib
 
 
 def build_variant(out, extra):

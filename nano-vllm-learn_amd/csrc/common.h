@@ -120,6 +120,18 @@ __device__ __forceinline__ bool argmax_better(float v, int i, float best, int bi
 __device__ __forceinline__ float fast_exp2(float x) { return __builtin_amdgcn_exp2f(x); }   // v_exp_f32
 __device__ __forceinline__ float fast_rcp(float x) { return __builtin_amdgcn_rcpf(x); }
 
+// gated unit with clamped inputs: g sigmoid(alpha g) (u + 1), g = min(gate, limit), u = clamp(up, -limit, limit)
+__device__ __forceinline__ float clamped_glu(float gate, float up, float limit, float alpha) {
+    const float g = fminf(gate, limit), u = fminf(fmaxf(up, -limit), limit);
+    return g / (1.f + __expf(-alpha * g)) * (u + 1.f);
+}
+
+// the gated unit of a gate_up projection: the clamped one when alpha != 0, SiLU(g) u with the gate rounded to bf16 first otherwise
+__device__ __forceinline__ float gated_unit(float g, float u, float limit, float alpha) {
+    if (alpha != 0.f) return clamped_glu(g, u, limit, alpha);
+    return (float)(__bf16)(g / (1.f + __expf(-g))) * u;
+}
+
 // ---- host-side error plumbing ------------------------------------------------------------------
 void set_error(const char* fmt, ...);
 int check_launch(const char* what);

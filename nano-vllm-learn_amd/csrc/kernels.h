@@ -100,6 +100,7 @@ struct LinearArgs {
     float norm_eps;
     int norm_mode;               // 0 none; 1 exact RMSNorm prologue; 2 folded RMSNorm (w already multiplied by the norm weight)
     int epi;
+    float glu_limit, glu_alpha;  // SILU epilogue with glu_alpha != 0: the clamped gated unit of common.h instead of SiLU(g) * u
     const int64_t* positions;    // ROPE: [M]
     const float* cos_sin;        // ROPE: [max_position, D]
     uint16_t* k_cache;           // ROPE: paged caches and slots of this step's rows

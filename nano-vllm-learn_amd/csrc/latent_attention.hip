@@ -1,0 +1,500 @@
+// Latent attention over a paged cache of one shared row per token: [normed latent c (kv_cols) | rotated key part (rot_cols)].
+//   prep     query latent norm, key latent norm, interleaved rotation of the shared key part, cache store: one launch over the projection's rows
+//   absorb   per head  q_lat = W_uk^T q_unrotated  and the rotation of the rotated part: queries in the cache's own space
+//   attend   softmax(scale q_lat . row) over the rows a query sees, un-normalised sums of c per split of the context
+//   value    combine the splits, per head  W_uv (latent sum)
+// A query's score against a key needs the cache row only, so one stream over the context serves every head (the decode form; prompts use the
+// expanded form of latent_prefill.hip).  Scores, weights and sums are fp32; the weights enter the MFMA as bf16 hi + lo halves.
+// Every step exists for bf16 on MFMA tiles and in a plain form for any size and for fp32 activations.
+#include <type_traits>
+
+#include "hybrid.h"
+
+namespace nvh {
+
+namespace {
+
+typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
+
+// ------------------------------------------------------------------------------------------------ prep
+template <typename T>
+__global__ __launch_bounds__(256) void latent_prep_kernel(const LatentPrepArgs a) {
+    __shared__ float lds[8];
+    const int row = blockIdx.x;
+    const T* x = reinterpret_cast<const T*>(a.a) + (int64_t)row * a.a_stride;
+    const T* c = x + a.q_cols;
+    float sq = 0.f, sc = 0.f;
+    for (int i = threadIdx.x * 4; i < a.q_cols; i += 1024) {
+        const f32x4 v = act_ld4(x + i);
+        sq += v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3];
+    }
+    for (int i = threadIdx.x * 4; i < a.kv_cols; i += 1024) {
+        const f32x4 v = act_ld4(c + i);
+        sc += v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3];
+    }
+    const float iq = 1.f / sqrtf(block_sum256(sq, lds) / a.q_rank + a.eps);
+    for (int i = threadIdx.x * 4; i < a.q_cols; i += 1024) {
+        const f32x4 v = act_ld4(x + i) * iq * *reinterpret_cast<const f32x4*>(a.q_w + i);
+        if (a.cq_packed) act_st4(reinterpret_cast<uint16_t*>(a.cq_packed) + pack_index(row, i, a.q_cols), v);
+        else act_st4(reinterpret_cast<T*>(a.cq) + (int64_t)row * a.q_cols + i, v);
+    }
+    if (a.kv_cols == 0) return;                      // (uniform over the launch)
+    const float ic = 1.f / sqrtf(block_sum256(sc, lds + 4) / a.kv_rank + a.eps);
+    const int slot = a.slots[row];
+    if (slot < 0) return;
+    T* out = reinterpret_cast<T*>(a.cache) + (int64_t)slot * (a.kv_cols + a.rot_cols);
+    for (int i = threadIdx.x * 4; i < a.kv_cols; i += 1024)
+        act_st4(out + i, act_ld4(c + i) * ic * *reinterpret_cast<const f32x4*>(a.kv_w + i));
+    int64_t pos = a.positions[row];
+    if (pos >= a.max_position) pos = a.max_position - 1;
+    const float* cs = a.cos_sin + pos * a.rot;
+    for (int i = threadIdx.x; i < a.rot / 2; i += 256) {
+        const float u = act_ld(c + a.kv_cols + 2 * i), v = act_ld(c + a.kv_cols + 2 * i + 1), co = cs[i], si = cs[a.rot / 2 + i];
+        act_st(out + a.kv_cols + 2 * i, u * co - v * si);
+        act_st(out + a.kv_cols + 2 * i + 1, v * co + u * si);
+    }
+}
+
+// ------------------------------------------------------------------------------------------------ absorb
+// rotated part of this workgroup's (row, head): qa[kv_cols ..] = rotate(q[dim_cols ..]); columns past `rot` are zero
+template <typename T>
+__device__ __forceinline__ void rotate_query(const LatentAttnArgs& a, int row, int head, int first, int step) {
+    const T* q = reinterpret_cast<const T*>(a.q) + (int64_t)row * a.q_stride + head * (a.dim_cols + a.qrot_cols) + a.dim_cols;
+    T* o = reinterpret_cast<T*>(a.qa) + ((int64_t)row * a.heads + head) * (a.kv_cols + a.rot_cols) + a.kv_cols;
+    int64_t pos = a.positions[row];
+    if (pos >= a.max_position) pos = a.max_position - 1;
+    const float* cs = a.cos_sin + pos * a.rot;
+    for (int i = first; i < a.rot_cols / 2; i += step) {
+        float r0 = 0.f, r1 = 0.f;
+        if (i < a.rot / 2) {
+            const float u = act_ld(q + 2 * i), v = act_ld(q + 2 * i + 1), co = cs[i], si = cs[a.rot / 2 + i];
+            r0 = u * co - v * si;
+            r1 = v * co + u * si;
+        }
+        act_st(o + 2 * i, r0);
+        act_st(o + 2 * i + 1, r1);
+    }
+}
+
+// grid (heads, kv_cols / 64, row tiles of 16), 4 waves x 16 latent columns
+__global__ __launch_bounds__(256) void latent_absorb_kernel(const LatentAttnArgs a) {
+    const int head = blockIdx.x, r0 = blockIdx.z * 16;
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, lq = lane & 15, lg = lane >> 4;
+    const int n0 = blockIdx.y * 64 + wave * 16, cols = a.kv_cols + a.rot_cols;
+    const int row = r0 + lq < a.rows ? r0 + lq : a.rows - 1;
+    const uint16_t* q = reinterpret_cast<const uint16_t*>(a.q) + (int64_t)row * a.q_stride + head * (a.dim_cols + a.qrot_cols) + 8 * lg;
+    const uint16_t* w = reinterpret_cast<const uint16_t*>(a.w_uk) + ((int64_t)head * a.kv_cols + n0 + lq) * a.dim_cols + 8 * lg;
+    f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+    for (int k = 0; k < a.dim_cols; k += 32)
+        acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8*>(w + k), *reinterpret_cast<const bf16x8*>(q + k), acc, 0, 0, 0);
+    // C^T layout: lane = query row lq, latent columns n0 + 4 lg ..
+    if (r0 + lq < a.rows)
+        act_st4(reinterpret_cast<uint16_t*>(a.qa) + ((int64_t)(r0 + lq) * a.heads + head) * cols + n0 + 4 * lg, acc);
+    if (blockIdx.y == 0 && r0 + (tid >> 4) < a.rows) rotate_query<uint16_t>(a, r0 + (tid >> 4), head, tid & 15, 16);
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void latent_absorb_generic_kernel(const LatentAttnArgs a) {
+    extern __shared__ float q_lds[];
+    const int row = blockIdx.x, head = blockIdx.y;
+    const T* q = reinterpret_cast<const T*>(a.q) + (int64_t)row * a.q_stride + head * (a.dim_cols + a.qrot_cols);
+    for (int i = threadIdx.x; i < a.dim_cols; i += 256) q_lds[i] = act_ld(q + i);
+    __syncthreads();
+    T* o = reinterpret_cast<T*>(a.qa) + ((int64_t)row * a.heads + head) * (a.kv_cols + a.rot_cols);
+    for (int n = threadIdx.x; n < a.kv_cols; n += 256) {
+        const T* w = reinterpret_cast<const T*>(a.w_uk) + ((int64_t)head * a.kv_cols + n) * a.dim_cols;
+        float s = 0.f;
+        for (int k = 0; k < a.dim_cols; k += 4) {
+            const f32x4 v = act_ld4(w + k);
+            s += v[0] * q_lds[k] + v[1] * q_lds[k + 1] + v[2] * q_lds[k + 2] + v[3] * q_lds[k + 3];
+        }
+        act_st(o + n, s);
+    }
+    rotate_query<T>(a, row, head, threadIdx.x, 256);
+}
+
+// ------------------------------------------------------------------------------------------------ attend, any type and size
+// one workgroup per (row, head, split); 64 keys at a time: 4 lanes per key for the scores, one thread per latent column for the sums
+__device__ __forceinline__ void split_range(int ctx, int splits, int split, int& k0, int& k1) {
+    const int tiles = (ctx + 63) / 64, per = (tiles + splits - 1) / splits;
+    k0 = split * per * 64;
+    k1 = k0 + per * 64 < ctx ? k0 + per * 64 : ctx;
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void latent_attend_generic_kernel(const LatentAttnArgs a) {
+    constexpr int OC = 8;                            // latent columns per thread: kv_cols <= 2048
+    extern __shared__ float q_lds[];                 // [kv_cols + rot_cols]
+    __shared__ float p_lds[64];
+    const int row = blockIdx.x, head = blockIdx.y, split = blockIdx.z, cols = a.kv_cols + a.rot_cols, tid = threadIdx.x;
+    const int seq = a.row_seq ? a.row_seq[row] : row;
+    const int ctx = (int)a.positions[row] + 1;
+    int k0, k1;
+    split_range(ctx, a.splits, split, k0, k1);
+    const T* q = reinterpret_cast<const T*>(a.qa) + ((int64_t)row * a.heads + head) * cols;
+    for (int i = tid; i < cols; i += 256) q_lds[i] = act_ld(q + i);
+    float o[OC], m = -INFINITY, l = 0.f;
+#pragma unroll
+    for (int j = 0; j < OC; ++j) o[j] = 0.f;
+    const float sc = a.scale * kLog2e;
+    __syncthreads();
+    auto cache_row = [&](int key) {
+        const int64_t page = a.block_tables[seq * a.bt_stride + key / a.block_size];
+        return reinterpret_cast<const T*>(a.cache) + (page * a.block_size + key % a.block_size) * cols;
+    };
+    for (int t0 = k0; t0 < k1; t0 += 64) {
+        const int key = t0 + (tid >> 2);
+        float s = 0.f;
+        if (key < k1) {
+            const T* r = cache_row(key);
+            for (int i = (tid & 3) * 4; i < cols; i += 16) {
+                const f32x4 v = act_ld4(r + i);
+                s += v[0] * q_lds[i] + v[1] * q_lds[i + 1] + v[2] * q_lds[i + 2] + v[3] * q_lds[i + 3];
+            }
+        }
+        s += __shfl_xor(s, 1);
+        s += __shfl_xor(s, 2);
+        if ((tid & 3) == 0) p_lds[tid >> 2] = key < k1 ? s * sc : -INFINITY;
+        __syncthreads();
+        float v = p_lds[tid & 63], mx = v;
+        for (int d = 1; d < 64; d <<= 1) mx = fmaxf(mx, __shfl_xor(mx, d));
+        const float m_new = fmaxf(m, mx), alpha = exp2f(m - m_new);
+        v = exp2f(v - m_new);
+        float sum = v;
+        for (int d = 1; d < 64; d <<= 1) sum += __shfl_xor(sum, d);
+        l = l * alpha + sum;
+        m = m_new;
+        __syncthreads();
+        if (tid < 64) p_lds[tid] = v;
+        __syncthreads();
+#pragma unroll
+        for (int j = 0; j < OC; ++j) o[j] *= alpha;
+        const int cnt = k1 - t0 < 64 ? k1 - t0 : 64;
+        for (int k = 0; k < cnt; ++k) {
+            const T* r = cache_row(t0 + k);
+            const float p = p_lds[k];
+#pragma unroll
+            for (int j = 0; j < OC; ++j)
+                if (tid + 256 * j < a.kv_cols) o[j] += p * act_ld(r + tid + 256 * j);
+        }
+        __syncthreads();
+    }
+    const int64_t rec = ((int64_t)row * a.splits + split) * a.heads + head;
+#pragma unroll
+    for (int j = 0; j < OC; ++j)
+        if (tid + 256 * j < a.kv_cols) a.part_o[rec * a.kv_cols + tid + 256 * j] = o[j];
+    if (tid == 0) {
+        a.part_ml[rec * 2] = m;
+        a.part_ml[rec * 2 + 1] = l;
+    }
+}
+
+// ------------------------------------------------------------------------------------------------ attend, MFMA (bf16, one row per sequence)
+// grid (splits, rows, head tiles of 16), 4 waves.  64 keys at a time in ONE LDS image that serves as K (row reads) and as V (hardware-transposed
+// reads): wave w scores keys 16 w .. + 15 for all 16 heads (queries in registers), the waves agree on the tile's maxima through LDS, weights go to
+// LDS as bf16 hi + lo in the order the transposed reads deliver keys, and wave w sums its quarter of the latent columns.
+// Two workgroups per CU (one image each) cover each other's load and compute phases.
+template <int OFF>
+__device__ __forceinline__ u32x2 ds_read_tr16(uint32_t lds_addr) {
+    u32x2 r;
+    asm volatile("ds_read_b64_tr_b16 %0, %1 offset:%2" : "=v"(r) : "v"(lds_addr), "n"(OFF) : "memory");
+    return r;
+}
+__device__ __forceinline__ uint32_t lds_addr_of(const void* p) { return (uint32_t)(uintptr_t)(__attribute__((address_space(3))) const void*)p; }
+
+template <int NT>                                    // kv_cols = 64 * NT, rot_cols = 64
+__global__ __launch_bounds__(256) void latent_attend_kernel(const LatentAttnArgs a) {
+    constexpr int COLS = 64 * NT + 64, ROWB = COLS * 2, CPR = COLS / 8, KS = COLS / 32, NI = CPR / 4;   // NI: DMA instructions per wave
+    constexpr bool kOdd = ((ROWB / 128) & 1) != 0;
+    extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
+    unsigned char* img = smem;                       // [64][ROWB], 16-byte pieces swizzled inside groups of 8
+    uint16_t* p_lds = reinterpret_cast<uint16_t*>(smem + 64 * ROWB);             // [hi | lo][16 heads][64 + 8]
+    float* mx_lds = reinterpret_cast<float*>(smem + 64 * ROWB + 2 * 16 * 72 * 2);  // [4 waves][16]
+    const int split = blockIdx.x, row = blockIdx.y, h0 = blockIdx.z * 16;
+    const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lq = lane & 15, lg = lane >> 4;
+    const int ctx = (int)a.positions[row] + 1;
+    const bool head_ok = h0 + lq < a.heads;
+    int k0, k1;
+    split_range(ctx, a.splits, split, k0, k1);
+    const int64_t rec = ((int64_t)row * a.splits + split) * a.heads + h0 + lq;
+    if (k0 >= k1) {
+        if (wave == 0 && lg == 0 && head_ok) {
+            a.part_ml[rec * 2] = -INFINITY;
+            a.part_ml[rec * 2 + 1] = 0.f;
+        }
+        return;
+    }
+    auto swz = [](int r) { return kOdd ? ((r >> 1) & 7) : (r & 7); };
+    const uint16_t* cache = reinterpret_cast<const uint16_t*>(a.cache);
+    // staging: piece s of the image -> (row s / CPR, place s % CPR); the source piece is the place with its low three bits xor-ed
+    auto stage = [&](int t0) {
+        const int64_t page = a.block_tables[row * a.bt_stride + t0 / a.block_size];          // 64 divides the page: one page per tile
+        const uint16_t* base = cache + (page * a.block_size + t0 % a.block_size) * COLS;
+        const int live = k1 - t0 < 64 ? k1 - t0 : 64;
+#pragma unroll
+        for (int j = 0; j < NI; ++j) {
+            const int s = (wave * NI + j) * 64 + lane;
+            const int r = s / CPR, place = s - r * CPR, piece = place ^ swz(r);
+            const int rc = r < live ? r : live - 1;                                           // (rows past the context repeat its last one: masked)
+            __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)(base + rc * COLS + piece * 8),
+                                             (__attribute__((address_space(3))) void*)(img + (wave * NI + j) * 1024), 16, 0, 0);
+        }
+    };
+    stage(k0);
+    bf16x8 qf[KS];                                   // B operand: column = head lq, 8 consecutive columns
+    {
+        const uint16_t* q = reinterpret_cast<const uint16_t*>(a.qa) + ((int64_t)row * a.heads + (head_ok ? h0 + lq : a.heads - 1)) * COLS + 8 * lg;
+#pragma unroll
+        for (int s = 0; s < KS; ++s) qf[s] = *reinterpret_cast<const bf16x8*>(q + 32 * s);
+    }
+    f32x4 o[NT];                                     // latent columns 64 t' .. : tile index 4 t + wave -> columns 16 (4 t + wave) + 4 lg, head lq
+#pragma unroll
+    for (int t = 0; t < NT; ++t) o[t] = f32x4{0.f, 0.f, 0.f, 0.f};
+    float m = -INFINITY, l = 0.f;
+    const float sc = a.scale * kLog2e;
+    // transposed reads: lane 4 q + p of a 16-lane group addresses key row 4 lg + q (+ 16), columns 4 p .. of the 16-column tile
+    const int vr = 4 * lg + (lq >> 2), vp = lq & 3;
+    for (int t0 = k0; t0 < k1; t0 += 64) {
+        asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+        __syncthreads();
+        const int R = 16 * wave + lq;
+        f32x4 s4 = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int s = 0; s < KS; ++s) {
+            const bf16x8 kf = *reinterpret_cast<const bf16x8*>(img + R * ROWB + ((4 * s + lg) ^ swz(R)) * 16);
+            s4 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[s], s4, 0, 0, 0);
+        }
+        float mx = -INFINITY;
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+            s4[r] = t0 + 16 * wave + 4 * lg + r < k1 ? s4[r] * sc : -INFINITY;
+            mx = fmaxf(mx, s4[r]);
+        }
+        mx = fmaxf(mx, __shfl_xor(mx, 16));
+        mx = fmaxf(mx, __shfl_xor(mx, 32));
+        if (lg == 0) mx_lds[wave * 16 + lq] = mx;
+        __syncthreads();
+        mx = fmaxf(fmaxf(mx_lds[lq], mx_lds[16 + lq]), fmaxf(mx_lds[32 + lq], mx_lds[48 + lq]));   // finite: the tile holds a visible key
+        const float m_new = fmaxf(m, mx), alpha = fast_exp2(m - m_new);
+        m = m_new;
+        float p[4], hi[4];
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+            p[r] = fast_exp2(s4[r] - m_new);
+            hi[r] = (float)(__bf16)p[r];
+        }
+        l = l * alpha + (p[0] + p[1] + p[2] + p[3]);
+        // key 16 w + 4 lg + r -> 32-key half w / 2, slot 8 lg + 4 (w & 1) + r
+        const int at = lq * 72 + 32 * (wave >> 1) + 8 * lg + 4 * (wave & 1);
+        *reinterpret_cast<u32x2*>(p_lds + at) = u32x2{pack_bf16x2(p[0], p[1]), pack_bf16x2(p[2], p[3])};
+        *reinterpret_cast<u32x2*>(p_lds + 16 * 72 + at) = u32x2{pack_bf16x2(p[0] - hi[0], p[1] - hi[1]), pack_bf16x2(p[2] - hi[2], p[3] - hi[3])};
+        __syncthreads();
+#pragma unroll
+        for (int t = 0; t < NT; ++t) o[t] *= alpha;
+#pragma unroll
+        for (int hh = 0; hh < 2; ++hh) {
+            const bf16x8 ph = *reinterpret_cast<const bf16x8*>(p_lds + lq * 72 + 32 * hh + 8 * lg);
+            const bf16x8 pl = *reinterpret_cast<const bf16x8*>(p_lds + 16 * 72 + lq * 72 + 32 * hh + 8 * lg);
+            u32x2 v0[NT], v1[NT];
+#pragma unroll
+            for (int t = 0; t < NT; ++t) {
+                const int tile = 4 * t + wave, ra = 32 * hh + vr, rb = ra + 16;
+                v0[t] = ds_read_tr16<0>(lds_addr_of(img + ra * ROWB + ((2 * tile + (vp >> 1)) ^ swz(ra)) * 16 + (vp & 1) * 8));
+                v1[t] = ds_read_tr16<0>(lds_addr_of(img + rb * ROWB + ((2 * tile + (vp >> 1)) ^ swz(rb)) * 16 + (vp & 1) * 8));
+            }
+            asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+            __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+            for (int t = 0; t < NT; ++t) {
+                const u32x4 raw = {v0[t][0], v0[t][1], v1[t][0], v1[t][1]};
+                const bf16x8 vf = *reinterpret_cast<const bf16x8*>(&raw);
+                o[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, ph, o[t], 0, 0, 0);
+                o[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pl, o[t], 0, 0, 0);
+            }
+        }
+        __syncthreads();                             // every wave is done with the image and the weights
+        if (t0 + 64 < k1) stage(t0 + 64);
+    }
+    if (head_ok) {
+#pragma unroll
+        for (int t = 0; t < NT; ++t) *reinterpret_cast<f32x4*>(a.part_o + rec * a.kv_cols + 16 * (4 * t + wave) + 4 * lg) = o[t];
+    }
+    l += __shfl_xor(l, 16);
+    l += __shfl_xor(l, 32);
+    if (lg == 0) mx_lds[wave * 16 + lq] = l;
+    __syncthreads();
+    if (wave == 0 && lg == 0 && head_ok) {
+        a.part_ml[rec * 2] = m;
+        a.part_ml[rec * 2 + 1] = mx_lds[lq] + mx_lds[16 + lq] + mx_lds[32 + lq] + mx_lds[48 + lq];
+    }
+}
+
+// ------------------------------------------------------------------------------------------------ value
+// normalised latent sum of (row, head) at columns c .. c + 3 from the split records
+__device__ __forceinline__ f32x4 combine_splits(const LatentAttnArgs& a, int row, int head, int c, float m, float inv) {
+    f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+    for (int s = 0; s < a.splits; ++s) {
+        const int64_t rec = ((int64_t)row * a.splits + s) * a.heads + head;
+        const float ms = a.part_ml[rec * 2];
+        if (ms == -INFINITY) continue;               // an empty split wrote no sums
+        acc += *reinterpret_cast<const f32x4*>(a.part_o + rec * a.kv_cols + c) * (fast_exp2(ms - m) * inv);
+    }
+    return acc;
+}
+__device__ __forceinline__ void split_totals(const LatentAttnArgs& a, int row, int head, float& m, float& inv) {
+    m = -INFINITY;
+    for (int s = 0; s < a.splits; ++s) m = fmaxf(m, a.part_ml[(((int64_t)row * a.splits + s) * a.heads + head) * 2]);
+    float l = 0.f;
+    for (int s = 0; s < a.splits; ++s) {
+        const int64_t rec = ((int64_t)row * a.splits + s) * a.heads + head;
+        const float ms = a.part_ml[rec * 2];
+        if (ms != -INFINITY) l += a.part_ml[rec * 2 + 1] * fast_exp2(ms - m);
+    }
+    inv = l > 0.f ? 1.f / l : 0.f;
+}
+
+// grid (heads, row tiles of RW): latent sums of RW rows into LDS as the A operand (rows past RW are zero), waves share the value columns
+template <int RW>
+__global__ __launch_bounds__(256) void latent_value_kernel(const LatentAttnArgs a) {
+    extern __shared__ __attribute__((aligned(16))) uint16_t lat[];             // [16][kv_cols + 8]
+    const int head = blockIdx.x, r0 = blockIdx.y * RW, ld = a.kv_cols + 8, pieces = a.kv_cols / 4;
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, lq = lane & 15, lg = lane >> 4;
+    for (int e = tid; e < 16 * pieces; e += 256) {
+        const int r = e / pieces, c = (e - r * pieces) * 4;
+        f32x4 v = {0.f, 0.f, 0.f, 0.f};
+        if (r < RW && r0 + r < a.rows) {
+            float m, inv;
+            split_totals(a, r0 + r, head, m, inv);
+            v = combine_splits(a, r0 + r, head, c, m, inv);
+        }
+        act_st4(lat + r * ld + c, v);
+    }
+    __syncthreads();
+    for (int nt = wave; nt < a.v_cols / 16; nt += 4) {
+        const uint16_t* w = reinterpret_cast<const uint16_t*>(a.w_uv) + ((int64_t)head * a.v_cols + 16 * nt + lq) * a.kv_cols + 8 * lg;
+        f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+        for (int k = 0; k < a.kv_cols; k += 32)
+            acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8*>(w + k), *reinterpret_cast<const bf16x8*>(lat + lq * ld + 8 * lg + k), acc, 0, 0, 0);
+        if (lq < RW && r0 + lq < a.rows) {           // C^T: lane = row lq, value columns 16 nt + 4 lg ..
+            const int col = head * a.v_cols + 16 * nt + 4 * lg;
+            if (a.out) act_st4(reinterpret_cast<uint16_t*>(a.out) + (int64_t)(r0 + lq) * a.out_stride + col, acc);
+            if (a.out_packed) act_st4(reinterpret_cast<uint16_t*>(a.out_packed) + pack_index(r0 + lq, col, a.heads * a.v_cols), acc);
+        }
+    }
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void latent_value_generic_kernel(const LatentAttnArgs a) {
+    extern __shared__ float latf[];
+    const int row = blockIdx.x, head = blockIdx.y;
+    float m, inv;
+    split_totals(a, row, head, m, inv);
+    for (int c = threadIdx.x * 4; c < a.kv_cols; c += 1024) {
+        const f32x4 v = combine_splits(a, row, head, c, m, inv);
+#pragma unroll
+        for (int k = 0; k < 4; ++k) latf[c + k] = act_round(v[k], (const T*)nullptr);
+    }
+    __syncthreads();
+    for (int n = threadIdx.x; n < a.v_cols; n += 256) {
+        const T* w = reinterpret_cast<const T*>(a.w_uv) + ((int64_t)head * a.v_cols + n) * a.kv_cols;
+        float s = 0.f;
+        for (int k = 0; k < a.kv_cols; k += 4) {
+            const f32x4 v = act_ld4(w + k);
+            s += v[0] * latf[k] + v[1] * latf[k + 1] + v[2] * latf[k + 2] + v[3] * latf[k + 3];
+        }
+        act_st(reinterpret_cast<T*>(a.out) + (int64_t)row * a.out_stride + head * a.v_cols + n, s);
+    }
+}
+
+// ------------------------------------------------------------------------------------------------ gather
+// cache rows of every key of the sequences, packed: out[cu_k[b] + j] = row of key j of sequence b
+template <typename T>
+__global__ __launch_bounds__(256) void latent_gather_kernel(T* __restrict__ out, const T* __restrict__ cache, const int32_t* __restrict__ cu_k,
+                                                             const int32_t* __restrict__ block_tables, int64_t bt_stride, int batch, int cols, int block_size) {
+    const int row = blockIdx.x;
+    int lo = 0, hi = batch;                          // sequence of this row: the last b with cu_k[b] <= row
+    while (hi - lo > 1) {
+        const int mid = (lo + hi) / 2;
+        if (cu_k[mid] <= row) lo = mid;
+        else hi = mid;
+    }
+    const int key = row - cu_k[lo];
+    const int64_t page = block_tables[lo * bt_stride + key / block_size];
+    const T* src = cache + (page * block_size + key % block_size) * cols;
+    for (int c = threadIdx.x * 4; c < cols; c += 1024) act_st4(out + (int64_t)row * cols + c, act_ld4(src + c));
+}
+
+template <int NT>
+void attend_nt(const LatentAttnArgs& a, hipStream_t stream) {
+    constexpr size_t lds = 64 * (64 * NT + 64) * 2 + 2 * 16 * 72 * 2 + 4 * 16 * 4;
+    if (lds > 64 * 1024) (void)hipFuncSetAttribute(reinterpret_cast<const void*>(latent_attend_kernel<NT>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+    latent_attend_kernel<NT><<<dim3(a.splits, a.rows, (a.heads + 15) / 16), 256, lds, stream>>>(a);
+}
+
+}  // namespace
+
+int launch_latent_prep(const LatentPrepArgs& a, int f32, hipStream_t stream) {
+    if (f32) latent_prep_kernel<float><<<a.rows, 256, 0, stream>>>(a);
+    else latent_prep_kernel<uint16_t><<<a.rows, 256, 0, stream>>>(a);
+    return check_launch("latent_prep");
+}
+
+int launch_latent_absorb(const LatentAttnArgs& a, int f32, hipStream_t stream) {
+    if (!f32 && a.dim_cols % 32 == 0 && a.kv_cols % 64 == 0) {
+        latent_absorb_kernel<<<dim3(a.heads, a.kv_cols / 64, (a.rows + 15) / 16), 256, 0, stream>>>(a);
+    } else {
+        const dim3 grid(a.rows, a.heads);
+        if (f32) latent_absorb_generic_kernel<float><<<grid, 256, a.dim_cols * 4, stream>>>(a);
+        else latent_absorb_generic_kernel<uint16_t><<<grid, 256, a.dim_cols * 4, stream>>>(a);
+    }
+    return check_launch("latent_absorb");
+}
+
+bool latent_mfma_supported(int kv_cols, int rot_cols, int block_size) {
+    if (rot_cols != 64 || block_size % 64) return false;
+    switch (kv_cols) {
+        case 64: case 128: case 192: case 256: case 384: case 512: return true;
+        default: return false;
+    }
+}
+
+int launch_latent_attend(const LatentAttnArgs& a, int f32, int generic, hipStream_t stream) {
+    if (!f32 && !generic && !a.row_seq && latent_mfma_supported(a.kv_cols, a.rot_cols, a.block_size)) {
+        switch (a.kv_cols) {
+            case 64: attend_nt<1>(a, stream); break;
+            case 128: attend_nt<2>(a, stream); break;
+            case 192: attend_nt<3>(a, stream); break;
+            case 256: attend_nt<4>(a, stream); break;
+            case 384: attend_nt<6>(a, stream); break;
+            default: attend_nt<8>(a, stream); break;
+        }
+    } else {
+        const dim3 grid(a.rows, a.heads, a.splits);
+        const size_t lds = (size_t)(a.kv_cols + a.rot_cols) * 4;
+        if (f32) latent_attend_generic_kernel<float><<<grid, 256, lds, stream>>>(a);
+        else latent_attend_generic_kernel<uint16_t><<<grid, 256, lds, stream>>>(a);
+    }
+    return check_launch("latent_attend");
+}
+
+int launch_latent_value(const LatentAttnArgs& a, int f32, hipStream_t stream) {
+    if (!f32 && a.v_cols % 16 == 0 && a.kv_cols % 32 == 0) {
+        const size_t lds = (size_t)16 * (a.kv_cols + 8) * 2;
+        if (a.rows <= 128) latent_value_kernel<4><<<dim3(a.heads, (a.rows + 3) / 4), 256, lds, stream>>>(a);
+        else latent_value_kernel<16><<<dim3(a.heads, (a.rows + 15) / 16), 256, lds, stream>>>(a);
+    } else {
+        const dim3 grid(a.rows, a.heads);
+        if (f32) latent_value_generic_kernel<float><<<grid, 256, a.kv_cols * 4, stream>>>(a);
+        else latent_value_generic_kernel<uint16_t><<<grid, 256, a.kv_cols * 4, stream>>>(a);
+    }
+    return check_launch("latent_value");
+}
+
+int launch_latent_gather(void* out, const void* cache, const int32_t* cu_k, const int32_t* block_tables, int64_t bt_stride, int batch, int total, int cols,
+                         int block_size, int f32, hipStream_t stream) {
+    if (f32) latent_gather_kernel<float><<<total, 256, 0, stream>>>((float*)out, (const float*)cache, cu_k, block_tables, bt_stride, batch, cols, block_size);
+    else latent_gather_kernel<uint16_t><<<total, 256, 0, stream>>>((uint16_t*)out, (const uint16_t*)cache, cu_k, block_tables, bt_stride, batch, cols, block_size);
+    return check_launch("latent_gather");
+}
+
+}  // namespace nvh

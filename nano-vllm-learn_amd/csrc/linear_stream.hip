@@ -547,13 +547,13 @@ __global__ __launch_bounds__(NWV * 64) void linear_stream_kernel(
                     const int col = 24 * tile + 16 * hb + c;
                     if ((hb == 1 && c >= 8) || col >= p_inter) continue;
                     const float g = (float)(__bf16)y[hb], u = (float)(__bf16)y[2 + hb];
-                    const __bf16 o = (__bf16)((float)(__bf16)(g / (1.f + __expf(-g))) * u);
+                    const __bf16 o = (__bf16)gated_unit(g, u, a.glu_limit, a.glu_alpha);
                     if (out) out[(int64_t)row * e_out_stride + col] = o;
                     if (e_out_packed) e_out_packed[pack_index(row, col, p_inter)] = __builtin_bit_cast(uint16_t, o);
                 }
             } else if constexpr (EPI == EPI_SILU) {
                 const float g = (float)(__bf16)y[0], u = (float)(__bf16)y[1];          // the projection output is bf16 in the reference
-                const __bf16 o = (__bf16)((float)(__bf16)(g / (1.f + __expf(-g))) * u);
+                const __bf16 o = (__bf16)gated_unit(g, u, a.glu_limit, a.glu_alpha);
                 if (out) out[(int64_t)row * e_out_stride + n0 + c] = o;
                 if (e_out_packed) e_out_packed[pack_index(row, n0 + c, p_inter)] = __builtin_bit_cast(uint16_t, o);
             } else if constexpr (EPI == EPI_RESADD) {

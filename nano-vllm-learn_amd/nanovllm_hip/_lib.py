@@ -10,6 +10,7 @@ import torch  # noqa: F401  (imported first on purpose: libnvh_attn.so binds to 
 
 _HERE = os.path.dirname(os.path.abspath(__file__))
 LIB_PATH = os.environ.get("NVH_LIB_PATH") or os.path.join(_HERE, "lib", "libnvh_attn.so")   # override: A/B of two builds
+LAYERS_LIB_PATH = os.path.join(_HERE, "lib", "libnvh_layers.so")                            # the subset without paged K/V attention (build.py layers_only)
 
 NVH_BF16 = 0
 NVH_F32 = 1
@@ -27,7 +28,56 @@ class LinearDesc(ctypes.Structure):
                 ("norm_folded", ctypes.c_int32), ("x_packed", ctypes.c_int32), ("out_packed", ctypes.c_void_p),
                 ("workspace", ctypes.c_void_p), ("workspace_bytes", ctypes.c_size_t),
                 ("candidate_val", ctypes.c_void_p), ("candidate_idx", ctypes.c_void_p), ("candidate_stride", ctypes.c_int64),
-                ("prefetch", ctypes.c_void_p), ("prefetch_bytes", ctypes.c_size_t)]
+                ("prefetch", ctypes.c_void_p), ("prefetch_bytes", ctypes.c_size_t),
+                ("glu_limit", ctypes.c_float), ("glu_alpha", ctypes.c_float)]
+
+
+class NormResidualDesc(ctypes.Structure):
+    """nvh_norm_residual_desc (include/nvh_attn.h)."""
+    _fields_ = [("x", ctypes.c_void_p), ("xb", ctypes.c_void_p), ("packed", ctypes.c_void_p), ("y", ctypes.c_void_p),
+                ("w", ctypes.c_void_p), ("eps", ctypes.c_float), ("rows", ctypes.c_int32), ("cols", ctypes.c_int32), ("n", ctypes.c_int32),
+                ("y_stride", ctypes.c_int64)]
+
+
+class RglruDesc(ctypes.Structure):
+    """nvh_rglru_desc (include/nvh_attn.h)."""
+    _fields_ = [("yx", ctypes.c_void_p), ("yx_stride", ctypes.c_int64), ("width", ctypes.c_int32), ("block", ctypes.c_int32),
+                ("blocks", ctypes.c_int32), ("taps", ctypes.c_int32), ("conv_w", ctypes.c_void_p), ("conv_b", ctypes.c_void_p),
+                ("ra", ctypes.c_void_p), ("ri", ctypes.c_void_p), ("ra_b", ctypes.c_void_p), ("ri_b", ctypes.c_void_p),
+                ("rate", ctypes.c_void_p), ("chunks", ctypes.c_void_p), ("n_chunks", ctypes.c_int32), ("positions", ctypes.c_void_p),
+                ("state_slots", ctypes.c_void_p), ("state", ctypes.c_void_p), ("conv_state", ctypes.c_void_p), ("s_loc", ctypes.c_void_p),
+                ("a_cum", ctypes.c_void_p), ("out", ctypes.c_void_p), ("out_stride", ctypes.c_int64), ("out_packed", ctypes.c_void_p)]
+
+
+class LatentPrepDesc(ctypes.Structure):
+    """nvh_latent_prep_desc (include/nvh_attn.h)."""
+    _fields_ = [("a", ctypes.c_void_p), ("a_stride", ctypes.c_int64), ("rows", ctypes.c_int32), ("q_rank", ctypes.c_int32),
+                ("q_cols", ctypes.c_int32), ("kv_rank", ctypes.c_int32), ("kv_cols", ctypes.c_int32), ("rot", ctypes.c_int32),
+                ("rot_cols", ctypes.c_int32), ("q_w", ctypes.c_void_p), ("kv_w", ctypes.c_void_p), ("eps", ctypes.c_float),
+                ("cq", ctypes.c_void_p), ("cq_packed", ctypes.c_void_p), ("cache", ctypes.c_void_p), ("slots", ctypes.c_void_p),
+                ("positions", ctypes.c_void_p), ("cos_sin", ctypes.c_void_p), ("max_position", ctypes.c_int32)]
+
+
+class LatentAttnDesc(ctypes.Structure):
+    """nvh_latent_attn_desc (include/nvh_attn.h)."""
+    _fields_ = [("q", ctypes.c_void_p), ("q_stride", ctypes.c_int64), ("rows", ctypes.c_int32), ("heads", ctypes.c_int32),
+                ("dim_cols", ctypes.c_int32), ("qrot_cols", ctypes.c_int32), ("cache", ctypes.c_void_p), ("kv_cols", ctypes.c_int32),
+                ("rot", ctypes.c_int32), ("rot_cols", ctypes.c_int32), ("block_size", ctypes.c_int32), ("block_tables", ctypes.c_void_p),
+                ("bt_stride", ctypes.c_int64), ("max_blocks", ctypes.c_int32), ("row_seq", ctypes.c_void_p), ("positions", ctypes.c_void_p),
+                ("cos_sin", ctypes.c_void_p), ("max_position", ctypes.c_int32), ("w_uk", ctypes.c_void_p), ("w_uv", ctypes.c_void_p),
+                ("v_cols", ctypes.c_int32), ("scale", ctypes.c_float), ("qa", ctypes.c_void_p), ("part_o", ctypes.c_void_p),
+                ("part_ml", ctypes.c_void_p), ("splits", ctypes.c_int32), ("out", ctypes.c_void_p), ("out_stride", ctypes.c_int64),
+                ("out_packed", ctypes.c_void_p)]
+
+
+class LatentPrefillDesc(ctypes.Structure):
+    """nvh_latent_prefill_desc (include/nvh_attn.h)."""
+    _fields_ = [("q", ctypes.c_void_p), ("k", ctypes.c_void_p), ("k_rot", ctypes.c_void_p), ("v", ctypes.c_void_p),
+                ("out", ctypes.c_void_p), ("q_stride", ctypes.c_int64), ("k_stride", ctypes.c_int64), ("kr_stride", ctypes.c_int64),
+                ("v_stride", ctypes.c_int64), ("out_stride", ctypes.c_int64), ("cu_q", ctypes.c_void_p), ("cu_k", ctypes.c_void_p),
+                ("positions", ctypes.c_void_p), ("cos_sin", ctypes.c_void_p), ("max_position", ctypes.c_int32), ("rot", ctypes.c_int32),
+                ("batch", ctypes.c_int32), ("heads", ctypes.c_int32), ("dim_cols", ctypes.c_int32), ("dk", ctypes.c_int32),
+                ("dv", ctypes.c_int32), ("max_q", ctypes.c_int32), ("scale_log2", ctypes.c_float)]
 
 
 EPI_NONE, EPI_SILU_MUL, EPI_RESIDUAL_ADD, EPI_ROPE_STORE = 0, 1, 2, 3
@@ -100,6 +150,19 @@ _SIGS = {
                                                                       ctypes.c_void_p] +
                                             [ctypes.c_void_p, ctypes.c_int, ctypes.c_int, ctypes.c_void_p, ctypes.c_int64, ctypes.c_void_p, ctypes.c_int,
                                              ctypes.c_void_p]),
+    "nvh_embed_rows": (ctypes.c_int, [ctypes.c_void_p] * 5 + [ctypes.c_float] + [ctypes.c_int] * 4 + [ctypes.c_void_p]),
+    "nvh_norm_residual": (ctypes.c_int, [ctypes.POINTER(NormResidualDesc), ctypes.c_int, ctypes.c_void_p]),
+    "nvh_clamped_glu": (ctypes.c_int, [ctypes.c_void_p] * 2 + [ctypes.c_int] * 2 + [ctypes.c_int64] * 2 + [ctypes.c_float] * 2 + [ctypes.c_int, ctypes.c_void_p]),
+    "nvh_rglru_chunk_tokens": (ctypes.c_int, []),
+    "nvh_rglru_step_supported": (ctypes.c_int, [ctypes.c_int]),
+    "nvh_rglru_chunks": (ctypes.c_int, [ctypes.POINTER(RglruDesc), ctypes.c_int, ctypes.c_int, ctypes.c_void_p]),
+    "nvh_rglru_step": (ctypes.c_int, [ctypes.POINTER(RglruDesc), ctypes.c_int, ctypes.c_int, ctypes.c_void_p]),
+    "nvh_latent_prep": (ctypes.c_int, [ctypes.POINTER(LatentPrepDesc), ctypes.c_int, ctypes.c_void_p]),
+    "nvh_latent_attend_mfma": (ctypes.c_int, [ctypes.c_int] * 3),
+    "nvh_latent_attention": (ctypes.c_int, [ctypes.POINTER(LatentAttnDesc), ctypes.c_int, ctypes.c_int, ctypes.c_void_p]),
+    "nvh_latent_gather": (ctypes.c_int, [ctypes.c_void_p] * 4 + [ctypes.c_int64] + [ctypes.c_int] * 5 + [ctypes.c_void_p]),
+    "nvh_latent_prefill_supported": (ctypes.c_int, [ctypes.c_int] * 2),
+    "nvh_latent_prefill": (ctypes.c_int, [ctypes.POINTER(LatentPrefillDesc), ctypes.c_int, ctypes.c_void_p]),
 }
 EXPORTS = tuple(_SIGS)
 
@@ -110,28 +173,46 @@ class NvhLibraryError(RuntimeError):
     pass
 
 
+class _Subset:
+    """The layers-only library: entry points it does not hold raise when they are asked for."""
+
+    def __init__(self, lib, path):
+        self._lib, self._path = lib, path
+
+    def __getattr__(self, name):
+        try:
+            return getattr(self._lib, name)
+        except AttributeError as e:
+            raise NvhLibraryError(f"{self._path} does not hold {name}: build the whole library with `python nano-vllm-learn_amd/build.py`") from e
+
+
 def load():
-    """Load (once) and return the ctypes handle.  Raises NvhLibraryError if the .so is absent."""
+    """Load (once) and return the library: libnvh_attn.so, or the layers-only subset where only that is built.  Raises
+    NvhLibraryError if neither is there."""
     global _lib
     if _lib is not None:
         return _lib
-    if not os.path.exists(LIB_PATH):
+    path = LIB_PATH if os.path.exists(LIB_PATH) or "NVH_LIB_PATH" in os.environ else LAYERS_LIB_PATH
+    if not os.path.exists(path):
         raise NvhLibraryError(
             f"{LIB_PATH} not found: build it with `python nano-vllm-learn_amd/build.py` "
             "(the hip attention backend has no fallback path)")
     try:
-        lib = ctypes.CDLL(LIB_PATH)
+        lib = ctypes.CDLL(path)
     except OSError as e:
-        raise NvhLibraryError(f"cannot load {LIB_PATH}: {e}") from e
+        raise NvhLibraryError(f"cannot load {path}: {e}") from e
+    subset = path == LAYERS_LIB_PATH
     for name, (res, args) in _SIGS.items():
         try:
             fn = getattr(lib, name)
         except AttributeError as e:
-            raise NvhLibraryError(f"{LIB_PATH} does not export {name}") from e
+            if subset:
+                continue
+            raise NvhLibraryError(f"{path} does not export {name}") from e
         fn.restype = res
         fn.argtypes = args
-    _lib = lib
-    return lib
+    _lib = _Subset(lib, path) if subset else lib
+    return _lib
 
 
 def check(rc, what):

@@ -29,6 +29,15 @@ class BlockManager:
         for _ in range(need):
             seq.block_table.append(self._take())
 
+    def grow(self, seq, num_tokens):
+        """Blocks for the sequence's first `num_tokens` tokens; False (and nothing taken) when the pool does not hold that many more."""
+        need = (num_tokens + self.block_size - 1) // self.block_size - len(seq.block_table)
+        if need > len(self.free_block_ids):
+            return False
+        for _ in range(need):
+            seq.block_table.append(self._take())
+        return True
+
     def can_append(self, seq):
         return len(self.free_block_ids) >= (len(seq) % self.block_size == 1)
 
@@ -43,3 +52,23 @@ class BlockManager:
             self.free_block_ids.append(block_id)
         seq.num_cached_tokens = 0
         seq.block_table.clear()
+
+
+class StateSlots:
+    """Recurrent-state slots: one per live sequence.  A slot needs no clearing when it changes hands: a sequence's first token starts from zero
+    whatever the slot holds."""
+
+    def __init__(self, num_slots):
+        self.free = deque(range(num_slots))
+
+    def allocate(self, seq):
+        if seq.state_slot < 0:
+            if not self.free:
+                return False
+            seq.state_slot = self.free.popleft()
+        return True
+
+    def deallocate(self, seq):
+        if seq.state_slot >= 0:
+            self.free.append(seq.state_slot)
+            seq.state_slot = -1

@@ -22,8 +22,10 @@ import torch
 import torch.distributed as dist
 
 from .. import ops
-from ..models.qwen import ModelConfig, QwenForCausalLM, tp_partition
+from ..models import build_model
+from ..models.qwen import tp_partition
 from ..utils.context import reset_context, set_context
+from ..utils.step import StepMeta
 from .sequence import Sequence
 
 
@@ -85,21 +87,68 @@ def build_decode_meta(seqs, block_size=256):
                 block_tables=build_block_tables(seqs))
 
 
+def recurrence_chunks(first_row, rows, seq, chunk_tokens):
+    """Chunk table rows of one sequence's portion: (first row, rows, sequence, index in the portion)."""
+    return [(first_row + k, min(chunk_tokens, rows - k), seq, k // chunk_tokens) for k in range(0, rows, chunk_tokens)]
+
+
+def build_step_meta(portions, block_size, chunk_tokens=64):
+    """Rows of a mixed batch.  portions: [(sequence, tokens)] — the sequence's next tokens behind its num_cached_tokens.  Sequences that bring one
+    token come first (`order` gives the places in `portions`); returns host tensors."""
+    _check_block_size([s for s, _ in portions], block_size)
+    order = sorted(range(len(portions)), key=lambda i: portions[i][1] > 1)
+    input_ids, positions, slots, row_seq, chunks = [], [], [], [], []
+    cu_q, cu_k, max_q, num_decode = [0], [0], 0, 0
+    for j, i in enumerate(order):
+        seq, n = portions[i]
+        lo, hi = seq.num_cached_tokens, seq.num_cached_tokens + n
+        assert 0 < n and hi <= len(seq) and hi <= len(seq.block_table) * block_size
+        chunks += recurrence_chunks(len(input_ids), n, j, chunk_tokens)
+        input_ids += seq[lo:hi]
+        positions += range(lo, hi)
+        slots += [seq.block_table[p // block_size] * block_size + p % block_size for p in range(lo, hi)]
+        row_seq += [j] * n
+        if n == 1:
+            num_decode += 1
+        else:
+            cu_q.append(cu_q[-1] + n)
+            cu_k.append(cu_k[-1] + hi)
+            max_q = max(max_q, n)
+    seqs = [portions[i][0] for i in order]
+
+    def i32(v):
+        return torch.tensor(v, dtype=torch.int32)
+    return dict(order=order, input_ids=torch.tensor(input_ids, dtype=torch.int64), positions=torch.tensor(positions, dtype=torch.int64), num_decode=num_decode,
+                slot_mapping=i32(slots), block_tables=build_block_tables(seqs, pad=0), state_slots=i32([s.state_slot for s in seqs]), chunks=i32(chunks),
+                row_seq=i32(row_seq), cu_q=i32(cu_q), cu_k=i32(cu_k), max_q=max_q, total_k=cu_k[-1], max_context=max(positions) + 1)
+
+
 # ----------------------------------------------------------------------------- runner
 class ModelRunner:
-    def __init__(self, cfg: ModelConfig, num_kvcache_blocks: int, device=None, max_model_len=4096, seed=0):
+    """weights: folder of a checkpoint (None: random weights of `seed`).  max_num_seqs: recurrent-state slots, for models that keep state."""
+
+    def __init__(self, cfg, num_kvcache_blocks: int, device=None, max_model_len=4096, seed=0, weights=None, max_num_seqs=512):
         self.cfg = cfg
         self.block_size = cfg.kvcache_block_size
-        assert self.block_size == Sequence.block_size, (
-            f"kvcache_block_size {self.block_size} != Sequence.block_size {Sequence.block_size} (fixed at 256 as in the reference, "
-            "engine/sequence.py:15, config.py:20,31)")
         self.max_model_len = max_model_len
         self.rank = dist.get_rank() if dist.is_initialized() else 0
         self.world_size = dist.get_world_size() if dist.is_initialized() else 1
         self.device = torch.device(device if device is not None else f"cuda:{torch.cuda.current_device()}")
-        self.model = QwenForCausalLM(cfg).init_random(seed).to(device=self.device, dtype=torch.bfloat16)
+        if hasattr(cfg, "dtype"):
+            assert max_model_len <= cfg.max_position_embeddings, "max_model_len exceeds the rotation table"
+            assert self.world_size == 1, f"{cfg.name} runs on one GPU"
+            if cfg.dtype == torch.float32:
+                torch.set_float32_matmul_precision("highest")                     # true 32-bit products
+            self.dtype = cfg.dtype
+            self.model = build_model(cfg, weights, seed).to(device=self.device)     # (each tensor already has its own type)
+        else:
+            self.dtype = torch.bfloat16
+            self.model = build_model(cfg, weights, seed).to(device=self.device, dtype=self.dtype)
         self.model.eval()
+        self.mixed_batches = getattr(self.model, "uses_step_meta", False)
+        self.max_num_seqs = max_num_seqs
         self.num_kvcache_blocks = num_kvcache_blocks
+        self.state = {}
         self.allocate_kv_cache()
         # tensor parallel: choose the all-reduce path once, the same on every rank (one-shot over IPC-mapped peer buffers for the
         # decode-sized messages, RCCL otherwise / as the fallback); NVH_ALLREDUCE=rccl keeps everything on RCCL
@@ -109,7 +158,21 @@ class ModelRunner:
             self.comm = init_tensor_parallel_comm(64, cfg.hidden_size, prefer_oneshot=os.environ.get("NVH_ALLREDUCE", "oneshot") != "rccl")
 
     def allocate_kv_cache(self):
+        """Every module that declares what it keeps per token (`cache_row`) or per sequence (`state_spec`) gets its pool; attention modules with
+        k_cache / v_cache share one tensor."""
         cfg = self.cfg
+        if self.mixed_batches:
+            self.kv_cache = []
+            for name, module in self.model.named_modules():
+                if getattr(module, "cache_row", None) and module.cache_row() is not None:
+                    cols, dtype = module.cache_row()
+                    module.latent_cache = torch.zeros(self.num_kvcache_blocks, self.block_size, cols, dtype=dtype, device=self.device)
+                    self.kv_cache.append(module.latent_cache)
+                for attr, (shape, dtype) in (module.state_spec() if hasattr(module, "state_spec") else {}).items():
+                    pool = torch.zeros(self.max_num_seqs, *shape, dtype=dtype, device=self.device)
+                    setattr(module, attr, pool)
+                    self.state[f"{name}.{attr}"] = pool
+            return
         kvh = tp_partition(cfg.num_attention_heads, cfg.num_key_value_heads, self.world_size, self.rank)[3]
         self.kv_cache = torch.zeros(2, cfg.num_hidden_layers, self.num_kvcache_blocks, self.block_size, kvh, cfg.head_dim,
                                     dtype=torch.bfloat16, device=self.device)
@@ -124,10 +187,39 @@ class ModelRunner:
     def _dev(self, t):
         return t.to(self.device, non_blocking=True) if t is not None else None
 
+    @torch.inference_mode()
+    def run_step(self, portions, want=None):
+        """One batch of a model that takes mixed batches.  portions: [(sequence, tokens)]; want: per portion, the places among its tokens whose
+        logits are asked for (default: the last).  Returns logits rows in the order of `portions` and `want` (None when nothing is wanted) and
+        advances num_cached_tokens."""
+        m = build_step_meta(portions, self.block_size, ops.rglru_chunk_tokens())
+        assert int(m["positions"].max()) < self.max_model_len, "a sequence exceeds max_model_len"
+        assert 0 <= int(m["input_ids"].min()) and int(m["input_ids"].max()) < self.cfg.vocab_size, "a token id is outside the vocabulary"
+        first, row = {}, 0
+        for i in m["order"]:
+            first[i] = row
+            row += portions[i][1]
+        want = want if want is not None else [[n - 1] for _, n in portions]
+        rows = [first[i] + p for i, places in enumerate(want) for p in places]
+        assert all(0 <= p < portions[i][1] for i, places in enumerate(want) for p in places), "a wanted place is outside its portion"
+        decode_only = m["num_decode"] == row
+        step = StepMeta(m["num_decode"], self._dev(m["slot_mapping"]), self._dev(m["block_tables"]), self._dev(m["state_slots"]), self._dev(m["chunks"]),
+                        m["max_context"], *([] if decode_only else [self._dev(m["row_seq"]), self._dev(m["cu_q"]), self._dev(m["cu_k"]), m["max_q"], m["total_k"]]))
+        hidden = self.model(self._dev(m["input_ids"]), self._dev(m["positions"]), step)
+        for seq, n in portions:
+            seq.num_cached_tokens += n
+        if not rows:
+            return None
+        if rows != list(range(row)):
+            hidden = hidden[torch.tensor(rows, device=self.device)]
+        return self.model.compute_logits(hidden)
+
     def warmup_model(self, max_num_batched_tokens=16384, max_num_seqs=512):
         """One maximum-size prefill of dummy sequences without cache slots, as the reference does at start-up
         (engine/model_runner.py:107-121): loads every kernel, lets the GEMM library pick its solutions and sizes the
         allocator's pools, so that the first real prefill is not a cold start."""
+        if self.mixed_batches:
+            return                                                # nothing to size: state and cache pools are allocated, kernels load on first use
         num_seqs = max(1, min(max_num_batched_tokens // self.max_model_len, max_num_seqs))
         self.run([Sequence([0] * self.max_model_len) for _ in range(num_seqs)], True)
         torch.cuda.synchronize(self.device)
@@ -227,8 +319,13 @@ class DecodeSession:
         self.max_new_tokens = max_new_tokens
         self.steps_done = 0
         cfg = runner.cfg
-        h = tp_partition(cfg.num_attention_heads, cfg.num_key_value_heads, runner.world_size, runner.rank)[1]
-        ops.reserve_workspace(dev, ops.decode_workspace_bytes(b, h, cfg.head_dim, self.block_tables.shape[1], bs))
+        runner.model.reserve_decode_workspace(b, self.block_tables.shape[1], bs, dev)
+        self.step_meta = None
+        if runner.mixed_batches:
+            self.positions -= 1                                   # of the token that is fed (build_decode_meta has the reference's own convention)
+            slots = torch.tensor([s.state_slot for s in seqs], dtype=torch.int32)
+            chunks = torch.tensor([(i, 1, i, 0) for i in range(b)], dtype=torch.int32)
+            self.step_meta = StepMeta(b, self.slot_mapping, self.block_tables, slots.to(dev), chunks.to(dev), need_tokens)
         # the next step's embedding lookup rides in the arg-max launch when the model allows it: the session then owns the
         # embedded rows (row-major = the residual stream of the step, and in fragment order for layer 0's projection)
         self.fuse_embed = bool(getattr(runner.model, "fused_embedding_ok", lambda *_: False)(b, torch.device(dev)))
@@ -277,7 +374,9 @@ class DecodeSession:
     def _step(self):
         set_context(False, slot_mapping=self.slot_mapping, context_lens=self.context_lens, block_tables=self.block_tables)
         model = self.runner.model
-        if self.fuse_embed:
+        if self.step_meta is not None:
+            hidden = model(self.input_ids, self.positions, self.step_meta)
+        elif self.fuse_embed:
             hidden = model(self.input_ids, self.positions, embedded=(self.hidden_in, self.hidden_in_p))
         else:
             hidden = model(self.input_ids, self.positions)
@@ -299,7 +398,7 @@ class DecodeSession:
         reset_context()
 
     def _live(self):
-        return (self.input_ids, self.positions, self.context_lens, self.slot_mapping, self.tokens, self.step_idx, self.row_steps)
+        return (self.input_ids, self.positions, self.context_lens, self.slot_mapping, self.tokens, self.step_idx, self.row_steps, *self.runner.state.values())
 
     def _restore(self, saved):
         for t, s in zip(self._live(), saved):
@@ -362,14 +461,17 @@ class DecodeSession:
 
     def rewind(self, seqs_state):
         """Reset the device metadata to a saved state (benchmark use: time the same context window repeatedly)."""
-        for t, s in zip((self.input_ids, self.positions, self.context_lens, self.slot_mapping, self.step_idx, self.row_steps), seqs_state):
+        for t, s in zip(self._rewindable(), seqs_state):
             t.copy_(s)
         if self.fuse_embed:
             self._refresh_embedding()
         self.steps_done = int(self.row_steps.max().item())
 
+    def _rewindable(self):
+        return (self.input_ids, self.positions, self.context_lens, self.slot_mapping, self.step_idx, self.row_steps, *self.runner.state.values())
+
     def state(self):
-        return [t.clone() for t in (self.input_ids, self.positions, self.context_lens, self.slot_mapping, self.step_idx, self.row_steps)]
+        return [t.clone() for t in self._rewindable()]
 
     def finish(self):
         """Copy generated tokens back into the host sequences (one device->host sync for the whole generation)."""
@@ -378,4 +480,7 @@ class DecodeSession:
         for row in toks:
             for s, t in zip(self.seqs, row):
                 s.append_token(int(t))
+        if self.step_meta is not None:
+            for s in self.seqs:
+                s.num_cached_tokens = len(s) - 1
         return toks

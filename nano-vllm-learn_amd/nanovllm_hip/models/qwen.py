@@ -24,6 +24,7 @@ import torch.nn.functional as F
 from torch import nn
 
 from ..config import resolve_attention
+from ..layers.linear import linear
 
 
 @dataclass
@@ -44,6 +45,18 @@ class ModelConfig:
     max_position_embeddings: int = 32768
     attn_backend: str = "hip"
     kvcache_block_size: int = 256
+
+    @classmethod
+    def from_json(cls, d, **overrides):
+        """From a Hugging Face config.json (Qwen2ForCausalLM / Qwen3ForCausalLM)."""
+        qwen2 = d["architectures"][0].startswith("Qwen2")
+        heads = d["num_attention_heads"]
+        return cls(**{**dict(
+            name=d["architectures"][0], num_hidden_layers=d["num_hidden_layers"], hidden_size=d["hidden_size"], num_attention_heads=heads,
+            num_key_value_heads=d["num_key_value_heads"], head_dim=d.get("head_dim") or d["hidden_size"] // heads,
+            intermediate_size=d["intermediate_size"], vocab_size=d["vocab_size"], tie_word_embeddings=d.get("tie_word_embeddings", False),
+            qkv_bias=d.get("attention_bias", qwen2), qk_norm=not qwen2, rope_theta=d.get("rope_theta", 1000000.0),
+            rms_norm_eps=d.get("rms_norm_eps", 1e-6), max_position_embeddings=d.get("max_position_embeddings", 32768)), **overrides})
 
 
 # public HF config.json values (SURVEY.md App. A)
@@ -132,15 +145,6 @@ class RMSNorm(nn.Module):
             residual = x32.to(x.dtype)
         y = (x32 * torch.rsqrt(x32.pow(2).mean(dim=-1, keepdim=True) + self.eps)).to(x.dtype) * self.weight
         return y if residual is None else (y, residual)
-
-
-def linear(x, weight, bias=None):
-    """F.linear; decode-sized batches on the GPU take the weight-streaming HIP kernel (ops.linear_small_m), anything
-    else (prefill, CPU tests) goes to the vendor GEMM."""
-    if x.is_cuda and x.dtype == torch.bfloat16 and x.numel() // x.shape[-1] <= 64 and x.shape[-1] % 64 == 0 and weight.shape[0] % 16 == 0:
-        from .. import ops
-        return ops.linear_small_m(x, weight, bias)
-    return F.linear(x, weight, bias)
 
 
 def silu_and_mul(gate_up):
@@ -497,30 +501,71 @@ class QwenForCausalLM(nn.Module):
         """Deterministic N(0, 0.02) weights; every rank draws the full tensors and keeps its shard so that
         tp=N equals tp=1 on the same seed."""
         gen = torch.Generator(device="cpu").manual_seed(seed)
-        rank, tp = _tp()
         cfg = self.cfg
 
         def draw(*shape):
             return torch.randn(*shape, generator=gen) * 0.02
 
+        hq, hkv = cfg.num_attention_heads * cfg.head_dim, cfg.num_key_value_heads * cfg.head_dim
+        self.embed_tokens.weight.copy_(draw(cfg.vocab_size, cfg.hidden_size))
+        if not cfg.tie_word_embeddings:
+            self.lm_head.weight.copy_(draw(cfg.vocab_size, cfg.hidden_size))
+        for layer in self.layers:
+            qkv = draw(hq + 2 * hkv, cfg.hidden_size)
+            bias = draw(hq + 2 * hkv) if cfg.qkv_bias else None
+            o = draw(cfg.hidden_size, hq)
+            gate_up = draw(2 * cfg.intermediate_size, cfg.hidden_size)
+            self._fill_layer(layer, qkv, bias, o, gate_up, draw(cfg.hidden_size, cfg.intermediate_size))
+        return self
+
+    @torch.no_grad()
+    def load_weights(self, get):
+        """get(name) -> tensor under the Hugging Face names; every rank reads the full tensors and keeps its shard."""
+        cfg = self.cfg
+        self.embed_tokens.weight.copy_(get("model.embed_tokens.weight"))
+        self.norm.weight.copy_(get("model.norm.weight"))
+        if not cfg.tie_word_embeddings:
+            self.lm_head.weight.copy_(get("lm_head.weight"))
+        elif "lm_head.weight" in get:
+            get("lm_head.weight")                                  # a stored copy of the tied embedding
+        for i, layer in enumerate(self.layers):
+            p = f"model.layers.{i}."
+
+            def cat(names):
+                return torch.cat([get(p + n) for n in names])
+            qkv = ["self_attn.q_proj", "self_attn.k_proj", "self_attn.v_proj"]
+            self._fill_layer(layer, cat(n + ".weight" for n in qkv), cat(n + ".bias" for n in qkv) if cfg.qkv_bias else None,
+                             get(p + "self_attn.o_proj.weight"), cat(["mlp.gate_proj.weight", "mlp.up_proj.weight"]), get(p + "mlp.down_proj.weight"))
+            layer.input_layernorm.weight.copy_(get(p + "input_layernorm.weight"))
+            layer.post_attention_layernorm.weight.copy_(get(p + "post_attention_layernorm.weight"))
+            if cfg.qk_norm:
+                layer.self_attn.q_norm.weight.copy_(get(p + "self_attn.q_norm.weight"))
+                layer.self_attn.k_norm.weight.copy_(get(p + "self_attn.k_norm.weight"))
+        return self
+
+    def _fill_layer(self, layer, qkv, qkv_bias, o, gate_up, down):
+        """This rank's shard of one layer's full tensors."""
+        rank, tp = _tp()
+        cfg, a, m = self.cfg, layer.self_attn, layer.mlp
+        hq, hkv, d = cfg.num_attention_heads * cfg.head_dim, cfg.num_key_value_heads * cfg.head_dim, cfg.head_dim
         q0, qn, kv0, kvn = tp_partition(cfg.num_attention_heads, cfg.num_key_value_heads, tp, rank)
 
         def shard_qkv(full):                                       # rows of this rank's q heads | kv heads | kv heads
             wq, wk, wv = full.split([hq, hkv, hkv], dim=0)
             return torch.cat([wq[q0 * d:(q0 + qn) * d], wk[kv0 * d:(kv0 + kvn) * d], wv[kv0 * d:(kv0 + kvn) * d]], dim=0)
 
-        self.embed_tokens.weight.copy_(draw(cfg.vocab_size, cfg.hidden_size))
-        if not cfg.tie_word_embeddings:
-            self.lm_head.weight.copy_(draw(cfg.vocab_size, cfg.hidden_size))
-        hq, hkv, d = cfg.num_attention_heads * cfg.head_dim, cfg.num_key_value_heads * cfg.head_dim, cfg.head_dim
-        for layer in self.layers:
-            a, m = layer.self_attn, layer.mlp
-            a.qkv_proj.weight.copy_(shard_qkv(draw(hq + 2 * hkv, cfg.hidden_size)))
-            if cfg.qkv_bias:
-                a.qkv_proj.bias.copy_(shard_qkv(draw(hq + 2 * hkv)))
-            a.o_proj.weight.copy_(draw(cfg.hidden_size, hq)[:, q0 * d:(q0 + qn) * d])
-            pad = m.down_proj.weight.shape[1] - m.inter                   # zero rows / columns of a padded shard (QwenMLP)
-            gate_up = [F.pad(p.chunk(tp, dim=0)[rank], (0, 0, 0, pad)) for p in draw(2 * cfg.intermediate_size, cfg.hidden_size).chunk(2, dim=0)]
-            m.gate_up_proj.weight.copy_(torch.cat(gate_up, dim=0))
-            m.down_proj.weight.copy_(F.pad(draw(cfg.hidden_size, cfg.intermediate_size).chunk(tp, dim=1)[rank], (0, pad)))
-        return self
+        a.qkv_proj.weight.copy_(shard_qkv(qkv))
+        if qkv_bias is not None:
+            a.qkv_proj.bias.copy_(shard_qkv(qkv_bias))
+        a.o_proj.weight.copy_(o[:, q0 * d:(q0 + qn) * d])
+        pad = m.down_proj.weight.shape[1] - m.inter                   # zero rows / columns of a padded shard (QwenMLP)
+        parts = [F.pad(p.chunk(tp, dim=0)[rank], (0, 0, 0, pad)) for p in gate_up.chunk(2, dim=0)]
+        m.gate_up_proj.weight.copy_(torch.cat(parts, dim=0))
+        m.down_proj.weight.copy_(F.pad(down.chunk(tp, dim=1)[rank], (0, pad)))
+
+    def reserve_decode_workspace(self, batch, max_blocks, block_size, device):
+        """Allocate what a captured decode step must find in place."""
+        from .. import ops
+        rank, tp = _tp()
+        h = tp_partition(self.cfg.num_attention_heads, self.cfg.num_key_value_heads, tp, rank)[1]
+        ops.reserve_workspace(device, ops.decode_workspace_bytes(batch, h, self.cfg.head_dim, max_blocks, block_size))

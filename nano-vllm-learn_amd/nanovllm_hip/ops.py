@@ -378,7 +378,7 @@ _EPI_CODES = {"none": _lib.EPI_NONE, "silu_mul": _lib.EPI_SILU_MUL, "residual_ad
 
 
 def fused_linear(x, weight, *, bias=None, norm_weight=None, norm_eps=1e-6, norm_folded=False, epilogue="none", out=None, rope=None,
-                 x_packed_rows=None, out_packed=None, workspace=None, want_out=True, candidates=None, prefetch=None):
+                 x_packed_rows=None, out_packed=None, workspace=None, want_out=True, candidates=None, prefetch=None, glu=None):
     """nvh_linear_small_m_ex: x [M<=64, K] . weight[N, K]^T with an optional RMSNorm prologue and one of the epilogues
     "none" (+bias) | "silu_mul" | "residual_add" (out = the residual stream, updated in place) | "rope_store"
     (rope = dict(positions, cos_sin, k_cache, v_cache, slot_mapping, num_heads, num_kv_heads, head_dim); returns q [M, H*D]).
@@ -389,10 +389,13 @@ def fused_linear(x, weight, *, bias=None, norm_weight=None, norm_eps=1e-6, norm_
     per workgroup and row the best bf16 output and its column ("none" only) — with want_out=False the outputs themselves are
     never written (LM head + greedy arg-max in one pass; finish with greedy_advance_candidates).
     prefetch = a contiguous CUDA tensor the NEXT launch will stream (the following projection's weights): the CUs this launch
-    leaves idle read it into the caches first (a hint; results do not depend on it)."""
+    leaves idle read it into the caches first (a hint; results do not depend on it).
+    glu = (limit, alpha): "silu_mul" applies the clamped gated unit of clamped_glu() instead of SiLU(g) * u."""
     d, out = _linear_desc(x, weight, bias=bias, norm_weight=norm_weight, norm_eps=norm_eps, norm_folded=norm_folded, epilogue=epilogue, out=out,
                           rope=rope, x_packed_rows=x_packed_rows, out_packed=out_packed, workspace=workspace, want_out=want_out,
                           candidates=candidates, prefetch=prefetch)
+    if glu is not None:
+        d.glu_limit, d.glu_alpha = float(glu[0]), float(glu[1])
     rc = _lib.load().nvh_linear_small_m_ex(ctypes.byref(d), NVH_BF16, _stream())
     _lib.check(rc, "nvh_linear_small_m_ex")
     return out
@@ -571,3 +574,262 @@ def greedy_advance(logits, input_ids, positions, context_lens, slot_mapping, blo
                                         context_lens.data_ptr(), slot_mapping.data_ptr(), block_tables.data_ptr(), block_tables.stride(0),
                                         block_size, tokens_log.data_ptr(), tokens_log.stride(0), row_steps.data_ptr(), NVH_BF16, _stream())
     _lib.check(rc, "nvh_greedy_advance")
+
+
+# --------------------------------------------------------------------------------------- fp32-residual row ops, recurrence, latent attention
+def _act_code(*tensors):
+    """Activation type of a call: every tensor bf16, or every tensor fp32."""
+    dtype = tensors[0].dtype
+    for t in tensors:
+        if not t.is_cuda:
+            raise RuntimeError("the hip layers have no CPU path: GPU tensors only")
+        if t.dtype != dtype:
+            raise TypeError(f"activations and weights of one call share a type, got {dtype} and {t.dtype}")
+    return _out_code(dtype)
+
+
+def _require_f32(**tensors):
+    for name, t in tensors.items():
+        if not t.is_cuda or t.dtype != torch.float32 or not t.is_contiguous():
+            raise TypeError(f"{name} must be a contiguous fp32 GPU tensor, got {t.dtype} on {t.device}")
+
+
+def embed_rows(tokens, embed, scale, packed=None):
+    """(fp32 stream [rows, cols], the same in the activation type — the stream itself for fp32) = embed[tokens] * scale.  packed (bf16): the second
+    form in fragment order into this buffer instead."""
+    code = _act_code(embed)
+    assert tokens.dtype == torch.int64 and tokens.is_cuda and tokens.is_contiguous() and embed.is_contiguous()
+    rows, cols = tokens.numel(), embed.shape[1]
+    x = torch.empty((rows, cols), dtype=torch.float32, device=embed.device)
+    xb = torch.empty((rows, cols), dtype=embed.dtype, device=embed.device) if embed.dtype != torch.float32 and packed is None else None
+    if packed is not None:
+        _require_gpu_bf16(embed=embed, packed=packed)
+        assert packed.is_contiguous() and packed.numel() >= ((rows + 15) // 16) * 16 * cols
+    rc = _lib.load().nvh_embed_rows(x.data_ptr(), xb.data_ptr() if xb is not None else None, packed.data_ptr() if packed is not None else None, tokens.data_ptr(), embed.data_ptr(), float(scale), rows, cols,
+                                    embed.shape[0], code, _stream())
+    _lib.check(rc, "nvh_embed_rows")
+    return x, xb if xb is not None else x
+
+
+def norm_residual(x, weight, eps, n, dtype, y=None, packed=None, want_rows=True):
+    """y given: x (fp32 stream, in place) += rmsnorm(y) * weight; returns the new stream in `dtype` (x itself for fp32).  y None: returns
+    rmsnorm(x) * weight in `dtype`, x unchanged.  The mean runs over the first n columns; packed (bf16): the rows also in fragment order."""
+    _require_f32(x=x, weight=weight)
+    rows, cols = x.shape
+    assert weight.numel() == cols
+    xb = None
+    if want_rows and (dtype != torch.float32 or y is None):
+        xb = torch.empty((rows, cols), dtype=dtype, device=x.device)
+    d = _lib.NormResidualDesc()
+    d.x, d.w, d.eps, d.rows, d.cols, d.n = x.data_ptr(), weight.data_ptr(), float(eps), rows, cols, int(n)
+    d.xb = xb.data_ptr() if xb is not None else None
+    if packed is not None:
+        _require_gpu_bf16(packed=packed)
+        assert packed.is_contiguous() and packed.numel() >= ((rows + 15) // 16) * 16 * cols
+        d.packed = packed.data_ptr()
+    if y is not None:
+        assert y.shape == x.shape and y.stride(1) == 1 and y.dtype == dtype and y.is_cuda
+        d.y, d.y_stride = y.data_ptr(), y.stride(0)
+    _lib.check(_lib.load().nvh_norm_residual(ctypes.byref(d), _out_code(dtype), _stream()), "nvh_norm_residual")
+    return xb if xb is not None else x
+
+
+def clamped_glu(gate_up, limit, alpha):
+    """g sigmoid(alpha g) (u + 1) with g = min(gate, limit), u = clamp(up, -limit, limit); rows hold gate | up."""
+    code = _act_code(gate_up)
+    inter = gate_up.shape[1] // 2
+    assert gate_up.dim() == 2 and gate_up.stride(1) == 1
+    out = torch.empty((gate_up.shape[0], inter), dtype=gate_up.dtype, device=gate_up.device)
+    rc = _lib.load().nvh_clamped_glu(out.data_ptr(), gate_up.data_ptr(), gate_up.shape[0], inter, gate_up.stride(0), out.stride(0), float(limit), float(alpha),
+                                     code, _stream())
+    _lib.check(rc, "nvh_clamped_glu")
+    return out
+
+
+def rglru_chunk_tokens() -> int:
+    return int(_lib.load().nvh_rglru_chunk_tokens())
+
+
+def rglru_step_supported(block) -> bool:
+    return bool(_lib.load().nvh_rglru_step_supported(int(block)))
+
+
+def _rglru_desc(yx, p, positions, state_slots, state, conv_state):
+    code = _act_code(yx, p["ra"], p["ri"], conv_state)
+    blocks, block, _ = p["ra"].shape
+    width = blocks * block
+    taps = p["conv_w"].shape[0]
+    _require_f32(conv_w=p["conv_w"], conv_b=p["conv_b"], ra_b=p["ra_b"], ri_b=p["ri_b"], rate=p["rate"], state=state)
+    _require_i32(state_slots=state_slots)
+    assert yx.stride(1) == 1 and yx.shape[1] == 2 * width and p["ra"].is_contiguous() and p["ri"].is_contiguous() and p["ri"].shape == p["ra"].shape
+    assert p["conv_w"].shape == (taps, width) and all(p[n].numel() == width for n in ("conv_b", "ra_b", "ri_b", "rate"))
+    assert state.shape[1] == width and conv_state.shape == (state.shape[0], taps, width) and conv_state.is_contiguous()
+    assert positions.dtype == torch.int64 and positions.is_contiguous() and positions.numel() == yx.shape[0]
+    d = _lib.RglruDesc()
+    d.yx, d.yx_stride, d.width, d.block, d.blocks, d.taps = yx.data_ptr(), yx.stride(0), width, block, blocks, taps
+    d.conv_w, d.conv_b, d.ra, d.ri = p["conv_w"].data_ptr(), p["conv_b"].data_ptr(), p["ra"].data_ptr(), p["ri"].data_ptr()
+    d.ra_b, d.ri_b, d.rate = p["ra_b"].data_ptr(), p["ri_b"].data_ptr(), p["rate"].data_ptr()
+    d.positions, d.state_slots, d.state, d.conv_state = positions.data_ptr(), state_slots.data_ptr(), state.data_ptr(), conv_state.data_ptr()
+    return d, width, code
+
+
+def rglru_chunks(yx, params, positions, state_slots, chunks, state, conv_state, out=None, generic=False):
+    """Gated linear recurrence over portions of sequences.  yx [rows, 2 * width] = gate branch | recurrent branch; params = dict(conv_w [taps, width],
+    conv_b, ra / ri [blocks, block, block], ra_b, ri_b, rate); chunks int32 [n, 4] = (first row, rows, sequence, index in its portion), built by
+    the host from portions cut every rglru_chunk_tokens() tokens.  state [slots, width] fp32 and conv_state [slots, taps, width] are updated.
+    Rows no chunk covers are left alone in `out` (they belong to another launch)."""
+    d, width, code = _rglru_desc(yx, params, positions, state_slots, state, conv_state)
+    _require_i32(chunks=chunks)
+    assert chunks.dim() == 2 and chunks.shape[1] == 4 and chunks.is_contiguous()
+    rows = yx.shape[0]
+    if out is None:
+        out = torch.empty((rows, width), dtype=yx.dtype, device=yx.device)
+    assert out.shape == (rows, width) and out.stride(1) == 1 and out.dtype == yx.dtype
+    scratch = torch.empty((2, rows, width), dtype=torch.float32, device=yx.device)
+    d.chunks, d.n_chunks, d.s_loc, d.a_cum = chunks.data_ptr(), chunks.shape[0], scratch[0].data_ptr(), scratch[1].data_ptr()
+    d.out, d.out_stride = out.data_ptr(), out.stride(0)
+    _lib.check(_lib.load().nvh_rglru_chunks(ctypes.byref(d), int(generic), code, _stream()), "nvh_rglru_chunks")
+    return out
+
+
+def rglru_step(yx, params, positions, state_slots, state, conv_state, out=None, out_packed=None, want_out=True):
+    """One new token per sequence (row i = sequence i), the whole recurrence in one launch (bf16).  out_packed: also in fragment order."""
+    d, width, code = _rglru_desc(yx, params, positions, state_slots, state, conv_state)
+    rows = yx.shape[0]
+    assert state_slots.numel() >= rows
+    if out is None and want_out:
+        out = torch.empty((rows, width), dtype=yx.dtype, device=yx.device)
+    if out is not None:
+        assert out.shape == (rows, width) and out.stride(1) == 1 and out.dtype == yx.dtype
+        d.out, d.out_stride = out.data_ptr(), out.stride(0)
+    if out_packed is not None:
+        _require_gpu_bf16(out_packed=out_packed)
+        assert out_packed.is_contiguous() and out_packed.numel() >= ((rows + 15) // 16) * 16 * width
+        d.out_packed = out_packed.data_ptr()
+    _lib.check(_lib.load().nvh_rglru_step(ctypes.byref(d), rows, code, _stream()), "nvh_rglru_step")
+    return out
+
+
+def latent_prep(a, q_rank, q_weight, eps, positions, cos_sin, kv_rank=0, kv_weight=None, cache=None, slots=None, cq_packed=None):
+    """Row ops behind the down-projections: returns the normed query latent [rows, q_cols]; with `cache` given also norms the key latent, rotates the
+    shared key part and stores the row.  `a` rows: query latent (q_cols) | key latent (kv_cols) | shared key part (rot_cols)."""
+    code = _act_code(a)
+    rows, q_cols = a.shape[0], q_weight.numel()
+    _require_f32(q_weight=q_weight, cos_sin=cos_sin)
+    assert a.stride(1) == 1 and positions.dtype == torch.int64 and positions.is_contiguous() and positions.numel() == rows
+    d = _lib.LatentPrepDesc()
+    d.a, d.a_stride, d.rows, d.q_rank, d.q_cols, d.q_w, d.eps = a.data_ptr(), a.stride(0), rows, q_rank, q_cols, q_weight.data_ptr(), float(eps)
+    cq = None
+    if cq_packed is None:
+        cq = torch.empty((rows, q_cols), dtype=a.dtype, device=a.device)
+        d.cq = cq.data_ptr()
+    else:
+        _require_gpu_bf16(cq_packed=cq_packed)
+        assert cq_packed.is_contiguous() and cq_packed.numel() >= ((rows + 15) // 16) * 16 * q_cols
+        d.cq_packed = cq_packed.data_ptr()
+    if cache is not None:
+        _require_f32(kv_weight=kv_weight)
+        _require_i32(slots=slots)
+        _act_code(a, cache)
+        kv_cols = kv_weight.numel()
+        assert cache.is_contiguous() and slots.numel() == rows and slots.is_contiguous() and a.shape[1] >= q_cols + cache.shape[-1]
+        d.kv_rank, d.kv_cols, d.kv_w, d.rot, d.rot_cols = kv_rank, kv_cols, kv_weight.data_ptr(), cos_sin.shape[1], cache.shape[-1] - kv_cols
+        d.cache, d.slots, d.positions, d.cos_sin, d.max_position = cache.data_ptr(), slots.data_ptr(), positions.data_ptr(), cos_sin.data_ptr(), cos_sin.shape[0]
+    _lib.check(_lib.load().nvh_latent_prep(ctypes.byref(d), code, _stream()), "nvh_latent_prep")
+    return cq
+
+
+def latent_attend_mfma(kv_cols, rot_cols, block_size) -> bool:
+    return bool(_lib.load().nvh_latent_attend_mfma(kv_cols, rot_cols, block_size))
+
+
+def latent_splits(rows, heads, max_context, mfma) -> int:
+    """Context splits of one latent-attention launch: two workgroups per CU where the context is long enough to share."""
+    per_row = (heads + 15) // 16 if mfma else heads
+    return max(1, min(512 // max(1, rows * per_row), (max_context + 63) // 64, 64))
+
+
+def latent_attention(q, cache, block_tables, positions, cos_sin, w_uk, w_uv, scale, rot, max_context, row_seq=None, out=None, out_packed=None, want_out=True,
+                     splits=None, generic=False):
+    """Causal latent attention of single rows (row i attends positions 0 .. positions[i] of sequence row_seq[i], or i): q [rows, heads, dim_cols +
+    qrot_cols] unrotated | rotated part (turned here); cache pages [blocks, block_size, kv_cols + rot_cols]; w_uk [heads, kv_cols, dim_cols],
+    w_uv [heads, v_cols, kv_cols].  Returns [rows, heads * v_cols].  generic=True forces the plain kernel (tests)."""
+    code = _act_code(q, cache, w_uk, w_uv)
+    rows = q.shape[0]
+    heads, kv_cols, dim_cols = w_uk.shape
+    v_cols, cols, block_size = w_uv.shape[1], cache.shape[2], cache.shape[1]
+    _require_f32(cos_sin=cos_sin)
+    _require_i32(block_tables=block_tables)
+    assert q.dim() == 2 and q.stride(1) == 1 and q.shape[1] % heads == 0 and w_uk.is_contiguous() and w_uv.is_contiguous() and cache.is_contiguous()
+    assert w_uv.shape == (heads, v_cols, kv_cols) and block_tables.dim() == 2 and block_tables.stride(1) == 1
+    assert positions.dtype == torch.int64 and positions.is_contiguous() and positions.numel() == rows
+    mfma = code == NVH_BF16 and row_seq is None and not generic and latent_attend_mfma(kv_cols, cols - kv_cols, block_size)
+    splits = splits or latent_splits(rows, heads, max_context, mfma)
+    qa = torch.empty((rows, heads, cols), dtype=q.dtype, device=q.device)
+    part_o = torch.empty((rows, splits, heads, kv_cols), dtype=torch.float32, device=q.device)
+    part_ml = torch.empty((rows, splits, heads, 2), dtype=torch.float32, device=q.device)
+    if out is None and want_out:
+        out = torch.empty((rows, heads * v_cols), dtype=q.dtype, device=q.device)
+    d = _lib.LatentAttnDesc()
+    d.q, d.q_stride, d.rows, d.heads, d.dim_cols, d.qrot_cols = q.data_ptr(), q.stride(0), rows, heads, dim_cols, q.shape[1] // heads - dim_cols
+    d.cache, d.kv_cols, d.rot, d.rot_cols, d.block_size = cache.data_ptr(), kv_cols, int(rot), cols - kv_cols, block_size
+    d.block_tables, d.bt_stride, d.max_blocks = block_tables.data_ptr(), block_tables.stride(0), block_tables.shape[1]
+    if row_seq is not None:
+        _require_i32(row_seq=row_seq)
+        assert row_seq.numel() == rows and row_seq.is_contiguous()
+        d.row_seq = row_seq.data_ptr()
+    else:
+        assert block_tables.shape[0] >= rows
+    d.positions, d.cos_sin, d.max_position = positions.data_ptr(), cos_sin.data_ptr(), cos_sin.shape[0]
+    d.w_uk, d.w_uv, d.v_cols, d.scale = w_uk.data_ptr(), w_uv.data_ptr(), v_cols, float(scale)
+    d.qa, d.part_o, d.part_ml, d.splits = qa.data_ptr(), part_o.data_ptr(), part_ml.data_ptr(), splits
+    if out is not None:
+        assert out.shape == (rows, heads * v_cols) and out.stride(1) == 1 and out.dtype == q.dtype
+        d.out, d.out_stride = out.data_ptr(), out.stride(0)
+    if out_packed is not None:
+        _require_gpu_bf16(out_packed=out_packed)
+        assert out_packed.is_contiguous() and out_packed.numel() >= ((rows + 15) // 16) * 16 * heads * v_cols
+        d.out_packed = out_packed.data_ptr()
+    _lib.check(_lib.load().nvh_latent_attention(ctypes.byref(d), int(generic), code, _stream()), "nvh_latent_attention")
+    return out
+
+
+def latent_gather(cache, cu_k, total, block_tables):
+    """The cache rows of every key of the sequences, packed [total, cols]."""
+    code = _act_code(cache)
+    _require_i32(cu_k=cu_k, block_tables=block_tables)
+    batch = cu_k.numel() - 1
+    assert cache.is_contiguous() and cu_k.is_contiguous() and block_tables.shape[0] >= batch and block_tables.stride(1) == 1
+    out = torch.empty((total, cache.shape[2]), dtype=cache.dtype, device=cache.device)
+    rc = _lib.load().nvh_latent_gather(out.data_ptr(), cache.data_ptr(), cu_k.data_ptr(), block_tables.data_ptr(), block_tables.stride(0), batch, total,
+                                       cache.shape[2], cache.shape[1], code, _stream())
+    _lib.check(rc, "nvh_latent_gather")
+    return out
+
+
+def latent_prefill_supported(dk, dv) -> bool:
+    return bool(_lib.load().nvh_latent_prefill_supported(dk, dv))
+
+
+def latent_prefill(q, k, k_rot, v, cu_q, cu_k, max_q, positions, cos_sin, scale, out=None):
+    """Causal attention of prompt portions in expanded form: q [rows, heads, dk] (rotated part not turned yet), k [keys, heads, dim_cols], k_rot
+    [keys, >= dk - dim_cols] shared by the heads, v [keys, heads, dv] (all with any row stride).  Returns [rows, heads * dv] (bf16)."""
+    _require_gpu_bf16(q=q, k=k, k_rot=k_rot, v=v)
+    _require_i32(cu_q=cu_q, cu_k=cu_k)
+    _require_f32(cos_sin=cos_sin)
+    rows, heads, dk = q.shape
+    dim_cols, dv = k.shape[2], v.shape[2]
+    assert k.shape[1] == heads and v.shape[1] == heads and q.stride(1) == dk and k.stride(1) == dim_cols and v.stride(1) == dv
+    assert q.stride(2) == 1 and k.stride(2) == 1 and v.stride(2) == 1 and k_rot.stride(1) == 1 and k_rot.shape[1] >= dk - dim_cols
+    assert positions.dtype == torch.int64 and positions.is_contiguous() and positions.numel() == rows and cu_q.numel() == cu_k.numel()
+    if out is None:
+        out = torch.empty((rows, heads * dv), dtype=torch.bfloat16, device=q.device)
+    assert out.shape == (rows, heads * dv) and out.stride(1) == 1
+    d = _lib.LatentPrefillDesc()
+    d.q, d.k, d.k_rot, d.v, d.out = q.data_ptr(), k.data_ptr(), k_rot.data_ptr(), v.data_ptr(), out.data_ptr()
+    d.q_stride, d.k_stride, d.kr_stride, d.v_stride, d.out_stride = q.stride(0), k.stride(0), k_rot.stride(0), v.stride(0), out.stride(0)
+    d.cu_q, d.cu_k, d.positions, d.cos_sin, d.max_position, d.rot = (cu_q.data_ptr(), cu_k.data_ptr(), positions.data_ptr(), cos_sin.data_ptr(),
+                                                                     cos_sin.shape[0], cos_sin.shape[1])
+    d.batch, d.heads, d.dim_cols, d.dk, d.dv, d.max_q, d.scale_log2 = cu_q.numel() - 1, heads, dim_cols, dk, dv, int(max_q), float(scale) * 1.4426950408889634
+    _lib.check(_lib.load().nvh_latent_prefill(ctypes.byref(d), NVH_BF16, _stream()), "nvh_latent_prefill")
+    return out
