@@ -31,6 +31,11 @@ class Scheduler:
             self.state_slots.deallocate(seq)
         return False
 
+    def _acquire_whole(self, seq):
+        """Blocks for the prompt and, while the pool has them, for everything the sequence will generate: a block table that never changes
+        gives every decode step the same launch geometry."""
+        return self.acquire(seq, len(seq) + seq.max_tokens - seq.num_completion_tokens) or self.acquire(seq, len(seq))
+
     def release(self, seq):
         self.block_manager.deallocate(seq)                      # (num_cached_tokens back to zero)
         if self.state_slots is not None:
@@ -57,7 +62,7 @@ class Scheduler:
         """[(sequence, tokens of it that run now)] with blocks and slots in place."""
         batch, budget = [], self.max_num_batched_tokens
         if not self.mixed:
-            while self.waiting and len(self.running) < self.max_num_seqs and len(self.waiting[0]) <= budget and self.acquire(self.waiting[0], len(self.waiting[0])):
+            while self.waiting and len(self.running) < self.max_num_seqs and len(self.waiting[0]) <= budget and self._acquire_whole(self.waiting[0]):
                 seq = self.waiting.popleft()
                 self.running.append(seq)
                 batch.append((seq, len(seq)))
