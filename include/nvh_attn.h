@@ -460,8 +460,8 @@ int nvh_norm_residual(const nvh_norm_residual_desc* d, int dtype, void* stream);
 int nvh_clamped_glu(void* out, const void* gate_up, int rows, int inter, int64_t gate_up_row_stride, int64_t out_row_stride, float limit, float alpha,
                     int dtype, void* stream);
 /* Real-gated linear recurrent unit behind a causal depthwise convolution: log a = -rate sigmoid(ra u), S = a S + sqrt(1 - a^2) sigmoid(ri u) u,
- * out = S gelu(y).  nvh_rglru_chunks: portions of prompts (and single tokens), cut by the caller into chunks of at most nvh_rglru_chunk_tokens()
- * tokens; chunks of one portion are consecutive.  nvh_rglru_step: row i is one new token of sequence i (bf16; nvh_rglru_step_supported(block)).
+ * out = S gelu(y).  nvh_rglru_chunks: portions of prompts (and single tokens), cut by the caller into segments that are
+ * scanned side by side; segments of one portion are consecutive.  nvh_rglru_step: row i is one new token of sequence i (bf16; nvh_rglru_step_supported(block)).
  * generic != 0 forces the plain kernel (tests). */
 typedef struct nvh_rglru_desc {
     const void* yx;              /* [rows, 2 * width]: gate branch | recurrent branch (biases added), row stride yx_stride */
@@ -475,14 +475,16 @@ typedef struct nvh_rglru_desc {
     const float* ra_b;           /* [width] */
     const float* ri_b;
     const float* rate;           /* [width]: log a = -rate * r */
-    const int32_t* chunks;       /* [n_chunks, 4]: first row, rows (<= nvh_rglru_chunk_tokens()), sequence, index of the chunk in its sequence's portion */
+    const int32_t* chunks;       /* [n_chunks, 4]: first row, rows, sequence, index of the segment in its sequence's portion */
     int32_t n_chunks;
+    int32_t segment;             /* tokens of every segment but a portion's last; a multiple of nvh_rglru_chunk_tokens() */
+    int32_t summaries;           /* != 0: some portion has more than one segment */
     const int64_t* positions;    /* [rows] */
     const int32_t* state_slots;  /* [sequences]; < 0: nothing is read or kept */
     float* state;                /* [slots, width] */
     void* conv_state;            /* [slots, taps, width]: input of position p at ring entry p % taps */
-    float* s_loc;                /* [rows, width] scratch: scan inside the chunk */
-    float* a_cum;                /* [rows, width] scratch: product of the decays since the chunk began */
+    float* s_loc;                /* [n_chunks, width] scratch: value at a segment's end */
+    float* a_cum;                /* [n_chunks, width] scratch: product of a segment's decays */
     void* out;                   /* [rows, width]: S * gelu(y), row stride out_stride */
     int64_t out_stride;
     void* out_packed;            /* nullable (bf16, step form): the result in MFMA-fragment order */

@@ -76,6 +76,7 @@ int nvh_rglru_chunks(const nvh_rglru_desc* d, int generic, int dtype, void* stre
     const int rc = check_rglru("rglru_chunks", d, dtype);
     if (rc) return rc;
     REQUIRE(d->chunks && d->s_loc && d->a_cum && d->out && d->n_chunks > 0, NVH_E_NULL, "rglru_chunks: null pointer");
+    REQUIRE(d->segment > 0 && d->segment % kRglruChunk == 0, NVH_E_SHAPE, "rglru_chunks: segment %d must be a positive multiple of %d", d->segment, kRglruChunk);
     REQUIRE(!d->out_packed, NVH_E_SHAPE, "rglru_chunks: packed output belongs to the step form");
     REQUIRE(aligned16(d->s_loc) && aligned16(d->a_cum), NVH_E_ALIGN, "rglru_chunks: scratch must be 16-byte aligned");
     return launch_rglru_chunks(*d, dtype == NVH_F32, generic, (hipStream_t)stream);
@@ -118,7 +119,7 @@ int nvh_latent_attention(const nvh_latent_attn_desc* d, int generic, int dtype, 
             NVH_E_NULL, "latent_attention: null pointer");
     REQUIRE(d->rows > 0 && d->heads > 0 && d->dim_cols % 8 == 0 && d->dim_cols > 0 && d->qrot_cols >= d->rot && d->qrot_cols % 8 == 0 && d->kv_cols > 0 && d->kv_cols % 8 == 0 &&
             d->kv_cols <= 2048 && d->rot % 2 == 0 && d->rot <= d->rot_cols && d->rot_cols % 8 == 0 && d->v_cols > 0 && d->v_cols % 8 == 0 && d->block_size > 0 &&
-            d->splits >= 1 && d->splits <= 1024 && d->max_position > 0 && d->max_blocks > 0, NVH_E_SHAPE,
+            d->splits >= 1 && d->splits <= 64 && d->max_position > 0 && d->max_blocks > 0, NVH_E_SHAPE,
             "latent_attention: heads %d dim %d rot %d/%d/%d latent %d value %d page %d splits %d", d->heads, d->dim_cols, d->rot, d->qrot_cols, d->rot_cols, d->kv_cols,
             d->v_cols, d->block_size, d->splits);
     REQUIRE(!d->out_packed || (dtype == NVH_BF16 && d->v_cols % 16 == 0 && d->kv_cols % 32 == 0 && (d->heads * d->v_cols) % 32 == 0), NVH_E_SHAPE,

@@ -46,7 +46,7 @@ int launch_norm_residual(const NormResidualArgs& a, int f32, hipStream_t stream)
 int launch_clamped_glu(void* out, const void* gate_up, int rows, int inter, int64_t gu_stride, int64_t out_stride, float limit, float alpha, int f32, hipStream_t stream);
 
 // ---- gated linear recurrence (rglru.hip)
-constexpr int kRglruChunk = 64;  // tokens of one sequence one workgroup scans
+constexpr int kRglruChunk = 64;  // tokens a workgroup scans at a time
 using RglruArgs = nvh_rglru_desc;
 int launch_rglru_chunks(const RglruArgs& a, int f32, int generic, hipStream_t stream);
 int launch_rglru_step(const RglruArgs& a, int rows, hipStream_t stream);

@@ -17,38 +17,56 @@ namespace {
 typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
 
 // ------------------------------------------------------------------------------------------------ prep
+__device__ __forceinline__ float wave_sum(float v) {
+    v = group_sum<16>(v);
+    v = sum_xor16(v);
+    return sum_xor32(v);
+}
+__device__ __forceinline__ float dot4(f32x4 v) { return v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3]; }
+
+// one wave norms one row part: out(column, 4 values).  Pieces of 4 columns, the first RC per lane kept in registers between the two passes
+template <typename T, typename Out>
+__device__ __forceinline__ void norm_part(const T* x, int cols, int n, float eps, const float* w, int lane, Out out) {
+    constexpr int RC = 6;
+    f32x4 keep[RC];
+    float ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < RC; ++i) {
+        const int c = (lane + 64 * i) * 4;
+        keep[i] = c < cols ? act_ld4(x + c) : f32x4{0.f, 0.f, 0.f, 0.f};
+    }
+#pragma unroll
+    for (int i = 0; i < RC; ++i) ss += dot4(keep[i]);
+    for (int c = (lane + 64 * RC) * 4; c < cols; c += 256) ss += dot4(act_ld4(x + c));
+    const float inv = 1.f / sqrtf(wave_sum(ss) / n + eps);
+#pragma unroll
+    for (int i = 0; i < RC; ++i) {
+        const int c = (lane + 64 * i) * 4;
+        if (c < cols) out(c, keep[i] * inv * *reinterpret_cast<const f32x4*>(w + c));
+    }
+    for (int c = (lane + 64 * RC) * 4; c < cols; c += 256) out(c, act_ld4(x + c) * inv * *reinterpret_cast<const f32x4*>(w + c));
+}
+
+// one wave per row, four rows per workgroup: no barrier
 template <typename T>
 __global__ __launch_bounds__(256) void latent_prep_kernel(const LatentPrepArgs a) {
-    __shared__ float lds[8];
-    const int row = blockIdx.x;
+    const int row = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
+    if (row >= a.rows) return;
     const T* x = reinterpret_cast<const T*>(a.a) + (int64_t)row * a.a_stride;
     const T* c = x + a.q_cols;
-    float sq = 0.f, sc = 0.f;
-    for (int i = threadIdx.x * 4; i < a.q_cols; i += 1024) {
-        const f32x4 v = act_ld4(x + i);
-        sq += v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3];
-    }
-    for (int i = threadIdx.x * 4; i < a.kv_cols; i += 1024) {
-        const f32x4 v = act_ld4(c + i);
-        sc += v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3];
-    }
-    const float iq = 1.f / sqrtf(block_sum256(sq, lds) / a.q_rank + a.eps);
-    for (int i = threadIdx.x * 4; i < a.q_cols; i += 1024) {
-        const f32x4 v = act_ld4(x + i) * iq * *reinterpret_cast<const f32x4*>(a.q_w + i);
+    norm_part<T>(x, a.q_cols, a.q_rank, a.eps, a.q_w, lane, [&](int i, f32x4 v) {
         if (a.cq_packed) act_st4(reinterpret_cast<uint16_t*>(a.cq_packed) + pack_index(row, i, a.q_cols), v);
         else act_st4(reinterpret_cast<T*>(a.cq) + (int64_t)row * a.q_cols + i, v);
-    }
-    if (a.kv_cols == 0) return;                      // (uniform over the launch)
-    const float ic = 1.f / sqrtf(block_sum256(sc, lds + 4) / a.kv_rank + a.eps);
+    });
+    if (a.kv_cols == 0) return;
     const int slot = a.slots[row];
     if (slot < 0) return;
     T* out = reinterpret_cast<T*>(a.cache) + (int64_t)slot * (a.kv_cols + a.rot_cols);
-    for (int i = threadIdx.x * 4; i < a.kv_cols; i += 1024)
-        act_st4(out + i, act_ld4(c + i) * ic * *reinterpret_cast<const f32x4*>(a.kv_w + i));
+    norm_part<T>(c, a.kv_cols, a.kv_rank, a.eps, a.kv_w, lane, [&](int i, f32x4 v) { act_st4(out + i, v); });
     int64_t pos = a.positions[row];
     if (pos >= a.max_position) pos = a.max_position - 1;
     const float* cs = a.cos_sin + pos * a.rot;
-    for (int i = threadIdx.x; i < a.rot / 2; i += 256) {
+    for (int i = lane; i < a.rot / 2; i += 64) {
         const float u = act_ld(c + a.kv_cols + 2 * i), v = act_ld(c + a.kv_cols + 2 * i + 1), co = cs[i], si = cs[a.rot / 2 + i];
         act_st(out + a.kv_cols + 2 * i, u * co - v * si);
         act_st(out + a.kv_cols + 2 * i + 1, v * co + u * si);
@@ -193,7 +211,12 @@ __global__ __launch_bounds__(256) void latent_attend_generic_kernel(const Latent
 // grid (splits, rows, head tiles of 16), 4 waves.  64 keys at a time in ONE LDS image that serves as K (row reads) and as V (hardware-transposed
 // reads): wave w scores keys 16 w .. + 15 for all 16 heads (queries in registers), the waves agree on the tile's maxima through LDS, weights go to
 // LDS as bf16 hi + lo in the order the transposed reads deliver keys, and wave w sums its quarter of the latent columns.
-// Two workgroups per CU (one image each) cover each other's load and compute phases.
+// Two images: the next tile's DMA is issued behind the barrier that finds this tile landed, and travels under its whole computation.
+__device__ __forceinline__ void lds_only_barrier() {     // (a __syncthreads() would drain the DMA in flight)
+    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+    __builtin_amdgcn_s_barrier();
+    asm volatile("" ::: "memory");
+}
 template <int OFF>
 __device__ __forceinline__ u32x2 ds_read_tr16(uint32_t lds_addr) {
     u32x2 r;
@@ -206,10 +229,10 @@ template <int NT>                                    // kv_cols = 64 * NT, rot_c
 __global__ __launch_bounds__(256) void latent_attend_kernel(const LatentAttnArgs a) {
     constexpr int COLS = 64 * NT + 64, ROWB = COLS * 2, CPR = COLS / 8, KS = COLS / 32, NI = CPR / 4;   // NI: DMA instructions per wave
     constexpr bool kOdd = ((ROWB / 128) & 1) != 0;
-    extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
-    unsigned char* img = smem;                       // [64][ROWB], 16-byte pieces swizzled inside groups of 8
-    uint16_t* p_lds = reinterpret_cast<uint16_t*>(smem + 64 * ROWB);             // [hi | lo][16 heads][64 + 8]
-    float* mx_lds = reinterpret_cast<float*>(smem + 64 * ROWB + 2 * 16 * 72 * 2);  // [4 waves][16]
+    constexpr int IMG = 64 * ROWB;
+    extern __shared__ __attribute__((aligned(16))) unsigned char smem[];       // [2 images][64][ROWB], 16-byte pieces swizzled inside groups of 8
+    uint16_t* p_lds = reinterpret_cast<uint16_t*>(smem + 2 * IMG);               // [hi | lo][16 heads][64 + 8]
+    float* mx_lds = reinterpret_cast<float*>(smem + 2 * IMG + 2 * 16 * 72 * 2);  // [4 waves][16]
     const int split = blockIdx.x, row = blockIdx.y, h0 = blockIdx.z * 16;
     const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lq = lane & 15, lg = lane >> 4;
     const int ctx = (int)a.positions[row] + 1;
@@ -227,7 +250,8 @@ __global__ __launch_bounds__(256) void latent_attend_kernel(const LatentAttnArgs
     auto swz = [](int r) { return kOdd ? ((r >> 1) & 7) : (r & 7); };
     const uint16_t* cache = reinterpret_cast<const uint16_t*>(a.cache);
     // staging: piece s of the image -> (row s / CPR, place s % CPR); the source piece is the place with its low three bits xor-ed
-    auto stage = [&](int t0) {
+    auto stage = [&](int t0, int buf) {
+        unsigned char* img = smem + buf * IMG;
         const int64_t page = a.block_tables[row * a.bt_stride + t0 / a.block_size];          // 64 divides the page: one page per tile
         const uint16_t* base = cache + (page * a.block_size + t0 % a.block_size) * COLS;
         const int live = k1 - t0 < 64 ? k1 - t0 : 64;
@@ -240,7 +264,7 @@ __global__ __launch_bounds__(256) void latent_attend_kernel(const LatentAttnArgs
                                              (__attribute__((address_space(3))) void*)(img + (wave * NI + j) * 1024), 16, 0, 0);
         }
     };
-    stage(k0);
+    stage(k0, 0);
     bf16x8 qf[KS];                                   // B operand: column = head lq, 8 consecutive columns
     {
         const uint16_t* q = reinterpret_cast<const uint16_t*>(a.qa) + ((int64_t)row * a.heads + (head_ok ? h0 + lq : a.heads - 1)) * COLS + 8 * lg;
@@ -254,9 +278,12 @@ __global__ __launch_bounds__(256) void latent_attend_kernel(const LatentAttnArgs
     const float sc = a.scale * kLog2e;
     // transposed reads: lane 4 q + p of a 16-lane group addresses key row 4 lg + q (+ 16), columns 4 p .. of the 16-column tile
     const int vr = 4 * lg + (lq >> 2), vp = lq & 3;
-    for (int t0 = k0; t0 < k1; t0 += 64) {
+    auto tile_body = [&](auto bufc, const int t0) {
+        constexpr int buf = decltype(bufc)::value;
+        const unsigned char* img = smem + buf * IMG;
         asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
-        __syncthreads();
+        lds_only_barrier();                          // the tile is in LDS, and every wave is done with the one before it
+        if (t0 + 64 < k1) stage(t0 + 64, buf ^ 1);
         const int R = 16 * wave + lq;
         f32x4 s4 = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
@@ -273,7 +300,7 @@ __global__ __launch_bounds__(256) void latent_attend_kernel(const LatentAttnArgs
         mx = fmaxf(mx, __shfl_xor(mx, 16));
         mx = fmaxf(mx, __shfl_xor(mx, 32));
         if (lg == 0) mx_lds[wave * 16 + lq] = mx;
-        __syncthreads();
+        lds_only_barrier();
         mx = fmaxf(fmaxf(mx_lds[lq], mx_lds[16 + lq]), fmaxf(mx_lds[32 + lq], mx_lds[48 + lq]));   // finite: the tile holds a visible key
         const float m_new = fmaxf(m, mx), alpha = fast_exp2(m - m_new);
         m = m_new;
@@ -288,7 +315,7 @@ __global__ __launch_bounds__(256) void latent_attend_kernel(const LatentAttnArgs
         const int at = lq * 72 + 32 * (wave >> 1) + 8 * lg + 4 * (wave & 1);
         *reinterpret_cast<u32x2*>(p_lds + at) = u32x2{pack_bf16x2(p[0], p[1]), pack_bf16x2(p[2], p[3])};
         *reinterpret_cast<u32x2*>(p_lds + 16 * 72 + at) = u32x2{pack_bf16x2(p[0] - hi[0], p[1] - hi[1]), pack_bf16x2(p[2] - hi[2], p[3] - hi[3])};
-        __syncthreads();
+        lds_only_barrier();
 #pragma unroll
         for (int t = 0; t < NT; ++t) o[t] *= alpha;
 #pragma unroll
@@ -312,8 +339,10 @@ __global__ __launch_bounds__(256) void latent_attend_kernel(const LatentAttnArgs
                 o[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pl, o[t], 0, 0, 0);
             }
         }
-        __syncthreads();                             // every wave is done with the image and the weights
-        if (t0 + 64 < k1) stage(t0 + 64);
+    };
+    for (int t0 = k0; t0 < k1; t0 += 128) {
+        tile_body(std::integral_constant<int, 0>{}, t0);
+        if (t0 + 64 < k1) tile_body(std::integral_constant<int, 1>{}, t0 + 64);
     }
     if (head_ok) {
 #pragma unroll
@@ -353,28 +382,63 @@ __device__ __forceinline__ void split_totals(const LatentAttnArgs& a, int row, i
     inv = l > 0.f ? 1.f / l : 0.f;
 }
 
-// grid (heads, row tiles of RW): latent sums of RW rows into LDS as the A operand (rows past RW are zero), waves share the value columns
+// grid (heads, row tiles of RW), 8 waves: weights of the splits into LDS, latent sums of the rows into LDS as the second operand, waves share the
+// value columns.  The first value columns' weights are asked for before anything else.
 template <int RW>
-__global__ __launch_bounds__(256) void latent_value_kernel(const LatentAttnArgs a) {
-    extern __shared__ __attribute__((aligned(16))) uint16_t lat[];             // [16][kv_cols + 8]
-    const int head = blockIdx.x, r0 = blockIdx.y * RW, ld = a.kv_cols + 8, pieces = a.kv_cols / 4;
+__global__ __launch_bounds__(512) void latent_value_kernel(const LatentAttnArgs a) {
+    extern __shared__ __attribute__((aligned(16))) uint16_t lat[];             // [RW][kv_cols + 8]
+    __shared__ float wsp[RW][64];
+    constexpr int PRE = 8;
+    const int head = blockIdx.x, r0 = blockIdx.y * RW, ld = a.kv_cols + 8, pieces = a.kv_cols / 4, ksteps = a.kv_cols / 32;
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, lq = lane & 15, lg = lane >> 4;
-    for (int e = tid; e < 16 * pieces; e += 256) {
+    const uint16_t* w_head = reinterpret_cast<const uint16_t*>(a.w_uv) + ((int64_t)head * a.v_cols + lq) * a.kv_cols + 8 * lg;
+    bf16x8 pre[PRE];
+    {
+        const uint16_t* w = w_head + (int64_t)(16 * wave < a.v_cols ? 16 * wave : 0) * a.kv_cols;
+#pragma unroll
+        for (int k = 0; k < PRE; ++k) pre[k] = *reinterpret_cast<const bf16x8*>(w + 32 * (k < ksteps ? k : 0));
+    }
+    auto live_splits = [&](int row) {                // splits that hold keys of this row
+        const int tiles = ((int)a.positions[row] + 64) / 64, per = (tiles + a.splits - 1) / a.splits;
+        return (tiles + per - 1) / per;
+    };
+    for (int r = wave; r < RW; r += 8) {
+        if (r0 + r >= a.rows) break;
+        const bool ok = lane < live_splits(r0 + r);
+        const int64_t rec = ((int64_t)(r0 + r) * a.splits + (ok ? lane : 0)) * a.heads + head;
+        const float ms = ok ? a.part_ml[rec * 2] : -INFINITY, ls = ok ? a.part_ml[rec * 2 + 1] : 0.f;
+        float m = ms;
+        for (int d = 1; d < 64; d <<= 1) m = fmaxf(m, __shfl_xor(m, d));
+        const float e = fast_exp2(ms - m);
+        float l = ls * e;
+        for (int d = 1; d < 64; d <<= 1) l += __shfl_xor(l, d);
+        wsp[r][lane] = e * (l > 0.f ? 1.f / l : 0.f);
+    }
+    __syncthreads();
+    for (int e = tid; e < RW * pieces; e += 512) {
         const int r = e / pieces, c = (e - r * pieces) * 4;
         f32x4 v = {0.f, 0.f, 0.f, 0.f};
-        if (r < RW && r0 + r < a.rows) {
-            float m, inv;
-            split_totals(a, r0 + r, head, m, inv);
-            v = combine_splits(a, r0 + r, head, c, m, inv);
+        if (r0 + r < a.rows) {
+            const int n = live_splits(r0 + r);
+            const float* p = a.part_o + ((int64_t)(r0 + r) * a.splits * a.heads + head) * a.kv_cols + c;
+            const int64_t step = (int64_t)a.heads * a.kv_cols;
+#pragma unroll 4
+            for (int s = 0; s < n; ++s) v += *reinterpret_cast<const f32x4*>(p + s * step) * wsp[r][s];
         }
         act_st4(lat + r * ld + c, v);
     }
     __syncthreads();
-    for (int nt = wave; nt < a.v_cols / 16; nt += 4) {
-        const uint16_t* w = reinterpret_cast<const uint16_t*>(a.w_uv) + ((int64_t)head * a.v_cols + 16 * nt + lq) * a.kv_cols + 8 * lg;
+    const uint16_t* l_row = lat + (lq < RW ? lq : 0) * ld + 8 * lg;            // (columns past RW are computed and dropped)
+    for (int nt = wave; nt < a.v_cols / 16; nt += 8) {
+        const uint16_t* w = w_head + (int64_t)16 * nt * a.kv_cols;
         f32x4 acc = {0.f, 0.f, 0.f, 0.f};
-        for (int k = 0; k < a.kv_cols; k += 32)
-            acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8*>(w + k), *reinterpret_cast<const bf16x8*>(lat + lq * ld + 8 * lg + k), acc, 0, 0, 0);
+        if (nt == wave) {
+#pragma unroll
+            for (int k = 0; k < PRE; ++k)
+                if (k < ksteps) acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(pre[k], *reinterpret_cast<const bf16x8*>(l_row + 32 * k), acc, 0, 0, 0);
+        }
+        for (int k = nt == wave ? PRE : 0; k < ksteps; ++k)
+            acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8*>(w + 32 * k), *reinterpret_cast<const bf16x8*>(l_row + 32 * k), acc, 0, 0, 0);
         if (lq < RW && r0 + lq < a.rows) {           // C^T: lane = row lq, value columns 16 nt + 4 lg ..
             const int col = head * a.v_cols + 16 * nt + 4 * lg;
             if (a.out) act_st4(reinterpret_cast<uint16_t*>(a.out) + (int64_t)(r0 + lq) * a.out_stride + col, acc);
@@ -407,11 +471,13 @@ __global__ __launch_bounds__(256) void latent_value_generic_kernel(const LatentA
 }
 
 // ------------------------------------------------------------------------------------------------ gather
-// cache rows of every key of the sequences, packed: out[cu_k[b] + j] = row of key j of sequence b
-template <typename T>
-__global__ __launch_bounds__(256) void latent_gather_kernel(T* __restrict__ out, const T* __restrict__ cache, const int32_t* __restrict__ cu_k,
-                                                             const int32_t* __restrict__ block_tables, int64_t bt_stride, int batch, int cols, int block_size) {
-    const int row = blockIdx.x;
+// cache rows of every key of the sequences, packed: out[cu_k[b] + j] = row of key j of sequence b.  One 16-byte piece per thread
+__global__ __launch_bounds__(256) void latent_gather_kernel(u32x4* __restrict__ out, const u32x4* __restrict__ cache, const int32_t* __restrict__ cu_k,
+                                                             const int32_t* __restrict__ block_tables, int64_t bt_stride, int batch, int total, int pieces,
+                                                             int block_size) {
+    const int64_t e = (int64_t)blockIdx.x * 256 + threadIdx.x;
+    const int row = (int)(e / pieces), p = (int)(e - (int64_t)row * pieces);
+    if (row >= total) return;
     int lo = 0, hi = batch;                          // sequence of this row: the last b with cu_k[b] <= row
     while (hi - lo > 1) {
         const int mid = (lo + hi) / 2;
@@ -420,13 +486,12 @@ __global__ __launch_bounds__(256) void latent_gather_kernel(T* __restrict__ out,
     }
     const int key = row - cu_k[lo];
     const int64_t page = block_tables[lo * bt_stride + key / block_size];
-    const T* src = cache + (page * block_size + key % block_size) * cols;
-    for (int c = threadIdx.x * 4; c < cols; c += 1024) act_st4(out + (int64_t)row * cols + c, act_ld4(src + c));
+    out[e] = cache[(page * block_size + key % block_size) * pieces + p];
 }
 
 template <int NT>
 void attend_nt(const LatentAttnArgs& a, hipStream_t stream) {
-    constexpr size_t lds = 64 * (64 * NT + 64) * 2 + 2 * 16 * 72 * 2 + 4 * 16 * 4;
+    constexpr size_t lds = 2 * 64 * (64 * NT + 64) * 2 + 2 * 16 * 72 * 2 + 4 * 16 * 4;
     if (lds > 64 * 1024) (void)hipFuncSetAttribute(reinterpret_cast<const void*>(latent_attend_kernel<NT>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
     latent_attend_kernel<NT><<<dim3(a.splits, a.rows, (a.heads + 15) / 16), 256, lds, stream>>>(a);
 }
@@ -434,8 +499,9 @@ void attend_nt(const LatentAttnArgs& a, hipStream_t stream) {
 }  // namespace
 
 int launch_latent_prep(const LatentPrepArgs& a, int f32, hipStream_t stream) {
-    if (f32) latent_prep_kernel<float><<<a.rows, 256, 0, stream>>>(a);
-    else latent_prep_kernel<uint16_t><<<a.rows, 256, 0, stream>>>(a);
+    const int grid = (a.rows + 3) / 4;
+    if (f32) latent_prep_kernel<float><<<grid, 256, 0, stream>>>(a);
+    else latent_prep_kernel<uint16_t><<<grid, 256, 0, stream>>>(a);
     return check_launch("latent_prep");
 }
 
@@ -478,10 +544,9 @@ int launch_latent_attend(const LatentAttnArgs& a, int f32, int generic, hipStrea
 }
 
 int launch_latent_value(const LatentAttnArgs& a, int f32, hipStream_t stream) {
-    if (!f32 && a.v_cols % 16 == 0 && a.kv_cols % 32 == 0) {
-        const size_t lds = (size_t)16 * (a.kv_cols + 8) * 2;
-        if (a.rows <= 128) latent_value_kernel<4><<<dim3(a.heads, (a.rows + 3) / 4), 256, lds, stream>>>(a);
-        else latent_value_kernel<16><<<dim3(a.heads, (a.rows + 15) / 16), 256, lds, stream>>>(a);
+    if (!f32 && a.v_cols % 16 == 0 && a.kv_cols % 32 == 0 && a.splits <= 64) {
+        if (a.rows <= 128) latent_value_kernel<4><<<dim3(a.heads, (a.rows + 3) / 4), 512, (size_t)4 * (a.kv_cols + 8) * 2, stream>>>(a);
+        else latent_value_kernel<16><<<dim3(a.heads, (a.rows + 15) / 16), 512, (size_t)16 * (a.kv_cols + 8) * 2, stream>>>(a);
     } else {
         const dim3 grid(a.rows, a.heads);
         if (f32) latent_value_generic_kernel<float><<<grid, 256, a.kv_cols * 4, stream>>>(a);
@@ -492,8 +557,9 @@ int launch_latent_value(const LatentAttnArgs& a, int f32, hipStream_t stream) {
 
 int launch_latent_gather(void* out, const void* cache, const int32_t* cu_k, const int32_t* block_tables, int64_t bt_stride, int batch, int total, int cols,
                          int block_size, int f32, hipStream_t stream) {
-    if (f32) latent_gather_kernel<float><<<total, 256, 0, stream>>>((float*)out, (const float*)cache, cu_k, block_tables, bt_stride, batch, cols, block_size);
-    else latent_gather_kernel<uint16_t><<<total, 256, 0, stream>>>((uint16_t*)out, (const uint16_t*)cache, cu_k, block_tables, bt_stride, batch, cols, block_size);
+    const int pieces = cols * (f32 ? 4 : 2) / 16;
+    const int64_t grid = ((int64_t)total * pieces + 255) / 256;
+    latent_gather_kernel<<<(unsigned)grid, 256, 0, stream>>>((u32x4*)out, (const u32x4*)cache, cu_k, block_tables, bt_stride, batch, total, pieces, block_size);
     return check_launch("latent_gather");
 }
 

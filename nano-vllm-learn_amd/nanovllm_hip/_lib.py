@@ -44,7 +44,7 @@ class RglruDesc(ctypes.Structure):
     _fields_ = [("yx", ctypes.c_void_p), ("yx_stride", ctypes.c_int64), ("width", ctypes.c_int32), ("block", ctypes.c_int32),
                 ("blocks", ctypes.c_int32), ("taps", ctypes.c_int32), ("conv_w", ctypes.c_void_p), ("conv_b", ctypes.c_void_p),
                 ("ra", ctypes.c_void_p), ("ri", ctypes.c_void_p), ("ra_b", ctypes.c_void_p), ("ri_b", ctypes.c_void_p),
-                ("rate", ctypes.c_void_p), ("chunks", ctypes.c_void_p), ("n_chunks", ctypes.c_int32), ("positions", ctypes.c_void_p),
+                ("rate", ctypes.c_void_p), ("chunks", ctypes.c_void_p), ("n_chunks", ctypes.c_int32), ("segment", ctypes.c_int32), ("summaries", ctypes.c_int32), ("positions", ctypes.c_void_p),
                 ("state_slots", ctypes.c_void_p), ("state", ctypes.c_void_p), ("conv_state", ctypes.c_void_p), ("s_loc", ctypes.c_void_p),
                 ("a_cum", ctypes.c_void_p), ("out", ctypes.c_void_p), ("out_stride", ctypes.c_int64), ("out_packed", ctypes.c_void_p)]
 

@@ -87,12 +87,12 @@ def build_decode_meta(seqs, block_size=256):
                 block_tables=build_block_tables(seqs))
 
 
-def recurrence_chunks(first_row, rows, seq, chunk_tokens):
-    """Chunk table rows of one sequence's portion: (first row, rows, sequence, index in the portion)."""
-    return [(first_row + k, min(chunk_tokens, rows - k), seq, k // chunk_tokens) for k in range(0, rows, chunk_tokens)]
+def recurrence_chunks(first_row, rows, seq, segment):
+    """Segment table rows of one sequence's portion: (first row, rows, sequence, index in the portion)."""
+    return [(first_row + k, min(segment, rows - k), seq, k // segment) for k in range(0, rows, segment)]
 
 
-def build_step_meta(portions, block_size, chunk_tokens=64):
+def build_step_meta(portions, block_size, segment=64):
     """Rows of a mixed batch.  portions: [(sequence, tokens)] — the sequence's next tokens behind its num_cached_tokens.  Sequences that bring one
     token come first (`order` gives the places in `portions`); returns host tensors."""
     _check_block_size([s for s, _ in portions], block_size)
@@ -103,7 +103,7 @@ def build_step_meta(portions, block_size, chunk_tokens=64):
         seq, n = portions[i]
         lo, hi = seq.num_cached_tokens, seq.num_cached_tokens + n
         assert 0 < n and hi <= len(seq) and hi <= len(seq.block_table) * block_size
-        chunks += recurrence_chunks(len(input_ids), n, j, chunk_tokens)
+        chunks += recurrence_chunks(len(input_ids), n, j, segment)
         input_ids += seq[lo:hi]
         positions += range(lo, hi)
         slots += [seq.block_table[p // block_size] * block_size + p % block_size for p in range(lo, hi)]
@@ -119,7 +119,8 @@ def build_step_meta(portions, block_size, chunk_tokens=64):
     def i32(v):
         return torch.tensor(v, dtype=torch.int32)
     return dict(order=order, input_ids=torch.tensor(input_ids, dtype=torch.int64), positions=torch.tensor(positions, dtype=torch.int64), num_decode=num_decode,
-                slot_mapping=i32(slots), block_tables=build_block_tables(seqs, pad=0), state_slots=i32([s.state_slot for s in seqs]), chunks=i32(chunks),
+                slot_mapping=i32(slots), block_tables=build_block_tables(seqs, pad=0), state_slots=i32([s.state_slot for s in seqs]), chunks=i32(chunks), segment=segment,
+                summaries=any(k for *_, k in chunks),
                 row_seq=i32(row_seq), cu_q=i32(cu_q), cu_k=i32(cu_k), max_q=max_q, total_k=cu_k[-1], max_context=max(positions) + 1)
 
 
@@ -192,7 +193,7 @@ class ModelRunner:
         """One batch of a model that takes mixed batches.  portions: [(sequence, tokens)]; want: per portion, the places among its tokens whose
         logits are asked for (default: the last).  Returns logits rows in the order of `portions` and `want` (None when nothing is wanted) and
         advances num_cached_tokens."""
-        m = build_step_meta(portions, self.block_size, ops.rglru_chunk_tokens())
+        m = build_step_meta(portions, self.block_size, self.model.recurrence_segment([n for _, n in portions if n > 1]))
         assert int(m["positions"].max()) < self.max_model_len, "a sequence exceeds max_model_len"
         assert 0 <= int(m["input_ids"].min()) and int(m["input_ids"].max()) < self.cfg.vocab_size, "a token id is outside the vocabulary"
         first, row = {}, 0
@@ -204,7 +205,7 @@ class ModelRunner:
         assert all(0 <= p < portions[i][1] for i, places in enumerate(want) for p in places), "a wanted place is outside its portion"
         decode_only = m["num_decode"] == row
         step = StepMeta(m["num_decode"], self._dev(m["slot_mapping"]), self._dev(m["block_tables"]), self._dev(m["state_slots"]), self._dev(m["chunks"]),
-                        m["max_context"], *([] if decode_only else [self._dev(m["row_seq"]), self._dev(m["cu_q"]), self._dev(m["cu_k"]), m["max_q"], m["total_k"]]))
+                        m["segment"], m["summaries"], m["max_context"], *([] if decode_only else [self._dev(m["row_seq"]), self._dev(m["cu_q"]), self._dev(m["cu_k"]), m["max_q"], m["total_k"]]))
         hidden = self.model(self._dev(m["input_ids"]), self._dev(m["positions"]), step)
         for seq, n in portions:
             seq.num_cached_tokens += n
@@ -325,7 +326,7 @@ class DecodeSession:
             self.positions -= 1                                   # of the token that is fed (build_decode_meta has the reference's own convention)
             slots = torch.tensor([s.state_slot for s in seqs], dtype=torch.int32)
             chunks = torch.tensor([(i, 1, i, 0) for i in range(b)], dtype=torch.int32)
-            self.step_meta = StepMeta(b, self.slot_mapping, self.block_tables, slots.to(dev), chunks.to(dev), need_tokens)
+            self.step_meta = StepMeta(b, self.slot_mapping, self.block_tables, slots.to(dev), chunks.to(dev), ops.rglru_chunk_tokens(), False, need_tokens)
         # the next step's embedding lookup rides in the arg-max launch when the model allows it: the session then owns the
         # embedded rows (row-major = the residual stream of the step, and in fragment order for layer 0's projection)
         self.fuse_embed = bool(getattr(runner.model, "fused_embedding_ok", lambda *_: False)(b, torch.device(dev)))

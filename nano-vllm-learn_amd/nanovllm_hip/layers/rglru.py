@@ -12,6 +12,25 @@ from .. import ops
 from .linear import linear, padded, round_up
 
 
+CUS = 256                     # compute units of an MI355X: one walking workgroup keeps one busy
+
+
+def choose_segment(portions, blocks, chunk=64):
+    """Tokens per segment for portions of these lengths: one workgroup walks one (segment, diagonal block), and cutting a portion into more than one
+    costs a summary walk (about 0.7 of a full one) over all its segments but the last.  Returns the cheapest power-of-two multiple of `chunk`."""
+    best, longest = None, max(portions, default=1)
+    seg = chunk
+    while True:
+        pieces = [-(-n // seg) for n in portions]
+        steps = min(seg, longest) / chunk
+        cost = -(-sum(pieces) * blocks // CUS) * steps + 0.7 * -(-sum(p - 1 for p in pieces) * blocks // CUS) * steps
+        if best is None or cost < best[0]:
+            best = (cost, seg)
+        if seg >= longest:
+            return best[1]
+        seg *= 2
+
+
 class RGLRU(nn.Module):
     """decay_scale: log a = -decay_scale * r * softplus(lam)."""
 
@@ -68,7 +87,8 @@ class RGLRU(nn.Module):
         if n:
             ops.rglru_step(yx[:n], self.params, positions[:n], step.state_slots, self.state, self.conv_state, out=out[:n])
         if n < x.shape[0]:
-            ops.rglru_chunks(yx, self.params, positions, step.state_slots, step.chunks[n:], self.state, self.conv_state, out=out)
+            ops.rglru_chunks(yx, self.params, positions, step.state_slots, step.chunks[n:], step.segment, step.summaries, self.state,
+                             self.conv_state, out=out)
         return linear(out, self.w_o)
 
     def decode(self, xp, rows, positions, step, bufs):

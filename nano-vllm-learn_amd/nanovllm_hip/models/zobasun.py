@@ -17,7 +17,7 @@ from .. import ops
 from ..layers.latent_attention import LatentAttention
 from ..layers.linear import linear, padded, round_up
 from ..layers.mlp import ClampedGLU
-from ..layers.rglru import RGLRU
+from ..layers.rglru import RGLRU, choose_segment
 from ..layers.rotary import rotation_table
 
 FUSED_DECODE = True          # tests flip this to compare the fused decode path with the plain one
@@ -168,9 +168,19 @@ class ZobasunForCausalLM(nn.Module):
                 ops.norm_residual(x, layer.norm2, eps, n, cfg.dtype, y=layer.mlp.decode(xp, rows, bufs), packed=xp, want_rows=False)
         return x
 
+    def recurrence_segment(self, portions):
+        """Tokens per recurrence segment for portions of these lengths (the layer with the fewest blocks fills the GPU last)."""
+        blocks = [layer.mixer.blocks for layer in self.layers if isinstance(layer.mixer, RGLRU)]
+        return choose_segment(portions, min(blocks), ops.rglru_chunk_tokens()) if blocks and portions else ops.rglru_chunk_tokens()
+
     def compute_logits(self, x):
         """Logits [rows, vocab] (a view of padded rows) of residual-stream rows."""
-        h = ops.norm_residual(x, self.final_norm, self.cfg.rms_norm_eps, self.cfg.hidden_size, self.cfg.dtype)
+        cfg, rows = self.cfg, x.shape[0]
+        if FUSED_DECODE and cfg.dtype == torch.bfloat16 and rows <= ops.LINEAR_SMALL_M_MAX:
+            bufs = self._decode_buffers(rows)
+            ops.norm_residual(x, self.final_norm, cfg.rms_norm_eps, cfg.hidden_size, cfg.dtype, packed=bufs.stream, want_rows=False)
+            return ops.fused_linear(bufs.stream, self.head, x_packed_rows=rows, workspace=bufs.workspace)[:, :cfg.vocab_size]
+        h = ops.norm_residual(x, self.final_norm, cfg.rms_norm_eps, cfg.hidden_size, cfg.dtype)
         return linear(h, self.head)[:, :self.cfg.vocab_size]
 
     def greedy_candidates(self, hidden):

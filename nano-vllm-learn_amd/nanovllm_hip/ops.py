@@ -673,11 +673,11 @@ def _rglru_desc(yx, p, positions, state_slots, state, conv_state):
     return d, width, code
 
 
-def rglru_chunks(yx, params, positions, state_slots, chunks, state, conv_state, out=None, generic=False):
+def rglru_chunks(yx, params, positions, state_slots, chunks, segment, summaries, state, conv_state, out=None, generic=False):
     """Gated linear recurrence over portions of sequences.  yx [rows, 2 * width] = gate branch | recurrent branch; params = dict(conv_w [taps, width],
-    conv_b, ra / ri [blocks, block, block], ra_b, ri_b, rate); chunks int32 [n, 4] = (first row, rows, sequence, index in its portion), built by
-    the host from portions cut every rglru_chunk_tokens() tokens.  state [slots, width] fp32 and conv_state [slots, taps, width] are updated.
-    Rows no chunk covers are left alone in `out` (they belong to another launch)."""
+    conv_b, ra / ri [blocks, block, block], ra_b, ri_b, rate); chunks int32 [n, 4] = (first row, rows, sequence, index in its portion), portions cut every
+    `segment` tokens (a multiple of rglru_chunk_tokens()); summaries: some portion has more than one segment.  state [slots, width] fp32 and conv_state
+    [slots, taps, width] are updated.  Rows no segment covers are left alone in `out` (they belong to another launch)."""
     d, width, code = _rglru_desc(yx, params, positions, state_slots, state, conv_state)
     _require_i32(chunks=chunks)
     assert chunks.dim() == 2 and chunks.shape[1] == 4 and chunks.is_contiguous()
@@ -685,8 +685,9 @@ def rglru_chunks(yx, params, positions, state_slots, chunks, state, conv_state, 
     if out is None:
         out = torch.empty((rows, width), dtype=yx.dtype, device=yx.device)
     assert out.shape == (rows, width) and out.stride(1) == 1 and out.dtype == yx.dtype
-    scratch = torch.empty((2, rows, width), dtype=torch.float32, device=yx.device)
+    scratch = torch.empty((2, chunks.shape[0], width), dtype=torch.float32, device=yx.device)
     d.chunks, d.n_chunks, d.s_loc, d.a_cum = chunks.data_ptr(), chunks.shape[0], scratch[0].data_ptr(), scratch[1].data_ptr()
+    d.segment, d.summaries = int(segment), int(summaries)
     d.out, d.out_stride = out.data_ptr(), out.stride(0)
     _lib.check(_lib.load().nvh_rglru_chunks(ctypes.byref(d), int(generic), code, _stream()), "nvh_rglru_chunks")
     return out
@@ -743,10 +744,16 @@ def latent_attend_mfma(kv_cols, rot_cols, block_size) -> bool:
     return bool(_lib.load().nvh_latent_attend_mfma(kv_cols, rot_cols, block_size))
 
 
-def latent_splits(rows, heads, max_context, mfma) -> int:
-    """Context splits of one latent-attention launch: two workgroups per CU where the context is long enough to share."""
-    per_row = (heads + 15) // 16 if mfma else heads
-    return max(1, min(512 // max(1, rows * per_row), (max_context + 63) // 64, 64))
+def latent_splits(rows, heads, max_context, mfma, cache_cols=576) -> int:
+    """Context splits of one latent-attention launch.  MFMA form: as many workgroups as the 256 CUs hold at once (two LDS images of 64 cache rows
+    each), every split the same number of 64-key tiles."""
+    tiles = (max_context + 63) // 64
+    if not mfma:
+        return max(1, min(512 // max(1, rows * heads), tiles, 64))
+    resident = 256 * (2 if 4 * 64 * cache_cols * 2 + 16384 <= 163840 else 1)
+    splits = max(1, min(resident // (rows * ((heads + 15) // 16)), tiles, 64))
+    per = -(-tiles // splits)
+    return -(-tiles // per)
 
 
 def latent_attention(q, cache, block_tables, positions, cos_sin, w_uk, w_uv, scale, rot, max_context, row_seq=None, out=None, out_packed=None, want_out=True,
@@ -764,7 +771,7 @@ def latent_attention(q, cache, block_tables, positions, cos_sin, w_uk, w_uv, sca
     assert w_uv.shape == (heads, v_cols, kv_cols) and block_tables.dim() == 2 and block_tables.stride(1) == 1
     assert positions.dtype == torch.int64 and positions.is_contiguous() and positions.numel() == rows
     mfma = code == NVH_BF16 and row_seq is None and not generic and latent_attend_mfma(kv_cols, cols - kv_cols, block_size)
-    splits = splits or latent_splits(rows, heads, max_context, mfma)
+    splits = splits or latent_splits(rows, heads, max_context, mfma, cols)
     qa = torch.empty((rows, heads, cols), dtype=q.dtype, device=q.device)
     part_o = torch.empty((rows, splits, heads, kv_cols), dtype=torch.float32, device=q.device)
     part_ml = torch.empty((rows, splits, heads, 2), dtype=torch.float32, device=q.device)

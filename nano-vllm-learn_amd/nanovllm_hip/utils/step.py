@@ -11,7 +11,9 @@ class StepMeta:
     slot_mapping: torch.Tensor                      # int32 [rows] cache slot of every row
     block_tables: torch.Tensor                      # int32 [sequences, width]
     state_slots: torch.Tensor                       # int32 [sequences]
-    chunks: torch.Tensor                            # int32 [n, 4] recurrence chunks, the decode rows' own first
+    chunks: torch.Tensor                            # int32 [n, 4] recurrence segments, the decode rows' own first
+    segment: int                                    # tokens of a full segment
+    summaries: bool                                 # some portion has more than one segment
     max_context: int                                # host bound on the context of any row
     row_seq: torch.Tensor | None = None             # int32 [rows] sequence of every row (None: decode rows only)
     cu_q: torch.Tensor | None = None                # int32 [portions + 1] row offsets of the portions, from the first portion row

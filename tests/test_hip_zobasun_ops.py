@@ -1,7 +1,5 @@
 """GPU: the recurrent and latent-attention layer ops, one mechanism at a time, against plain equations on the CPU (oracle/zobasun_ref.py, float64):
 bf16 on the MFMA kernels, bf16 and fp32 on the plain ones.  Inputs are given in the compared type, so fp32 results are held to fp32 rounding."""
-import math
-
 import pytest
 import torch
 
@@ -145,7 +143,7 @@ class Recurrence:
         s, last = Z.rglru_recurrence(u, r, i, d(self.lam))
         return s * Z.gelu_tanh(d(y)), last
 
-    def run(self, portions, generic=False, step=False):
+    def run(self, portions, generic=False, step=False, segment=64):
         """portions: [(slot, first position, y, x)] as one batch; returns the unpadded rows per portion."""
         from nanovllm_hip import ops
         from nanovllm_hip.engine.model_runner import recurrence_chunks
@@ -159,9 +157,10 @@ class Recurrence:
         else:
             table, row = [], 0
             for j, (_, _, y, _) in enumerate(portions):
-                table += recurrence_chunks(row, y.shape[0], j, ops.rglru_chunk_tokens())
+                table += recurrence_chunks(row, y.shape[0], j, segment)
                 row += y.shape[0]
-            out = ops.rglru_chunks(yx, self.params, pos, slots, torch.tensor(table, dtype=torch.int32, device="cuda"), self.state, self.conv_state, generic=generic)
+            out = ops.rglru_chunks(yx, self.params, pos, slots, torch.tensor(table, dtype=torch.int32, device="cuda"), segment, any(k for *_, k in table),
+                                   self.state, self.conv_state, generic=generic)
         out = self.unspread(out.cpu())
         return out.split([y.shape[0] for _, _, y, _ in portions])
 
@@ -170,16 +169,17 @@ SHAPES = [(1, 32, 64, 1), (3, 44, 64, 4), (2, 96, 96, 2), (4, 256, 256, 4), (1, 
 FORMS = [(torch.bfloat16, False), (torch.bfloat16, True), (torch.float32, False)]
 
 
+@pytest.mark.parametrize("segment", [64, 128, 4096])
 @pytest.mark.parametrize("dtype,generic", FORMS)
 @pytest.mark.parametrize("blocks,size,block,taps", SHAPES)
-def test_recurrence_portions(blocks, size, block, taps, dtype, generic):
+def test_recurrence_portions(blocks, size, block, taps, dtype, generic, segment):
     """Two unequal sequences in one batch, then their later portions (down to two tokens, across chunk edges) from the state."""
     r = Recurrence(blocks, size, block, taps, dtype)
-    (ya, xa), (yb, xb) = r.yx(205, 1), r.yx(77, 2)
+    (ya, xa), (yb, xb) = r.yx(341, 1), r.yx(77, 2)
     (wa, la), (wb, lb) = r.plain(ya, xa), r.plain(yb, xb)
-    cuts_a, cuts_b = [0, 130, 132, 133, 197, 205], [0, 2, 66, 68, 75, 77]
+    cuts_a, cuts_b = [0, 193, 195, 196, 330, 341], [0, 2, 66, 68, 75, 77]
     for (a0, a1), (b0, b1) in zip(zip(cuts_a, cuts_a[1:]), zip(cuts_b, cuts_b[1:])):
-        ga, gb = r.run([(2, a0, ya[a0:a1], xa[a0:a1]), (0, b0, yb[b0:b1], xb[b0:b1])], generic)
+        ga, gb = r.run([(2, a0, ya[a0:a1], xa[a0:a1]), (0, b0, yb[b0:b1], xb[b0:b1])], generic, segment=segment)
         close(ga, wa[a0:a1], dtype)
         close(gb, wb[b0:b1], dtype)
     close(r.unspread(r.state[[2, 0]].cpu()), torch.stack([la, lb]), torch.float32, 40 if dtype == torch.bfloat16 else 3)
@@ -212,7 +212,7 @@ def test_recurrence_remembers_for_long(dtype, generic):
     zeroed = x.clone()
     zeroed[3] = 0
     assert (want[600:] - r.plain(y, zeroed)[0][600:]).abs().max() > 0.5 * want[600:].abs().max()
-    got = torch.cat([r.run([(1, a, y[a:b], x[a:b])], generic)[0] for a, b in ((0, 300), (300, 302), (302, 640))])
+    got = torch.cat([r.run([(1, a, y[a:b], x[a:b])], generic, segment=128)[0] for a, b in ((0, 300), (300, 302), (302, 640))])
     close(got, want, dtype, 3)
 
 
@@ -426,4 +426,4 @@ def test_operand_checks():
         ops.clamped_glu(torch.zeros(2, 16, device="cuda", dtype=torch.float16), 1.0, 1.0)
     with pytest.raises(RuntimeError, match="inter"):
         ops.clamped_glu(torch.zeros(2, 6, device="cuda"), 1.0, 1.0)
-    assert math.isclose(ops.latent_splits(32, 16, 1536, True), 16)
+    assert ops.latent_splits(32, 16, 1536, True) == 8

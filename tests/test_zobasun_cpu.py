@@ -185,6 +185,12 @@ def test_step_meta_refuses_tokens_without_pages():
         build_step_meta([(_seq(70, 0, [1], 0), 70)], 64)
 
 
+def test_segment_choice():
+    from nanovllm_hip.layers.rglru import choose_segment
+    assert choose_segment([1024] * 32, 16) >= 1024                              # enough workgroups: one walk each
+    assert choose_segment([8192], 10) < 1024 and choose_segment([2], 4) == 64
+
+
 # ------------------------------------------------------------------------------------------------ scheduler
 def _scheduler(blocks, slots=4, mixed=True, **kw):
     from nanovllm_hip.engine.block_manager import BlockManager, StateSlots
