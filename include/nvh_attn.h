@@ -462,7 +462,7 @@ int nvh_clamped_glu(void* out, const void* gate_up, int rows, int inter, int64_t
 /* Real-gated linear recurrent unit behind a causal depthwise convolution: log a = -rate sigmoid(ra u), S = a S + sqrt(1 - a^2) sigmoid(ri u) u,
  * out = S gelu(y).  nvh_rglru_chunks: portions of prompts (and single tokens), cut by the caller into segments that are
  * scanned side by side; segments of one portion are consecutive.  nvh_rglru_step: row i is one new token of sequence i (bf16; nvh_rglru_step_supported(block)).
- * generic != 0 forces the plain kernel (tests). */
+ * generic: 0 = the fastest form the shape allows, 1 = the plain kernel, 2 = the MFMA walk without LDS-DMA (tests). */
 typedef struct nvh_rglru_desc {
     const void* yx;              /* [rows, 2 * width]: gate branch | recurrent branch (biases added), row stride yx_stride */
     int64_t yx_stride;

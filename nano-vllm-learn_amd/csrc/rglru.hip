@@ -35,8 +35,8 @@ __device__ __forceinline__ float fast_gelu(float z) {
 __device__ __forceinline__ void decay_and_input(float rate, float r, float ig, float u, float& a, float& b) {
     const float x = rate * r, y = 2.f * x;
     a = fast_exp2(-kLog2e * x);
-    const float series = y * (1.f - y * (1.f / 2) * (1.f - y * (1.f / 3) * (1.f - y * (1.f / 4) * (1.f - y * (1.f / 5) * (1.f - y * (1.f / 6))))));
-    b = fast_sqrt(y < 0.3f ? series : 1.f - a * a) * ig * u;
+    const float series = y * (1.f - y * (1.f / 2) * (1.f - y * (1.f / 3) * (1.f - y * (1.f / 4))));
+    b = fast_sqrt(y < 0.06f ? series : 1.f - a * a) * ig * u;
 }
 
 // convolution input of the token `t` rows after the portion's first row (negative: before it, from the ring; before position 0: zero)
@@ -240,6 +240,231 @@ __global__ __launch_bounds__(1024) void rglru_walk_kernel(const RglruArgs a) {
     if (mine && lg == 0 && (SUMMARY || !more)) {
         a.s_loc[(int64_t)seg * a.width + ch] = cs;
         if (SUMMARY && kth) a.a_cum[(int64_t)seg * a.width + ch] = ca;
+    }
+}
+
+// ------------------------------------------------------------------------------------------------ prompt portions, blocks of up to 256 channels
+// The same walk with everything in flight early: x of the next 64 tokens and y of these travel by LDS-DMA under this step's arithmetic, both gates' weights
+// of a wave's channels stay in registers for the whole segment (8 waves, 16 or 32 channels each), and u and y come into the accumulator layout through an
+// MFMA with a 0/1 selection matrix (exact) instead of single-element LDS reads.
+constexpr int HALO = 8;                              // rows in front of a step's 64 in the x image: taps <= HALO + 1
+
+__device__ __forceinline__ void lds_barrier() {      // (a __syncthreads() would drain the DMA in flight)
+    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+    __builtin_amdgcn_s_barrier();
+    asm volatile("" ::: "memory");
+}
+
+template <int KS> constexpr size_t scan_x_bytes() { return (size_t)(CH + HALO) * KS * 64 + 1024; }     // (the last DMA instruction may run over)
+template <int KS> constexpr size_t scan_lds_bytes(int taps) {
+    return 2 * scan_x_bytes<KS>() + (size_t)CH * (KS * 32 + 8) * 2 + (size_t)CH * KS * 64 + (size_t)(taps + 1) * KS * 128;
+}
+
+template <int KS, bool SUMMARY>                      // block = 32 KS
+__global__ __launch_bounds__(512) void rglru_scan_kernel(const RglruArgs a) {
+    constexpr int BLOCK = 32 * KS, OCT = 4 * KS, TILES = 2 * KS, NTW = (TILES + 7) / 8, LD = BLOCK + 8;
+    constexpr int SWZ = OCT % 8 == 0 ? 7 : 3;        // y image: piece p of row r sits at p ^ (r & SWZ)
+    constexpr int XINS = ((CH + HALO) * OCT + 63) / 64, YINS = OCT;
+    extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
+    uint16_t* x_lds = reinterpret_cast<uint16_t*>(smem);                       // [2][HALO + CH][BLOCK]
+    constexpr int XBUF = scan_x_bytes<KS>() / 2;
+    uint16_t* u_lds = x_lds + 2 * XBUF;                                        // [CH][LD]
+    uint16_t* y_lds = u_lds + CH * LD;                                         // [CH][BLOCK] swizzled; out after the scan
+    float* w_lds = reinterpret_cast<float*>(y_lds + CH * BLOCK);               // [taps + 1][BLOCK]: taps, then the bias
+    const int seg = blockIdx.x, blk = blockIdx.y, c0 = blk * BLOCK;
+    const int row0 = a.chunks[seg * 4], n = a.chunks[seg * 4 + 1], seq = a.chunks[seg * 4 + 2], kth = a.chunks[seg * 4 + 3];
+    const bool more = seg + 1 < a.n_chunks && a.chunks[seg * 4 + 6] == seq;
+    if (SUMMARY && !more) return;
+    const int off0 = kth * a.segment, seq_row0 = row0 - off0;
+    const int slot = a.state_slots[seq];
+    const int64_t pos0 = a.positions[seq_row0];
+    const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lq = lane & 15, lg = lane >> 4;
+    const uint16_t* yx = reinterpret_cast<const uint16_t*>(a.yx);
+    const uint16_t* xcol = yx + a.width + c0;
+    auto dma = [&](const uint16_t* src, void* dst) {
+        __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)src, (__attribute__((address_space(3))) void*)dst, 16, 0, 0);
+    };
+    auto stage_x = [&](int t0, int buf) {            // rows t0 - HALO .. t0 + CH - 1 of the segment, clamped to the portion's rows that exist
+        const int lo = -off0, hi = n - 1;
+#pragma unroll
+        for (int j = 0; j < (XINS + 7) / 8; ++j) {
+            const int ins = wave + 8 * j;
+            if (ins < XINS) {
+                const int s = ins * 64 + lane;
+                int t = t0 - HALO + s / OCT;
+                t = t < lo ? lo : (t > hi ? hi : t);
+                dma(xcol + (int64_t)(row0 + t) * a.yx_stride + (s % OCT) * 8, x_lds + buf * XBUF + ins * 512);
+            }
+        }
+    };
+    auto stage_y = [&](int t0) {
+#pragma unroll
+        for (int j = 0; j < (YINS + 7) / 8; ++j) {
+            const int ins = wave + 8 * j;
+            if (ins < YINS) {
+                const int s = ins * 64 + lane, r = s / OCT, t = t0 + r < n ? t0 + r : n - 1;
+                dma(yx + (int64_t)(row0 + t) * a.yx_stride + c0 + ((s % OCT) ^ (r & SWZ)) * 8, y_lds + ins * 512);
+            }
+        }
+    };
+    stage_x(0, 0);
+    for (int e = tid; e < (a.taps + 1) * BLOCK; e += 512) w_lds[e] = e < a.taps * BLOCK ? a.conv_w[(int64_t)(e / BLOCK) * a.width + c0 + e % BLOCK] : a.conv_b[c0 + e % BLOCK];
+
+    // ---- this wave's channels: 16-channel tiles wave, wave + 8
+    bf16x8 wr[NTW][KS], wi[NTW][KS], sel;
+    float ca[NTW], cs[NTW], rb[NTW], ib[NTW], rate[NTW];
+    {
+        u32x4 one;                                   // 1.0 where this lane's k-slot is its own channel (tiles wave and wave + 8: the same half of a k-step)
+#pragma unroll
+        for (int k = 0; k < 4; ++k) {
+            const int want = 16 * (wave & 1) + lq - 8 * lg - 2 * k;
+            one[k] = want == 0 ? 0x3F80u : (want == 1 ? 0x3F800000u : 0u);
+        }
+        sel = __builtin_bit_cast(bf16x8, one);
+    }
+#pragma unroll
+    for (int j = 0; j < NTW; ++j) {
+        const int nt = wave + 8 * j < TILES ? wave + 8 * j : 0, cb = 16 * nt + lq, ch = c0 + cb;
+        const uint16_t* pr = reinterpret_cast<const uint16_t*>(a.ra) + ((int64_t)c0 + cb) * BLOCK + 8 * lg;
+        const uint16_t* pi = reinterpret_cast<const uint16_t*>(a.ri) + ((int64_t)c0 + cb) * BLOCK + 8 * lg;
+#pragma unroll
+        for (int k = 0; k < KS; ++k) {
+            wr[j][k] = *reinterpret_cast<const bf16x8*>(pr + 32 * k);
+            wi[j][k] = *reinterpret_cast<const bf16x8*>(pi + 32 * k);
+        }
+        rb[j] = -kLog2e * a.ra_b[ch], ib[j] = -kLog2e * a.ri_b[ch], rate[j] = a.rate[ch];
+        ca[j] = 1.f;
+        cs[j] = walk_start(a, SUMMARY, more, seg, kth, slot, pos0, ch);
+        if (SUMMARY && kth == 0 && wave + 8 * j < TILES && lg == 0) a.a_cum[(int64_t)seg * a.width + ch] = cs[j];
+    }
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+    lds_barrier();
+    if (off0 == 0)                                   // inputs in front of the portion: from the ring, zero in front of the sequence
+        for (int e = tid; e < (a.taps - 1) * OCT; e += 512) {
+            const int back = e / OCT + 1, o = e % OCT;
+            const uint16_t* p = conv_input<uint16_t>(a, seq_row0, -back, pos0, slot, c0 + o * 8);
+            *reinterpret_cast<u32x4*>(x_lds + (HALO - back) * BLOCK + o * 8) = p ? *reinterpret_cast<const u32x4*>(p) : u32x4{0, 0, 0, 0};
+        }
+
+    for (int t0 = 0, buf = 0; t0 < n; t0 += CH, buf ^= 1) {
+        const int cnt = n - t0 < CH ? n - t0 : CH;
+        // x of this step was asked for a step ago; only that step's own stores were issued behind it (vector-memory operations complete in order)
+        if (t0 > 0) asm volatile("s_waitcnt vmcnt(%0)" ::"n"(SUMMARY ? 0 : KS / 2) : "memory");
+        lds_barrier();                               // x is in LDS for everyone; the last step's reads of u and y are done
+        if (!SUMMARY) stage_y(t0);
+        if (t0 + CH < n) stage_x(t0 + CH, buf ^ 1);
+        // ---- u, four tokens x 8 channels a time
+        const uint16_t* xs = x_lds + buf * XBUF;
+        for (int e = tid; e < CH / 4 * OCT; e += 512) {
+            const int t = 4 * (e / OCT), o = e % OCT;
+            const float* wp = w_lds + o * 8;
+            float acc[4][8];
+            {
+                const f32x4 b0 = *reinterpret_cast<const f32x4*>(wp + a.taps * BLOCK), b1 = *reinterpret_cast<const f32x4*>(wp + a.taps * BLOCK + 4);
+#pragma unroll
+                for (int i = 0; i < 4; ++i)
+#pragma unroll
+                    for (int k = 0; k < 8; ++k) acc[i][k] = k < 4 ? b0[k] : b1[k - 4];
+            }
+            const uint16_t* xp = xs + (HALO + t - (a.taps - 1)) * BLOCK + o * 8;
+            if (a.taps == 4) {
+                u32x4 v[7];
+#pragma unroll
+                for (int j = 0; j < 7; ++j) v[j] = *reinterpret_cast<const u32x4*>(xp + j * BLOCK);
+#pragma unroll
+                for (int j = 0; j < 4; ++j)
+#pragma unroll
+                    for (int i = 0; i < 4; ++i) fma8(acc[i], v[i + j], wp + j * BLOCK);
+            } else {
+                for (int j = 0; j < a.taps; ++j)
+#pragma unroll
+                    for (int i = 0; i < 4; ++i) fma8(acc[i], *reinterpret_cast<const u32x4*>(xp + (i + j) * BLOCK), wp + j * BLOCK);
+            }
+#pragma unroll
+            for (int i = 0; i < 4; ++i) *reinterpret_cast<u32x4*>(u_lds + (t + i) * LD + o * 8) = pack8(acc[i]);
+        }
+        lds_barrier();
+#pragma unroll 1
+        for (int tm = 0; tm < CH; tm += 16) {        // 16 tokens at a time
+            if (tm > 0 && tm >= cnt) break;
+            f32x4 gr[NTW], gi[NTW];
+#pragma unroll
+            for (int j = 0; j < NTW; ++j) gr[j] = gi[j] = f32x4{0.f, 0.f, 0.f, 0.f};
+            const uint16_t* u_row = u_lds + (tm + lq) * LD + 8 * lg;
+#pragma unroll
+            for (int k = 0; k < KS; ++k) {
+                const bf16x8 ua = *reinterpret_cast<const bf16x8*>(u_row + 32 * k);
+#pragma unroll
+                for (int j = 0; j < NTW; ++j) {
+                    gr[j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ua, wr[j][k], gr[j], 0, 0, 0);
+                    gi[j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ua, wi[j][k], gi[j], 0, 0, 0);
+                }
+            }
+            if (!SUMMARY && tm == 0) {               // y of this step is in LDS; x of the next may still travel
+                if (t0 + CH < n) asm volatile("s_waitcnt vmcnt(%0)" ::"n"(XINS / 8) : "memory");
+                else asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+                lds_barrier();
+            }
+#pragma unroll
+            for (int j = 0; j < NTW; ++j) {
+                if (wave + 8 * j >= TILES) break;
+                const int nt = wave + 8 * j, cb = 16 * nt + lq, r = tm + lq;
+                const f32x4 zero = {0.f, 0.f, 0.f, 0.f};
+                const f32x4 uu = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8*>(u_row + 32 * (nt >> 1)), sel, zero, 0, 0, 0);
+                f32x4 yv = zero;
+                if (!SUMMARY)
+                    yv = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8*>(y_lds + r * BLOCK + (((nt >> 1) * 4 + lg) ^ (r & SWZ)) * 8), sel, zero,
+                                                                 0, 0, 0);
+                float av[4], sv[4];
+                float pa = 1.f, ps = 0.f;
+#pragma unroll
+                for (int i = 0; i < 4; ++i) {
+                    const float rg = fast_rcp(1.f + fast_exp2(gr[j][i] * -kLog2e + rb[j])), ig = fast_rcp(1.f + fast_exp2(gi[j][i] * -kLog2e + ib[j]));
+                    float dec, inp;
+                    decay_and_input(rate[j], rg, ig, uu[i], dec, inp);
+                    if (tm + 4 * lg + i >= cnt) dec = 1.f, inp = 0.f;
+                    ps = dec * ps + inp;
+                    pa *= dec;
+                    av[i] = pa;
+                    sv[i] = ps;
+                }
+                // across the four lane groups (4 tokens each): e = the even group of the pair, then both pairs' totals to everyone
+                const auto swap16 = [](float v) { return __builtin_amdgcn_permlane16_swap(__float_as_uint(v), __float_as_uint(v), false, false); };
+                const auto swap32 = [](float v) { return __builtin_amdgcn_permlane32_swap(__float_as_uint(v), __float_as_uint(v), false, false); };
+                const bool odd = lg & 1;
+                const float ea = __uint_as_float(swap16(pa)[0]), es = __uint_as_float(swap16(ps)[0]);
+                const float ia = odd ? pa * ea : pa, is = odd ? pa * es + ps : ps;                  // inclusive inside the pair
+                const auto ha = swap32(__uint_as_float(swap16(ia)[1])), hs = swap32(__uint_as_float(swap16(is)[1]));
+                const float la = __uint_as_float(ha[0]), ls = __uint_as_float(hs[0]), ua_ = __uint_as_float(ha[1]), us_ = __uint_as_float(hs[1]);
+                if (!SUMMARY) {
+                    float before = lg >= 2 ? la * cs[j] + ls : cs[j];
+                    before = odd ? ea * before + es : before;                                       // the state in front of this lane's first token
+#pragma unroll
+                    for (int i = 0; i < 4; ++i) {
+                        const int ro = tm + 4 * lg + i;
+                        act_st(y_lds + ro * BLOCK + ((cb >> 3) ^ (ro & SWZ)) * 8 + (cb & 7), (av[i] * before + sv[i]) * fast_gelu(yv[i]));
+                    }
+                }
+                cs[j] = ua_ * (la * cs[j] + ls) + us_;
+                ca[j] *= la * ua_;
+            }
+        }
+        if (!SUMMARY) {
+            lds_barrier();
+            for (int e = tid; e < cnt * OCT; e += 512) {
+                const int r = e / OCT, p = e % OCT;
+                *reinterpret_cast<u32x4*>(reinterpret_cast<uint16_t*>(a.out) + (int64_t)(row0 + t0 + r) * a.out_stride + c0 + p * 8) =
+                    *reinterpret_cast<const u32x4*>(y_lds + r * BLOCK + (p ^ (r & SWZ)) * 8);
+            }
+        }
+    }
+#pragma unroll
+    for (int j = 0; j < NTW; ++j) {
+        const int nt = wave + 8 * j, ch = c0 + 16 * nt + lq;
+        if (nt < TILES && lg == 0 && (SUMMARY || !more)) {
+            a.s_loc[(int64_t)seg * a.width + ch] = cs[j];
+            if (SUMMARY && kth) a.a_cum[(int64_t)seg * a.width + ch] = ca[j];
+        }
     }
 }
 
@@ -455,14 +680,37 @@ __global__ __launch_bounds__(256) void rglru_step_kernel(const RglruArgs a, cons
 constexpr size_t kMaxLds = 160 * 1024;
 size_t walk_lds(int block) { return (size_t)CH * ((block + 8) + ((block < kGroup ? block : kGroup) + 8)) * 2; }
 size_t step_lds(int block) { return (size_t)32 * (block + 8) * 2 + 16 * 64 * sizeof(f32x4); }
+template <bool SUMMARY, int KS>
+bool scan_ks(const RglruArgs& a, hipStream_t stream) {
+    const size_t lds = scan_lds_bytes<KS>(a.taps);
+    (void)hipFuncSetAttribute(reinterpret_cast<const void*>(rglru_scan_kernel<KS, SUMMARY>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)kMaxLds);
+    rglru_scan_kernel<KS, SUMMARY><<<dim3(a.n_chunks, a.blocks), 512, lds, stream>>>(a);
+    return true;
+}
+template <bool SUMMARY>
+bool scan(const RglruArgs& a, hipStream_t stream) {
+    if (a.taps > HALO + 1 || scan_lds_bytes<8>(a.taps) > kMaxLds) return false;
+    switch (a.block / 32) {
+        case 1: return scan_ks<SUMMARY, 1>(a, stream);
+        case 2: return scan_ks<SUMMARY, 2>(a, stream);
+        case 3: return scan_ks<SUMMARY, 3>(a, stream);
+        case 4: return scan_ks<SUMMARY, 4>(a, stream);
+        case 5: return scan_ks<SUMMARY, 5>(a, stream);
+        case 6: return scan_ks<SUMMARY, 6>(a, stream);
+        case 7: return scan_ks<SUMMARY, 7>(a, stream);
+        case 8: return scan_ks<SUMMARY, 8>(a, stream);
+        default: return false;
+    }
+}
+
 template <bool SUMMARY>
 int walk(const RglruArgs& a, int f32, int generic, hipStream_t stream) {
     const size_t lds = walk_lds(a.block);
-    if (f32 || generic || lds > kMaxLds) {
+    if (f32 || generic == 1 || lds > kMaxLds) {
         const dim3 grid(a.n_chunks, a.blocks * ((a.block + 63) / 64));
         if (f32) rglru_walk_generic_kernel<float, SUMMARY><<<grid, 256, 0, stream>>>(a);
         else rglru_walk_generic_kernel<uint16_t, SUMMARY><<<grid, 256, 0, stream>>>(a);
-    } else {
+    } else if (generic == 2 || !scan<SUMMARY>(a, stream)) {
         const int waves = a.block < kGroup ? a.block / 16 : kGroup / 16;
         if (lds > 64 * 1024) (void)hipFuncSetAttribute(reinterpret_cast<const void*>(rglru_walk_kernel<SUMMARY>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)kMaxLds);
         rglru_walk_kernel<SUMMARY><<<dim3(a.n_chunks, a.blocks * ((a.block + kGroup - 1) / kGroup)), waves * 64, lds, stream>>>(a);
