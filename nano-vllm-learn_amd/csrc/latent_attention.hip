@@ -47,18 +47,20 @@ __device__ __forceinline__ void norm_part(const T* x, int cols, int n, float eps
     for (int c = (lane + 64 * RC) * 4; c < cols; c += 256) out(c, act_ld4(x + c) * inv * *reinterpret_cast<const f32x4*>(w + c));
 }
 
-// one wave per row, four rows per workgroup: no barrier
+// one wave per row part (query latent, cache row), four per workgroup: no barrier
 template <typename T>
 __global__ __launch_bounds__(256) void latent_prep_kernel(const LatentPrepArgs a) {
-    const int row = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
+    const int parts = a.kv_cols ? 2 : 1, unit = blockIdx.x * 4 + (threadIdx.x >> 6), row = unit / parts, lane = threadIdx.x & 63;
     if (row >= a.rows) return;
     const T* x = reinterpret_cast<const T*>(a.a) + (int64_t)row * a.a_stride;
     const T* c = x + a.q_cols;
-    norm_part<T>(x, a.q_cols, a.q_rank, a.eps, a.q_w, lane, [&](int i, f32x4 v) {
-        if (a.cq_packed) act_st4(reinterpret_cast<uint16_t*>(a.cq_packed) + pack_index(row, i, a.q_cols), v);
-        else act_st4(reinterpret_cast<T*>(a.cq) + (int64_t)row * a.q_cols + i, v);
-    });
-    if (a.kv_cols == 0) return;
+    if (unit - row * parts == 0) {
+        norm_part<T>(x, a.q_cols, a.q_rank, a.eps, a.q_w, lane, [&](int i, f32x4 v) {
+            if (a.cq_packed) act_st4(reinterpret_cast<uint16_t*>(a.cq_packed) + pack_index(row, i, a.q_cols), v);
+            else act_st4(reinterpret_cast<T*>(a.cq) + (int64_t)row * a.q_cols + i, v);
+        });
+        return;
+    }
     const int slot = a.slots[row];
     if (slot < 0) return;
     T* out = reinterpret_cast<T*>(a.cache) + (int64_t)slot * (a.kv_cols + a.rot_cols);
@@ -208,10 +210,10 @@ __global__ __launch_bounds__(256) void latent_attend_generic_kernel(const Latent
 }
 
 // ------------------------------------------------------------------------------------------------ attend, MFMA (bf16, one row per sequence)
-// grid (splits, rows, head tiles of 16), 4 waves.  64 keys at a time in ONE LDS image that serves as K (row reads) and as V (hardware-transposed
+// grid (splits, rows, groups of HT head tiles of 16), 4 waves per head tile.  64 keys at a time in ONE LDS image that serves as K (row reads) and as V (hardware-transposed
 // reads): wave w scores keys 16 w .. + 15 for all 16 heads (queries in registers), the waves agree on the tile's maxima through LDS, weights go to
 // LDS as bf16 hi + lo in the order the transposed reads deliver keys, and wave w sums its quarter of the latent columns.
-// Two images: the next tile's DMA is issued behind the barrier that finds this tile landed, and travels under its whole computation.
+// Two images, refilled as soon as a tile has been summed: up to two tiles travel at once, so the stream does not pause for a round trip per tile.
 __device__ __forceinline__ void lds_only_barrier() {     // (a __syncthreads() would drain the DMA in flight)
     asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
     __builtin_amdgcn_s_barrier();
@@ -225,16 +227,19 @@ __device__ __forceinline__ u32x2 ds_read_tr16(uint32_t lds_addr) {
 }
 __device__ __forceinline__ uint32_t lds_addr_of(const void* p) { return (uint32_t)(uintptr_t)(__attribute__((address_space(3))) const void*)p; }
 
-template <int NT>                                    // kv_cols = 64 * NT, rot_cols = 64
-__global__ __launch_bounds__(256) void latent_attend_kernel(const LatentAttnArgs a) {
-    constexpr int COLS = 64 * NT + 64, ROWB = COLS * 2, CPR = COLS / 8, KS = COLS / 32, NI = CPR / 4;   // NI: DMA instructions per wave
+constexpr int kAttendTileBytes = 2 * 16 * 72 * 2 + 4 * 16 * 4;                 // weights and maxima of one head tile
+
+template <int NT, int HT>                            // kv_cols = 64 * NT, rot_cols = 64
+__global__ __launch_bounds__(256 * HT) void latent_attend_kernel(const LatentAttnArgs a) {
+    constexpr int COLS = 64 * NT + 64, ROWB = COLS * 2, CPR = COLS / 8, KS = COLS / 32, NI = CPR / (4 * HT);   // NI: DMA instructions per wave
     constexpr bool kOdd = ((ROWB / 128) & 1) != 0;
     constexpr int IMG = 64 * ROWB;
     extern __shared__ __attribute__((aligned(16))) unsigned char smem[];       // [2 images][64][ROWB], 16-byte pieces swizzled inside groups of 8
-    uint16_t* p_lds = reinterpret_cast<uint16_t*>(smem + 2 * IMG);               // [hi | lo][16 heads][64 + 8]
-    float* mx_lds = reinterpret_cast<float*>(smem + 2 * IMG + 2 * 16 * 72 * 2);  // [4 waves][16]
-    const int split = blockIdx.x, row = blockIdx.y, h0 = blockIdx.z * 16;
-    const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lq = lane & 15, lg = lane >> 4;
+    const int tid = threadIdx.x, lane = tid & 63, all_wave = __builtin_amdgcn_readfirstlane(tid >> 6), lq = lane & 15, lg = lane >> 4;
+    const int ht = all_wave >> 2, wave = all_wave & 3;                         // head tile of this workgroup, wave of the tile
+    uint16_t* p_lds = reinterpret_cast<uint16_t*>(smem + 2 * IMG + ht * kAttendTileBytes);     // [hi | lo][16 heads][64 + 8]
+    float* mx_lds = reinterpret_cast<float*>(p_lds + 2 * 16 * 72);                              // [4 waves][16]
+    const int split = blockIdx.x, row = blockIdx.y, h0 = (blockIdx.z * HT + ht) * 16;
     const int ctx = (int)a.positions[row] + 1;
     const bool head_ok = h0 + lq < a.heads;
     int k0, k1;
@@ -257,20 +262,22 @@ __global__ __launch_bounds__(256) void latent_attend_kernel(const LatentAttnArgs
         const int live = k1 - t0 < 64 ? k1 - t0 : 64;
 #pragma unroll
         for (int j = 0; j < NI; ++j) {
-            const int s = (wave * NI + j) * 64 + lane;
+            const int s = (all_wave * NI + j) * 64 + lane;
             const int r = s / CPR, place = s - r * CPR, piece = place ^ swz(r);
             const int rc = r < live ? r : live - 1;                                           // (rows past the context repeat its last one: masked)
             __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)(base + rc * COLS + piece * 8),
-                                             (__attribute__((address_space(3))) void*)(img + (wave * NI + j) * 1024), 16, 0, 0);
+                                             (__attribute__((address_space(3))) void*)(img + (all_wave * NI + j) * 1024), 16, 0, 0);
         }
     };
-    stage(k0, 0);
     bf16x8 qf[KS];                                   // B operand: column = head lq, 8 consecutive columns
     {
         const uint16_t* q = reinterpret_cast<const uint16_t*>(a.qa) + ((int64_t)row * a.heads + (head_ok ? h0 + lq : a.heads - 1)) * COLS + 8 * lg;
 #pragma unroll
         for (int s = 0; s < KS; ++s) qf[s] = *reinterpret_cast<const bf16x8*>(q + 32 * s);
     }
+    // (the queries' loads are issued in front of the tiles': vector-memory operations complete in order)
+    stage(k0, 0);
+    if (k0 + 64 < k1) stage(k0 + 64, 1);
     f32x4 o[NT];                                     // latent columns 64 t' .. : tile index 4 t + wave -> columns 16 (4 t + wave) + 4 lg, head lq
 #pragma unroll
     for (int t = 0; t < NT; ++t) o[t] = f32x4{0.f, 0.f, 0.f, 0.f};
@@ -281,16 +288,18 @@ __global__ __launch_bounds__(256) void latent_attend_kernel(const LatentAttnArgs
     auto tile_body = [&](auto bufc, const int t0) {
         constexpr int buf = decltype(bufc)::value;
         const unsigned char* img = smem + buf * IMG;
-        asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
-        lds_only_barrier();                          // the tile is in LDS, and every wave is done with the one before it
-        if (t0 + 64 < k1) stage(t0 + 64, buf ^ 1);
+        if (t0 + 64 < k1) asm volatile("s_waitcnt vmcnt(%0)" ::"n"(NI) : "memory");
+        else asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+        lds_only_barrier();                          // this tile is in LDS, the next one travels
         const int R = 16 * wave + lq;
-        f32x4 s4 = {0.f, 0.f, 0.f, 0.f};
+        f32x4 s4 = {0.f, 0.f, 0.f, 0.f}, s4b = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
         for (int s = 0; s < KS; ++s) {
             const bf16x8 kf = *reinterpret_cast<const bf16x8*>(img + R * ROWB + ((4 * s + lg) ^ swz(R)) * 16);
-            s4 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[s], s4, 0, 0, 0);
+            if (s & 1) s4b = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[s], s4b, 0, 0, 0);
+            else s4 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[s], s4, 0, 0, 0);
         }
+        s4 += s4b;
         float mx = -INFINITY;
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
@@ -338,6 +347,10 @@ __global__ __launch_bounds__(256) void latent_attend_kernel(const LatentAttnArgs
                 o[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, ph, o[t], 0, 0, 0);
                 o[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pl, o[t], 0, 0, 0);
             }
+        }
+        if (t0 + 128 < k1) {
+            lds_only_barrier();                      // every wave is done with this image: the tile after the next may have it
+            stage(t0 + 128, buf);
         }
     };
     for (int t0 = k0; t0 < k1; t0 += 128) {
@@ -388,10 +401,19 @@ template <int RW>
 __global__ __launch_bounds__(512) void latent_value_kernel(const LatentAttnArgs a) {
     extern __shared__ __attribute__((aligned(16))) uint16_t lat[];             // [RW][kv_cols + 8]
     __shared__ float wsp[RW][64];
-    constexpr int PRE = 8;
+    constexpr int PRE = 16;
     const int head = blockIdx.x, r0 = blockIdx.y * RW, ld = a.kv_cols + 8, pieces = a.kv_cols / 4, ksteps = a.kv_cols / 32;
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, lq = lane & 15, lg = lane >> 4;
     const uint16_t* w_head = reinterpret_cast<const uint16_t*>(a.w_uv) + ((int64_t)head * a.v_cols + lq) * a.kv_cols + 8 * lg;
+    // this thread's first piece: the sums of the first PS splits, asked for before their weights are known (places past the live splits are dropped)
+    constexpr int PS = 8;
+    f32x4 first[PS];
+    {
+        const int r = tid / pieces, row = r0 + r < a.rows && r < RW ? r0 + r : r0;
+        const float* p = a.part_o + ((int64_t)row * a.splits * a.heads + head) * a.kv_cols + (tid - r * pieces) * 4;
+#pragma unroll
+        for (int s = 0; s < PS; ++s) first[s] = *reinterpret_cast<const f32x4*>(p + (s < a.splits ? s : 0) * (int64_t)a.heads * a.kv_cols);
+    }
     bf16x8 pre[PRE];
     {
         const uint16_t* w = w_head + (int64_t)(16 * wave < a.v_cols ? 16 * wave : 0) * a.kv_cols;
@@ -422,8 +444,13 @@ __global__ __launch_bounds__(512) void latent_value_kernel(const LatentAttnArgs 
             const int n = live_splits(r0 + r);
             const float* p = a.part_o + ((int64_t)(r0 + r) * a.splits * a.heads + head) * a.kv_cols + c;
             const int64_t step = (int64_t)a.heads * a.kv_cols;
+            if (e == tid) {
+#pragma unroll
+                for (int s = 0; s < PS; ++s)
+                    if (s < n) v += first[s] * wsp[r][s];
+            }
 #pragma unroll 4
-            for (int s = 0; s < n; ++s) v += *reinterpret_cast<const f32x4*>(p + s * step) * wsp[r][s];
+            for (int s = e == tid ? PS : 0; s < n; ++s) v += *reinterpret_cast<const f32x4*>(p + s * step) * wsp[r][s];
         }
         act_st4(lat + r * ld + c, v);
     }
@@ -433,9 +460,14 @@ __global__ __launch_bounds__(512) void latent_value_kernel(const LatentAttnArgs 
         const uint16_t* w = w_head + (int64_t)16 * nt * a.kv_cols;
         f32x4 acc = {0.f, 0.f, 0.f, 0.f};
         if (nt == wave) {
+            f32x4 acc2 = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
             for (int k = 0; k < PRE; ++k)
-                if (k < ksteps) acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(pre[k], *reinterpret_cast<const bf16x8*>(l_row + 32 * k), acc, 0, 0, 0);
+                if (k < ksteps) {
+                    f32x4& c = k & 1 ? acc2 : acc;
+                    c = __builtin_amdgcn_mfma_f32_16x16x32_bf16(pre[k], *reinterpret_cast<const bf16x8*>(l_row + 32 * k), c, 0, 0, 0);
+                }
+            acc += acc2;
         }
         for (int k = nt == wave ? PRE : 0; k < ksteps; ++k)
             acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8*>(w + 32 * k), *reinterpret_cast<const bf16x8*>(l_row + 32 * k), acc, 0, 0, 0);
@@ -489,17 +521,22 @@ __global__ __launch_bounds__(256) void latent_gather_kernel(u32x4* __restrict__ 
     out[e] = cache[(page * block_size + key % block_size) * pieces + p];
 }
 
+template <int NT, int HT>
+void attend_ht(const LatentAttnArgs& a, hipStream_t stream) {
+    constexpr size_t lds = 2 * 64 * (64 * NT + 64) * 2 + HT * kAttendTileBytes;
+    if (lds > 64 * 1024) (void)hipFuncSetAttribute(reinterpret_cast<const void*>(latent_attend_kernel<NT, HT>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+    latent_attend_kernel<NT, HT><<<dim3(a.splits, a.rows, (a.heads + 16 * HT - 1) / (16 * HT)), 256 * HT, lds, stream>>>(a);
+}
 template <int NT>
 void attend_nt(const LatentAttnArgs& a, hipStream_t stream) {
-    constexpr size_t lds = 2 * 64 * (64 * NT + 64) * 2 + 2 * 16 * 72 * 2 + 4 * 16 * 4;
-    if (lds > 64 * 1024) (void)hipFuncSetAttribute(reinterpret_cast<const void*>(latent_attend_kernel<NT>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
-    latent_attend_kernel<NT><<<dim3(a.splits, a.rows, (a.heads + 15) / 16), 256, lds, stream>>>(a);
+    if (a.heads > 16) attend_ht<NT, 2>(a, stream);   // two head tiles share the images: one stream over the cache for 32 heads
+    else attend_ht<NT, 1>(a, stream);
 }
 
 }  // namespace
 
 int launch_latent_prep(const LatentPrepArgs& a, int f32, hipStream_t stream) {
-    const int grid = (a.rows + 3) / 4;
+    const int grid = (a.rows * (a.kv_cols ? 2 : 1) + 3) / 4;
     if (f32) latent_prep_kernel<float><<<grid, 256, 0, stream>>>(a);
     else latent_prep_kernel<uint16_t><<<grid, 256, 0, stream>>>(a);
     return check_launch("latent_prep");

@@ -15,20 +15,25 @@ from .linear import linear, padded, round_up
 CUS = 256                     # compute units of an MI355X: one walking workgroup keeps one busy
 
 
+SEGMENT_OVERHEAD = 0.8        # start of a walk (gate weights into registers, first rows) in units of one 64-token step
+SUMMARY_SHARE = 0.7           # a summary walk's step against a full one's
+
+
 def choose_segment(portions, blocks, chunk=64):
     """Tokens per segment for portions of these lengths: one workgroup walks one (segment, diagonal block), and cutting a portion into more than one
-    costs a summary walk (about 0.7 of a full one) over all its segments but the last.  Returns the cheapest power-of-two multiple of `chunk`."""
-    best, longest = None, max(portions, default=1)
-    seg = chunk
-    while True:
-        pieces = [-(-n // seg) for n in portions]
-        steps = min(seg, longest) / chunk
-        cost = -(-sum(pieces) * blocks // CUS) * steps + 0.7 * -(-sum(p - 1 for p in pieces) * blocks // CUS) * steps
-        if best is None or cost < best[0]:
-            best = (cost, seg)
-        if seg >= longest:
-            return best[1]
-        seg *= 2
+    costs a summary walk over all its segments but the last.  Returns the cheapest multiple of `chunk` among about ten per octave of lengths."""
+    longest = max(portions, default=1)
+    last = -(-longest // chunk)
+
+    def cost(k):
+        pieces = [-(-n // (k * chunk)) for n in portions]
+        walk, summary = -(-sum(pieces) * blocks // CUS), -(-sum(p - 1 for p in pieces) * blocks // CUS)
+        return (walk + SUMMARY_SHARE * summary) * (min(k, last) + SEGMENT_OVERHEAD)
+    steps, k = [last], 1
+    while k < last:
+        steps.append(k)
+        k += max(1, k // 8)
+    return chunk * min(steps, key=cost)
 
 
 class RGLRU(nn.Module):

@@ -751,7 +751,8 @@ def latent_splits(rows, heads, max_context, mfma, cache_cols=576) -> int:
     if not mfma:
         return max(1, min(512 // max(1, rows * heads), tiles, 64))
     resident = 256 * (2 if 4 * 64 * cache_cols * 2 + 16384 <= 163840 else 1)
-    splits = max(1, min(resident // (rows * ((heads + 15) // 16)), tiles, 64))
+    groups = 1 if heads <= 16 else (heads + 31) // 32
+    splits = max(1, min(resident // (rows * groups), tiles, 64))
     per = -(-tiles // splits)
     return -(-tiles // per)
 
