@@ -405,6 +405,16 @@ __global__ __launch_bounds__(512) void latent_value_kernel(const LatentAttnArgs 
     const int head = blockIdx.x, r0 = blockIdx.y * RW, ld = a.kv_cols + 8, pieces = a.kv_cols / 4, ksteps = a.kv_cols / 32;
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, lq = lane & 15, lg = lane >> 4;
     const uint16_t* w_head = reinterpret_cast<const uint16_t*>(a.w_uv) + ((int64_t)head * a.v_cols + lq) * a.kv_cols + 8 * lg;
+    // everything this workgroup reads is asked for at once: maxima and sums of its rows' splits (lane = split; places past the live ones are dropped)
+    constexpr int RPW = (RW + 7) / 8;
+    float ms_all[RPW], ls_all[RPW];
+#pragma unroll
+    for (int i = 0; i < RPW; ++i) {
+        const int r = wave + 8 * i, row = r < RW && r0 + r < a.rows ? r0 + r : r0;
+        const int64_t rec = ((int64_t)row * a.splits + (lane < a.splits ? lane : 0)) * a.heads + head;
+        ms_all[i] = a.part_ml[rec * 2];
+        ls_all[i] = a.part_ml[rec * 2 + 1];
+    }
     // this thread's first piece: the sums of the first PS splits, asked for before their weights are known (places past the live splits are dropped)
     constexpr int PS = 8;
     f32x4 first[PS];
@@ -424,11 +434,12 @@ __global__ __launch_bounds__(512) void latent_value_kernel(const LatentAttnArgs 
         const int tiles = ((int)a.positions[row] + 64) / 64, per = (tiles + a.splits - 1) / a.splits;
         return (tiles + per - 1) / per;
     };
-    for (int r = wave; r < RW; r += 8) {
-        if (r0 + r >= a.rows) break;
+#pragma unroll
+    for (int i = 0; i < RPW; ++i) {
+        const int r = wave + 8 * i;
+        if (r >= RW || r0 + r >= a.rows) break;
         const bool ok = lane < live_splits(r0 + r);
-        const int64_t rec = ((int64_t)(r0 + r) * a.splits + (ok ? lane : 0)) * a.heads + head;
-        const float ms = ok ? a.part_ml[rec * 2] : -INFINITY, ls = ok ? a.part_ml[rec * 2 + 1] : 0.f;
+        const float ms = ok ? ms_all[i] : -INFINITY, ls = ok ? ls_all[i] : 0.f;
         float m = ms;
         for (int d = 1; d < 64; d <<= 1) m = fmaxf(m, __shfl_xor(m, d));
         const float e = fast_exp2(ms - m);

@@ -378,8 +378,7 @@ __device__ __forceinline__ bool prefill_varlen_body(const PrefillArgs& a, unsign
                 const float m_new = max2(m_run[qs], mx);
                 // rows that have seen no key yet keep m = -inf; use 0 as the reference point so exp2 stays finite
                 const float m_use = m_new == -INFINITY ? 0.f : m_new;
-                // scale-and-subtract and the row sum on element PAIRS (v_pk_fma_f32 / v_pk_add_f32: two lanes' worth per issue slot;
-                // the loop is VALU-bound), exp2 per element
+                // scale-and-subtract and the row sum on element pairs (plain fp32 instructions: packed ones are switched off in the build), exp2 per element
                 const f32x2 sc2 = {a.scale_log2, a.scale_log2}, mm2 = {-m_use, -m_use};
                 f32x2 psum2 = {0.f, 0.f};
 #pragma unroll
