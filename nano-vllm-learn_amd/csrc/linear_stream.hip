@@ -716,14 +716,17 @@ int linear_stream_candidate_groups(int n, int k) {
     return tiles > 1024 ? (int)kMultiWgs : tiles;
 }
 
-// counters [tiles], ONE PER 128-BYTE LINE (the memory side executes the adds on one line one after the other: dense tickets made every
+// A FIXED ticket header (the same bytes whatever the shape: launches of different tile counts share one workspace, and one's partials must never lie
+// where another's tickets are), tickets ONE PER 128-BYTE LINE (the memory side executes the adds on one line one after the other: dense tickets made every
 // tile's last arriver queue behind its neighbours' adds), then partial records [tiles][ksplit][NB*MT*256 + MT*16] fp32; 0 when K needs no split
+constexpr size_t kTicketTiles = 32768;             // n up to 524288 columns
+constexpr size_t kTicketHeader = kTicketTiles * kTicketWords * 4;
 size_t linear_stream_workspace_bytes(int m, int n, int k, int epi) {
     const int pieces = k / 64, ksplit = (pieces + SW * PMAX - 1) / (SW * PMAX);
     if (ksplit <= 1) return 0;
     const int nb = (epi == EPI_SILU || epi == EPI_ROPE) ? 2 : 1, mt = (m + 15) / 16;
     const int tiles = nb == 2 ? n / 32 : n / 16;
-    return (size_t)tiles * kTicketWords * 4 + (size_t)tiles * ksplit * (nb * mt * 256 + mt * 16) * 4;
+    return kTicketHeader + (size_t)tiles * ksplit * (nb * mt * 256 + mt * 16) * 4;
 }
 
 // Returns -100 when the call is not this kernel's (the caller falls back to skinny_gemm.hip's loop kernel).
@@ -736,11 +739,11 @@ int launch_linear_stream(const LinearArgs& a_in, hipStream_t stream) {
     const int pieces = a.K / 64;
     a.ksplit = (pieces + SW * PMAX - 1) / (SW * PMAX);
     if (a.ksplit > 1) {
-        const size_t counters_bytes = (size_t)a.tiles * kTicketWords * 4;
+        if ((size_t)a.tiles > kTicketTiles) return -100;
         const int nb = (a.epi == EPI_SILU || a.epi == EPI_ROPE) ? 2 : 1, mt = (a.M + 15) / 16;
-        if (!a.ws_raw || a.ws_bytes < counters_bytes + (size_t)a.tiles * a.ksplit * (nb * mt * 256 + mt * 16) * 4) return -100;
+        if (!a.ws_raw || a.ws_bytes < kTicketHeader + (size_t)a.tiles * a.ksplit * (nb * mt * 256 + mt * 16) * 4) return -100;
         a.counters = reinterpret_cast<unsigned*>(a.ws_raw);
-        a.ws = reinterpret_cast<float*>(reinterpret_cast<unsigned char*>(a.ws_raw) + counters_bytes);
+        a.ws = reinterpret_cast<float*>(reinterpret_cast<unsigned char*>(a.ws_raw) + kTicketHeader);
     }
     switch ((a.M + 15) / 16) {
         case 1: return launch_mt<1>(a, stream);

@@ -61,7 +61,7 @@ class ZobasunConfig:
 
 
 class _DecodeBuffers:
-    """Scratch of the fused decode path for one batch size: fragment-order activations by width and the split-K workspace (zero-filled once)."""
+    """Scratch of the fused decode path for one number of 16-row tiles: fragment-order activations by width and the split-K workspace (zero-filled once)."""
 
     def __init__(self, rows, device, linears, stream_cols):
         self.rows16, self.device, self._packed = round_up(rows, 16), device, {}
@@ -151,6 +151,7 @@ class ZobasunForCausalLM(nn.Module):
                 and all(getattr(layer.mixer, "step_ok", True) for layer in self.layers))
 
     def _decode_buffers(self, rows):
+        rows = round_up(rows, 16)
         if rows not in self._bufs:
             lin = [l for layer in self.layers for l in layer.mixer.linears() + (layer.mlp.linears() if layer.mlp is not None else [])]
             self._bufs[rows] = _DecodeBuffers(rows, self.embed.device, lin + [(self.head, "none")], self.cols)

@@ -290,6 +290,21 @@ def test_stream_linear_split_k_residual_add(m, n, k):
     assert int(ws[: tiles * 128].view(torch.int32).abs().sum()) == 0       # one ticket per 128-byte line, all back at zero
 
 
+def test_stream_linear_shapes_share_a_workspace():
+    """Split-K launches of different tile counts and splits, interleaved on ONE workspace: a launch's partial sums must not land on another's tickets."""
+    from nanovllm_hip import ops
+    m, shapes = 20, [(4096, 1536, "none"), (192, 5120, "none"), (2560, 2048, "silu_mul"), (1024, 3072, "none"), (4800, 1088, "none")]
+    g = torch.Generator().manual_seed(5)
+    data = [(torch.randn(m, k, generator=g).bfloat16().cuda(), (torch.randn(n, k, generator=g) * k ** -0.5).bfloat16().cuda(), e) for n, k, e in shapes]
+    ws = _zero_ws(max(ops.linear_workspace_bytes(m, n, k, e) for n, k, e in shapes))
+    for _ in range(4):
+        for x, w, e in data:
+            alone = ops.fused_linear(x, w, epilogue=e, workspace=_zero_ws(ops.linear_workspace_bytes(m, w.shape[0], w.shape[1], e)))
+            out = torch.full_like(alone, float("nan"))
+            ops.fused_linear(x, w, epilogue=e, workspace=ws, out=out)
+            assert torch.equal(out, alone)
+
+
 def test_stream_linear_split_k_silu_and_rope():
     """The non-linear epilogues run in the last arriver on the complete sums (Qwen2-7B tp=4 shapes: hidden 3584, heads 7/1 x 128)."""
     from nanovllm_hip import ops

@@ -37,6 +37,9 @@ CONFIGS = {
                               latent(4, 128, 64, 64, 64, 512, 0.07)], eps=1e-6, scale=1.0),
     # beyond the MFMA kernels: wide latent, wide rotation, wide keys; these layers run on the plain kernels in bf16 too
     "plain": config(136, 90, [latent(2, 210, 80, 150, 40, 530, 0.08), recurrent(40, 5, 4, mlp=dense(72, 1.0)), latent(3, 30, 80, 20, 24, 530, 0.1, kv_from=0)]),
+    # contractions longer than 1024, each projection with its own split: the decode path's shared split-K workspace
+    "long": config(1280, 300, [recurrent(1536, 6, 4, mlp=dense(1700, 1.0)), latent(10, 64, 32, 128, 1100, 320, 0.1, mlp=dense(2100, 2.0)), recurrent(1100, 5, 3)],
+                   scale=2.0),
 }
 
 
