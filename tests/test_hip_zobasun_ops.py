@@ -293,7 +293,7 @@ class Latent:
 
 
 #            heads dim dim_cols rot vdim v_cols kv kv_cols rot_cols
-LAT = {"one": (1, 8, 32, 8, 16, 64, 20, 64, 64), "small": (6, 32, 32, 32, 48, 64, 64, 64, 64), "many": (20, 64, 64, 64, 128, 128, 250, 256, 64),
+LAT = {"one": (1, 8, 32, 8, 16, 64, 20, 64, 64), "small": (7, 32, 32, 24, 40, 64, 56, 64, 64), "many": (20, 64, 64, 64, 128, 128, 250, 256, 64),
        "big": (16, 128, 128, 64, 128, 128, 512, 512, 64), "three": (3, 40, 64, 24, 50, 64, 129, 192, 64), "heads40": (40, 32, 32, 16, 64, 64, 384, 384, 64), "wide": (2, 70, 96, 90, 130, 192, 600, 640, 128)}
 
 
