@@ -565,6 +565,147 @@ typedef struct nvh_latent_prefill_desc {
 int nvh_latent_prefill(const nvh_latent_prefill_desc* d, int dtype, void* stream);
 int nvh_latent_prefill_supported(int dk, int dv);
 
+/* ================================================================================================================================
+ * Softmax attention over pages with windows, kept first tokens and sinks; lightning attention; mixture of experts; row ops of models whose
+ * sublayers share one layer norm.  `dtype` and "cols" as in the section above.
+ *
+ * Cache pages of one attention layer: [pages][kv_heads][block_size rows of dk keys, then block_size rows of dv values].
+ */
+/* Row ops behind a q | k | v projection, in place: optional RMS norm over all query columns and over all key columns at once, rotation of
+ * interleaved pairs of queries and keys, keys and values into the cache. */
+typedef struct nvh_attn_prep_desc {
+    void* qkv;                   /* [rows, heads * dk | kv_heads * dk | kv_heads * dv], row stride qkv_stride; queries are rewritten */
+    int64_t qkv_stride;
+    int32_t rows, heads, kv_heads, dk, dv;
+    const float* q_w;            /* nullable: [heads * dk] norm weight (then k_w too) */
+    const float* k_w;            /* [kv_heads * dk] */
+    int32_t q_n, k_n;            /* columns the means run over (the rest is zero padding) */
+    float eps;
+    const int64_t* positions;    /* [rows] */
+    const float* cos_sin;        /* [max_position, rot]: cos(0..rot/2) | sin(0..rot/2) */
+    int32_t max_position, rot;   /* rot <= dk: leading dimensions of a head that turn */
+    void* cache;
+    const int32_t* slots;        /* [rows] page * block_size + offset; < 0: not stored */
+    int32_t block_size;
+} nvh_attn_prep_desc;
+int nvh_attn_prep(const nvh_attn_prep_desc* d, int dtype, void* stream);
+/* softmax(scale q . k) v over the keys a query sees: position j of its sequence if j <= its own and (window == 0 or nearer than `window` or
+ * j < keep_first).  sink (nullable): exp(sink[head]) joins the denominator.  Query head h reads key/value head h / (heads / kv_heads).
+ *   rows form   (nvh_paged_attend_rows): row i belongs to sequence row_seq[i] (or i); splits > 1: context splits, merged by the last workgroup to arrive
+ *   portions    (nvh_paged_attend_prompt, bf16): rows cu_q[b] .. of sequence b are its last ones, cu_k[b + 1] - cu_k[b] keys in all
+ * MFMA / streaming forms for the widths nvh_paged_attend_supported names; `generic` (rows form): the plain kernel, any width up to 2048. */
+typedef struct nvh_paged_attend_desc {
+    const void* q;               /* [rows, heads, dk], row stride q_stride */
+    int64_t q_stride;
+    int32_t rows, heads, kv_heads, dk, dv;
+    const void* cache;
+    int32_t block_size;
+    const int32_t* block_tables; /* [sequences, bt_stride] */
+    int64_t bt_stride;
+    const int32_t* row_seq;      /* nullable */
+    const int64_t* positions;    /* [rows] (rows form) */
+    const int32_t* cu_q;         /* [batch + 1] (portions) */
+    const int32_t* cu_k;
+    int32_t batch, max_q;
+    float scale;
+    int32_t window, keep_first;
+    const float* sink;           /* nullable: [heads] */
+    int32_t splits;
+    float* part_o;               /* splits > 1: [rows, heads, splits, dv] scratch */
+    float* part_ml;              /* [rows, heads, splits, 2] */
+    uint32_t* tickets;           /* zero before the launch, left zero: nvh_paged_attend_ticket_bytes(rows, kv_heads, heads) */
+    void* out;                   /* nullable: [rows, heads * dv], row stride out_stride */
+    int64_t out_stride;
+    void* out_packed;            /* nullable (bf16, rows form): the same in MFMA-fragment order */
+} nvh_paged_attend_desc;
+int nvh_paged_attend_supported(int dk, int dv, int block_size);
+size_t nvh_paged_attend_ticket_bytes(int rows, int kv_heads, int heads);
+int nvh_paged_attend_rows(const nvh_paged_attend_desc* d, int generic, int dtype, void* stream);
+int nvh_paged_attend_prompt(const nvh_paged_attend_desc* d, int dtype, void* stream);
+
+/* Lightning attention: per head S = decay S + k v^T, o = S^T q with q, k, v = silu of the projection's columns (rounded to the activation type);
+ * the state is fp32.  nvh_lightning_chunks: portions cut into segments as for nvh_rglru_chunks; nvh_lightning_step: row i is one new token of
+ * sequence i.  A token at position 0 takes the state as zero.  generic (chunks): the plain token-by-token kernel, any width; the MFMA form and the step need
+ * nvh_lightning_supported(dk, dv). */
+typedef struct nvh_lightning_desc {
+    const void* qkv;             /* [rows, heads * dk | heads * dk | heads * dv], row stride qkv_stride */
+    int64_t qkv_stride;
+    int32_t rows, heads, dk, dv;
+    const float* decay;          /* [heads] */
+    const int64_t* positions;    /* [rows] */
+    const int32_t* state_slots;  /* [sequences]; < 0: nothing is read or kept */
+    float* state;                /* [slots, heads, dk, dv] */
+    const int32_t* chunks;       /* [n_chunks, 4]: first row, rows, sequence, index of the segment in its sequence's portion */
+    int32_t n_chunks;
+    int32_t summaries;           /* != 0: some portion has more than one segment */
+    float* seg_state;            /* summaries: [n_chunks, heads, dk, dv] scratch */
+    void* out;                   /* [rows, heads * dv], row stride out_stride */
+    int64_t out_stride;
+} nvh_lightning_desc;
+int nvh_lightning_supported(int dk, int dv);
+int nvh_lightning_chunks(const nvh_lightning_desc* d, int generic, int dtype, void* stream);
+int nvh_lightning_step(const nvh_lightning_desc* d, int dtype, void* stream);
+/* out = rmsnorm(x over n columns) * w * sigmoid(gate); packed (nullable, bf16): in fragment order instead. */
+int nvh_norm_gate(void* out, void* packed, const void* x, const void* gate, const float* w, float eps, int rows, int cols, int n, int64_t x_stride,
+                  int64_t gate_stride, int64_t out_stride, int dtype, void* stream);
+
+/* Mixture of experts.  Route: s = sigmoid(h . router_e) in 32-bit; choice scores s + correction; the experts form `groups` equal groups of neighbours,
+ * a group counts the sum of its two largest choice scores, the best `keep` groups stay open, the `top` largest choice scores among them win;
+ * weights s / (sum + 1e-20) * scale.  Pair p = row * top + k. */
+typedef struct nvh_moe_route_desc {
+    const void* x;               /* [rows, cols], row stride x_stride */
+    int64_t x_stride;
+    const void* router;          /* [experts, cols] */
+    const float* correction;     /* [experts] */
+    int32_t rows, cols, experts, top, groups, keep;
+    float scale;
+    int32_t* ids;                /* [rows, top] */
+    float* weights;              /* [rows, top] */
+} nvh_moe_route_desc;
+int nvh_moe_route(const nvh_moe_route_desc* d, int dtype, void* stream);
+/* Pairs sorted by expert: slot_pair[slot], tiles [max_tiles][4] = (expert, first slot, slots, tiles in use), unused ones with
+ * 0 slots, tile_rows slots each;
+ * counts: [nvh_moe_dispatch_blocks(pairs), experts] scratch.  max_tiles >= pairs / tile_rows + experts. */
+int nvh_moe_dispatch_blocks(int pairs);
+int nvh_moe_dispatch(int32_t* slot_pair, int32_t* tiles, int32_t* counts, const int32_t* ids, int pairs, int experts, int tile_rows, int max_tiles, void* stream);
+/* Expert products.  glu: act[p] = silu(x[p / top] . gate_e) * (x . up_e), w = [experts, 2 * n, k] (gate rows, then up rows); otherwise
+ * out[p] = x[p] . w_e, w = [experts, n, k].
+ * tiles == NULL: small batches (bf16, at most 64 rows), the pairs of an expert found from ids; otherwise tiles from nvh_moe_dispatch (nvh_moe_tile_rows(dtype)
+ * rows each).  n and k multiples of 64. */
+typedef struct nvh_moe_gemm_desc {
+    void* out;                   /* [pairs, n] */
+    const void* x;               /* glu: [rows, k], row stride x_stride; otherwise [pairs, k] */
+    int64_t x_stride;
+    const void* w;
+    int32_t pairs, top, experts, n, k, glu;
+    const int32_t* ids;          /* [pairs] (small form) */
+    const int32_t* slot_pair;    /* [pairs] */
+    const int32_t* tiles;
+    int32_t max_tiles;
+} nvh_moe_gemm_desc;
+int nvh_moe_tile_rows(int dtype);
+int nvh_moe_gemm(const nvh_moe_gemm_desc* d, int dtype, void* stream);
+
+/* x (fp32 stream) += y + sum_k ew[row, k] * e[row * top + k]  (each part nullable), then, with w given, the layer norm of the new row:
+ * (x - mean) / sqrt(var + eps) * w + b. */
+typedef struct nvh_residual_norm_desc {
+    float* x;                    /* [rows, cols] */
+    const void* y;               /* nullable: [rows, cols], row stride y_stride */
+    int64_t y_stride;
+    const void* e;               /* nullable: [rows * top, cols] expert outputs */
+    const float* ew;             /* [rows, top] */
+    int32_t top;
+    const float* w;              /* nullable: no norm */
+    const float* b;
+    float eps;
+    int32_t rows, cols, n;       /* n: elements mean and variance run over */
+    void* xb;                    /* nullable: the normed rows in the activation type */
+    void* packed;                /* nullable (bf16): the same in MFMA-fragment order */
+} nvh_residual_norm_desc;
+int nvh_residual_norm(const nvh_residual_norm_desc* d, int dtype, void* stream);
+/* x = cap * tanh(x / cap) in place, rows of `cols` elements. */
+int nvh_softcap(void* x, float cap, int rows, int cols, int64_t stride, int dtype, void* stream);
+
 #ifdef __cplusplus
 }
 #endif

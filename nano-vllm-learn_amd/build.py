@@ -18,12 +18,15 @@ CSRC = os.path.join(HERE, "csrc")
 OUT_DIR = os.path.join(HERE, "nanovllm_hip", "lib")
 OBJ_DIR = os.path.join(HERE, "build")
 LIB = os.path.join(OUT_DIR, "libnvh_attn.so")
-LAYERS_LIB = os.path.join(OUT_DIR, "libnvh_layers.so")       # the LAYER_SOURCES subset of the same library
-# the linear layer, row ops, recurrence and latent attention: all that a model without paged K/V attention needs
-LAYER_SOURCES = ["api_layers.hip", "api_hybrid.hip", "layer_ops.hip", "skinny_gemm.hip", "linear_stream.hip", "hybrid_ops.hip", "rglru.hip", "latent_attention.hip",
-                 "latent_prefill.hip"]
-SOURCES = ["api.hip", "store_kvcache.hip", "paged_decode.hip", "prefill_mfma.hip", "rope_store.hip", "allreduce_oneshot.hip", "qkv_attend.hip", *LAYER_SOURCES]
-HEADERS = ["common.h", "kernels.h", "hybrid.h", "api_common.h", "decode_chunked.h", os.path.join("..", "..", "include", "nvh_attn.h")]
+# what a model needs beside the linear layer and the row ops (both in LINEAR_SOURCES): the kernels of its mixers and feed-forwards
+LINEAR_SOURCES = ["api_layers.hip", "api_rows.hip", "layer_ops.hip", "skinny_gemm.hip", "linear_stream.hip", "hybrid_ops.hip"]
+MODEL_SOURCES = {
+    "Zobasun": ["api_hybrid.hip", "rglru.hip", "latent_attention.hip", "latent_prefill.hip"],
+    "Galirax": ["api_mixers.hip", "paged_attend.hip", "paged_prompt.hip", "lightning.hip", "moe.hip"],
+}
+SOURCES = ["api.hip", "store_kvcache.hip", "paged_decode.hip", "prefill_mfma.hip", "rope_store.hip", "allreduce_oneshot.hip", "qkv_attend.hip", *LINEAR_SOURCES,
+           *[s for sources in MODEL_SOURCES.values() for s in sources]]
+HEADERS = ["common.h", "kernels.h", "hybrid.h", "mixers.h", "attend_tile.h", "api_common.h", "decode_chunked.h", os.path.join("..", "..", "include", "nvh_attn.h")]
 HIPCC = os.environ.get("HIPCC", "/opt/rocm/bin/hipcc")
 # -amdgpu-mfma-vgpr-form: MFMA results stay in the architectural VGPRs.  By default hipcc parks accumulators in the AGPR file
 # and pays a v_accvgpr_read/write per element wherever VALU code touches them (softmax on S, rescale of O): 159 such moves in
@@ -64,10 +67,14 @@ def _compile(src, asm, extra=(), obj_dir=None):
     return obj
 
 
-def build(force=False, asm=False, verbose=True, layers_only=False):
-    """Compile every HIP source for gfx950 and link libnvh_attn.so — or, with layers_only, the LAYER_SOURCES subset into
-    libnvh_layers.so.  Returns the library path."""
-    sources, lib = (LAYER_SOURCES, LAYERS_LIB) if layers_only else (SOURCES, LIB)
+def subset_lib(model):
+    return os.path.join(OUT_DIR, f"libnvh_{model.lower()}.so")
+
+
+def build(force=False, asm=False, verbose=True, model=None):
+    """Compile every HIP source for gfx950 and link libnvh_attn.so — or, with the name of a model in MODEL_SOURCES, what that model needs into a
+    library of its own.  Returns the library path."""
+    sources, lib = (LINEAR_SOURCES + MODEL_SOURCES[model], subset_lib(model)) if model else (SOURCES, LIB)
     os.makedirs(OUT_DIR, exist_ok=True)
     os.makedirs(OBJ_DIR, exist_ok=True)
     stamp = os.path.join(OBJ_DIR, f"digest_{os.path.basename(lib)}.txt")
@@ -105,6 +112,7 @@ if __name__ == "__main__":
     ap = argparse.ArgumentParser()
     ap.add_argument("--force", action="store_true")
     ap.add_argument("--asm", action="store_true", help="also emit .s and register/LDS usage per kernel into build/")
+    ap.add_argument("--model", choices=sorted(MODEL_SOURCES), help="only the kernels this model needs, into a library of their own")
     ap.add_argument("--variant", help="output path of an A/B build with --extra flags (the default library is untouched)")
     ap.add_argument("--extra", nargs="*", default=[], help="extra hipcc flags of the variant, e.g. =-DNVH_DMA_AUX=2 (leading '=' keeps argparse off them)")
     args = ap.parse_args()
@@ -112,6 +120,6 @@ if __name__ == "__main__":
         if args.variant:
             build_variant(args.variant, [e.lstrip("=") for e in args.extra])
             sys.exit(0)
-        build(force=args.force, asm=args.asm)
+        build(force=args.force, asm=args.asm, model=args.model)
     except subprocess.CalledProcessError as e:
         sys.exit(e.returncode)

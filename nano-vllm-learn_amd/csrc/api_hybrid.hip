@@ -7,14 +7,6 @@ using namespace nvh;
 
 namespace {
 
-#define REQUIRE(cond, code, ...) do { if (!(cond)) { set_error(__VA_ARGS__); return code; } } while (0)
-
-int check_dtype(const char* fn, int dtype) {
-    REQUIRE(dtype == NVH_BF16 || dtype == NVH_F32, NVH_E_DTYPE, "%s: dtype %d unsupported (bf16 or f32)", fn, dtype);
-    return 0;
-}
-#define DTYPE(fn) do { const int rc_ = check_dtype(fn, dtype); if (rc_) return rc_; } while (0)
-
 int check_rglru(const char* fn, const nvh_rglru_desc* d, int dtype) {
     DTYPE(fn);
     REQUIRE(d->yx && d->conv_w && d->conv_b && d->ra && d->ri && d->ra_b && d->ri_b && d->rate && d->positions && d->state_slots && d->state && d->conv_state,
@@ -31,41 +23,6 @@ int check_rglru(const char* fn, const nvh_rglru_desc* d, int dtype) {
 }  // namespace
 
 extern "C" {
-
-int nvh_embed_rows(float* x, void* xb, void* packed, const int64_t* tokens, const void* embed, float scale, int rows, int cols, int vocab, int dtype, void* stream) {
-    if (rows == 0) return 0;
-    DTYPE("embed_rows");
-    REQUIRE(x && tokens && embed, NVH_E_NULL, "embed_rows: null pointer");
-    REQUIRE(rows > 0 && cols > 0 && cols % 8 == 0 && vocab > 0, NVH_E_SHAPE, "embed_rows: rows %d cols %d (%%8) vocab %d", rows, cols, vocab);
-    REQUIRE(!packed || (dtype == NVH_BF16 && cols % 32 == 0), NVH_E_SHAPE, "embed_rows: packed rows are bf16, cols %% 32 == 0");
-    REQUIRE(aligned16(x) && aligned16(embed) && (!xb || aligned16(xb)) && (!packed || aligned16(packed)), NVH_E_ALIGN, "embed_rows: pointers must be 16-byte aligned");
-    return launch_embed_rows(x, xb, packed, tokens, embed, scale, rows, cols, vocab, dtype == NVH_F32, (hipStream_t)stream);
-}
-
-int nvh_norm_residual(const nvh_norm_residual_desc* d, int dtype, void* stream) {
-    REQUIRE(d, NVH_E_NULL, "norm_residual: null descriptor");
-    if (d->rows == 0) return 0;
-    DTYPE("norm_residual");
-    REQUIRE(d->x && d->w && (d->y || d->xb || d->packed), NVH_E_NULL, "norm_residual: null pointer");
-    REQUIRE(d->rows > 0 && d->cols > 0 && d->cols % 8 == 0 && d->cols <= 16384 && d->n > 0 && d->n <= d->cols, NVH_E_SHAPE,
-            "norm_residual: cols %d (%%8, <= 16384), mean over %d", d->cols, d->n);
-    REQUIRE(!d->packed || (dtype == NVH_BF16 && d->cols % 32 == 0), NVH_E_SHAPE, "norm_residual: packed rows are bf16, cols %% 32 == 0");
-    REQUIRE(!d->y || (d->y_stride % 4 == 0 && d->y_stride >= d->cols), NVH_E_STRIDE, "norm_residual: y row stride");
-    REQUIRE(aligned16(d->x) && aligned16(d->w) && (!d->y || aligned16(d->y)) && (!d->xb || aligned16(d->xb)) && (!d->packed || aligned16(d->packed)), NVH_E_ALIGN,
-            "norm_residual: pointers must be 16-byte aligned");
-    return launch_norm_residual(*d, dtype == NVH_F32, (hipStream_t)stream);
-}
-
-int nvh_clamped_glu(void* out, const void* gate_up, int rows, int inter, int64_t gate_up_row_stride, int64_t out_row_stride, float limit, float alpha,
-                    int dtype, void* stream) {
-    if (rows == 0) return 0;
-    DTYPE("clamped_glu");
-    REQUIRE(out && gate_up, NVH_E_NULL, "clamped_glu: null pointer");
-    REQUIRE(rows > 0 && inter > 0 && inter % 8 == 0 && gate_up_row_stride >= 2 * (int64_t)inter && gate_up_row_stride % 8 == 0 && out_row_stride >= inter && out_row_stride % 8 == 0,
-            NVH_E_SHAPE, "clamped_glu: inter %d (%%8) / row strides", inter);
-    REQUIRE(aligned16(out) && aligned16(gate_up), NVH_E_ALIGN, "clamped_glu: pointers must be 16-byte aligned");
-    return launch_clamped_glu(out, gate_up, rows, inter, gate_up_row_stride, out_row_stride, limit, alpha, dtype == NVH_F32, (hipStream_t)stream);
-}
 
 int nvh_rglru_chunk_tokens(void) { return kRglruChunk; }
 int nvh_rglru_step_supported(int block) { return block > 0 && block % 32 == 0 && rglru_step_supported(block); }

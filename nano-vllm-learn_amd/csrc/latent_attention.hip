@@ -6,15 +6,11 @@
 // A query's score against a key needs the cache row only, so one stream over the context serves every head (the decode form; prompts use the
 // expanded form of latent_prefill.hip).  Scores, weights and sums are fp32; the weights enter the MFMA as bf16 hi + lo halves.
 // Every step exists for bf16 on MFMA tiles and in a plain form for any size and for fp32 activations.
-#include <type_traits>
-
-#include "hybrid.h"
+#include "attend_tile.h"
 
 namespace nvh {
 
 namespace {
-
-typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
 
 // ------------------------------------------------------------------------------------------------ prep
 __device__ __forceinline__ float wave_sum(float v) {
@@ -214,19 +210,6 @@ __global__ __launch_bounds__(256) void latent_attend_generic_kernel(const Latent
 // reads): wave w scores keys 16 w .. + 15 for all 16 heads (queries in registers), the waves agree on the tile's maxima through LDS, weights go to
 // LDS as bf16 hi + lo in the order the transposed reads deliver keys, and wave w sums its quarter of the latent columns.
 // Two images, refilled as soon as a tile has been summed: up to two tiles travel at once, so the stream does not pause for a round trip per tile.
-__device__ __forceinline__ void lds_only_barrier() {     // (a __syncthreads() would drain the DMA in flight)
-    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
-    __builtin_amdgcn_s_barrier();
-    asm volatile("" ::: "memory");
-}
-template <int OFF>
-__device__ __forceinline__ u32x2 ds_read_tr16(uint32_t lds_addr) {
-    u32x2 r;
-    asm volatile("ds_read_b64_tr_b16 %0, %1 offset:%2" : "=v"(r) : "v"(lds_addr), "n"(OFF) : "memory");
-    return r;
-}
-__device__ __forceinline__ uint32_t lds_addr_of(const void* p) { return (uint32_t)(uintptr_t)(__attribute__((address_space(3))) const void*)p; }
-
 constexpr int kAttendTileBytes = 2 * 16 * 72 * 2 + 4 * 16 * 4;                 // weights and maxima of one head tile
 
 template <int NT, int HT>                            // kv_cols = 64 * NT, rot_cols = 64

@@ -1,0 +1,566 @@
+// Mixture of experts with a sigmoid router, choice corrections and expert groups.
+//   route     32-bit logits of a row tile against every expert (MFMA for bf16), sigmoid, group and expert choice, weights: one launch
+//   dispatch  pairs (row, chosen expert) sorted by expert and cut into tiles of one expert each: two launches, no host round trip
+//   gemm      expert products: gate | up with the SiLU product in the epilogue, and down.  Large batches: 128 x 128 MFMA tiles over the sorted pairs, the
+//             rows gathered by the DMA that fills LDS.  At most 64 rows: every wave streams 16 weight rows once for all the rows that chose the expert.
+// Outputs stay per pair; the weighted sum over a row's experts belongs to the residual add (hybrid_ops.hip).
+#include "attend_tile.h"
+#include "mixers.h"
+
+namespace nvh {
+
+namespace {
+
+__device__ __forceinline__ void wave_lds_sync() {    // LDS written by other lanes of this wave is visible behind it
+    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+    __builtin_amdgcn_wave_barrier();
+}
+
+// ------------------------------------------------------------------------------------------------ choice (one wave per row)
+// index of the wave's largest value; ties go to the lower index
+__device__ __forceinline__ void wave_argmax(float& v, int& i) {
+    for (int d = 1; d < 64; d <<= 1) {
+        const float ov = __shfl_xor(v, d);
+        const int oi = __shfl_xor(i, d);
+        if (ov > v || (ov == v && oi < i)) {
+            v = ov;
+            i = oi;
+        }
+    }
+}
+// z [E]: logits in, scores out; choice [E], gs [groups]: scratch in LDS
+__device__ __forceinline__ void choose_experts(const MoeRouteArgs& a, int row, int lane, float* z, float* choice, float* gs) {
+    for (int e = lane; e < a.experts; e += 64) {
+        const float s = 1.f / (1.f + expf(-z[e]));
+        z[e] = s;
+        choice[e] = s + a.correction[e];
+    }
+    wave_lds_sync();
+    const int size = a.experts / a.groups;
+    if (a.keep < a.groups) {
+        for (int g = lane; g < a.groups; g += 64) {
+            float b0 = -INFINITY, b1 = -INFINITY;
+            for (int k = 0; k < size; ++k) {
+                const float c = choice[g * size + k];
+                if (c > b0) {
+                    b1 = b0;
+                    b0 = c;
+                } else if (c > b1) {
+                    b1 = c;
+                }
+            }
+            gs[g] = size > 1 ? b0 + b1 : b0;
+        }
+        wave_lds_sync();
+        for (int k = 0; k < a.keep; ++k) {           // an open group is marked by +inf
+            float v = -INFINITY;
+            int i = 0x7fffffff;
+            for (int g = lane; g < a.groups; g += 64) {
+                const float s = gs[g];
+                if (s < INFINITY && (s > v || i == 0x7fffffff)) {
+                    v = s;
+                    i = g;
+                }
+            }
+            wave_argmax(v, i);
+            if (lane == 0 && i < a.groups) gs[i] = INFINITY;
+            wave_lds_sync();
+        }
+        for (int e = lane; e < a.experts; e += 64)
+            if (!(gs[e / size] == INFINITY)) choice[e] = -INFINITY;
+        wave_lds_sync();
+    }
+    float total = 0.f, mine = 0.f;
+    int my_id = 0;
+    for (int k = 0; k < a.top; ++k) {
+        float v = -INFINITY;
+        int i = 0x7fffffff;
+        for (int e = lane; e < a.experts; e += 64) {
+            const float c = choice[e];
+            if (c > v) {
+                v = c;
+                i = e;
+            }
+        }
+        wave_argmax(v, i);
+        if (i >= a.experts) i = 0;                   // (only where a router delivers no number)
+        const float s = z[i];
+        total += s;
+        if (lane == k) {
+            mine = s;
+            my_id = i;
+        }
+        if (lane == 0) choice[i] = -INFINITY;
+        wave_lds_sync();
+    }
+    if (lane < a.top) {
+        a.ids[(int64_t)row * a.top + lane] = my_id;
+        a.weights[(int64_t)row * a.top + lane] = mine / (total + 1e-20f) * a.scale;
+    }
+}
+
+// 16 rows per workgroup, the contraction shared by 8 waves, 64 experts at a time
+__global__ __launch_bounds__(512) void moe_route_kernel(const MoeRouteArgs a) {
+    extern __shared__ __attribute__((aligned(16))) float lds_r[];
+    const int ez = (a.experts + 63) / 64 * 64;
+    float *part = lds_r, *z = part + 8 * 16 * 68, *choice = z + 16 * ez, *gs = choice + 8 * ez;     // [8][16][64 + 4], [16][ez], per wave [ez], [groups]
+    const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lq = lane & 15, lg = lane >> 4;
+    const int r0 = blockIdx.x * 16, row = r0 + lq < a.rows ? r0 + lq : a.rows - 1;
+    const int steps = a.cols / 32, per = (steps + 7) / 8, s0 = wave * per, s1 = s0 + per < steps ? s0 + per : steps;
+    const uint16_t* x = reinterpret_cast<const uint16_t*>(a.x) + (int64_t)row * a.x_stride + 8 * lg;
+    for (int e0 = 0; e0 < a.experts; e0 += 64) {
+        const uint16_t* w[4];
+#pragma unroll
+        for (int t = 0; t < 4; ++t) {
+            const int e = e0 + 16 * t + lq;
+            w[t] = reinterpret_cast<const uint16_t*>(a.router) + (int64_t)(e < a.experts ? e : a.experts - 1) * a.cols + 8 * lg;
+        }
+        f32x4 acc[4];
+#pragma unroll
+        for (int t = 0; t < 4; ++t) acc[t] = f32x4{0.f, 0.f, 0.f, 0.f};
+        auto walk = [&](auto ntc) {                  // (tiles that hold no expert are not read)
+            constexpr int NT = decltype(ntc)::value;
+            constexpr int UN = 4;
+            int s = s0;
+            for (; s + UN <= s1; s += UN) {
+                bf16x8 xf[UN], wf[UN][NT];
+#pragma unroll
+                for (int i = 0; i < UN; ++i) {
+                    xf[i] = *reinterpret_cast<const bf16x8*>(x + 32 * (s + i));
+#pragma unroll
+                    for (int t = 0; t < NT; ++t) wf[i][t] = *reinterpret_cast<const bf16x8*>(w[t] + 32 * (s + i));
+                }
+#pragma unroll
+                for (int i = 0; i < UN; ++i)
+#pragma unroll
+                    for (int t = 0; t < NT; ++t) acc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf[i][t], xf[i], acc[t], 0, 0, 0);
+            }
+            for (; s < s1; ++s) {
+                const bf16x8 xf = *reinterpret_cast<const bf16x8*>(x + 32 * s);
+#pragma unroll
+                for (int t = 0; t < NT; ++t) acc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8*>(w[t] + 32 * s), xf, acc[t], 0, 0, 0);
+            }
+        };
+        switch ((a.experts - e0 + 15) / 16) {
+            case 1: walk(std::integral_constant<int, 1>{}); break;
+            case 2: walk(std::integral_constant<int, 2>{}); break;
+            case 3: walk(std::integral_constant<int, 3>{}); break;
+            default: walk(std::integral_constant<int, 4>{}); break;
+        }
+        // D: lane = row lq, experts 16 t + 4 lg ..
+#pragma unroll
+        for (int t = 0; t < 4; ++t) *reinterpret_cast<f32x4*>(part + (wave * 16 + lq) * 68 + 16 * t + 4 * lg) = acc[t];
+        __syncthreads();
+        for (int i = tid; i < 16 * 64; i += 512) {
+            const int r = i >> 6, e = i & 63;
+            float s = 0.f;
+#pragma unroll
+            for (int k = 0; k < 8; ++k) s += part[(k * 16 + r) * 68 + e];
+            z[r * ez + e0 + e] = s;
+        }
+        __syncthreads();
+    }
+    for (int r = wave; r < 16 && r0 + r < a.rows; r += 8) choose_experts(a, r0 + r, lane, z + r * ez, choice + wave * ez, gs + wave * a.groups);
+}
+
+// any type and width: one workgroup per row, a wave per expert in turn
+template <typename T>
+__global__ __launch_bounds__(256) void moe_route_generic_kernel(const MoeRouteArgs a) {
+    extern __shared__ __attribute__((aligned(16))) float lds_r[];
+    float *z = lds_r, *choice = z + a.experts, *gs = choice + a.experts;
+    const int row = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+    const T* x = reinterpret_cast<const T*>(a.x) + (int64_t)row * a.x_stride;
+    for (int e = wave; e < a.experts; e += 4) {
+        const T* w = reinterpret_cast<const T*>(a.router) + (int64_t)e * a.cols;
+        float s = 0.f;
+        for (int c = lane * 4; c < a.cols; c += 256) s += sum4(act_ld4(x + c) * act_ld4(w + c));
+        s = wave_sum64(s);
+        if (lane == 0) z[e] = s;
+    }
+    __syncthreads();
+    if (wave == 0) choose_experts(a, row, lane, z, choice, gs);
+}
+
+// ------------------------------------------------------------------------------------------------ dispatch
+constexpr int DP = 2048;                             // pairs per workgroup
+
+__global__ __launch_bounds__(256) void moe_count_kernel(int32_t* __restrict__ counts, const int32_t* __restrict__ ids, int pairs, int experts) {
+    __shared__ int hist[kMoeMaxExperts];
+    for (int e = threadIdx.x; e < experts; e += 256) hist[e] = 0;
+    __syncthreads();
+    const int p0 = blockIdx.x * DP;
+    for (int p = p0 + threadIdx.x; p < p0 + DP && p < pairs; p += 256) atomicAdd(&hist[ids[p]], 1);
+    __syncthreads();
+    for (int e = threadIdx.x; e < experts; e += 256) counts[(int64_t)blockIdx.x * experts + e] = hist[e];
+}
+
+// every workgroup sums the counts in front of its own pairs; the first one also writes the tiles
+__global__ __launch_bounds__(256) void moe_scatter_kernel(int32_t* __restrict__ slot_pair, int32_t* __restrict__ tiles, const int32_t* __restrict__ counts,
+                                                          const int32_t* __restrict__ ids, int pairs, int experts, int tile_rows, int max_tiles) {
+    __shared__ int at[kMoeMaxExperts], total[kMoeMaxExperts], start[kMoeMaxExperts], tile0[kMoeMaxExperts];
+    __shared__ int n_tiles;
+    for (int e = threadIdx.x; e < experts; e += 256) {
+        int before = 0, all = 0;
+        for (int b = 0; b < (int)gridDim.x; ++b) {
+            const int c = counts[(int64_t)b * experts + e];
+            if (b < (int)blockIdx.x) before += c;
+            all += c;
+        }
+        at[e] = before;
+        total[e] = all;
+    }
+    __syncthreads();
+    if (threadIdx.x < 64) {                          // exclusive scans over the experts, 64 at a time
+        int base = 0, tbase = 0;
+        for (int e0 = 0; e0 < experts; e0 += 64) {
+            const int e = e0 + threadIdx.x, n = e < experts ? total[e] : 0, t = (n + tile_rows - 1) / tile_rows;
+            int s = n, u = t;
+            for (int d = 1; d < 64; d <<= 1) {
+                const int ps = __shfl_up(s, d), pu = __shfl_up(u, d);
+                if ((int)threadIdx.x >= d) {
+                    s += ps;
+                    u += pu;
+                }
+            }
+            if (e < experts) {
+                start[e] = base + s - n;
+                tile0[e] = tbase + u - t;
+            }
+            base += __shfl(s, 63);
+            tbase += __shfl(u, 63);
+        }
+        if (threadIdx.x == 0) n_tiles = tbase;
+    }
+    __syncthreads();
+    for (int e = threadIdx.x; e < experts; e += 256) at[e] += start[e];
+    __syncthreads();
+    const int p0 = blockIdx.x * DP;
+    for (int p = p0 + threadIdx.x; p < p0 + DP && p < pairs; p += 256) slot_pair[atomicAdd(&at[ids[p]], 1)] = p;
+    if (blockIdx.x == 0) {
+        for (int e = threadIdx.x; e < experts; e += 256)
+            for (int t = 0; t * tile_rows < total[e]; ++t) {
+                const int left = total[e] - t * tile_rows;
+                reinterpret_cast<int4*>(tiles)[tile0[e] + t] = int4{e, start[e] + t * tile_rows, left < tile_rows ? left : tile_rows, n_tiles};
+            }
+        for (int t = n_tiles + threadIdx.x; t < max_tiles; t += 256) reinterpret_cast<int4*>(tiles)[t] = int4{0, 0, 0, n_tiles};
+    }
+}
+
+// ------------------------------------------------------------------------------------------------ products, large batches (bf16)
+// 128 pairs x 128 weight rows per workgroup, 64 of the contraction at a time, both operands by LDS-DMA, double-buffered; 4 waves of 64 x 64.
+// GLU: weight rows alternate 16 of gate, 16 of up, so a lane holds both halves of its outputs.
+constexpr int TM = 128, TN = 128, TK = 64;
+
+template <bool GLU>
+__global__ __launch_bounds__(256) void moe_gemm_kernel(const MoeGemmArgs a) {
+    constexpr int IMG = TM * TK * 2;
+    extern __shared__ __attribute__((aligned(16))) unsigned char lds[];        // [2][weights | rows]
+    constexpr int OUTS = GLU ? TN / 2 : TN;
+    int nt, mt;
+    {
+        // one XCD takes a run of column tiles of the same pairs: the gathered rows and the expert's weights are shared in its L2
+        const int total = (int)gridDim.x * a.tiles[3], lin = (int)(blockIdx.x + gridDim.x * blockIdx.y), per = total >> 3;
+        if (lin >= total) return;
+        const int idx = lin < per * 8 ? (lin & 7) * per + (lin >> 3) : lin;
+        mt = idx / (int)gridDim.x;
+        nt = idx - mt * (int)gridDim.x;
+    }
+    const int expert = a.tiles[4 * mt], first = a.tiles[4 * mt + 1], live = a.tiles[4 * mt + 2];
+    const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lq = lane & 15, lg = lane >> 4, wm = wave >> 1, wn = wave & 1;
+    const uint16_t* w = reinterpret_cast<const uint16_t*>(a.w) + (int64_t)expert * (GLU ? 2 : 1) * a.n * a.k;
+    // this lane's piece of each DMA instruction: 4 for the weights, 4 for the rows
+    const uint16_t *wp[4], *xp[4];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+        const int s = (wave * 4 + j) * 64 + lane, R = s >> 3, piece = (s & 7) ^ (R & 7);
+        int col;                                     // weight row
+        if constexpr (GLU) col = nt * OUTS + (R >> 5) * 16 + (R & 15);
+        else col = nt * OUTS + R;
+        if (col >= a.n) col = a.n - 1;
+        wp[j] = w + (int64_t)(GLU && (R & 16) ? a.n + col : col) * a.k + piece * 8;
+        const int slot = first + (R < live ? R : live - 1), pair = a.slot_pair[slot];
+        xp[j] = reinterpret_cast<const uint16_t*>(a.x) + (GLU ? (int64_t)(pair / a.top) * a.x_stride : (int64_t)pair * a.k) + piece * 8;
+    }
+    auto stage = [&](int it, int buf) {
+        unsigned char* base = lds + buf * 2 * IMG;
+#pragma unroll
+        for (int j = 0; j < 4; ++j) dma16(wp[j] + it * TK, base + (wave * 4 + j) * 1024);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) dma16(xp[j] + it * TK, base + IMG + (wave * 4 + j) * 1024);
+    };
+    f32x4 acc[4][4];                                 // [weight tile][row tile]: D[weight row 4 lg + r][pair lq]
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+#pragma unroll
+        for (int j = 0; j < 4; ++j) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
+    const int iters = a.k / TK;
+    stage(0, 0);
+    auto body = [&](auto bufc, const int it) {
+        constexpr int buf = decltype(bufc)::value;
+        if (it + 1 < iters) {
+            stage(it + 1, buf ^ 1);
+            asm volatile("s_waitcnt vmcnt(8)" ::: "memory");
+        } else {
+            asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+        }
+        __builtin_amdgcn_s_barrier();
+        asm volatile("" ::: "memory");
+        const unsigned char* wimg = lds + buf * 2 * IMG + wn * 64 * 128;
+        const unsigned char* ximg = lds + buf * 2 * IMG + IMG + wm * 64 * 128;
+#pragma unroll
+        for (int st = 0; st < 2; ++st) {
+            const int at = lq * 128 + ((4 * st + lg) ^ (lq & 7)) * 16;
+            bf16x8 wf[4], xf[4];
+#pragma unroll
+            for (int t = 0; t < 4; ++t) wf[t] = *reinterpret_cast<const bf16x8*>(wimg + t * 16 * 128 + at);
+#pragma unroll
+            for (int t = 0; t < 4; ++t) xf[t] = *reinterpret_cast<const bf16x8*>(ximg + t * 16 * 128 + at);
+#pragma unroll
+            for (int i = 0; i < 4; ++i)
+#pragma unroll
+                for (int j = 0; j < 4; ++j) acc[i][j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf[i], xf[j], acc[i][j], 0, 0, 0);
+        }
+        lds_only_barrier();                          // everyone's reads of this buffer are done
+    };
+    for (int it = 0; it < iters; it += 2) {
+        body(std::integral_constant<int, 0>{}, it);
+        if (it + 1 < iters) body(std::integral_constant<int, 1>{}, it + 1);
+    }
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+        const int R = wm * 64 + 16 * j + lq;
+        if (R >= live) continue;
+        uint16_t* out = reinterpret_cast<uint16_t*>(a.out) + (int64_t)a.slot_pair[first + R] * a.n;
+        if constexpr (GLU) {
+#pragma unroll
+            for (int i = 0; i < 2; ++i) {
+                const int col = nt * OUTS + wn * 32 + 16 * i + 4 * lg;
+                f32x4 v;
+#pragma unroll
+                for (int r = 0; r < 4; ++r) v[r] = silu_f(acc[2 * i][j][r]) * acc[2 * i + 1][j][r];
+                if (col < a.n) act_st4(out + col, v);
+            }
+        } else {
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+                const int col = nt * OUTS + wn * 64 + 16 * i + 4 * lg;
+                if (col < a.n) act_st4(out + col, acc[i][j]);
+            }
+        }
+    }
+}
+
+// ------------------------------------------------------------------------------------------------ products, at most 64 rows (bf16)
+// grid (n / (16 x waves' tiles), experts): the pairs of the expert are found from the ids; an expert nobody chose costs one scan.
+// SPLIT: the 4 waves share one 16-column tile and split the contraction; otherwise every wave owns a tile.
+template <bool GLU, int MT, bool SPLIT>
+__device__ __forceinline__ void moe_small_tile(const MoeGemmArgs& a, int expert, int n0, int s0, int s1, const int* list, int count, float* red, int wave, int lane) {
+    const int lq = lane & 15, lg = lane >> 4;
+    const uint16_t* w = reinterpret_cast<const uint16_t*>(a.w) + ((int64_t)expert * (GLU ? 2 : 1) * a.n + n0 + lq) * a.k + 8 * lg;
+    const uint16_t* x[MT];
+#pragma unroll
+    for (int m = 0; m < MT; ++m) {
+        const int p = list[16 * m + lq < count ? 16 * m + lq : count - 1];
+        x[m] = reinterpret_cast<const uint16_t*>(a.x) + (GLU ? (int64_t)(p / a.top) * a.x_stride : (int64_t)p * a.k) + 8 * lg;
+    }
+    f32x4 g[MT], u[MT];
+#pragma unroll
+    for (int m = 0; m < MT; ++m) g[m] = u[m] = f32x4{0.f, 0.f, 0.f, 0.f};
+    constexpr int UN = GLU ? (MT > 2 ? 2 : 4) : (MT > 2 ? 4 : 8);
+    const int64_t up = (int64_t)a.n * a.k;
+    int s = s0;
+    for (; s + UN <= s1; s += UN) {
+        bf16x8 wg[UN], wu[UN], xf[UN][MT];
+#pragma unroll
+        for (int i = 0; i < UN; ++i) {
+            wg[i] = __builtin_nontemporal_load(reinterpret_cast<const bf16x8*>(w + 32 * (s + i)));
+            if constexpr (GLU) wu[i] = __builtin_nontemporal_load(reinterpret_cast<const bf16x8*>(w + up + 32 * (s + i)));
+        }
+#pragma unroll
+        for (int i = 0; i < UN; ++i)
+#pragma unroll
+            for (int m = 0; m < MT; ++m) xf[i][m] = *reinterpret_cast<const bf16x8*>(x[m] + 32 * (s + i));
+#pragma unroll
+        for (int i = 0; i < UN; ++i)
+#pragma unroll
+            for (int m = 0; m < MT; ++m) {
+                g[m] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wg[i], xf[i][m], g[m], 0, 0, 0);
+                if constexpr (GLU) u[m] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wu[i], xf[i][m], u[m], 0, 0, 0);
+            }
+    }
+    for (; s < s1; ++s) {
+        const bf16x8 wg = *reinterpret_cast<const bf16x8*>(w + 32 * s);
+        bf16x8 wu = wg;
+        if constexpr (GLU) wu = *reinterpret_cast<const bf16x8*>(w + up + 32 * s);
+#pragma unroll
+        for (int m = 0; m < MT; ++m) {
+            const bf16x8 xf = *reinterpret_cast<const bf16x8*>(x[m] + 32 * s);
+            g[m] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wg, xf, g[m], 0, 0, 0);
+            if constexpr (GLU) u[m] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wu, xf, u[m], 0, 0, 0);
+        }
+    }
+    if constexpr (SPLIT) {                           // red [4 waves][2][MT][64 lanes][4]
+        constexpr int W = 2 * MT * 256;
+#pragma unroll
+        for (int m = 0; m < MT; ++m) {
+            *reinterpret_cast<f32x4*>(red + wave * W + m * 256 + lane * 4) = g[m];
+            if constexpr (GLU) *reinterpret_cast<f32x4*>(red + wave * W + (MT + m) * 256 + lane * 4) = u[m];
+        }
+        __syncthreads();
+        if (wave) return;
+#pragma unroll
+        for (int k = 1; k < 4; ++k)
+#pragma unroll
+            for (int m = 0; m < MT; ++m) {
+                g[m] += *reinterpret_cast<const f32x4*>(red + k * W + m * 256 + lane * 4);
+                if constexpr (GLU) u[m] += *reinterpret_cast<const f32x4*>(red + k * W + (MT + m) * 256 + lane * 4);
+            }
+    }
+#pragma unroll
+    for (int m = 0; m < MT; ++m) {
+        if (16 * m + lq >= count) continue;
+        f32x4 v = g[m];
+        if constexpr (GLU) {
+#pragma unroll
+            for (int r = 0; r < 4; ++r) v[r] = silu_f(g[m][r]) * u[m][r];
+        }
+        act_st4(reinterpret_cast<uint16_t*>(a.out) + (int64_t)list[16 * m + lq] * a.n + n0 + 4 * lg, v);
+    }
+}
+
+template <bool GLU, bool SPLIT>
+__global__ __launch_bounds__(256) void moe_small_kernel(const MoeGemmArgs a) {
+    __shared__ int list[64];
+    __shared__ int count_s;
+    __shared__ __attribute__((aligned(16))) float red[SPLIT ? 4 * 2 * 4 * 256 : 4];
+    const int expert = blockIdx.y, tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+    if (wave == 0) {                                 // (an expert is chosen at most once per row: at most 64 pairs)
+        int n = 0;
+        for (int p0 = 0; p0 < a.pairs; p0 += 64) {
+            const bool mine = p0 + lane < a.pairs && a.ids[p0 + lane] == expert;
+            const uint64_t ball = __builtin_amdgcn_ballot_w64(mine);
+            const int at = n + __popcll(ball & ((1ull << lane) - 1));
+            if (mine && at < 64) list[at] = p0 + lane;
+            n += __popcll(ball);
+        }
+        if (lane == 0) count_s = n < 64 ? n : 64;
+    }
+    __syncthreads();
+    const int count = __builtin_amdgcn_readfirstlane(count_s);
+    if (count == 0) return;
+    const int tile = SPLIT ? blockIdx.x : blockIdx.x * 4 + wave, steps = a.k / 32;
+    if (tile * 16 >= a.n) return;                    // (whole waves; only the form without a later barrier has such tiles)
+    const int per = (steps + 3) / 4, s0 = SPLIT ? wave * per : 0, s1 = SPLIT ? (s0 + per < steps ? s0 + per : steps) : steps;
+    if (count <= 16) moe_small_tile<GLU, 1, SPLIT>(a, expert, tile * 16, s0, s1, list, count, red, wave, lane);
+    else if (count <= 32) moe_small_tile<GLU, 2, SPLIT>(a, expert, tile * 16, s0, s1, list, count, red, wave, lane);
+    else moe_small_tile<GLU, 4, SPLIT>(a, expert, tile * 16, s0, s1, list, count, red, wave, lane);
+}
+
+// ------------------------------------------------------------------------------------------------ products in 32-bit
+// 64 pairs x 64 outputs per workgroup, 16 of the contraction at a time through LDS, 4 x 4 outputs per thread
+constexpr int FM = 64;
+
+template <bool GLU>
+__global__ __launch_bounds__(256) void moe_gemm_f32_kernel(const MoeGemmArgs a) {
+    __shared__ __attribute__((aligned(16))) float xs[16][FM + 4], ws[2][16][64 + 4];
+    const int mt = blockIdx.y, n0 = blockIdx.x * 64, tid = threadIdx.x;
+    const int expert = a.tiles[4 * mt], first = a.tiles[4 * mt + 1], live = a.tiles[4 * mt + 2];
+    if (live <= 0) return;
+    const float* w = reinterpret_cast<const float*>(a.w) + (int64_t)expert * (GLU ? 2 : 1) * a.n * a.k;
+    const int lr = tid >> 2, lc = (tid & 3) * 4;     // staging: row lr, 4 of the contraction
+    const int pair = a.slot_pair[first + (lr < live ? lr : live - 1)];
+    const float* x = reinterpret_cast<const float*>(a.x) + (GLU ? (int64_t)(pair / a.top) * a.x_stride : (int64_t)pair * a.k) + lc;
+    const float* wr = w + (int64_t)(n0 + lr) * a.k + lc;
+    const int tm = (tid >> 4) * 4, tn = (tid & 15) * 4;
+    float g[4][4] = {}, u[4][4] = {};
+    for (int k0 = 0; k0 < a.k; k0 += 16) {
+        const f32x4 xv = *reinterpret_cast<const f32x4*>(x + k0), gv = *reinterpret_cast<const f32x4*>(wr + k0);
+        f32x4 uv = gv;
+        if constexpr (GLU) uv = *reinterpret_cast<const f32x4*>(wr + (int64_t)a.n * a.k + k0);
+        __syncthreads();
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+            xs[lc + i][lr] = xv[i];
+            ws[0][lc + i][lr] = gv[i];
+            if constexpr (GLU) ws[1][lc + i][lr] = uv[i];
+        }
+        __syncthreads();
+#pragma unroll
+        for (int k = 0; k < 16; ++k) {
+            const f32x4 m = *reinterpret_cast<const f32x4*>(&xs[k][tm]), n = *reinterpret_cast<const f32x4*>(&ws[0][k][tn]);
+            f32x4 n2 = n;
+            if constexpr (GLU) n2 = *reinterpret_cast<const f32x4*>(&ws[1][k][tn]);
+#pragma unroll
+            for (int i = 0; i < 4; ++i)
+#pragma unroll
+                for (int j = 0; j < 4; ++j) {
+                    g[i][j] += m[i] * n[j];
+                    if constexpr (GLU) u[i][j] += m[i] * n2[j];
+                }
+        }
+    }
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+        if (tm + i >= live) continue;
+        f32x4 v;
+#pragma unroll
+        for (int j = 0; j < 4; ++j) v[j] = GLU ? g[i][j] / (1.f + expf(-g[i][j])) * u[i][j] : g[i][j];
+        *reinterpret_cast<f32x4*>(reinterpret_cast<float*>(a.out) + (int64_t)a.slot_pair[first + tm + i] * a.n + n0 + tn) = v;
+    }
+}
+
+}  // namespace
+
+int launch_moe_route(const MoeRouteArgs& a, int f32, hipStream_t stream) {
+    if (!f32 && a.cols % 32 == 0) {
+        const int ez = (a.experts + 63) / 64 * 64;
+        const size_t lds = (size_t)(8 * 16 * 68 + 24 * ez + 8 * a.groups) * 4;
+        if (lds > 64 * 1024) (void)hipFuncSetAttribute(reinterpret_cast<const void*>(moe_route_kernel), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+        moe_route_kernel<<<(a.rows + 15) / 16, 512, lds, stream>>>(a);
+    } else {
+        const size_t lds = (size_t)(2 * a.experts + a.groups) * 4;
+        if (f32) moe_route_generic_kernel<float><<<a.rows, 256, lds, stream>>>(a);
+        else moe_route_generic_kernel<uint16_t><<<a.rows, 256, lds, stream>>>(a);
+    }
+    return check_launch("moe_route");
+}
+
+int moe_dispatch_blocks(int pairs) { return (pairs + DP - 1) / DP; }
+
+int launch_moe_dispatch(int32_t* slot_pair, int32_t* tiles, int32_t* counts, const int32_t* ids, int pairs, int experts, int tile_rows, int max_tiles,
+                        hipStream_t stream) {
+    const int grid = moe_dispatch_blocks(pairs);
+    moe_count_kernel<<<grid, 256, 0, stream>>>(counts, ids, pairs, experts);
+    const int rc = check_launch("moe_count");
+    if (rc) return rc;
+    moe_scatter_kernel<<<grid, 256, 0, stream>>>(slot_pair, tiles, counts, ids, pairs, experts, tile_rows, max_tiles);
+    return check_launch("moe_scatter");
+}
+
+int moe_tile_rows(int f32) { return f32 ? FM : TM; }
+
+int launch_moe_gemm(const MoeGemmArgs& a, int f32, hipStream_t stream) {
+    if (f32) {
+        const dim3 grid(a.n / 64, a.max_tiles);
+        if (a.glu) moe_gemm_f32_kernel<true><<<grid, 256, 0, stream>>>(a);
+        else moe_gemm_f32_kernel<false><<<grid, 256, 0, stream>>>(a);
+    } else if (!a.tiles) {
+        const int tiles = a.n / 16, busy = a.pairs < a.experts ? a.pairs : a.experts;
+        const bool split = (int64_t)busy * tiles < 4 * 512;                    // too few waves with a tile each: four share one
+        const dim3 grid(split ? tiles : (tiles + 3) / 4, a.experts);
+        if (a.glu && split) moe_small_kernel<true, true><<<grid, 256, 0, stream>>>(a);
+        else if (a.glu) moe_small_kernel<true, false><<<grid, 256, 0, stream>>>(a);
+        else if (split) moe_small_kernel<false, true><<<grid, 256, 0, stream>>>(a);
+        else moe_small_kernel<false, false><<<grid, 256, 0, stream>>>(a);
+    } else {
+        constexpr size_t lds = 2 * (TM + TN) * TK * 2;
+        const int outs = a.glu ? TN / 2 : TN;
+        const dim3 grid((a.n + outs - 1) / outs, a.max_tiles);
+        if (a.glu) moe_gemm_kernel<true><<<grid, 256, lds, stream>>>(a);
+        else moe_gemm_kernel<false><<<grid, 256, lds, stream>>>(a);
+    }
+    return check_launch("moe_gemm");
+}
+
+}  // namespace nvh

@@ -1,0 +1,465 @@
+// Softmax attention over pages of one layer, [page][kv head][block_size keys | block_size values], with windows, kept first tokens and sinks.
+//   prep      norm over all query / key columns, rotation of interleaved pairs, store of keys and values: one launch over the projection's rows
+//   rows      one query row at a time (decoding): a workgroup streams the visible keys of one (row, key/value head, split)
+// A sink is an entry of the softmax with score sink[head], no key and no value: it starts the running maximum and sum.
+// Keys a window hides are not read: the walk covers the tiles of the kept first tokens, then those of the window.
+#include "mixers.h"
+
+namespace nvh {
+
+namespace {
+
+// ------------------------------------------------------------------------------------------------ prep
+// one workgroup per row; a thread keeps its 8-element pieces of [q | k | v] in registers between the sums and the second pass
+template <typename T, int CH>
+__global__ __launch_bounds__(256) void attn_prep_kernel(const AttnPrepArgs a) {
+    __shared__ float lds[8];
+    const int64_t row = blockIdx.x;
+    T* x = reinterpret_cast<T*>(a.qkv) + row * a.qkv_stride;
+    const int nq = a.heads * a.dk, nk = a.kv_heads * a.dk, total = nq + nk + a.kv_heads * a.dv;
+    f32x8 v[CH];
+    float sq = 0.f, sk = 0.f;
+#pragma unroll
+    for (int i = 0; i < CH; ++i) {
+        const int c = (threadIdx.x + i * 256) * 8;
+        v[i] = {f32x4{0.f, 0.f, 0.f, 0.f}, f32x4{0.f, 0.f, 0.f, 0.f}};
+        if (c < total) v[i] = act_ld8(x + c);
+    }
+    if (a.q_w) {
+#pragma unroll
+        for (int i = 0; i < CH; ++i) {
+            const int c = (threadIdx.x + i * 256) * 8;
+            const float ss = sum4(v[i].a * v[i].a) + sum4(v[i].b * v[i].b);
+            if (c < nq) sq += ss;
+            else if (c < nq + nk) sk += ss;
+        }
+        block_sum256x2(sq, sk, lds);
+        sq = 1.f / sqrtf(sq / a.q_n + a.eps);
+        sk = 1.f / sqrtf(sk / a.k_n + a.eps);
+    }
+    int64_t pos = a.positions[row];
+    if (pos >= a.max_position) pos = a.max_position - 1;
+    const float* cs = a.cos_sin + pos * a.rot;
+    const int slot = a.slots[row];
+    const int page = slot >= 0 ? slot / a.block_size : 0, off = slot >= 0 ? slot - page * a.block_size : 0;
+    T* cache = reinterpret_cast<T*>(a.cache) + (int64_t)page * a.kv_heads * a.block_size * (a.dk + a.dv);
+#pragma unroll
+    for (int i = 0; i < CH; ++i) {
+        const int c = (threadIdx.x + i * 256) * 8;
+        if (c >= total) continue;
+        f32x8 r = v[i];
+        if (c < nq + nk) {
+            const bool is_q = c < nq;
+            const int h = is_q ? c / a.dk : (c - nq) / a.dk, d = (is_q ? c : c - nq) - h * a.dk;
+            if (a.q_w) {
+                const float* w = is_q ? a.q_w + c : a.k_w + (c - nq);
+                const float inv = is_q ? sq : sk;
+                r.a *= inv * *reinterpret_cast<const f32x4*>(w);
+                r.b *= inv * *reinterpret_cast<const f32x4*>(w + 4);
+            }
+            float e[8] = {r.a[0], r.a[1], r.a[2], r.a[3], r.b[0], r.b[1], r.b[2], r.b[3]};
+#pragma unroll
+            for (int p = 0; p < 4; ++p) {
+                const int pair = d / 2 + p;
+                if (pair < a.rot / 2) {
+                    const float co = cs[pair], si = cs[a.rot / 2 + pair], u = e[2 * p], w = e[2 * p + 1];
+                    e[2 * p] = u * co - w * si;
+                    e[2 * p + 1] = w * co + u * si;
+                }
+            }
+            r = {f32x4{e[0], e[1], e[2], e[3]}, f32x4{e[4], e[5], e[6], e[7]}};
+            if (is_q) act_st8(x + c, r);
+            else if (slot >= 0) act_st8(cache + (int64_t)h * a.block_size * (a.dk + a.dv) + off * a.dk + d, r);
+        } else if (slot >= 0) {
+            const int h = (c - nq - nk) / a.dv, d = c - nq - nk - h * a.dv;
+            act_st8(cache + (int64_t)h * a.block_size * (a.dk + a.dv) + (int64_t)a.block_size * a.dk + (int64_t)off * a.dv + d, r);
+        }
+    }
+}
+
+// ------------------------------------------------------------------------------------------------ rows, any type and size
+// one workgroup per (row, head); 64 keys at a time: 4 lanes per key for the scores, one thread per value column for the sums
+template <typename T>
+__global__ __launch_bounds__(256) void paged_rows_generic_kernel(const PagedAttendArgs a) {
+    constexpr int OC = 8;                            // value columns per thread: dv <= 2048
+    extern __shared__ float q_lds[];                 // [dk]
+    __shared__ float p_lds[64];
+    const int row = blockIdx.x, head = blockIdx.y, tid = threadIdx.x, g = head / (a.heads / a.kv_heads);
+    const int seq = a.row_seq ? a.row_seq[row] : row;
+    const int pos = (int)a.positions[row];
+    const T* q = reinterpret_cast<const T*>(a.q) + (int64_t)row * a.q_stride + head * a.dk;
+    for (int i = tid; i < a.dk; i += 256) q_lds[i] = act_ld(q + i);
+    float o[OC], m = -INFINITY, l = 0.f;
+    if (a.sink) {
+        m = a.sink[head] * kLog2e;
+        l = 1.f;
+    }
+#pragma unroll
+    for (int j = 0; j < OC; ++j) o[j] = 0.f;
+    const float sc = a.scale * kLog2e;
+    const int64_t head_elems = (int64_t)a.block_size * (a.dk + a.dv);
+    __syncthreads();
+    auto head_base = [&](int key) {
+        const int64_t page = a.block_tables[seq * a.bt_stride + key / a.block_size];
+        return reinterpret_cast<const T*>(a.cache) + (page * a.kv_heads + g) * head_elems;
+    };
+    const VisibleTiles vis = visible_tiles(pos, pos, a.window, a.keep_first);
+    for (int it = 0; it < vis.count; ++it) {
+        const int t0 = vis.tile(it) * 64, key = t0 + (tid >> 2);
+        const bool sees = key <= pos && (a.window <= 0 || pos - key < a.window || key < a.keep_first);
+        float s = 0.f;
+        if (sees) {
+            const T* r = head_base(key) + (int64_t)(key % a.block_size) * a.dk;
+            for (int i = (tid & 3) * 4; i < a.dk; i += 16) {
+                const f32x4 v = act_ld4(r + i);
+                s += v[0] * q_lds[i] + v[1] * q_lds[i + 1] + v[2] * q_lds[i + 2] + v[3] * q_lds[i + 3];
+            }
+        }
+        s += __shfl_xor(s, 1);
+        s += __shfl_xor(s, 2);
+        if ((tid & 3) == 0) p_lds[tid >> 2] = sees ? s * sc : -INFINITY;
+        __syncthreads();
+        float v = p_lds[tid & 63], mx = v;
+        for (int d = 1; d < 64; d <<= 1) mx = fmaxf(mx, __shfl_xor(mx, d));
+        const float m_new = fmaxf(m, mx), m_use = m_new == -INFINITY ? 0.f : m_new, alpha = exp2f(m - m_use);
+        v = exp2f(v - m_use);
+        float sum = v;
+        for (int d = 1; d < 64; d <<= 1) sum += __shfl_xor(sum, d);
+        l = l * alpha + sum;
+        m = m_new;
+        __syncthreads();
+        if (tid < 64) p_lds[tid] = v;
+        __syncthreads();
+#pragma unroll
+        for (int j = 0; j < OC; ++j) o[j] *= alpha;
+        for (int k = 0; k < 64; ++k) {
+            const float p = p_lds[k];
+            if (p == 0.f) continue;                  // (unseen, or a weight that vanished)
+            const T* r = head_base(t0 + k) + (int64_t)a.block_size * a.dk + (int64_t)((t0 + k) % a.block_size) * a.dv;
+#pragma unroll
+            for (int j = 0; j < OC; ++j)
+                if (tid + 256 * j < a.dv) o[j] += p * act_ld(r + tid + 256 * j);
+        }
+        __syncthreads();
+    }
+    const float inv = l > 0.f ? 1.f / l : 0.f;
+#pragma unroll
+    for (int j = 0; j < OC; ++j) {
+        const int c = tid + 256 * j;
+        if (c >= a.dv) continue;
+        if (a.out) act_st(reinterpret_cast<T*>(a.out) + (int64_t)row * a.out_stride + head * a.dv + c, o[j] * inv);
+        if (a.out_packed) act_st(reinterpret_cast<uint16_t*>(a.out_packed) + pack_index(row, head * a.dv + c, a.heads * a.dv), o[j] * inv);
+    }
+}
+
+// ------------------------------------------------------------------------------------------------ rows, streaming (bf16)
+// grid (splits, kv heads x passes, rows), 4 waves.  A wave takes units of UK keys: LPR lanes hold a row of keys or values, so one load instruction covers
+// 64 / LPR rows and the lanes that scored a key also weigh its value: no exchange until the end.  Every group of LPR lanes keeps its own running maximum,
+// sum and output; groups, waves and splits are merged once.  Loads of the next unit's keys are issued behind the scores of this one, its values behind
+// the sums, so about a unit per wave is always in flight.
+// Split partials: write-through stores, drained by every storing wave, a ticket per (row, key/value head, pass); the last workgroup to arrive merges.
+__device__ __forceinline__ void st_through(float* p, float v) {
+    __hip_atomic_store(reinterpret_cast<unsigned*>(p), __builtin_bit_cast(unsigned, v), __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+}
+__device__ __forceinline__ float ld_through(const float* p) {
+    return __builtin_bit_cast(float, __hip_atomic_load(reinterpret_cast<const unsigned*>(p), __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT));
+}
+
+// this lane's share of a row of W elements: W / LPR of them, in pieces of 8 (and one of 4)
+template <int W, int LPR>
+struct LanePiece {
+    static constexpr int E = W / LPR, P8 = E / 8, P4 = (E % 8) / 4, DW = E / 2;
+    static_assert(E % 4 == 0, "a lane holds whole pieces");
+    static __device__ __forceinline__ int column(int lane, int e) {            // of element e of lane `lane`
+        return e < 8 * P8 ? (e / 8) * 8 * LPR + lane * 8 + (e & 7) : P8 * 8 * LPR + lane * 4 + (e & 3);
+    }
+    static __device__ __forceinline__ void load(const uint16_t* row, int lane, uint32_t (&d)[DW]) {
+#pragma unroll
+        for (int p = 0; p < P8; ++p) {
+            const u32x4 r = __builtin_nontemporal_load(reinterpret_cast<const u32x4*>(row + p * 8 * LPR + lane * 8));
+#pragma unroll
+            for (int k = 0; k < 4; ++k) d[4 * p + k] = r[k];
+        }
+        if constexpr (P4) {
+            const u32x2 r = __builtin_nontemporal_load(reinterpret_cast<const u32x2*>(row + P8 * 8 * LPR + lane * 4));
+            d[4 * P8] = r[0];
+            d[4 * P8 + 1] = r[1];
+        }
+    }
+};
+template <int LPR>
+__device__ __forceinline__ float lanes_sum(float x) { return group_sum<LPR>(x); }
+
+constexpr int kRowsHeads = 8;                        // query heads a pass holds at most
+
+template <int DK, int DV, int R>
+__global__ __launch_bounds__(256) void paged_rows_kernel(const PagedAttendArgs a) {
+    constexpr int LPR = DK == 64 && DV == 64 ? 8 : 16, SLOTS = 64 / LPR, NI = DK + DV > 256 ? 4 : 8, UK = NI * SLOTS;
+    using KL = LanePiece<DK, LPR>;
+    using VL = LanePiece<DV, LPR>;
+    constexpr int RECW = DV + 4;                     // floats of one head's record in LDS: sums, max, sum
+    __shared__ __attribute__((aligned(16))) float rec[4 * R * RECW];
+    __shared__ int last_flag;
+    const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), ll = lane % LPR, ls = lane / LPR;
+    const int split = blockIdx.x, row = blockIdx.z, ratio = a.heads / a.kv_heads, passes = (ratio + kRowsHeads - 1) / kRowsHeads;
+    const int g = blockIdx.y / passes, h0 = g * ratio + (blockIdx.y - g * passes) * kRowsHeads;
+    const int nh = (g + 1) * ratio - h0 < R ? (g + 1) * ratio - h0 : R;
+    const int pos = (int)a.positions[row];
+    const VisibleTiles vis = visible_tiles(pos, pos, a.window, a.keep_first);
+    const int per = (vis.count + a.splits - 1) / a.splits, t_beg = split * per, t_end = t_beg + per < vis.count ? t_beg + per : vis.count;
+    const int units = t_end > t_beg ? (t_end - t_beg) * (64 / UK) : 0;
+
+    uint32_t q[R][KL::DW];
+#pragma unroll
+    for (int r = 0; r < R; ++r) {
+        const uint16_t* qr = reinterpret_cast<const uint16_t*>(a.q) + (int64_t)row * a.q_stride + (int64_t)(h0 + (r < nh ? r : nh - 1)) * DK;
+        KL::load(qr, ll, q[r]);
+    }
+    float m[R], l[R], o[R][VL::E];
+#pragma unroll
+    for (int r = 0; r < R; ++r) {
+        m[r] = -INFINITY;
+        l[r] = 0.f;
+#pragma unroll
+        for (int e = 0; e < VL::E; ++e) o[r][e] = 0.f;
+    }
+    const float sc = a.scale * kLog2e;
+    const int64_t head_elems = (int64_t)a.block_size * (DK + DV);
+    const int32_t* table = a.block_tables + (int64_t)row * a.bt_stride;
+    auto unit_key = [&](int u) { return vis.tile(t_beg + u / (64 / UK)) * 64 + (u % (64 / UK)) * UK; };
+    uint32_t kd[NI][KL::DW], vd[NI][VL::DW];
+    auto load_k = [&](int k0, int page) {            // rows past the query's own position repeat it: not seen
+        const uint16_t* base = reinterpret_cast<const uint16_t*>(a.cache) + ((int64_t)page * a.kv_heads + g) * head_elems;
+        const int o0 = k0 % a.block_size - k0;
+#pragma unroll
+        for (int i = 0; i < NI; ++i) {
+            const int key = k0 + i * SLOTS + ls;
+            KL::load(base + (int64_t)((key < pos ? key : pos) + o0) * DK, ll, kd[i]);
+        }
+    };
+    auto load_v = [&](int k0, int page) {
+        const uint16_t* base = reinterpret_cast<const uint16_t*>(a.cache) + ((int64_t)page * a.kv_heads + g) * head_elems + (int64_t)a.block_size * DK;
+        const int o0 = k0 % a.block_size - k0;
+#pragma unroll
+        for (int i = 0; i < NI; ++i) {
+            const int key = k0 + i * SLOTS + ls;
+            VL::load(base + (int64_t)((key < pos ? key : pos) + o0) * DV, ll, vd[i]);
+        }
+    };
+    // a unit that starts past the query's position (the second half of its tile) holds nothing to see
+    auto live = [&](int u) { return u < units && unit_key(u) <= pos; };
+    int u = wave;
+    int page = live(u) ? table[unit_key(u) / a.block_size] : 0;
+    if (live(u)) {
+        load_k(unit_key(u), page);
+        load_v(unit_key(u), page);
+    }
+    int next_page = live(u + 4) ? table[unit_key(u + 4) / a.block_size] : 0;
+    for (; live(u); u += 4) {
+        const int k0 = unit_key(u);
+        float s[R][NI];
+#pragma unroll
+        for (int r = 0; r < R; ++r)
+#pragma unroll
+            for (int i = 0; i < NI; ++i) {
+                float acc = 0.f;
+#pragma unroll
+                for (int d = 0; d < KL::DW; ++d) acc = dot2_bf16(kd[i][d], q[r][d], acc);
+                s[r][i] = acc;
+            }
+        const bool more = live(u + 4);
+        if (more) load_k(unit_key(u + 4), next_page);
+        bool sees[NI];
+#pragma unroll
+        for (int i = 0; i < NI; ++i) {
+            const int key = k0 + i * SLOTS + ls;
+            sees[i] = key <= pos && (a.window <= 0 || pos - key < a.window || key < a.keep_first);
+        }
+#pragma unroll
+        for (int r = 0; r < R; ++r) {
+            float mx = m[r];
+#pragma unroll
+            for (int i = 0; i < NI; ++i) {
+                s[r][i] = sees[i] ? lanes_sum<LPR>(s[r][i]) * sc : -INFINITY;
+                mx = max2(mx, s[r][i]);
+            }
+            const float m_use = mx == -INFINITY ? 0.f : mx, alpha = fast_exp2(m[r] - m_use);
+            float sum = 0.f;
+#pragma unroll
+            for (int i = 0; i < NI; ++i) {
+                s[r][i] = fast_exp2(s[r][i] - m_use);
+                sum += s[r][i];
+            }
+            l[r] = l[r] * alpha + sum;
+            m[r] = mx;
+#pragma unroll
+            for (int e = 0; e < VL::E; ++e) o[r][e] *= alpha;
+        }
+#pragma unroll
+        for (int i = 0; i < NI; ++i)
+#pragma unroll
+            for (int d = 0; d < VL::DW; ++d) {
+                const float v0 = bf16_lo(vd[i][d]), v1 = bf16_hi(vd[i][d]);
+#pragma unroll
+                for (int r = 0; r < R; ++r) {
+                    o[r][2 * d] += s[r][i] * v0;
+                    o[r][2 * d + 1] += s[r][i] * v1;
+                }
+            }
+        if (more) {
+            load_v(unit_key(u + 4), next_page);
+            next_page = live(u + 8) ? table[unit_key(u + 8) / a.block_size] : 0;
+        }
+    }
+    // ---- merge the lane groups of the wave, then the waves
+#pragma unroll
+    for (int r = 0; r < R; ++r) {
+        float mx = m[r];
+        if constexpr (LPR == 8) mx = max2(mx, __shfl_xor(mx, 8));
+        mx = max_xor16(mx);
+        mx = max_xor32(mx);
+        const float f = mx == -INFINITY ? 0.f : fast_exp2(m[r] - mx);
+        float sum = l[r] * f;
+        if constexpr (LPR == 8) sum += __shfl_xor(sum, 8);
+        sum = sum_xor16(sum);
+        sum = sum_xor32(sum);
+        float* dst = rec + (wave * R + r) * RECW;
+#pragma unroll
+        for (int e = 0; e < VL::E; ++e) {
+            float v = o[r][e] * f;
+            if constexpr (LPR == 8) v += __shfl_xor(v, 8);
+            v = sum_xor16(v);
+            v = sum_xor32(v);
+            if (ls == 0) dst[VL::column(ll, e)] = v;
+        }
+        if (lane == 0) {
+            dst[DV] = mx;
+            dst[DV + 1] = sum;
+        }
+    }
+    __syncthreads();
+    constexpr int PIECES = DV / 4;
+    auto finish = [&](int r, int c, f32x4 v) {       // 4 normalised columns of head h0 + r
+        const int col = (h0 + r) * DV + c;
+        if (a.out) act_st4(reinterpret_cast<uint16_t*>(a.out) + (int64_t)row * a.out_stride + col, v);
+        if (a.out_packed) act_st4(reinterpret_cast<uint16_t*>(a.out_packed) + pack_index(row, col, a.heads * DV), v);
+    };
+    for (int e = tid; e < nh * PIECES; e += 256) {
+        const int r = e / PIECES, c = (e - r * PIECES) * 4;
+        float mw[4], mx = -INFINITY, sum = 0.f;
+#pragma unroll
+        for (int w = 0; w < 4; ++w) {
+            mw[w] = rec[(w * R + r) * RECW + DV];
+            mx = fmaxf(mx, mw[w]);
+        }
+        const float sink = a.splits == 1 && a.sink ? a.sink[h0 + r] * kLog2e : -INFINITY;
+        mx = fmaxf(mx, sink);
+        const float m_use = mx == -INFINITY ? 0.f : mx;
+        f32x4 v = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int w = 0; w < 4; ++w) {
+            const float f = fast_exp2(mw[w] - m_use);
+            v += *reinterpret_cast<const f32x4*>(rec + (w * R + r) * RECW + c) * f;
+            sum += rec[(w * R + r) * RECW + DV + 1] * f;
+        }
+        if (a.splits == 1) {
+            sum += fast_exp2(sink - m_use);
+            finish(r, c, v * (sum > 0.f ? 1.f / sum : 0.f));
+        } else {
+            const int64_t at = ((int64_t)row * a.heads + h0 + r) * a.splits + split;
+#pragma unroll
+            for (int k = 0; k < 4; ++k) st_through(a.part_o + at * DV + c + k, v[k]);
+            if (c == 0) {
+                st_through(a.part_ml + at * 2, mx);
+                st_through(a.part_ml + at * 2 + 1, sum);
+            }
+        }
+    }
+    if (a.splits == 1) return;
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+    __syncthreads();
+    if (tid == 0) {
+        uint32_t* ticket = a.tickets + ((int64_t)row * gridDim.y + blockIdx.y) * kAttendTicketWords;
+        const uint32_t seen = __hip_atomic_fetch_add(ticket, 1u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+        last_flag = seen == (uint32_t)a.splits - 1;
+        if (last_flag) __hip_atomic_store(ticket, 0u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+    }
+    __syncthreads();
+    if (!last_flag) return;
+    for (int e = tid; e < nh * PIECES; e += 256) {
+        const int r = e / PIECES, c = (e - r * PIECES) * 4;
+        const int64_t at = ((int64_t)row * a.heads + h0 + r) * a.splits;
+        const float sink = a.sink ? a.sink[h0 + r] * kLog2e : -INFINITY;
+        float mx = sink;
+        for (int s = 0; s < a.splits; ++s) mx = fmaxf(mx, ld_through(a.part_ml + (at + s) * 2));
+        const float m_use = mx == -INFINITY ? 0.f : mx;
+        float sum = fast_exp2(sink - m_use);
+        f32x4 v = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
+        for (int s = 0; s < a.splits; ++s) {
+            const float f = fast_exp2(ld_through(a.part_ml + (at + s) * 2) - m_use);
+            sum += f * ld_through(a.part_ml + (at + s) * 2 + 1);
+#pragma unroll
+            for (int k = 0; k < 4; ++k) v[k] += f * ld_through(a.part_o + (at + s) * DV + c + k);
+        }
+        finish(r, c, v * (sum > 0.f ? 1.f / sum : 0.f));
+    }
+}
+
+template <int DK, int DV>
+void rows_dims(const PagedAttendArgs& a, hipStream_t stream) {
+    const int ratio = a.heads / a.kv_heads;
+    const dim3 grid(a.splits, a.kv_heads * paged_attend_groups(a.heads, a.kv_heads), a.rows);
+    if (ratio == 1) paged_rows_kernel<DK, DV, 1><<<grid, 256, 0, stream>>>(a);
+    else if (ratio == 2) paged_rows_kernel<DK, DV, 2><<<grid, 256, 0, stream>>>(a);
+    else if (ratio <= 4) paged_rows_kernel<DK, DV, 4><<<grid, 256, 0, stream>>>(a);
+    else paged_rows_kernel<DK, DV, 8><<<grid, 256, 0, stream>>>(a);
+}
+
+template <typename T>
+void prep_t(const AttnPrepArgs& a, hipStream_t stream) {
+    const int ch = (a.heads * a.dk + a.kv_heads * (a.dk + a.dv) + 2047) / 2048;
+    if (ch <= 1) attn_prep_kernel<T, 1><<<a.rows, 256, 0, stream>>>(a);
+    else if (ch <= 2) attn_prep_kernel<T, 2><<<a.rows, 256, 0, stream>>>(a);
+    else if (ch <= 4) attn_prep_kernel<T, 4><<<a.rows, 256, 0, stream>>>(a);
+    else if (ch <= 8) attn_prep_kernel<T, 8><<<a.rows, 256, 0, stream>>>(a);
+    else attn_prep_kernel<T, kRowPieces><<<a.rows, 256, 0, stream>>>(a);
+}
+
+}  // namespace
+
+int launch_attn_prep(const AttnPrepArgs& a, int f32, hipStream_t stream) {
+    if (f32) prep_t<float>(a, stream);
+    else prep_t<uint16_t>(a, stream);
+    return check_launch("attn_prep");
+}
+
+bool paged_attend_supported(int dk, int dv, int block_size) {
+    if (block_size % 64) return false;
+    return ((dk == 64 || dk == 128 || dk == 192 || dk == 256) && (dv == 64 || dv == 128)) || (dk == 256 && dv == 256);
+}
+
+int paged_attend_groups(int heads, int kv_heads) { return (heads / kv_heads + kRowsHeads - 1) / kRowsHeads; }
+
+int launch_paged_attend_rows(const PagedAttendArgs& a, int f32, int generic, hipStream_t stream) {
+    if (!f32 && !generic && !a.row_seq && paged_attend_supported(a.dk, a.dv, a.block_size)) {
+        switch (a.dk * 1000 + a.dv) {
+            case 64064: rows_dims<64, 64>(a, stream); break;
+            case 64128: rows_dims<64, 128>(a, stream); break;
+            case 128064: rows_dims<128, 64>(a, stream); break;
+            case 128128: rows_dims<128, 128>(a, stream); break;
+            case 192064: rows_dims<192, 64>(a, stream); break;
+            case 192128: rows_dims<192, 128>(a, stream); break;
+            case 256064: rows_dims<256, 64>(a, stream); break;
+            case 256128: rows_dims<256, 128>(a, stream); break;
+            default: rows_dims<256, 256>(a, stream); break;
+        }
+    } else {
+        const dim3 grid(a.rows, a.heads);
+        if (f32) paged_rows_generic_kernel<float><<<grid, 256, a.dk * 4, stream>>>(a);
+        else paged_rows_generic_kernel<uint16_t><<<grid, 256, a.dk * 4, stream>>>(a);
+    }
+    return check_launch("paged_attend_rows");
+}
+
+}  // namespace nvh

@@ -10,7 +10,7 @@ import torch  # noqa: F401  (imported first on purpose: libnvh_attn.so binds to 
 
 _HERE = os.path.dirname(os.path.abspath(__file__))
 LIB_PATH = os.environ.get("NVH_LIB_PATH") or os.path.join(_HERE, "lib", "libnvh_attn.so")   # override: A/B of two builds
-LAYERS_LIB_PATH = os.path.join(_HERE, "lib", "libnvh_layers.so")                            # the subset without paged K/V attention (build.py layers_only)
+_subset = None                                                                             # architecture whose kernels alone may be built (build.py --model)
 
 NVH_BF16 = 0
 NVH_F32 = 1
@@ -78,6 +78,59 @@ class LatentPrefillDesc(ctypes.Structure):
                 ("positions", ctypes.c_void_p), ("cos_sin", ctypes.c_void_p), ("max_position", ctypes.c_int32), ("rot", ctypes.c_int32),
                 ("batch", ctypes.c_int32), ("heads", ctypes.c_int32), ("dim_cols", ctypes.c_int32), ("dk", ctypes.c_int32),
                 ("dv", ctypes.c_int32), ("max_q", ctypes.c_int32), ("scale_log2", ctypes.c_float)]
+
+
+class AttnPrepDesc(ctypes.Structure):
+    """nvh_attn_prep_desc (include/nvh_attn.h)."""
+    _fields_ = [("qkv", ctypes.c_void_p), ("qkv_stride", ctypes.c_int64), ("rows", ctypes.c_int32), ("heads", ctypes.c_int32),
+                ("kv_heads", ctypes.c_int32), ("dk", ctypes.c_int32), ("dv", ctypes.c_int32), ("q_w", ctypes.c_void_p),
+                ("k_w", ctypes.c_void_p), ("q_n", ctypes.c_int32), ("k_n", ctypes.c_int32), ("eps", ctypes.c_float),
+                ("positions", ctypes.c_void_p), ("cos_sin", ctypes.c_void_p), ("max_position", ctypes.c_int32), ("rot", ctypes.c_int32),
+                ("cache", ctypes.c_void_p), ("slots", ctypes.c_void_p), ("block_size", ctypes.c_int32)]
+
+
+class PagedAttendDesc(ctypes.Structure):
+    """nvh_paged_attend_desc (include/nvh_attn.h)."""
+    _fields_ = [("q", ctypes.c_void_p), ("q_stride", ctypes.c_int64), ("rows", ctypes.c_int32), ("heads", ctypes.c_int32),
+                ("kv_heads", ctypes.c_int32), ("dk", ctypes.c_int32), ("dv", ctypes.c_int32), ("cache", ctypes.c_void_p),
+                ("block_size", ctypes.c_int32), ("block_tables", ctypes.c_void_p), ("bt_stride", ctypes.c_int64),
+                ("row_seq", ctypes.c_void_p), ("positions", ctypes.c_void_p), ("cu_q", ctypes.c_void_p), ("cu_k", ctypes.c_void_p),
+                ("batch", ctypes.c_int32), ("max_q", ctypes.c_int32), ("scale", ctypes.c_float), ("window", ctypes.c_int32),
+                ("keep_first", ctypes.c_int32), ("sink", ctypes.c_void_p), ("splits", ctypes.c_int32), ("part_o", ctypes.c_void_p),
+                ("part_ml", ctypes.c_void_p), ("tickets", ctypes.c_void_p), ("out", ctypes.c_void_p), ("out_stride", ctypes.c_int64),
+                ("out_packed", ctypes.c_void_p)]
+
+
+class LightningDesc(ctypes.Structure):
+    """nvh_lightning_desc (include/nvh_attn.h)."""
+    _fields_ = [("qkv", ctypes.c_void_p), ("qkv_stride", ctypes.c_int64), ("rows", ctypes.c_int32), ("heads", ctypes.c_int32),
+                ("dk", ctypes.c_int32), ("dv", ctypes.c_int32), ("decay", ctypes.c_void_p), ("positions", ctypes.c_void_p),
+                ("state_slots", ctypes.c_void_p), ("state", ctypes.c_void_p), ("chunks", ctypes.c_void_p), ("n_chunks", ctypes.c_int32),
+                ("summaries", ctypes.c_int32), ("seg_state", ctypes.c_void_p), ("out", ctypes.c_void_p), ("out_stride", ctypes.c_int64)]
+
+
+class MoeRouteDesc(ctypes.Structure):
+    """nvh_moe_route_desc (include/nvh_attn.h)."""
+    _fields_ = [("x", ctypes.c_void_p), ("x_stride", ctypes.c_int64), ("router", ctypes.c_void_p), ("correction", ctypes.c_void_p),
+                ("rows", ctypes.c_int32), ("cols", ctypes.c_int32), ("experts", ctypes.c_int32), ("top", ctypes.c_int32),
+                ("groups", ctypes.c_int32), ("keep", ctypes.c_int32), ("scale", ctypes.c_float), ("ids", ctypes.c_void_p),
+                ("weights", ctypes.c_void_p)]
+
+
+class MoeGemmDesc(ctypes.Structure):
+    """nvh_moe_gemm_desc (include/nvh_attn.h)."""
+    _fields_ = [("out", ctypes.c_void_p), ("x", ctypes.c_void_p), ("x_stride", ctypes.c_int64), ("w", ctypes.c_void_p),
+                ("pairs", ctypes.c_int32), ("top", ctypes.c_int32), ("experts", ctypes.c_int32), ("n", ctypes.c_int32),
+                ("k", ctypes.c_int32), ("glu", ctypes.c_int32), ("ids", ctypes.c_void_p), ("slot_pair", ctypes.c_void_p),
+                ("tiles", ctypes.c_void_p), ("max_tiles", ctypes.c_int32)]
+
+
+class ResidualNormDesc(ctypes.Structure):
+    """nvh_residual_norm_desc (include/nvh_attn.h)."""
+    _fields_ = [("x", ctypes.c_void_p), ("y", ctypes.c_void_p), ("y_stride", ctypes.c_int64), ("e", ctypes.c_void_p),
+                ("ew", ctypes.c_void_p), ("top", ctypes.c_int32), ("w", ctypes.c_void_p), ("b", ctypes.c_void_p), ("eps", ctypes.c_float),
+                ("rows", ctypes.c_int32), ("cols", ctypes.c_int32), ("n", ctypes.c_int32), ("xb", ctypes.c_void_p),
+                ("packed", ctypes.c_void_p)]
 
 
 EPI_NONE, EPI_SILU_MUL, EPI_RESIDUAL_ADD, EPI_ROPE_STORE = 0, 1, 2, 3
@@ -163,6 +216,22 @@ _SIGS = {
     "nvh_latent_gather": (ctypes.c_int, [ctypes.c_void_p] * 4 + [ctypes.c_int64] + [ctypes.c_int] * 5 + [ctypes.c_void_p]),
     "nvh_latent_prefill_supported": (ctypes.c_int, [ctypes.c_int] * 2),
     "nvh_latent_prefill": (ctypes.c_int, [ctypes.POINTER(LatentPrefillDesc), ctypes.c_int, ctypes.c_void_p]),
+    "nvh_attn_prep": (ctypes.c_int, [ctypes.POINTER(AttnPrepDesc), ctypes.c_int, ctypes.c_void_p]),
+    "nvh_paged_attend_supported": (ctypes.c_int, [ctypes.c_int] * 3),
+    "nvh_paged_attend_ticket_bytes": (ctypes.c_size_t, [ctypes.c_int] * 3),
+    "nvh_paged_attend_rows": (ctypes.c_int, [ctypes.POINTER(PagedAttendDesc), ctypes.c_int, ctypes.c_int, ctypes.c_void_p]),
+    "nvh_paged_attend_prompt": (ctypes.c_int, [ctypes.POINTER(PagedAttendDesc), ctypes.c_int, ctypes.c_void_p]),
+    "nvh_lightning_supported": (ctypes.c_int, [ctypes.c_int] * 2),
+    "nvh_lightning_chunks": (ctypes.c_int, [ctypes.POINTER(LightningDesc), ctypes.c_int, ctypes.c_int, ctypes.c_void_p]),
+    "nvh_lightning_step": (ctypes.c_int, [ctypes.POINTER(LightningDesc), ctypes.c_int, ctypes.c_void_p]),
+    "nvh_norm_gate": (ctypes.c_int, [ctypes.c_void_p] * 5 + [ctypes.c_float] + [ctypes.c_int] * 3 + [ctypes.c_int64] * 3 + [ctypes.c_int, ctypes.c_void_p]),
+    "nvh_moe_route": (ctypes.c_int, [ctypes.POINTER(MoeRouteDesc), ctypes.c_int, ctypes.c_void_p]),
+    "nvh_moe_dispatch_blocks": (ctypes.c_int, [ctypes.c_int]),
+    "nvh_moe_dispatch": (ctypes.c_int, [ctypes.c_void_p] * 4 + [ctypes.c_int] * 4 + [ctypes.c_void_p]),
+    "nvh_moe_tile_rows": (ctypes.c_int, [ctypes.c_int]),
+    "nvh_moe_gemm": (ctypes.c_int, [ctypes.POINTER(MoeGemmDesc), ctypes.c_int, ctypes.c_void_p]),
+    "nvh_residual_norm": (ctypes.c_int, [ctypes.POINTER(ResidualNormDesc), ctypes.c_int, ctypes.c_void_p]),
+    "nvh_softcap": (ctypes.c_int, [ctypes.c_void_p, ctypes.c_float, ctypes.c_int, ctypes.c_int, ctypes.c_int64, ctypes.c_int, ctypes.c_void_p]),
 }
 EXPORTS = tuple(_SIGS)
 
@@ -174,7 +243,7 @@ class NvhLibraryError(RuntimeError):
 
 
 class _Subset:
-    """The layers-only library: entry points it does not hold raise when they are asked for."""
+    """A library with the kernels of one model: entry points it does not hold raise when they are asked for."""
 
     def __init__(self, lib, path):
         self._lib, self._path = lib, path
@@ -186,13 +255,24 @@ class _Subset:
             raise NvhLibraryError(f"{self._path} does not hold {name}: build the whole library with `python nano-vllm-learn_amd/build.py`") from e
 
 
+def subset_path(architecture):
+    return os.path.join(_HERE, "lib", f"libnvh_{architecture.lower()}.so")
+
+
+def use_subset(architecture):
+    """Where the whole library is not built, load the one with this architecture's kernels (before anything is loaded)."""
+    global _subset
+    _subset = architecture
+
+
 def load():
-    """Load (once) and return the library: libnvh_attn.so, or the layers-only subset where only that is built.  Raises
+    """Load (once) and return the library: libnvh_attn.so, or the subset chosen by use_subset() where only that is built.  Raises
     NvhLibraryError if neither is there."""
     global _lib
     if _lib is not None:
         return _lib
-    path = LIB_PATH if os.path.exists(LIB_PATH) or "NVH_LIB_PATH" in os.environ else LAYERS_LIB_PATH
+    whole = os.path.exists(LIB_PATH) or "NVH_LIB_PATH" in os.environ or _subset is None
+    path = LIB_PATH if whole else subset_path(_subset)
     if not os.path.exists(path):
         raise NvhLibraryError(
             f"{LIB_PATH} not found: build it with `python nano-vllm-learn_amd/build.py` "
@@ -201,7 +281,7 @@ def load():
         lib = ctypes.CDLL(path)
     except OSError as e:
         raise NvhLibraryError(f"cannot load {path}: {e}") from e
-    subset = path == LAYERS_LIB_PATH
+    subset = not whole
     for name, (res, args) in _SIGS.items():
         try:
             fn = getattr(lib, name)

@@ -159,18 +159,20 @@ class ModelRunner:
             self.comm = init_tensor_parallel_comm(64, cfg.hidden_size, prefer_oneshot=os.environ.get("NVH_ALLREDUCE", "oneshot") != "rccl")
 
     def allocate_kv_cache(self):
-        """Every module that declares what it keeps per token (`cache_row`) or per sequence (`state_spec`) gets its pool; attention modules with
-        k_cache / v_cache share one tensor."""
+        """Every module that declares what it keeps per token (`cache_row`) or per sequence (`state_spec`) gets its pool, one per pass where a module
+        runs in several (`passes`: a leading dimension); attention modules with k_cache / v_cache share one tensor."""
         cfg = self.cfg
         if self.mixed_batches:
             self.kv_cache = []
             for name, module in self.model.named_modules():
+                passes = (module.passes,) if hasattr(module, "passes") else ()
                 if getattr(module, "cache_row", None) and module.cache_row() is not None:
                     cols, dtype = module.cache_row()
-                    module.latent_cache = torch.zeros(self.num_kvcache_blocks, self.block_size, cols, dtype=dtype, device=self.device)
-                    self.kv_cache.append(module.latent_cache)
+                    pool = torch.zeros(*passes, self.num_kvcache_blocks, self.block_size, cols, dtype=dtype, device=self.device)
+                    setattr(module, getattr(module, "cache_name", "latent_cache"), pool)
+                    self.kv_cache.append(pool)
                 for attr, (shape, dtype) in (module.state_spec() if hasattr(module, "state_spec") else {}).items():
-                    pool = torch.zeros(self.max_num_seqs, *shape, dtype=dtype, device=self.device)
+                    pool = torch.zeros(*passes, self.max_num_seqs, *shape, dtype=dtype, device=self.device)
                     setattr(module, attr, pool)
                     self.state[f"{name}.{attr}"] = pool
             return
@@ -326,7 +328,7 @@ class DecodeSession:
             self.positions -= 1                                   # of the token that is fed (build_decode_meta has the reference's own convention)
             slots = torch.tensor([s.state_slot for s in seqs], dtype=torch.int32)
             chunks = torch.tensor([(i, 1, i, 0) for i in range(b)], dtype=torch.int32)
-            self.step_meta = StepMeta(b, self.slot_mapping, self.block_tables, slots.to(dev), chunks.to(dev), ops.rglru_chunk_tokens(), False, need_tokens)
+            self.step_meta = StepMeta(b, self.slot_mapping, self.block_tables, slots.to(dev), chunks.to(dev), 64, False, need_tokens)
         # the next step's embedding lookup rides in the arg-max launch when the model allows it: the session then owns the
         # embedded rows (row-major = the residual stream of the step, and in fragment order for layer 0's projection)
         self.fuse_embed = bool(getattr(runner.model, "fused_embedding_ok", lambda *_: False)(b, torch.device(dev)))

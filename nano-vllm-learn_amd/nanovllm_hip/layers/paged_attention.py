@@ -1,0 +1,104 @@
+"""Softmax attention with grouped heads over its own pages: optional projection biases, RMS norm over the whole query and key projections, rotation of the
+leading dimensions, a sliding window with kept first tokens, a learned sink per head.  Every pass over the layer (a looped layer has several) has its own
+cache, bound by the runner (`page_cache` [passes, pages, block_size, kv_heads * (dk + dv)], inside a page [kv head][keys | values]).
+
+Single rows (decode) stream the visible keys; prompt portions run the MFMA kernel over the pages.  Widths those kernels do not take, and fp32 models, use
+the plain kernel for both.  Padded widths (zeros): keys to 64 / 128 / 192 / 256, values to 64 / 128 / 256.
+"""
+import torch
+from torch import nn
+
+from .. import ops
+from .linear import linear, padded, round_up
+
+
+def padded_widths(dim, vdim):
+    """Key and value widths of the MFMA kernels that hold `dim` and `vdim`, or the next multiples of 8."""
+    if dim > 256 or vdim > 256:
+        return round_up(dim, 8), round_up(vdim, 8)
+    dk, dv = round_up(dim, 64), (64 if vdim <= 64 else 128 if vdim <= 128 else 256)
+    return (256, 256) if dv == 256 else (dk, dv)
+
+
+class PagedAttention(nn.Module):
+    cache_name = "page_cache"
+
+    def __init__(self, in_width, in_cols, heads, kv_heads, dim, vdim, scale, rope, dtype, eps, bias=False, qk_norm=False, sink=False, window=0, keep_first=0, passes=1,
+                 block_size=64):
+        super().__init__()
+        assert heads % kv_heads == 0, f"{heads} query heads must share {kv_heads} key/value heads evenly"
+        self.in_width, self.in_cols, self.dtype, self.eps, self.rope = in_width, in_cols, dtype, eps, rope
+        self.heads, self.kv_heads, self.dim, self.vdim, self.scale = heads, kv_heads, dim, vdim, float(scale)
+        self.bias, self.qk_norm, self.has_sink, self.window, self.keep_first, self.passes = bias, qk_norm, sink, int(window), int(keep_first), passes
+        self.dk, self.dv = padded_widths(dim, vdim)
+        self.q_cols, self.k_cols, self.v_cols = heads * self.dk, kv_heads * self.dk, kv_heads * self.dv
+        self.out_cols = round_up(heads * self.dv, 64)
+        self.proj_cols = round_up(self.q_cols + self.k_cols + self.v_cols, 64)
+        self.page_cache = torch.tensor([])
+        # the MFMA prompt kernel takes the maximum before the scale
+        self.fast = dtype == torch.bfloat16 and self.scale > 0 and heads * self.dv == self.out_cols and ops.paged_attend_supported(self.dk, self.dv, block_size)
+
+    def cache_row(self):
+        """Elements and type of one token's cache row."""
+        return self.k_cols + self.v_cols, self.dtype
+
+    def load(self, get):
+        """get(name) -> tensor of the checkpoint (names below the mixer's prefix)."""
+        h, g, c, reg = self.heads, self.kv_heads, self.in_cols, self.register_buffer
+        assert get("q").shape == (h * self.dim, self.in_width) and get("v").shape == (g * self.vdim, self.in_width)
+
+        def head_rows(t, n, width, to):                      # [n * width, ...] -> [n * to, ...]
+            t = t.reshape(n, width, -1)
+            return padded(t, n, to, t.shape[2]).reshape(n * to, -1)
+        parts = [("q", h, self.dim, self.dk), ("k", g, self.dim, self.dk), ("v", g, self.vdim, self.dv)]
+        w = torch.cat([padded(head_rows(get(n), *s), s[0] * s[2], c) for n, *s in parts])
+        reg("w_qkv", padded(w, self.proj_cols, c).to(self.dtype).contiguous())
+        reg("b_qkv", padded(torch.cat([head_rows(get(n + ".b"), *s).reshape(-1) for n, *s in parts]), self.proj_cols).to(self.dtype).contiguous() if self.bias else None)
+        for n, heads in (("q", h), ("k", g)):
+            reg(n + "_norm", head_rows(get(n + ".norm").float(), heads, self.dim, self.dk).reshape(-1).contiguous() if self.qk_norm else None)
+        reg("sink", get("sink").float().contiguous() if self.has_sink else None)
+        o = padded(get("o").reshape(self.in_width, h, self.vdim), self.in_width, h, self.dv).reshape(self.in_width, h * self.dv)
+        reg("w_o", padded(o, c, self.out_cols).to(self.dtype).contiguous())
+
+    def _prep(self, qkv, positions, step, cache):
+        norm = dict(q_weight=self.q_norm, k_weight=self.k_norm, q_n=self.heads * self.dim, k_n=self.kv_heads * self.dim, eps=self.eps) if self.qk_norm else {}
+        ops.attn_prep(qkv, self.heads, self.kv_heads, self.dk, self.dv, positions, self.rope(qkv.device), cache, step.slot_mapping, **norm)
+
+    def _mask(self):
+        return dict(window=self.window, keep_first=self.keep_first, sink=self.sink)
+
+    def _rows(self, q, positions, step, cache, row_seq=None, **kw):
+        return ops.paged_attend_rows(q, cache, step.block_tables, positions, self.heads, self.kv_heads, self.dk, self.dv, self.scale, step.max_context,
+                                     row_seq=row_seq, **self._mask(), **kw)
+
+    def forward(self, x, positions, step, run=0):
+        """x [rows, in_cols] in the activation type -> the mixer's output, same shape; run: which pass over the layer this is."""
+        rows, n, cache = x.shape[0], step.num_decode, self.page_cache[run]
+        qkv = linear(x, self.w_qkv, self.b_qkv)
+        self._prep(qkv, positions, step, cache)
+        alloc = torch.empty if self.heads * self.dv == self.out_cols else torch.zeros
+        out = alloc((rows, self.out_cols), dtype=x.dtype, device=x.device)
+        o = out[:, :self.heads * self.dv]
+        if n:
+            self._rows(qkv[:n], positions[:n], step, cache, out=o[:n])
+        if n < rows and self.fast:
+            ops.paged_attend_prompt(qkv[n:], cache, step.block_tables[n:], step.cu_q, step.cu_k, step.max_q, self.heads, self.kv_heads, self.dk, self.dv, self.scale,
+                                    out=o[n:], **self._mask())
+        elif n < rows:
+            self._rows(qkv[n:], positions[n:], step, cache, row_seq=step.row_seq[n:], out=o[n:])
+        return linear(out, self.w_o)
+
+    @property
+    def step_ok(self):
+        return self.fast
+
+    def decode(self, xp, rows, positions, step, bufs, run=0):
+        """Fused decode: fragment-packed rows in, output rows out (four launches)."""
+        qkv = ops.fused_linear(xp, self.w_qkv, bias=self.b_qkv, x_packed_rows=rows, workspace=bufs.workspace)
+        self._prep(qkv, positions, step, self.page_cache[run])
+        mid = bufs.packed(self.out_cols)
+        self._rows(qkv, positions, step, self.page_cache[run], out_packed=mid, want_out=False)
+        return ops.fused_linear(mid, self.w_o, x_packed_rows=rows, workspace=bufs.workspace)
+
+    def linears(self):
+        return [(self.w_qkv, "none"), (self.w_o, "none")]

@@ -9,12 +9,17 @@ def _zobasun():
     return ZobasunConfig.from_json, ZobasunForCausalLM
 
 
+def _galirax():
+    from .galirax import GaliraxConfig, GaliraxForCausalLM
+    return GaliraxConfig.from_json, GaliraxForCausalLM
+
+
 def _qwen():
     from .qwen import ModelConfig, QwenForCausalLM
     return ModelConfig.from_json, QwenForCausalLM
 
 
-REGISTRY = {"Zobasun": _zobasun, "Qwen2ForCausalLM": _qwen, "Qwen3ForCausalLM": _qwen}
+REGISTRY = {"Zobasun": _zobasun, "Galirax": _galirax, "Qwen2ForCausalLM": _qwen, "Qwen3ForCausalLM": _qwen}
 
 
 def architecture(config_json):
@@ -31,9 +36,10 @@ def load_config(path, **overrides):
 
 
 def model_class(cfg):
+    from .galirax import GaliraxConfig, GaliraxForCausalLM
     from .qwen import ModelConfig, QwenForCausalLM
     from .zobasun import ZobasunConfig, ZobasunForCausalLM
-    return {ModelConfig: QwenForCausalLM, ZobasunConfig: ZobasunForCausalLM}[type(cfg)]
+    return {ModelConfig: QwenForCausalLM, ZobasunConfig: ZobasunForCausalLM, GaliraxConfig: GaliraxForCausalLM}[type(cfg)]
 
 
 def build_model(cfg, path=None, seed=0):

@@ -15,7 +15,7 @@ from torch import nn
 
 from .. import ops
 from ..layers.latent_attention import LatentAttention
-from ..layers.linear import linear, padded, round_up
+from ..layers.linear import DecodeBuffers, linear, padded, round_up
 from ..layers.mlp import ClampedGLU
 from ..layers.rglru import RGLRU, choose_segment
 from ..layers.rotary import rotation_table
@@ -58,24 +58,6 @@ class ZobasunConfig:
     @property
     def num_hidden_layers(self):
         return len(self.layers)
-
-
-class _DecodeBuffers:
-    """Scratch of the fused decode path for one number of 16-row tiles: fragment-order activations by width and the split-K workspace (zero-filled once)."""
-
-    def __init__(self, rows, device, linears, stream_cols):
-        self.rows16, self.device, self._packed = round_up(rows, 16), device, {}
-        need = max([16] + [ops.linear_workspace_bytes(rows, w.shape[0], w.shape[1], epi) for w, epi in linears])
-        self.workspace = torch.zeros(need, dtype=torch.uint8, device=device)
-        self.stream = torch.zeros(self.rows16 * stream_cols, dtype=torch.bfloat16, device=device)       # the residual stream in fragment order
-        for w, _ in linears:
-            self.packed(w.shape[1])
-
-    def packed(self, cols):
-        """One buffer per width, never the stream's: what one launch writes the next launch on the stream consumes, so equal widths can share."""
-        if cols not in self._packed:
-            self._packed[cols] = torch.zeros(self.rows16 * cols, dtype=torch.bfloat16, device=self.device)
-        return self._packed[cols]
 
 
 class ZobasunLayer(nn.Module):
@@ -154,7 +136,7 @@ class ZobasunForCausalLM(nn.Module):
         rows = round_up(rows, 16)
         if rows not in self._bufs:
             lin = [l for layer in self.layers for l in layer.mixer.linears() + (layer.mlp.linears() if layer.mlp is not None else [])]
-            self._bufs[rows] = _DecodeBuffers(rows, self.embed.device, lin + [(self.head, "none")], self.cols)
+            self._bufs[rows] = DecodeBuffers(rows, self.embed.device, lin + [(self.head, "none")], self.cols)
         return self._bufs[rows]
 
     def _forward_decode(self, input_ids, positions, step):

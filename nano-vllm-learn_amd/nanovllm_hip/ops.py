@@ -841,3 +841,275 @@ def latent_prefill(q, k, k_rot, v, cu_q, cu_k, max_q, positions, cos_sin, scale,
     d.batch, d.heads, d.dim_cols, d.dk, d.dv, d.max_q, d.scale_log2 = cu_q.numel() - 1, heads, dim_cols, dk, dv, int(max_q), float(scale) * 1.4426950408889634
     _lib.check(_lib.load().nvh_latent_prefill(ctypes.byref(d), NVH_BF16, _stream()), "nvh_latent_prefill")
     return out
+
+
+# --------------------------------------------------------------------------------------- paged sink/window attention
+def _packed_ok(packed, rows, cols):
+    _require_gpu_bf16(packed=packed)
+    assert packed.is_contiguous() and packed.numel() >= ((rows + 15) // 16) * 16 * cols
+
+
+def attn_prep(qkv, heads, kv_heads, dk, dv, positions, cos_sin, cache, slots, q_weight=None, k_weight=None, q_n=0, k_n=0, eps=0.0):
+    """Row ops behind a q | k | v projection: optional RMS norm over all query and all key columns (means over q_n / k_n of them), rotation of
+    interleaved pairs of the first cos_sin.shape[1] dimensions of every head, keys and values into the cache [pages, block_size, kv_heads * (dk + dv)]
+    (inside a page: [kv head][keys | values]).  The queries are rewritten in place."""
+    code = _act_code(qkv, cache)
+    rows = qkv.shape[0]
+    _require_f32(cos_sin=cos_sin)
+    _require_i32(slots=slots)
+    assert qkv.dim() == 2 and qkv.stride(1) == 1 and qkv.shape[1] >= heads * dk + kv_heads * (dk + dv)
+    assert cache.dim() == 3 and cache.is_contiguous() and cache.shape[2] == kv_heads * (dk + dv)
+    assert positions.dtype == torch.int64 and positions.is_contiguous() and positions.numel() == rows and slots.numel() == rows and slots.is_contiguous()
+    d = _lib.AttnPrepDesc()
+    d.qkv, d.qkv_stride, d.rows, d.heads, d.kv_heads, d.dk, d.dv = qkv.data_ptr(), qkv.stride(0), rows, heads, kv_heads, dk, dv
+    if q_weight is not None:
+        _require_f32(q_weight=q_weight, k_weight=k_weight)
+        assert q_weight.numel() == heads * dk and k_weight.numel() == kv_heads * dk
+        d.q_w, d.k_w, d.q_n, d.k_n, d.eps = q_weight.data_ptr(), k_weight.data_ptr(), int(q_n), int(k_n), float(eps)
+    d.positions, d.cos_sin, d.max_position, d.rot = positions.data_ptr(), cos_sin.data_ptr(), cos_sin.shape[0], cos_sin.shape[1]
+    d.cache, d.slots, d.block_size = cache.data_ptr(), slots.data_ptr(), cache.shape[1]
+    _lib.check(_lib.load().nvh_attn_prep(ctypes.byref(d), code, _stream()), "nvh_attn_prep")
+
+
+def paged_attend_supported(dk, dv, block_size) -> bool:
+    return bool(_lib.load().nvh_paged_attend_supported(int(dk), int(dv), int(block_size)))
+
+
+def paged_attend_splits(rows, kv_heads, heads, max_context, window=0, keep_first=0) -> int:
+    """Context splits of one launch over single rows: about two workgroups per CU, none with fewer than four 64-key tiles' worth of work."""
+    seen = min(max_context, window + keep_first + 126) if window else max_context
+    tiles = (seen + 63) // 64
+    groups = rows * kv_heads * ((heads // kv_heads + 7) // 8)
+    splits = max(1, min(512 // max(1, groups), (tiles + 3) // 4, 64))
+    per = -(-tiles // splits)
+    return -(-tiles // per)
+
+
+def _paged_desc(q, cache, block_tables, heads, kv_heads, dk, dv, scale, window, keep_first, sink, out):
+    code = _act_code(q, cache)
+    rows = q.shape[0]
+    _require_i32(block_tables=block_tables)
+    assert q.dim() == 2 and q.stride(1) == 1 and q.shape[1] >= heads * dk and cache.dim() == 3 and cache.is_contiguous() and cache.shape[2] == kv_heads * (dk + dv)
+    assert block_tables.dim() == 2 and block_tables.stride(1) == 1
+    d = _lib.PagedAttendDesc()
+    d.q, d.q_stride, d.rows, d.heads, d.kv_heads, d.dk, d.dv = q.data_ptr(), q.stride(0), rows, heads, kv_heads, dk, dv
+    d.cache, d.block_size, d.block_tables, d.bt_stride = cache.data_ptr(), cache.shape[1], block_tables.data_ptr(), block_tables.stride(0)
+    d.scale, d.window, d.keep_first, d.splits = float(scale), int(window), int(keep_first), 1
+    if sink is not None:
+        _require_f32(sink=sink)
+        assert sink.numel() == heads
+        d.sink = sink.data_ptr()
+    if out is not None:
+        assert out.shape == (rows, heads * dv) and out.stride(1) == 1 and out.dtype == q.dtype
+        d.out, d.out_stride = out.data_ptr(), out.stride(0)
+    return d, code
+
+
+def paged_attend_rows(q, cache, block_tables, positions, heads, kv_heads, dk, dv, scale, max_context, window=0, keep_first=0, sink=None, row_seq=None, out=None,
+                      out_packed=None, want_out=True, splits=None, generic=False):
+    """Attention of single query rows over the pages (row i: sequence row_seq[i], or i; sees its own position and before, with window > 0 only what is
+    nearer than `window` or among the first keep_first tokens; sink [heads] joins the softmax).  Returns [rows, heads * dv].
+    generic=True forces the plain kernel (tests)."""
+    rows = q.shape[0]
+    if out is None and want_out:
+        out = torch.empty((rows, heads * dv), dtype=q.dtype, device=q.device)
+    d, code = _paged_desc(q, cache, block_tables, heads, kv_heads, dk, dv, scale, window, keep_first, sink, out)
+    assert positions.dtype == torch.int64 and positions.is_contiguous() and positions.numel() == rows
+    d.positions = positions.data_ptr()
+    if row_seq is not None:
+        _require_i32(row_seq=row_seq)
+        assert row_seq.numel() == rows and row_seq.is_contiguous()
+        d.row_seq = row_seq.data_ptr()
+    else:
+        assert block_tables.shape[0] >= rows
+    if code == NVH_BF16 and row_seq is None and not generic and paged_attend_supported(dk, dv, cache.shape[1]):
+        d.splits = splits or paged_attend_splits(rows, kv_heads, heads, max_context, window, keep_first)
+    if d.splits > 1:
+        part_o = torch.empty((rows, heads, d.splits, dv), dtype=torch.float32, device=q.device)
+        part_ml = torch.empty((rows, heads, d.splits, 2), dtype=torch.float32, device=q.device)
+        tickets = reserve_workspace(q.device, paged_attend_ticket_bytes(rows, kv_heads, heads), "paged_attend")
+        d.part_o, d.part_ml, d.tickets = part_o.data_ptr(), part_ml.data_ptr(), tickets.data_ptr()
+    if out_packed is not None:
+        _packed_ok(out_packed, rows, heads * dv)
+        d.out_packed = out_packed.data_ptr()
+    _lib.check(_lib.load().nvh_paged_attend_rows(ctypes.byref(d), int(generic), code, _stream()), "nvh_paged_attend_rows")
+    return out
+
+
+def paged_attend_ticket_bytes(rows, kv_heads, heads) -> int:
+    return int(_lib.load().nvh_paged_attend_ticket_bytes(rows, kv_heads, heads))
+
+
+def paged_attend_prompt(q, cache, block_tables, cu_q, cu_k, max_q, heads, kv_heads, dk, dv, scale, window=0, keep_first=0, sink=None, out=None):
+    """Attention of prompt portions over the pages (bf16): rows cu_q[b] .. of q are the last ones of sequence b, which has cu_k[b + 1] - cu_k[b] keys;
+    visibility and sink as in paged_attend_rows.  Returns [rows, heads * dv]."""
+    _require_gpu_bf16(q=q)
+    _require_i32(cu_q=cu_q, cu_k=cu_k)
+    if out is None:
+        out = torch.empty((q.shape[0], heads * dv), dtype=q.dtype, device=q.device)
+    d, code = _paged_desc(q, cache, block_tables, heads, kv_heads, dk, dv, scale, window, keep_first, sink, out)
+    assert cu_q.numel() == cu_k.numel() and cu_q.is_contiguous() and cu_k.is_contiguous() and block_tables.shape[0] >= cu_q.numel() - 1
+    d.cu_q, d.cu_k, d.batch, d.max_q = cu_q.data_ptr(), cu_k.data_ptr(), cu_q.numel() - 1, int(max_q)
+    _lib.check(_lib.load().nvh_paged_attend_prompt(ctypes.byref(d), code, _stream()), "nvh_paged_attend_prompt")
+    return out
+
+
+# --------------------------------------------------------------------------------------- lightning attention
+def lightning_supported(dk, dv) -> bool:
+    return bool(_lib.load().nvh_lightning_supported(int(dk), int(dv)))
+
+
+def _lightning_desc(qkv, decay, positions, state_slots, state, out):
+    code = _act_code(qkv)
+    slots, heads, dk, dv = state.shape
+    rows = qkv.shape[0]
+    _require_f32(decay=decay, state=state)
+    _require_i32(state_slots=state_slots)
+    assert qkv.dim() == 2 and qkv.stride(1) == 1 and qkv.shape[1] >= heads * (2 * dk + dv) and decay.numel() == heads
+    assert positions.dtype == torch.int64 and positions.is_contiguous() and positions.numel() == rows
+    if out is None:
+        out = torch.empty((rows, heads * dv), dtype=qkv.dtype, device=qkv.device)
+    assert out.shape == (rows, heads * dv) and out.stride(1) == 1 and out.dtype == qkv.dtype
+    d = _lib.LightningDesc()
+    d.qkv, d.qkv_stride, d.rows, d.heads, d.dk, d.dv = qkv.data_ptr(), qkv.stride(0), rows, heads, dk, dv
+    d.decay, d.positions, d.state_slots, d.state = decay.data_ptr(), positions.data_ptr(), state_slots.data_ptr(), state.data_ptr()
+    d.out, d.out_stride = out.data_ptr(), out.stride(0)
+    return d, out, code
+
+
+def lightning_chunks(qkv, decay, positions, state_slots, chunks, summaries, state, out=None, generic=False):
+    """Lightning attention over portions of sequences.  qkv rows: q (heads * dk) | k (heads * dk) | v (heads * dv), SiLU not applied yet; chunks int32 [n, 4] =
+    (first row, rows, sequence, index in its portion); summaries: some portion has more than one segment; state [slots, heads, dk, dv] fp32 is
+    updated.  Rows no segment covers are left alone in `out`."""
+    d, out, code = _lightning_desc(qkv, decay, positions, state_slots, state, out)
+    _require_i32(chunks=chunks)
+    assert chunks.dim() == 2 and chunks.shape[1] == 4 and chunks.is_contiguous()
+    d.chunks, d.n_chunks, d.summaries = chunks.data_ptr(), chunks.shape[0], int(summaries)
+    if summaries:
+        seg = torch.empty((chunks.shape[0], *state.shape[1:]), dtype=torch.float32, device=qkv.device)
+        d.seg_state = seg.data_ptr()
+    _lib.check(_lib.load().nvh_lightning_chunks(ctypes.byref(d), int(generic), code, _stream()), "nvh_lightning_chunks")
+    return out
+
+
+def lightning_step(qkv, decay, positions, state_slots, state, out=None):
+    """One new token per sequence (row i = sequence i), bf16."""
+    d, out, code = _lightning_desc(qkv, decay, positions, state_slots, state, out)
+    assert state_slots.numel() >= qkv.shape[0]
+    _lib.check(_lib.load().nvh_lightning_step(ctypes.byref(d), code, _stream()), "nvh_lightning_step")
+    return out
+
+
+def norm_gate(x, gate, weight, eps, n, packed=None):
+    """rmsnorm(x over n columns) * weight * sigmoid(gate); packed (bf16): in fragment order into this buffer, returns None."""
+    code = _act_code(x, gate)
+    _require_f32(weight=weight)
+    rows, cols = x.shape
+    assert gate.shape == x.shape and x.stride(1) == 1 and gate.stride(1) == 1 and weight.numel() == cols
+    out = None
+    if packed is None:
+        out = torch.empty((rows, cols), dtype=x.dtype, device=x.device)
+    else:
+        _packed_ok(packed, rows, cols)
+    rc = _lib.load().nvh_norm_gate(out.data_ptr() if out is not None else None, packed.data_ptr() if packed is not None else None, x.data_ptr(), gate.data_ptr(),
+                                   weight.data_ptr(), float(eps), rows, cols, int(n), x.stride(0), gate.stride(0), cols, code, _stream())
+    _lib.check(rc, "nvh_norm_gate")
+    return out
+
+
+# --------------------------------------------------------------------------------------- mixture of experts
+def moe_route(x, router, correction, top, groups, keep, scale):
+    """(chosen experts int32 [rows, top], weights fp32 [rows, top]) of rows x against router [experts, cols]."""
+    code = _act_code(x, router)
+    _require_f32(correction=correction)
+    rows, cols = x.shape
+    experts = router.shape[0]
+    assert router.is_contiguous() and router.shape[1] == cols and x.stride(1) == 1 and correction.numel() == experts
+    ids = torch.empty((rows, top), dtype=torch.int32, device=x.device)
+    weights = torch.empty((rows, top), dtype=torch.float32, device=x.device)
+    d = _lib.MoeRouteDesc()
+    d.x, d.x_stride, d.router, d.correction = x.data_ptr(), x.stride(0), router.data_ptr(), correction.data_ptr()
+    d.rows, d.cols, d.experts, d.top, d.groups, d.keep, d.scale = rows, cols, experts, int(top), int(groups), int(keep), float(scale)
+    d.ids, d.weights = ids.data_ptr(), weights.data_ptr()
+    _lib.check(_lib.load().nvh_moe_route(ctypes.byref(d), code, _stream()), "nvh_moe_route")
+    return ids, weights
+
+
+def moe_dispatch(ids, experts, dtype):
+    """(slot_pair, tiles): the pairs row * top + k sorted by expert, cut into tiles of one expert each; nothing comes back to the host."""
+    _require_i32(ids=ids)
+    assert ids.is_contiguous()
+    lib, pairs = _lib.load(), ids.numel()
+    tile_rows = int(lib.nvh_moe_tile_rows(_out_code(dtype)))
+    max_tiles = pairs // tile_rows + min(experts, pairs)
+    slots = torch.empty(pairs, dtype=torch.int32, device=ids.device)
+    tiles = torch.empty((pairs // tile_rows + experts, 4), dtype=torch.int32, device=ids.device)
+    counts = torch.empty((lib.nvh_moe_dispatch_blocks(pairs), experts), dtype=torch.int32, device=ids.device)
+    _lib.check(lib.nvh_moe_dispatch(slots.data_ptr(), tiles.data_ptr(), counts.data_ptr(), ids.data_ptr(), pairs, experts, tile_rows, tiles.shape[0], _stream()),
+               "nvh_moe_dispatch")
+    return slots, tiles[:max_tiles]
+
+
+def moe_gemm(x, weight, ids, glu, dispatch=None):
+    """Expert products per pair p = row * top + k: glu: silu(x[row] . gate_e) * (x[row] . up_e) with weight [experts, 2 * n, k]; otherwise x[p] . w_e with
+    weight [experts, n, k].  dispatch: what moe_dispatch returned; None: the form for at most 64 rows (bf16)."""
+    code = _act_code(x, weight)
+    experts, n, k = weight.shape
+    n = n // 2 if glu else n
+    pairs, top = ids.numel(), ids.shape[1]
+    assert weight.is_contiguous() and x.dim() == 2 and x.stride(1) == 1 and x.shape == (ids.shape[0] if glu else pairs, k) and (glu or x.is_contiguous())
+    out = torch.empty((pairs, n), dtype=x.dtype, device=x.device)
+    d = _lib.MoeGemmDesc()
+    d.out, d.x, d.x_stride, d.w = out.data_ptr(), x.data_ptr(), x.stride(0), weight.data_ptr()
+    d.pairs, d.top, d.experts, d.n, d.k, d.glu = pairs, top, experts, n, k, int(glu)
+    if dispatch is None:
+        _require_i32(ids=ids)
+        assert ids.is_contiguous()
+        d.ids = ids.data_ptr()
+    else:
+        slots, tiles = dispatch
+        assert slots.numel() == pairs and tiles.is_contiguous()
+        d.slot_pair, d.tiles, d.max_tiles = slots.data_ptr(), tiles.data_ptr(), tiles.shape[0]
+    _lib.check(_lib.load().nvh_moe_gemm(ctypes.byref(d), code, _stream()), "nvh_moe_gemm")
+    return out
+
+
+# --------------------------------------------------------------------------------------- residual and output of models with one norm per layer
+def residual_norm(x, dtype, y=None, experts=None, weight=None, bias=None, eps=0.0, n=0, packed=None, want_rows=True):
+    """x (fp32 stream, in place) += y + the weighted sum of experts = (outputs [rows * top, cols], weights [rows, top]); with weight given returns the layer norm
+    of the new rows (mean and variance over n columns) in `dtype`, and in fragment order into `packed` (bf16)."""
+    _require_f32(x=x)
+    rows, cols = x.shape
+    code = _out_code(dtype)
+    d = _lib.ResidualNormDesc()
+    d.x, d.rows, d.cols, d.n, d.eps = x.data_ptr(), rows, cols, int(n) or cols, float(eps)
+    if y is not None:
+        assert y.shape == x.shape and y.stride(1) == 1 and y.dtype == dtype and y.is_cuda
+        d.y, d.y_stride = y.data_ptr(), y.stride(0)
+    if experts is not None:
+        e, ew = experts
+        _require_f32(ew=ew)
+        assert ew.shape[0] == rows and e.shape == (ew.numel(), cols) and e.is_contiguous() and e.dtype == dtype and e.is_cuda
+        d.e, d.ew, d.top = e.data_ptr(), ew.data_ptr(), ew.shape[1]
+    out = None
+    if weight is not None:
+        _require_f32(weight=weight, bias=bias)
+        assert weight.numel() == cols and bias.numel() == cols
+        d.w, d.b = weight.data_ptr(), bias.data_ptr()
+        if want_rows:
+            out = torch.empty((rows, cols), dtype=dtype, device=x.device)
+            d.xb = out.data_ptr()
+        if packed is not None:
+            _packed_ok(packed, rows, cols)
+            d.packed = packed.data_ptr()
+    _lib.check(_lib.load().nvh_residual_norm(ctypes.byref(d), code, _stream()), "nvh_residual_norm")
+    return out
+
+
+def softcap_(x, cap):
+    """cap * tanh(x / cap) in place (rows with any stride)."""
+    code = _act_code(x)
+    assert x.dim() == 2 and x.stride(1) == 1
+    for rows in x.split(65535):
+        _lib.check(_lib.load().nvh_softcap(rows.data_ptr(), float(cap), rows.shape[0], rows.shape[1], rows.stride(0), code, _stream()), "nvh_softcap")
+    return x

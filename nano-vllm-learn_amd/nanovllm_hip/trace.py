@@ -44,13 +44,16 @@ class TraceRunner:
         return out
 
 
-def main(argv=None):
+def main(argv=None, prepare=None):
+    """prepare(model folder): called before anything is loaded (compiles what is missing)."""
     ap = argparse.ArgumentParser(prog="trace_run", description=__doc__, formatter_class=argparse.RawDescriptionHelpFormatter)
     ap.add_argument("--model", required=True)
     ap.add_argument("--dtype", required=True, choices=["bfloat16", "float32"])
     ap.add_argument("--out", required=True)
     ap.add_argument("--max-tokens", required=True, type=int)
     a = ap.parse_args(argv)
+    if prepare is not None:
+        prepare(a.model)
     runner = TraceRunner(a.model, getattr(torch, a.dtype), a.max_tokens)
     for line in sys.stdin:
         if not line.strip():
