@@ -38,7 +38,7 @@ int nvh_attn_prep(const nvh_attn_prep_desc* d, int dtype, void* stream) {
     REQUIRE(d, NVH_E_NULL, "attn_prep: null descriptor");
     if (d->rows == 0) return 0;
     DTYPE("attn_prep");
-    REQUIRE(d->qkv && d->positions && d->cos_sin && d->cache && d->slots && (!d->q_w == !d->k_w), NVH_E_NULL, "attn_prep: null pointer");
+    REQUIRE(d->qkv && d->positions && (d->cos_sin || d->rot == 0) && d->cache && d->slots && (!d->q_w == !d->k_w), NVH_E_NULL, "attn_prep: null pointer");
     const int64_t cols = (int64_t)d->heads * d->dk + (int64_t)d->kv_heads * (d->dk + d->dv);
     REQUIRE(d->rows > 0 && d->heads > 0 && d->kv_heads > 0 && d->dk > 0 && d->dk % 8 == 0 && d->dv > 0 && d->dv % 8 == 0 && cols <= kMaxRowCols && d->rot >= 0 && d->rot % 2 == 0 &&
             d->rot <= d->dk && d->max_position > 0 && d->block_size > 0 && (!d->q_w || (d->q_n > 0 && d->k_n > 0)), NVH_E_SHAPE,

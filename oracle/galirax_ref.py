@@ -109,29 +109,36 @@ def lightning_mixer(w, p, m, h, eps):
 
 
 def route(z, correction, r):
-    """One token: logits [experts] -> (chosen experts, their weights)."""
+    """One token: logits [experts] -> (chosen experts, their weights, how far the nearest other choice was)."""
     s = torch.sigmoid(z)
-    choice = s + correction
-    groups, keep = r["groups"]["count"], r["groups"]["keep"]
+    choice = (s + correction).tolist()
+    groups, keep, top = r["groups"]["count"], r["groups"]["keep"], r["top"]
     size = len(z) // groups
-    rank = sorted(range(groups), key=lambda g: -sum(sorted(choice[g * size:(g + 1) * size].tolist())[-2:]))[:keep]
-    open_to = [e for e in range(len(z)) if e // size in rank]
-    chosen = sorted(open_to, key=lambda e: -choice[e].item())[:r["top"]]
+    score = [sum(sorted(choice[g * size:(g + 1) * size])[-2:]) for g in range(groups)]
+    rank = sorted(range(groups), key=lambda g: -score[g])
+    open_to = sorted((e for e in range(len(z)) if e // size in rank[:keep]), key=lambda e: -choice[e])
+    chosen = open_to[:top]
+    gaps = [choice[chosen[-1]] - choice[open_to[top]]] if top < len(open_to) else []
+    if keep < groups:
+        gaps.append(score[rank[keep - 1]] - score[rank[keep]])
     weights = s[chosen]
-    return chosen, weights / (weights.sum() + 1e-20) * r["scale"]
+    return chosen, weights / (weights.sum() + 1e-20) * r["scale"], min(gaps, default=math.inf)
 
 
 def expert(w, p, h):
     return (silu(h @ w[p + "gate"].T) * (h @ w[p + "up"].T)) @ w[p + "down"].T
 
 
-def moe(w, p, m, h):
+def moe(w, p, m, h, margins=None):
     out = torch.zeros_like(h)
     z = h @ w[p + "router"].T
     picks = {}
     for t in range(h.shape[0]):
-        for e, g in zip(*route(z[t], w[p + "correction"], m["router"])):
+        chosen, weights, gap = route(z[t], w[p + "correction"], m["router"])
+        for e, g in zip(chosen, weights):
             picks.setdefault(e, []).append((t, g))
+        if margins is not None:
+            margins[t] = min(margins[t], gap)
     for e, rows in picks.items():
         t = [r[0] for r in rows]
         out[t] += torch.stack([r[1] for r in rows])[:, None] * expert(w, f"{p}e{e}.", h[t])
@@ -150,8 +157,9 @@ def softcap(z, cap):
     return cap * torch.tanh(z / cap)
 
 
-def forward(cfg, weights, tokens, collect=None):
-    """Logits [T, vocab] of one whole sequence; `collect`, a list, receives the residual stream after every layer run."""
+def forward(cfg, weights, tokens, collect=None, margins=None):
+    """Logits [T, vocab] of one whole sequence; `collect`, a list, receives the residual stream after every layer run, `margins`, a list of a number per
+    token, the closest call of its expert choices."""
     w = {k: v.to(F64) for k, v in weights.items()}
     eps = cfg["norm"]["eps"]
     x = w["embed"][torch.as_tensor(tokens)]
@@ -161,7 +169,7 @@ def forward(cfg, weights, tokens, collect=None):
         m = layer["mixer"]
         y = lightning_mixer(w, p + "mix.", m, h, eps) if layer["type"] == "lightning" else attention_mixer(w, p + "mix.", layer["type"], m, h, eps)
         if layer["mlp"] is not None:
-            y = y + moe(w, p + "mlp.", layer["mlp"], h)
+            y = y + moe(w, p + "mlp.", layer["mlp"], h, margins)
         x = x + y
         if collect is not None:
             collect.append(x.clone())
