@@ -311,13 +311,14 @@ def main():
     ap.add_argument("--no-full-window", action="store_true", help="skip the extra replay of bench_my's whole decode window (out = in tokens)")
     ap.add_argument("--no-sweep", action="store_true", help="skip the attention_sweep of the other BASELINE configs")
     ap.add_argument("--prefill-leg", action="store_true", help="time the prefill attention op for models other than the headline one too")
-    ap.add_argument("--beside", choices=["1k", "2k", "4k"], help="instead of the default workload: the Zobasun model beside a Qwen2-shaped one of this size "
+    ap.add_argument("--beside", choices=["1k", "2k", "4k"], help="instead of the default workload: another model beside a Qwen2-shaped one of this size "
                     "(engine throughput and kernels against their rooflines), one JSON line")
+    ap.add_argument("--beside-model", choices=["zobasun", "galirax"], default="zobasun")
     ap.add_argument("--beside-only", choices=["kernels", "engine"])
     args = ap.parse_args()
     if args.beside:
         from nanovllm_hip.bench_models import run
-        print(json.dumps(run(args.beside, args.beside_only)), flush=True)
+        print(json.dumps(run(args.beside, args.beside_only, args.beside_model)), flush=True)
         return
 
     world = int(os.environ.get("WORLD_SIZE", "1"))

@@ -1,44 +1,62 @@
-"""Zobasun beside the closest other model (a Qwen2-shaped stack) at equal size, on random weights: prefill and decode throughput through the engine,
-and each hot kernel against its roofline.  bench.py --beside SIZE prints the result as one JSON line."""
+"""Zobasun or Galirax beside the closest other model (a Qwen2-shaped stack) at equal size, on random weights: prefill and decode throughput through the
+engine, and each hot kernel against its roofline.  bench.py --beside SIZE [--beside-model NAME] prints the result as one JSON line."""
 from __future__ import annotations
 
 import time
 
 import torch
 
+import torch.nn.functional as F
+
 from . import ops
 from .engine.llm_engine import LLMEngine
 from .engine.model_runner import recurrence_chunks
 from .layers.rglru import choose_segment
 from .layers.rotary import rotation_table
+from .models.galirax import GaliraxConfig
 from .models.qwen import ModelConfig
 from .models.zobasun import ZobasunConfig
 
 HBM_GBPS, MFMA_TFLOPS = 8000.0, 2500.0          # MI355X peaks (dense bf16)
 
-# width, feed-forward, layers; attention heads (128 wide); latent ranks and widths; recurrence width, blocks
+# width, feed-forward, layers; attention heads (128 wide); latent ranks and widths; recurrence width, blocks; experts (each ff / top wide)
 SIZES = {
-    "1k": dict(width=1024, ff=3072, layers=12, heads=8, kv_heads=2, q_rank=384, kv_rank=256, dim=64, rot=64, vdim=64, rec=1024, blocks=4),
-    "2k": dict(width=2048, ff=6144, layers=12, heads=16, kv_heads=4, q_rank=768, kv_rank=512, dim=128, rot=64, vdim=128, rec=2560, blocks=10),
-    "4k": dict(width=4096, ff=12288, layers=6, heads=32, kv_heads=8, q_rank=1536, kv_rank=512, dim=128, rot=64, vdim=128, rec=4096, blocks=16),
+    "1k": dict(width=1024, ff=3072, layers=12, heads=8, kv_heads=2, q_rank=384, kv_rank=256, dim=64, rot=64, vdim=64, rec=1024, blocks=4, experts=32, top=4),
+    "2k": dict(width=2048, ff=6144, layers=12, heads=16, kv_heads=4, q_rank=768, kv_rank=512, dim=128, rot=64, vdim=128, rec=2560, blocks=10, experts=32, top=4),
+    "4k": dict(width=4096, ff=12288, layers=6, heads=32, kv_heads=8, q_rank=1536, kv_rank=512, dim=128, rot=64, vdim=128, rec=4096, blocks=16, experts=32, top=4),
 }
 VOCAB = 32000
+WINDOW, KEEP = 512, 4                           # Galirax's windowed layers
 
 
-def configs(size):
-    """(Zobasun configuration: two recurrent layers for every latent-attention one; Qwen2-shaped configuration of the same width, depth and feed-forward)."""
+def qwen_config(size):
+    s = SIZES[size]
+    return ModelConfig(name=f"Qwen2-shaped {size}", num_hidden_layers=s["layers"], hidden_size=s["width"], num_attention_heads=s["heads"],
+                       num_key_value_heads=s["kv_heads"], head_dim=128, intermediate_size=s["ff"], vocab_size=VOCAB, tie_word_embeddings=False, qkv_bias=True,
+                       qk_norm=False)
+
+
+def galirax_config(size):
+    """Windowed attention, lightning attention, full attention in turn; the experts a token uses are together as wide as the Qwen stack's feed-forward."""
+    s = SIZES[size]
+    mlp = {"kind": "moe", "expert": {"ff": s["ff"] // s["top"]}, "router": {"experts": s["experts"], "top": s["top"], "groups": {"count": 8, "keep": 4}, "scale": 2.5}}
+    att = dict(heads=s["heads"], kv_heads=s["kv_heads"], dim=128, vdim=128, scale=128 ** -0.5, rot={"base": 10000.0, "dims": 128})
+    kinds = [("attention_2", {**att, "mask": {"size": WINDOW, "keep_first": KEEP}}),
+             ("lightning", dict(heads=s["heads"], dim=128, vdim=128, decay=[1 - 2.0 ** -(3 + 6 * i / s["heads"]) for i in range(s["heads"])])), ("attention", att)]
+    return GaliraxConfig.from_json({"width": s["width"], "vocab": VOCAB, "norm": {"eps": 1e-6}, "logit_softcap": 15.0,
+                                    "layers": [dict(type=kinds[i % 3][0], mixer=kinds[i % 3][1], mlp=mlp) for i in range(s["layers"])]})
+
+
+def zobasun_config(size):
+    """Two recurrent layers for every latent-attention one."""
     s = SIZES[size]
     mlp = {"kind": "dense", "ff": s["ff"], "limit": 7.0}
     rec = {"type": "rglru", "mixer": {"width": s["rec"], "blocks": s["blocks"], "conv": 4}, "mlp": mlp}
     att = {"type": "latent_attention", "mlp": mlp, "mixer": dict(
         heads=s["heads"], dim=s["dim"], rot_dim=s["rot"], vdim=s["vdim"], q_rank=s["q_rank"], kv_rank=s["kv_rank"], scale=(s["dim"] + s["rot"]) ** -0.5,
         rot={"base": 10000.0, "dims": s["rot"]})}
-    new = ZobasunConfig.from_json({"width": s["width"], "vocab": VOCAB, "norm": {"eps": 1e-6}, "embedding": {"scale": 1.0},
-                                   "layers": [(rec, rec, att)[i % 3] for i in range(s["layers"])]})
-    old = ModelConfig(name=f"Qwen2-shaped {size}", num_hidden_layers=s["layers"], hidden_size=s["width"], num_attention_heads=s["heads"],
-                      num_key_value_heads=s["kv_heads"], head_dim=128, intermediate_size=s["ff"], vocab_size=VOCAB, tie_word_embeddings=False, qkv_bias=True,
-                      qk_norm=False)
-    return new, old
+    return ZobasunConfig.from_json({"width": s["width"], "vocab": VOCAB, "norm": {"eps": 1e-6}, "embedding": {"scale": 1.0},
+                                    "layers": [(rec, rec, att)[i % 3] for i in range(s["layers"])]})
 
 
 def _engine_throughput(cfg, batch, prompt, decode_steps, repeats=3):
@@ -107,10 +125,144 @@ def _randn(*shape, dtype=torch.bfloat16):
     return torch.randn(*shape, device="cuda", dtype=dtype)
 
 
+def qwen_attention(size, batch, ctx, seqs, prompt):
+    """The Qwen stack's prompt and decode attention."""
+    s, out, rows = SIZES[size], {}, seqs * prompt
+    h, hk = s["heads"], s["kv_heads"]
+    cu = torch.arange(0, rows + 1, prompt, dtype=torch.int32, device="cuda")
+    pairs = seqs * prompt * (prompt + 1) / 2
+    qkv = [_randn(rows, (h + 2 * hk) * 128) for _ in range(2)]
+
+    def old_prefill(x, pv_fp16):
+        p = x.view(rows, -1, 128)
+        ops.flash_attn_varlen_func(p[:, :h], p[:, h:h + hk], p[:, h + hk:], prompt, cu, prompt, cu, pv_fp16=pv_fp16)
+    for name, form in (("qwen_prefill_attention", None), ("qwen_prefill_attention_exact", False)):
+        us = _time([lambda x=x: old_prefill(x, form) for x in qkv] * 2)
+        out[name] = _line(us, 4 * rows * (h + hk) * 128, 4 * 128 * h * pairs)
+    opages = -(-ctx // 256)
+    n = max(2, int(3e8 // (4 * batch * opages * 256 * hk * 128)) + 1)
+    caches = [_randn(2, batch * opages, 256, hk, 128) for _ in range(n)]
+    obt = torch.randperm(batch * opages).view(batch, opages).int().cuda()
+    cl = torch.full((batch,), ctx, dtype=torch.int32, device="cuda")
+    oq = _randn(batch, h, 128)
+    us = _time([lambda c=c: ops.flash_attn_with_kvcache(oq, c[0], c[1], cl, obt) for c in caches] * 3)
+    out["qwen_decode_attention"] = _line(us, batch * (4 * ctx * hk * 128 + 4 * h * 128))
+    return out
+
+
 @torch.inference_mode()
-def kernels(size, batch=32, ctx=1536, seqs=16, prompt=1024):
+def galirax_kernels(size, batch=32, ctx=1536, seqs=16, prompt=1024):
+    """Each hot kernel of Galirax alone, and the Qwen stack's like ones; operands cycle through more than the memory-side cache holds where that matters."""
+    s, out, rows = SIZES[size], qwen_attention(size, batch, ctx, seqs, prompt), seqs * prompt
+    h, g, d, width, experts, top = s["heads"], s["kv_heads"], 128, s["width"], s["experts"], s["top"]
+    ff = s["ff"] // top
+    cu = torch.arange(0, rows + 1, prompt, dtype=torch.int32, device="cuda")
+    pos = torch.arange(prompt, device="cuda").repeat(seqs)
+    table = rotation_table(d, 10000.0, 4096, "cuda")
+    sink = torch.ones(h, device="cuda")
+    # ---- attention over prompts, row ops in front
+    cols = (h + 2 * g) * d
+    qkv = [_randn(rows, cols) for _ in range(3)]
+    cache = torch.zeros(rows // 64, 64, 2 * g * d, dtype=torch.bfloat16, device="cuda")
+    slot = torch.arange(rows, dtype=torch.int32, device="cuda")
+    qw, kw = torch.ones(h * d, device="cuda"), torch.ones(g * d, device="cuda")
+    us = _time([lambda x=x: ops.attn_prep(x, h, g, d, d, pos, table, cache, slot, qw, kw, h * d, g * d, 1e-6) for x in qkv])
+    out["attn_prep"] = _line(us, rows * 4 * cols)
+    bt = torch.arange(rows // 64, dtype=torch.int32, device="cuda").view(seqs, -1)
+    o = torch.empty(rows, h * d, device="cuda", dtype=torch.bfloat16)
+    nbytes = 4 * rows * (h + g) * d
+    for name, mask in (("paged_prompt", {}), ("paged_prompt_window", dict(window=WINDOW, keep_first=KEEP))):
+        us = _time([lambda x=x: ops.paged_attend_prompt(x, cache, bt, cu, cu, prompt, h, g, d, d, d ** -0.5, sink=sink, out=o, **mask) for x in qkv] * 2)
+        seen = sum(min(t + 1, WINDOW) + min(KEEP, max(0, t + 1 - WINDOW)) for t in range(prompt)) if mask else prompt * (prompt + 1) / 2
+        out[name] = _line(us, nbytes, 4 * d * h * seqs * seen)
+    del qkv, o, cache
+    # ---- decode attention
+    pages = -(-ctx // 64)
+    n = max(2, int(3e8 // (batch * pages * 64 * 4 * g * d)) + 1)
+    caches = [_randn(batch * pages, 64, 2 * g * d) for _ in range(n)]
+    bt = torch.randperm(batch * pages).view(batch, pages).int().cuda()
+    dpos = torch.full((batch,), ctx - 1, device="cuda")
+    q, o = _randn(batch, h * d), torch.empty(batch, h * d, device="cuda", dtype=torch.bfloat16)
+    for name, mask, seen in (("paged_rows", {}, ctx), ("paged_rows_window", dict(window=WINDOW, keep_first=KEEP), WINDOW + KEEP)):
+        us = _time([lambda c=c: ops.paged_attend_rows(q, c, bt, dpos, h, g, d, d, d ** -0.5, ctx, sink=sink, out=o, **mask) for c in caches] * 3)
+        out[name] = _line(us, batch * (4 * seen * g * d + 4 * h * d))
+    del caches
+    # ---- lightning attention
+    x = [_randn(rows, 4 * h * d) for _ in range(2)]
+    decay = torch.linspace(0.8, 0.999, h, device="cuda")
+    slots = torch.arange(max(seqs, batch), dtype=torch.int32, device="cuda")
+    state = torch.zeros(max(seqs, batch), h, d, d, device="cuda")
+    o = torch.empty(rows, h * d, device="cuda", dtype=torch.bfloat16)
+    seg = choose_segment([prompt] * seqs, h * 2)
+    chunks = torch.tensor([c for i in range(seqs) for c in recurrence_chunks(i * prompt, prompt, i, seg)], dtype=torch.int32, device="cuda")
+    us = _time([lambda a=a: ops.lightning_chunks(a, decay, pos, slots, chunks, seg < prompt, state, out=o) for a in x] * 2)
+    out["lightning_chunks"] = _line(us, rows * 8 * h * d, 4 * rows * h * d * d)
+    us = _time([lambda a=a: ops.norm_gate(o, a[:, 3 * h * d:], qw, 1e-6, h * d) for a in x])
+    out["norm_gate"] = _line(us, rows * 6 * h * d)
+    x1 = _randn(batch, 4 * h * d)
+    states = [torch.zeros(batch, h, d, d, device="cuda") for _ in range(max(2, int(3e8 // (4 * batch * h * d * d)) + 1))]
+    us = _time([lambda t=t: ops.lightning_step(x1, decay, dpos, slots, t) for t in states] * 3)
+    out["lightning_step"] = _line(us, 8 * batch * h * d * d)
+    del x, o, states, state
+    # ---- experts, large batch
+    xs, router, corr = [_randn(rows, width) for _ in range(2)], _randn(experts, width) * width ** -0.5, torch.zeros(experts, device="cuda")
+    us = _time([lambda a=a: ops.moe_route(a, router, corr, top, 8, 4, 2.5) for a in xs] * 2)
+    out["moe_route"] = _line(us, 2 * rows * width, 2 * rows * width * experts)
+    ids, ew = ops.moe_route(xs[0], router, corr, top, 8, 4, 2.5)
+    us = _time([lambda: ops.moe_dispatch(ids, experts, torch.bfloat16)] * 4)
+    out["moe_dispatch"] = _line(us, 8 * rows * top)
+    dispatch = ops.moe_dispatch(ids, experts, torch.bfloat16)
+    wgu = [_randn(experts, 2 * ff, width) * 0.02 for _ in range(max(1, int(3e8 // (4 * experts * ff * width)) + 1))]
+    wdn = [_randn(experts, width, ff) * 0.02 for _ in range(max(1, int(3e8 // (2 * experts * ff * width)) + 1))]
+    us = _time([lambda w=w: ops.moe_gemm(xs[0], w, ids, True, dispatch) for w in wgu[:2]])
+    out["moe_gate_up"] = _line(us, 0, 4 * rows * top * ff * width)
+    act = ops.moe_gemm(xs[0], wgu[0], ids, True, dispatch)
+    us = _time([lambda w=w: ops.moe_gemm(act, w, ids, False, dispatch) for w in wdn[:2]])
+    out["moe_down"] = _line(us, 0, 2 * rows * top * ff * width)
+    e = ops.moe_gemm(act, wdn[0], ids, False, dispatch)
+    del act
+    qgu, qdn = _randn(2 * s["ff"], width), _randn(width, s["ff"])
+    us = _time([lambda a=a: ops.silu_mul(F.linear(a, qgu)) for a in xs])
+    out["qwen_gate_up (product + silu_mul)"] = _line(us, 0, 4 * rows * s["ff"] * width)
+    t = _randn(rows, s["ff"])
+    out["qwen_down"] = _line(_time([lambda: F.linear(t, qdn)] * 2), 0, 2 * rows * s["ff"] * width)
+    del t
+    # ---- residual and norm
+    st, w32 = _randn(rows, width, dtype=torch.float32), torch.ones(width, device="cuda")
+    us = _time([lambda a=a: ops.residual_norm(st, torch.bfloat16, y=a, experts=(e, ew), weight=w32, bias=w32, eps=1e-6) for a in xs])
+    out["residual_norm"] = _line(us, rows * width * (8 + 2 + 2 * top + 2))
+    rs, wb = _randn(rows, width), _randn(width)
+    out["qwen_add_rmsnorm"] = _line(_time([lambda a=a: ops.add_rmsnorm(a, wb, 1e-6, rs) for a in xs]), rows * width * 8)
+    del xs, st, rs, e
+    # ---- experts, decode batch
+    x1 = _randn(batch, width)
+    ids, _ = ops.moe_route(x1, router, corr, top, 8, 4, 2.5)
+    used = ids.unique().numel()
+    us = _time([lambda w=w: ops.moe_gemm(x1, w, ids, True) for w in wgu] * 3)
+    out["moe_gate_up_decode"] = _line(us, used * 4 * ff * width)
+    a1 = ops.moe_gemm(x1, wgu[0], ids, True)
+    us = _time([lambda w=w: ops.moe_gemm(a1, w, ids, False) for w in wdn] * 3)
+    out["moe_down_decode"] = _line(us, used * 2 * ff * width)
+    del wgu, wdn
+    ws = torch.zeros(max(ops.linear_workspace_bytes(batch, 2 * s["ff"], width, "silu_mul"), ops.linear_workspace_bytes(batch, width, s["ff"]), 16), dtype=torch.uint8, device="cuda")
+    xp, mid = ops.pack_rows(x1), torch.zeros((batch + 15) // 16 * 16 * s["ff"], dtype=torch.bfloat16, device="cuda")
+    qgus = [_randn(2 * s["ff"], width) for _ in range(int(3e8 // (4 * s["ff"] * width)) + 2)]
+    us = _time([lambda w=w: ops.fused_linear(xp, w, x_packed_rows=batch, epilogue="silu_mul", out_packed=mid, want_out=False, workspace=ws) for w in qgus] * 2)
+    out["qwen_gate_up_decode"] = _line(us, 4 * s["ff"] * width)
+    del qgus
+    qdns = [_randn(width, s["ff"]) for _ in range(int(3e8 // (2 * s["ff"] * width)) + 2)]
+    us = _time([lambda w=w: ops.fused_linear(mid, w, x_packed_rows=batch, workspace=ws) for w in qdns] * 2)
+    out["qwen_down_decode"] = _line(us, 2 * s["ff"] * width)
+    us = _time([lambda: ops.moe_route(x1, router, corr, top, 8, 4, 2.5)] * 20)
+    out["moe_route_decode"] = _line(us, 2 * (batch + experts) * width)
+    torch.cuda.empty_cache()
+    return out
+
+
+@torch.inference_mode()
+def zobasun_kernels(size, batch=32, ctx=1536, seqs=16, prompt=1024):
     """Each hot kernel of the two models alone; operands cycle through more than the memory-side cache holds where that matters."""
-    s, out = SIZES[size], {}
+    s, out = SIZES[size], qwen_attention(size, batch, ctx, seqs, prompt)
     rows, h, dim, rot, vdim, kv = seqs * prompt, s["heads"], s["dim"], s["rot"], s["vdim"], s["kv_rank"]
     width, ff, rec, blocks = s["width"], s["ff"], s["rec"], s["blocks"]
     dk, cols, scale = dim + rot, kv + 64, (dim + rot) ** -0.5
@@ -123,15 +275,7 @@ def kernels(size, batch=32, ctx=1536, seqs=16, prompt=1024):
     o = torch.empty(rows, h * vdim, device="cuda", dtype=torch.bfloat16)
     us = _time([lambda: ops.latent_prefill(q, k, kr, v, cu, cu, prompt, pos, table, scale, out=o)] * 4)
     out["latent_prefill"] = _line(us, 2 * rows * (h * (dk + dim + 2 * vdim) + 64), 2 * h * (dk + vdim) * pairs)
-    qkv = [_randn(rows, (h + 2 * s["kv_heads"]) * 128) for _ in range(2)]
-
-    def old_prefill(x, pv_fp16):
-        p = x.view(rows, -1, 128)
-        ops.flash_attn_varlen_func(p[:, :h], p[:, h:h + s["kv_heads"]], p[:, h + s["kv_heads"]:], prompt, cu, prompt, cu, pv_fp16=pv_fp16)
-    for name, form in (("qwen_prefill_attention", None), ("qwen_prefill_attention_exact", False)):
-        us = _time([lambda x=x: old_prefill(x, form) for x in qkv] * 2)
-        out[name] = _line(us, 4 * rows * (h + s["kv_heads"]) * 128, 4 * 128 * h * pairs)
-    del q, k, v, qkv
+    del q, k, v
     # ---- decode attention
     pages = -(-ctx // 64)
     n = max(2, int(3e8 // (batch * pages * 64 * cols * 2)) + 1)
@@ -142,16 +286,6 @@ def kernels(size, batch=32, ctx=1536, seqs=16, prompt=1024):
     o = torch.empty(batch, h * vdim, device="cuda", dtype=torch.bfloat16)
     us = _time([lambda c=c: ops.latent_attention(q, c, bt, dpos, table, uk, uv, scale, rot, ctx, out=o) for c in caches] * 3)
     out["latent_decode (absorb + attend + value)"] = _line(us, batch * ctx * cols * 2 + 2 * (uk.numel() + uv.numel() + q.numel() + o.numel()))
-    del caches
-    hk = s["kv_heads"]
-    opages = -(-ctx // 256)
-    n = max(2, int(3e8 // (4 * batch * opages * 256 * hk * 128)) + 1)
-    caches = [_randn(2, batch * opages, 256, hk, 128) for _ in range(n)]
-    obt = torch.randperm(batch * opages).view(batch, opages).int().cuda()
-    cl = torch.full((batch,), ctx, dtype=torch.int32, device="cuda")
-    oq = _randn(batch, h, 128)
-    us = _time([lambda c=c: ops.flash_attn_with_kvcache(oq, c[0], c[1], cl, obt) for c in caches] * 3)
-    out["qwen_decode_attention"] = _line(us, batch * (4 * ctx * hk * 128 + 4 * h * 128))
     del caches
     # ---- recurrence
     p = dict(conv_w=_randn(4, rec, dtype=torch.float32), conv_b=_randn(rec, dtype=torch.float32), ra=_randn(blocks, rec // blocks, rec // blocks) * 0.05,
@@ -192,16 +326,20 @@ def kernels(size, batch=32, ctx=1536, seqs=16, prompt=1024):
     return out
 
 
-def run(size, only=None):
+MODELS = {"zobasun": (zobasun_config, zobasun_kernels), "galirax": (galirax_config, galirax_kernels)}
+
+
+def run(size, only=None, model="zobasun"):
     torch.manual_seed(0)
-    new, old = configs(size)
-    res = {"metric": "Zobasun beside a Qwen2-shaped stack of equal width, depth and feed-forward (random weights)", "size": size, "shape": SIZES[size], "dtype": "bf16"}
+    config, kernels = MODELS[model]
+    new, old = config(size), qwen_config(size)
+    res = {"metric": f"{new.name} beside a Qwen2-shaped stack of equal width, depth and feed-forward (random weights)", "size": size, "shape": SIZES[size], "dtype": "bf16"}
     if only in (None, "kernels"):
         res["kernels"] = kernels(size)
     if only in (None, "engine"):
         for batch, prompt in ((16, 1024), (2, 8192)):
-            for name, cfg in (("zobasun", new), ("qwen", old)):
+            for name, cfg in ((model, new), ("qwen", old)):
                 res[f"{name}_{batch}x{prompt}"] = _engine_throughput(cfg, batch, prompt, 64)
-        for name, cfg in (("zobasun", new), ("qwen", old)):
+        for name, cfg in ((model, new), ("qwen", old)):
             res[f"{name}_32x1024"] = _engine_throughput(cfg, 32, 1024, 256, repeats=1)
     return res

@@ -17,7 +17,8 @@ class MixtureOfExperts(nn.Module):
     def load(self, get):
         """get(name) -> tensor of the checkpoint (names below the feed-forward's prefix)."""
         e, f, c, d = self.experts, self.cols, self.in_cols, self.dtype
-        gate_up, down = torch.zeros(e, 2 * f, c, dtype=d), torch.zeros(e, c, f, dtype=d)
+        device = get("router").device
+        gate_up, down = torch.zeros(e, 2 * f, c, dtype=d, device=device), torch.zeros(e, c, f, dtype=d, device=device)
         assert get("router").shape == (e, self.in_width) and get("e0.gate").shape == (self.ff, self.in_width)
         for i in range(e):
             gate_up[i, :self.ff, :self.in_width], gate_up[i, f:f + self.ff, :self.in_width] = get(f"e{i}.gate"), get(f"e{i}.up")

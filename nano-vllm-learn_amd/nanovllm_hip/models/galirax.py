@@ -136,9 +136,11 @@ class GaliraxForCausalLM(nn.Module):
         return self
 
     def init_random(self, seed=0):
-        """Deterministic random weights: N(0, 0.02) matrices, norm weights around one."""
-        gen = torch.Generator().manual_seed(seed)
-        return self.load_weights(_RandomTensors(self.cfg, lambda shape, std=0.02: (torch.randn(shape, generator=gen) * std).bfloat16()))
+        """Deterministic random weights (per device kind: experts are many, so they are drawn on the GPU where there is one): N(0, 0.02) matrices, norm
+        weights around one."""
+        device = "cuda" if torch.cuda.is_available() else "cpu"
+        gen = torch.Generator(device).manual_seed(seed)
+        return self.load_weights(_RandomTensors(self.cfg, lambda shape, std=0.02: (torch.randn(shape, generator=gen, device=device) * std).bfloat16()))
 
     # ------------------------------------------------------------------ forward
     def forward(self, input_ids, positions, step):
