@@ -670,8 +670,8 @@ int nvh_moe_dispatch_blocks(int pairs);
 int nvh_moe_dispatch(int32_t* slot_pair, int32_t* tiles, int32_t* counts, const int32_t* ids, int pairs, int experts, int tile_rows, int max_tiles, void* stream);
 /* Expert products.  glu: act[p] = silu(x[p / top] . gate_e) * (x . up_e), w = [experts, 2 * n, k] (gate rows, then up rows); otherwise
  * out[p] = x[p] . w_e, w = [experts, n, k].
- * tiles == NULL: small batches (bf16, at most 64 rows), the pairs of an expert found from ids; otherwise tiles from nvh_moe_dispatch (nvh_moe_tile_rows(dtype)
- * rows each).  n and k multiples of 64. */
+ * tiles == NULL: small batches (bf16, at most 64 rows), the pairs of an expert found from ids; otherwise tiles of tile_rows from
+ * nvh_moe_dispatch (bf16: 128 or 256, f32: 64; nvh_moe_tile_rows picks).  n and k multiples of 64. */
 typedef struct nvh_moe_gemm_desc {
     void* out;                   /* [pairs, n] */
     const void* x;               /* glu: [rows, k], row stride x_stride; otherwise [pairs, k] */
@@ -681,9 +681,9 @@ typedef struct nvh_moe_gemm_desc {
     const int32_t* ids;          /* [pairs] (small form) */
     const int32_t* slot_pair;    /* [pairs] */
     const int32_t* tiles;
-    int32_t max_tiles;
+    int32_t max_tiles, tile_rows;
 } nvh_moe_gemm_desc;
-int nvh_moe_tile_rows(int dtype);
+int nvh_moe_tile_rows(int pairs, int experts, int dtype);
 int nvh_moe_gemm(const nvh_moe_gemm_desc* d, int dtype, void* stream);
 
 /* x (fp32 stream) += y + sum_k ew[row, k] * e[row * top + k]  (each part nullable), then, with w given, the layer norm of the new row:

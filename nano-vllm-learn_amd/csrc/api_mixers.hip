@@ -135,7 +135,7 @@ int nvh_moe_dispatch(int32_t* slot_pair, int32_t* tiles, int32_t* counts, const 
     return launch_moe_dispatch(slot_pair, tiles, counts, ids, pairs, experts, tile_rows, max_tiles, (hipStream_t)stream);
 }
 
-int nvh_moe_tile_rows(int dtype) { return moe_tile_rows(dtype == NVH_F32); }
+int nvh_moe_tile_rows(int pairs, int experts, int dtype) { return pairs > 0 && experts > 0 ? moe_tile_rows(pairs, experts, dtype == NVH_F32) : 0; }
 
 int nvh_moe_gemm(const nvh_moe_gemm_desc* d, int dtype, void* stream) {
     REQUIRE(d, NVH_E_NULL, "moe_gemm: null descriptor");
@@ -144,6 +144,7 @@ int nvh_moe_gemm(const nvh_moe_gemm_desc* d, int dtype, void* stream) {
     REQUIRE(d->out && d->x && d->w && (d->tiles ? d->slot_pair != nullptr : d->ids != nullptr), NVH_E_NULL, "moe_gemm: null pointer");
     REQUIRE(d->pairs > 0 && d->top > 0 && d->pairs % d->top == 0 && d->experts > 0 && d->experts <= kMoeMaxExperts && d->n > 0 && d->n % 64 == 0 && d->k > 0 && d->k % 64 == 0,
             NVH_E_SHAPE, "moe_gemm: %d pairs of top %d, n %d k %d (%%64)", d->pairs, d->top, d->n, d->k);
+    REQUIRE(!d->tiles || d->tile_rows == (dtype == NVH_F32 ? 64 : 128) || (dtype == NVH_BF16 && d->tile_rows == 256), NVH_E_SHAPE, "moe_gemm: tiles of %d rows", d->tile_rows);
     REQUIRE(d->tiles ? d->max_tiles > 0 && d->max_tiles <= 65535 : dtype == NVH_BF16 && d->pairs / d->top <= 64, NVH_E_SHAPE,
             "moe_gemm: %d tiles, or the small form with more than 64 rows", d->max_tiles);
     REQUIRE(!d->glu || (d->x_stride % 8 == 0 && d->x_stride >= d->k), NVH_E_STRIDE, "moe_gemm: row stride");

@@ -12,9 +12,9 @@ namespace nvh {
 namespace {
 
 template <int DK, int DV, int QT>
-__global__ __launch_bounds__(256) void latent_prefill_kernel(const LatentPrefillArgs a) {
-    using Tile = AttendTile<DK, DV, QT>;
-    constexpr int BM = Tile::BM, WR = Tile::WR, BN = Tile::BN, KP = Tile::KP, VP = Tile::VP, NK = Tile::NK, NV = Tile::NV, STEPS = Tile::STEPS;
+__global__ __launch_bounds__(256, DK + DV <= 320 ? 2 : 1) void latent_prefill_kernel(const LatentPrefillArgs a) {
+    using Images = TileImages<DK, DV>;
+    constexpr int BM = 64 * QT, WR = 16 * QT, BN = Images::BN, KP = Images::KP, VP = Images::VP, NK = Images::NK, NV = Images::NV;
     extern __shared__ __attribute__((aligned(16))) unsigned char lds[];
     int qt, head, b;
     attend_unit(a.heads, qt, head, b);
@@ -23,8 +23,6 @@ __global__ __launch_bounds__(256) void latent_prefill_kernel(const LatentPrefill
     if (q0 >= sq || sk <= 0) return;
     const int shift = sk - sq;                       // query r sees keys <= r + shift
     const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lq = lane & 15, lg = lane >> 4;
-    Tile tile;
-    tile.init(lds, lq, lg);
     int kv_end = q0 + BM + shift;
     if (kv_end > sk) kv_end = sk;
     const int n_tiles = (kv_end + BN - 1) / BN;
@@ -49,8 +47,8 @@ __global__ __launch_bounds__(256) void latent_prefill_kernel(const LatentPrefill
         vp_[j] = a.v + (int64_t)k_beg * a.v_stride + head * DV + piece * 8;
     }
     auto stage = [&](int it, int buf) {
-        unsigned char* kimg = Tile::k_image(lds, buf);
-        unsigned char* vimg = Tile::v_image(lds, buf);
+        unsigned char* kimg = Images::k(lds, buf);
+        unsigned char* vimg = Images::v(lds, buf);
         const int kv0 = it * BN;
 #pragma unroll
         for (int j = 0; j < NK; ++j) {
@@ -63,65 +61,44 @@ __global__ __launch_bounds__(256) void latent_prefill_kernel(const LatentPrefill
             dma16(vp_[j] + row * a.v_stride, vimg + (wave * NV + j) * 1024);
         }
     };
-    stage(0, 0);
-
-    // ---- query fragments, the rotated part turned here
+    // ---- queries, the rotated part turned while the fragments are loaded
     int my_q[QT];
     bool q_ok[QT];
+    const uint16_t* qp[QT];
+    const float* cs[QT];
 #pragma unroll
     for (int qs = 0; qs < QT; ++qs) {
         my_q[qs] = q0 + wave * WR + 16 * qs + lq;
         q_ok[qs] = my_q[qs] < sq;
         const int64_t qrow = q_beg + (q_ok[qs] ? my_q[qs] : sq - 1);
-        const uint16_t* qp = a.q + qrow * a.q_stride + (int64_t)head * DK + lg * 8;
+        qp[qs] = a.q + qrow * a.q_stride + (int64_t)head * DK + lg * 8;
         int64_t pos = a.positions[qrow];
         if (pos >= a.max_position) pos = a.max_position - 1;
-        const float* cs = a.cos_sin + pos * a.rot;
-#pragma unroll
-        for (int st = 0; st < STEPS; ++st) {
-            u32x4 raw = *reinterpret_cast<const u32x4*>(qp + st * 32);
-            const int i0 = (32 * st + 8 * lg - a.dim_cols) / 2;               // first pair of this piece (dim_cols is a multiple of 32)
-            if (32 * st >= a.dim_cols) {
-#pragma unroll
-                for (int k = 0; k < 4; ++k)
-                    if (i0 + k < a.rot / 2) {
-                        const float u = bf16_lo(raw[k]), v = bf16_hi(raw[k]), co = cs[i0 + k], si = cs[a.rot / 2 + i0 + k];
-                        raw[k] = pack_bf16x2(u * co - v * si, v * co + u * si);
-                    }
-            }
-            tile.qf[qs][st] = *reinterpret_cast<const bf16x8*>(&raw);
-        }
+        cs[qs] = a.cos_sin + pos * a.rot;
     }
-    auto tile_body = [&](auto bufc, const int it) {
-        constexpr int buf = decltype(bufc)::value;
-        if (it + 1 < n_tiles) {
-            stage(it + 1, buf ^ 1);
-            asm volatile("s_waitcnt vmcnt(%0)" ::"n"(NK + NV) : "memory");     // tile `it` has landed, tile it + 1 is in flight
-        } else {
-            asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
-        }
-        __builtin_amdgcn_s_barrier();
-        asm volatile("" ::: "memory");
-        const int kv0 = it * BN;
-        if (kv0 <= wave_last_key) {
-            int limit[QT];
+    auto query = [&](int qs, int st) {
+        u32x4 raw = *reinterpret_cast<const u32x4*>(qp[qs] + st * 32);
+        const int i0 = (32 * st + 8 * lg - a.dim_cols) / 2;                   // first pair of this piece (dim_cols is a multiple of 32)
+        if (32 * st >= a.dim_cols) {
 #pragma unroll
-            for (int qs = 0; qs < QT; ++qs) limit[qs] = (my_q[qs] + shift < sk - 1 ? my_q[qs] + shift : sk - 1) - kv0 - 4 * lg;
-            tile.template attend<buf>(lds, a.scale_log2, kv0 + BN - 1 > wave_first_key || kv0 + BN > sk, lq, lg, [&](int qs, int off) { return off <= limit[qs]; });
+            for (int k = 0; k < 4; ++k)
+                if (i0 + k < a.rot / 2) {
+                    const float u = bf16_lo(raw[k]), v = bf16_hi(raw[k]), co = cs[qs][i0 + k], si = cs[qs][a.rot / 2 + i0 + k];
+                    raw[k] = pack_bf16x2(u * co - v * si, v * co + u * si);
+                }
         }
-        lds_only_barrier();                                                    // everyone's reads of this buffer are done
+        return *reinterpret_cast<const bf16x8*>(&raw);
     };
-    for (int it = 0; it < n_tiles; it += 2) {
-        tile_body(std::integral_constant<int, 0>{}, it);
-        if (it + 1 < n_tiles) tile_body(std::integral_constant<int, 1>{}, it + 1);
-    }
-#pragma unroll
-    for (int qs = 0; qs < QT; ++qs) tile.store(qs, a.out + (int64_t)(q_beg + my_q[qs]) * a.out_stride + head * DV, lg, q_ok[qs]);
+    attend_walk<DK, DV, QT>(
+        lds, n_tiles, a.scale_log2, -INFINITY, lane, stage, query, [&](int it) { return it * BN; }, [&](int kv0) { return kv0 <= wave_last_key; },
+        [&](int kv0) { return kv0 + BN - 1 > wave_first_key || kv0 + BN > sk; },
+        [&](int kv0, int qs, int off) { return off <= (my_q[qs] + shift < sk - 1 ? my_q[qs] + shift : sk - 1) - kv0 - 4 * lg; },
+        [&](int qs) { return q_ok[qs] ? a.out + (int64_t)(q_beg + my_q[qs]) * a.out_stride + head * DV : nullptr; });
 }
 
 template <int DK, int DV, int QT>
 int launch_one(const LatentPrefillArgs& a, hipStream_t stream) {
-    constexpr size_t lds = AttendTile<DK, DV, QT>::LDS;
+    constexpr size_t lds = TileImages<DK, DV>::BYTES;
     if (lds > 64 * 1024) (void)hipFuncSetAttribute(reinterpret_cast<const void*>(latent_prefill_kernel<DK, DV, QT>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
     latent_prefill_kernel<DK, DV, QT><<<dim3(a.heads, a.batch, (a.max_q + 64 * QT - 1) / (64 * QT)), 256, lds, stream>>>(a);
     return check_launch("latent_prefill");

@@ -34,7 +34,7 @@ int launch_moe_route(const MoeRouteArgs& a, int f32, hipStream_t stream);
 int moe_dispatch_blocks(int pairs);
 int launch_moe_dispatch(int32_t* slot_pair, int32_t* tiles, int32_t* counts, const int32_t* ids, int pairs, int experts, int tile_rows, int max_tiles,
                         hipStream_t stream);
-int moe_tile_rows(int f32);
+int moe_tile_rows(int pairs, int experts, int f32);
 int launch_moe_gemm(const MoeGemmArgs& a, int f32, hipStream_t stream);
 
 int launch_residual_norm(const ResidualNormArgs& a, int f32, hipStream_t stream);

@@ -1,8 +1,8 @@
 // Mixture of experts with a sigmoid router, choice corrections and expert groups.
 //   route     32-bit logits of a row tile against every expert (MFMA for bf16), sigmoid, group and expert choice, weights: one launch
 //   dispatch  pairs (row, chosen expert) sorted by expert and cut into tiles of one expert each: two launches, no host round trip
-//   gemm      expert products: gate | up with the SiLU product in the epilogue, and down.  Large batches: 128 x 128 MFMA tiles over the sorted pairs, the
-//             rows gathered by the DMA that fills LDS.  At most 64 rows: every wave streams 16 weight rows once for all the rows that chose the expert.
+//   gemm      expert products: gate | up with the SiLU product in the epilogue, and down.  Large batches: 128 x 128 or 256 x 256 MFMA tiles over the
+//             sorted pairs, the rows gathered by the DMA that fills LDS.  At most 64 rows: every wave streams 16 weight rows once for all the rows that chose the expert.
 // Outputs stay per pair; the weighted sum over a row's experts belongs to the residual add (hybrid_ops.hip).
 #include "attend_tile.h"
 #include "mixers.h"
@@ -18,95 +18,124 @@ __device__ __forceinline__ void wave_lds_sync() {    // LDS written by other lan
 }
 
 // ------------------------------------------------------------------------------------------------ choice (one wave per row)
-// index of the wave's largest value; ties go to the lower index
-__device__ __forceinline__ void wave_argmax(float& v, int& i) {
-    for (int d = 1; d < 64; d <<= 1) {
-        const float ov = __shfl_xor(v, d);
-        const int oi = __shfl_xor(i, d);
-        if (ov > v || (ov == v && oi < i)) {
-            v = ov;
-            i = oi;
-        }
+__device__ __forceinline__ float wave_max64(float v) {
+    v = fmaxf(v, pair_in_row<1>(v));
+    v = fmaxf(v, pair_in_row<2>(v));
+    v = fmaxf(v, pair_in_row<4>(v));
+    v = fmaxf(v, pair_in_row<8>(v));
+    v = max_xor16(v);
+    return max_xor32(v);
+}
+// lane that holds the wave's largest value (the first of equal ones)
+__device__ __forceinline__ int wave_winner(float v) {
+    const uint64_t b = __builtin_amdgcn_ballot_w64(v == wave_max64(v));
+    return b ? __builtin_ctzll(b) : 0;               // (0 only where a router delivers no number)
+}
+__device__ __forceinline__ float lane_value(float v, int lane) { return __int_as_float(__builtin_amdgcn_readlane(__float_as_int(v), lane)); }
+
+__device__ __forceinline__ float group_score(const float* choice, int size) {
+    float b0 = -INFINITY, b1 = -INFINITY;            // the two largest
+    for (int k = 0; k < size; ++k) {
+        const float c = choice[k];
+        b1 = fmaxf(b1, fminf(b0, c));
+        b0 = fmaxf(b0, c);
+    }
+    return size > 1 ? b0 + b1 : b0;
+}
+
+__device__ __forceinline__ void store_choice(const MoeRouteArgs& a, int row, int lane, int id, float score, float total) {
+    if (lane < a.top) {
+        a.ids[(int64_t)row * a.top + lane] = id;
+        a.weights[(int64_t)row * a.top + lane] = score / (total + 1e-20f) * a.scale;
     }
 }
-// z [E]: logits in, scores out; choice [E], gs [groups]: scratch in LDS
+
+// z [E]: logits in, scores out; choice [E], gs [groups]: scratch in LDS.  Up to 64 experts: one per lane, LDS for the group scores only.
 __device__ __forceinline__ void choose_experts(const MoeRouteArgs& a, int row, int lane, float* z, float* choice, float* gs) {
+    const int size = a.experts / a.groups;
+    float total = 0.f, mine = 0.f;
+    int my_id = 0;
+    if (a.experts <= 64) {
+        const bool ok = lane < a.experts;
+        const float s = ok ? 1.f / (1.f + expf(-z[lane])) : 0.f;
+        float c = ok ? s + a.correction[lane] : -INFINITY;
+        if (a.keep < a.groups) {
+            choice[lane] = c;
+            wave_lds_sync();
+            float g = lane < a.groups ? group_score(choice + lane * size, size) : -INFINITY;
+            uint64_t open = 0;
+            for (int k = 0; k < a.keep; ++k) {
+                const int w = wave_winner(g);
+                open |= 1ull << w;
+                if (lane == w) g = -INFINITY;
+            }
+            if (!((open >> (lane / size)) & 1)) c = -INFINITY;
+        }
+        for (int k = 0; k < a.top; ++k) {
+            const int w = wave_winner(c);
+            const float sw = lane_value(s, w);
+            total += sw;
+            if (lane == k) {
+                mine = sw;
+                my_id = w < a.experts ? w : 0;
+            }
+            if (lane == w) c = -INFINITY;
+        }
+        store_choice(a, row, lane, my_id, mine, total);
+        return;
+    }
     for (int e = lane; e < a.experts; e += 64) {
         const float s = 1.f / (1.f + expf(-z[e]));
         z[e] = s;
         choice[e] = s + a.correction[e];
     }
     wave_lds_sync();
-    const int size = a.experts / a.groups;
-    if (a.keep < a.groups) {
-        for (int g = lane; g < a.groups; g += 64) {
-            float b0 = -INFINITY, b1 = -INFINITY;
-            for (int k = 0; k < size; ++k) {
-                const float c = choice[g * size + k];
-                if (c > b0) {
-                    b1 = b0;
-                    b0 = c;
-                } else if (c > b1) {
-                    b1 = c;
-                }
-            }
-            gs[g] = size > 1 ? b0 + b1 : b0;
-        }
-        wave_lds_sync();
-        for (int k = 0; k < a.keep; ++k) {           // an open group is marked by +inf
-            float v = -INFINITY;
-            int i = 0x7fffffff;
-            for (int g = lane; g < a.groups; g += 64) {
-                const float s = gs[g];
-                if (s < INFINITY && (s > v || i == 0x7fffffff)) {
-                    v = s;
-                    i = g;
-                }
-            }
-            wave_argmax(v, i);
-            if (lane == 0 && i < a.groups) gs[i] = INFINITY;
-            wave_lds_sync();
-        }
-        for (int e = lane; e < a.experts; e += 64)
-            if (!(gs[e / size] == INFINITY)) choice[e] = -INFINITY;
-        wave_lds_sync();
-    }
-    float total = 0.f, mine = 0.f;
-    int my_id = 0;
-    for (int k = 0; k < a.top; ++k) {
+    auto best = [&](const float* list, int n) {      // index of the list's largest value
         float v = -INFINITY;
-        int i = 0x7fffffff;
-        for (int e = lane; e < a.experts; e += 64) {
-            const float c = choice[e];
+        int i = 0;
+        for (int e = lane; e < n; e += 64) {
+            const float c = list[e];
             if (c > v) {
                 v = c;
                 i = e;
             }
         }
-        wave_argmax(v, i);
-        if (i >= a.experts) i = 0;                   // (only where a router delivers no number)
-        const float s = z[i];
+        return __builtin_amdgcn_readlane(i, wave_winner(v));
+    };
+    if (a.keep < a.groups) {
+        for (int g = lane; g < a.groups; g += 64) gs[g] = group_score(choice + g * size, size);
+        wave_lds_sync();
+        for (int k = 0; k < a.keep; ++k) {           // an open group is marked by NaN: it loses every comparison
+            const int g = best(gs, a.groups);
+            if (lane == 0) gs[g] = NAN;
+            wave_lds_sync();
+        }
+        for (int e = lane; e < a.experts; e += 64)
+            if (gs[e / size] == gs[e / size]) choice[e] = -INFINITY;
+        wave_lds_sync();
+    }
+    for (int k = 0; k < a.top; ++k) {
+        const int e = best(choice, a.experts);
+        const float s = z[e];
         total += s;
         if (lane == k) {
             mine = s;
-            my_id = i;
+            my_id = e;
         }
-        if (lane == 0) choice[i] = -INFINITY;
+        wave_lds_sync();
+        if (lane == 0) choice[e] = -INFINITY;
         wave_lds_sync();
     }
-    if (lane < a.top) {
-        a.ids[(int64_t)row * a.top + lane] = my_id;
-        a.weights[(int64_t)row * a.top + lane] = mine / (total + 1e-20f) * a.scale;
-    }
+    store_choice(a, row, lane, my_id, mine, total);
 }
 
-// 16 rows per workgroup, the contraction shared by 8 waves, 64 experts at a time
-__global__ __launch_bounds__(512) void moe_route_kernel(const MoeRouteArgs a) {
+// live rows (at most 16) per workgroup, the contraction shared by 8 waves, 64 experts at a time
+__global__ __launch_bounds__(512) void moe_route_kernel(const MoeRouteArgs a, const int live) {
     extern __shared__ __attribute__((aligned(16))) float lds_r[];
     const int ez = (a.experts + 63) / 64 * 64;
     float *part = lds_r, *z = part + 8 * 16 * 68, *choice = z + 16 * ez, *gs = choice + 8 * ez;     // [8][16][64 + 4], [16][ez], per wave [ez], [groups]
     const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lq = lane & 15, lg = lane >> 4;
-    const int r0 = blockIdx.x * 16, row = r0 + lq < a.rows ? r0 + lq : a.rows - 1;
+    const int r0 = blockIdx.x * live, rows = a.rows - r0 < live ? a.rows - r0 : live, row = r0 + (lq < rows ? lq : rows - 1);
     const int steps = a.cols / 32, per = (steps + 7) / 8, s0 = wave * per, s1 = s0 + per < steps ? s0 + per : steps;
     const uint16_t* x = reinterpret_cast<const uint16_t*>(a.x) + (int64_t)row * a.x_stride + 8 * lg;
     for (int e0 = 0; e0 < a.experts; e0 += 64) {
@@ -152,7 +181,7 @@ __global__ __launch_bounds__(512) void moe_route_kernel(const MoeRouteArgs a) {
 #pragma unroll
         for (int t = 0; t < 4; ++t) *reinterpret_cast<f32x4*>(part + (wave * 16 + lq) * 68 + 16 * t + 4 * lg) = acc[t];
         __syncthreads();
-        for (int i = tid; i < 16 * 64; i += 512) {
+        for (int i = tid; i < rows * 64; i += 512) {
             const int r = i >> 6, e = i & 63;
             float s = 0.f;
 #pragma unroll
@@ -161,7 +190,7 @@ __global__ __launch_bounds__(512) void moe_route_kernel(const MoeRouteArgs a) {
         }
         __syncthreads();
     }
-    for (int r = wave; r < 16 && r0 + r < a.rows; r += 8) choose_experts(a, r0 + r, lane, z + r * ez, choice + wave * ez, gs + wave * a.groups);
+    for (int r = wave; r < rows; r += 8) choose_experts(a, r0 + r, lane, z + r * ez, choice + wave * ez, gs + wave * a.groups);
 }
 
 // any type and width: one workgroup per row, a wave per expert in turn
@@ -248,15 +277,21 @@ __global__ __launch_bounds__(256) void moe_scatter_kernel(int32_t* __restrict__ 
 }
 
 // ------------------------------------------------------------------------------------------------ products, large batches (bf16)
-// 128 pairs x 128 weight rows per workgroup, 64 of the contraction at a time, both operands by LDS-DMA, double-buffered; 4 waves of 64 x 64.
-// GLU: weight rows alternate 16 of gate, 16 of up, so a lane holds both halves of its outputs.
-constexpr int TM = 128, TN = 128, TK = 64;
+// MW x NW waves of MT x NT tiles of 16 x 16: TM pairs by TN weight rows per workgroup, 64 of the contraction at a time, both operands by LDS-DMA,
+// double-buffered.  GLU: weight rows alternate 16 of gate, 16 of up, so a lane holds both halves of its outputs.
+constexpr int TK = 64;
+template <int MW, int NW, int MT, int NT>
+struct GemmShape {
+    static constexpr int WAVES = MW * NW, TM = MW * MT * 16, TN = NW * NT * 16, ROWS = TM + TN, DMA = ROWS / 8 / WAVES;
+    static constexpr size_t LDS = (size_t)2 * ROWS * TK * 2;
+    static_assert(ROWS % (8 * WAVES) == 0 && NT % 2 == 0, "DMA instructions and gate/up tiles divide evenly");
+};
 
-template <bool GLU>
-__global__ __launch_bounds__(256) void moe_gemm_kernel(const MoeGemmArgs a) {
-    constexpr int IMG = TM * TK * 2;
-    extern __shared__ __attribute__((aligned(16))) unsigned char lds[];        // [2][weights | rows]
-    constexpr int OUTS = GLU ? TN / 2 : TN;
+template <bool GLU, int MW, int NW, int MT, int NT>
+__global__ __launch_bounds__(64 * MW * NW) void moe_gemm_kernel(const MoeGemmArgs a) {
+    using G = GemmShape<MW, NW, MT, NT>;
+    constexpr int TN = G::TN, DMA = G::DMA, OUTS = GLU ? TN / 2 : TN;
+    extern __shared__ __attribute__((aligned(16))) unsigned char lds[];        // [2][TN weight rows | TM pairs][128 bytes]
     int nt, mt;
     {
         // one XCD takes a run of column tiles of the same pairs: the gathered rows and the expert's weights are shared in its L2
@@ -267,59 +302,57 @@ __global__ __launch_bounds__(256) void moe_gemm_kernel(const MoeGemmArgs a) {
         nt = idx - mt * (int)gridDim.x;
     }
     const int expert = a.tiles[4 * mt], first = a.tiles[4 * mt + 1], live = a.tiles[4 * mt + 2];
-    const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lq = lane & 15, lg = lane >> 4, wm = wave >> 1, wn = wave & 1;
+    const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lq = lane & 15, lg = lane >> 4, wm = wave / NW, wn = wave % NW;
     const uint16_t* w = reinterpret_cast<const uint16_t*>(a.w) + (int64_t)expert * (GLU ? 2 : 1) * a.n * a.k;
-    // this lane's piece of each DMA instruction: 4 for the weights, 4 for the rows
-    const uint16_t *wp[4], *xp[4];
+    // this lane's piece of each DMA instruction: 8 rows of 128 bytes, 16-byte pieces xor-ed with the row
+    const uint16_t* src[DMA];
 #pragma unroll
-    for (int j = 0; j < 4; ++j) {
-        const int s = (wave * 4 + j) * 64 + lane, R = s >> 3, piece = (s & 7) ^ (R & 7);
-        int col;                                     // weight row
-        if constexpr (GLU) col = nt * OUTS + (R >> 5) * 16 + (R & 15);
-        else col = nt * OUTS + R;
-        if (col >= a.n) col = a.n - 1;
-        wp[j] = w + (int64_t)(GLU && (R & 16) ? a.n + col : col) * a.k + piece * 8;
-        const int slot = first + (R < live ? R : live - 1), pair = a.slot_pair[slot];
-        xp[j] = reinterpret_cast<const uint16_t*>(a.x) + (GLU ? (int64_t)(pair / a.top) * a.x_stride : (int64_t)pair * a.k) + piece * 8;
+    for (int j = 0; j < DMA; ++j) {
+        const int R = (wave * DMA + j) * 8 + (lane >> 3), piece = ((lane & 7) ^ (R & 7)) * 8;
+        if (R < TN) {
+            int col = nt * OUTS + (GLU ? (R >> 5) * 16 + (R & 15) : R);
+            if (col >= a.n) col = a.n - 1;
+            src[j] = w + (int64_t)(GLU && (R & 16) ? a.n + col : col) * a.k + piece;
+        } else {
+            const int r = R - TN, pair = a.slot_pair[first + (r < live ? r : live - 1)];
+            src[j] = reinterpret_cast<const uint16_t*>(a.x) + (GLU ? (int64_t)(pair / a.top) * a.x_stride : (int64_t)pair * a.k) + piece;
+        }
     }
     auto stage = [&](int it, int buf) {
-        unsigned char* base = lds + buf * 2 * IMG;
 #pragma unroll
-        for (int j = 0; j < 4; ++j) dma16(wp[j] + it * TK, base + (wave * 4 + j) * 1024);
-#pragma unroll
-        for (int j = 0; j < 4; ++j) dma16(xp[j] + it * TK, base + IMG + (wave * 4 + j) * 1024);
+        for (int j = 0; j < DMA; ++j) dma16(src[j] + it * TK, lds + buf * G::ROWS * 128 + (wave * DMA + j) * 1024);
     };
-    f32x4 acc[4][4];                                 // [weight tile][row tile]: D[weight row 4 lg + r][pair lq]
+    f32x4 acc[NT][MT];                               // D[weight row 16 i + 4 lg + r][pair 16 j + lq]
 #pragma unroll
-    for (int i = 0; i < 4; ++i)
+    for (int i = 0; i < NT; ++i)
 #pragma unroll
-        for (int j = 0; j < 4; ++j) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
+        for (int j = 0; j < MT; ++j) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
     const int iters = a.k / TK;
     stage(0, 0);
     auto body = [&](auto bufc, const int it) {
         constexpr int buf = decltype(bufc)::value;
         if (it + 1 < iters) {
             stage(it + 1, buf ^ 1);
-            asm volatile("s_waitcnt vmcnt(8)" ::: "memory");
+            asm volatile("s_waitcnt vmcnt(%0)" ::"n"(DMA) : "memory");
         } else {
             asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
         }
         __builtin_amdgcn_s_barrier();
         asm volatile("" ::: "memory");
-        const unsigned char* wimg = lds + buf * 2 * IMG + wn * 64 * 128;
-        const unsigned char* ximg = lds + buf * 2 * IMG + IMG + wm * 64 * 128;
+        const unsigned char* wimg = lds + buf * G::ROWS * 128 + wn * NT * 16 * 128;
+        const unsigned char* ximg = lds + buf * G::ROWS * 128 + (TN + wm * MT * 16) * 128;
 #pragma unroll
         for (int st = 0; st < 2; ++st) {
             const int at = lq * 128 + ((4 * st + lg) ^ (lq & 7)) * 16;
-            bf16x8 wf[4], xf[4];
+            bf16x8 wf[NT], xf[MT];
 #pragma unroll
-            for (int t = 0; t < 4; ++t) wf[t] = *reinterpret_cast<const bf16x8*>(wimg + t * 16 * 128 + at);
+            for (int t = 0; t < NT; ++t) wf[t] = *reinterpret_cast<const bf16x8*>(wimg + t * 16 * 128 + at);
 #pragma unroll
-            for (int t = 0; t < 4; ++t) xf[t] = *reinterpret_cast<const bf16x8*>(ximg + t * 16 * 128 + at);
+            for (int t = 0; t < MT; ++t) xf[t] = *reinterpret_cast<const bf16x8*>(ximg + t * 16 * 128 + at);
 #pragma unroll
-            for (int i = 0; i < 4; ++i)
+            for (int j = 0; j < MT; ++j)
 #pragma unroll
-                for (int j = 0; j < 4; ++j) acc[i][j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf[i], xf[j], acc[i][j], 0, 0, 0);
+                for (int i = 0; i < NT; ++i) acc[i][j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf[i], xf[j], acc[i][j], 0, 0, 0);
         }
         lds_only_barrier();                          // everyone's reads of this buffer are done
     };
@@ -328,14 +361,14 @@ __global__ __launch_bounds__(256) void moe_gemm_kernel(const MoeGemmArgs a) {
         if (it + 1 < iters) body(std::integral_constant<int, 1>{}, it + 1);
     }
 #pragma unroll
-    for (int j = 0; j < 4; ++j) {
-        const int R = wm * 64 + 16 * j + lq;
+    for (int j = 0; j < MT; ++j) {
+        const int R = (wm * MT + j) * 16 + lq;
         if (R >= live) continue;
         uint16_t* out = reinterpret_cast<uint16_t*>(a.out) + (int64_t)a.slot_pair[first + R] * a.n;
         if constexpr (GLU) {
 #pragma unroll
-            for (int i = 0; i < 2; ++i) {
-                const int col = nt * OUTS + wn * 32 + 16 * i + 4 * lg;
+            for (int i = 0; i < NT / 2; ++i) {
+                const int col = nt * OUTS + (wn * NT / 2 + i) * 16 + 4 * lg;
                 f32x4 v;
 #pragma unroll
                 for (int r = 0; r < 4; ++r) v[r] = silu_f(acc[2 * i][j][r]) * acc[2 * i + 1][j][r];
@@ -343,12 +376,21 @@ __global__ __launch_bounds__(256) void moe_gemm_kernel(const MoeGemmArgs a) {
             }
         } else {
 #pragma unroll
-            for (int i = 0; i < 4; ++i) {
-                const int col = nt * OUTS + wn * 64 + 16 * i + 4 * lg;
+            for (int i = 0; i < NT; ++i) {
+                const int col = nt * OUTS + (wn * NT + i) * 16 + 4 * lg;
                 if (col < a.n) act_st4(out + col, acc[i][j]);
             }
         }
     }
+}
+
+template <bool GLU, int MW, int NW, int MT, int NT>
+void gemm_shape(const MoeGemmArgs& a, hipStream_t stream) {
+    using G = GemmShape<MW, NW, MT, NT>;
+    const int outs = GLU ? G::TN / 2 : G::TN;
+    if (G::LDS > 64 * 1024)
+        (void)hipFuncSetAttribute(reinterpret_cast<const void*>(moe_gemm_kernel<GLU, MW, NW, MT, NT>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)G::LDS);
+    moe_gemm_kernel<GLU, MW, NW, MT, NT><<<dim3((a.n + outs - 1) / outs, a.max_tiles), 64 * G::WAVES, G::LDS, stream>>>(a);
 }
 
 // ------------------------------------------------------------------------------------------------ products, at most 64 rows (bf16)
@@ -517,7 +559,8 @@ int launch_moe_route(const MoeRouteArgs& a, int f32, hipStream_t stream) {
         const int ez = (a.experts + 63) / 64 * 64;
         const size_t lds = (size_t)(8 * 16 * 68 + 24 * ez + 8 * a.groups) * 4;
         if (lds > 64 * 1024) (void)hipFuncSetAttribute(reinterpret_cast<const void*>(moe_route_kernel), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
-        moe_route_kernel<<<(a.rows + 15) / 16, 512, lds, stream>>>(a);
+        const int live = a.rows <= 256 ? 2 : a.rows <= 2048 ? 8 : 16;           // few rows: more workgroups, shorter choice
+        moe_route_kernel<<<(a.rows + live - 1) / live, 512, lds, stream>>>(a, live);
     } else {
         const size_t lds = (size_t)(2 * a.experts + a.groups) * 4;
         if (f32) moe_route_generic_kernel<float><<<a.rows, 256, lds, stream>>>(a);
@@ -538,7 +581,7 @@ int launch_moe_dispatch(int32_t* slot_pair, int32_t* tiles, int32_t* counts, con
     return check_launch("moe_scatter");
 }
 
-int moe_tile_rows(int f32) { return f32 ? FM : TM; }
+int moe_tile_rows(int pairs, int experts, int f32) { return f32 ? FM : pairs / experts >= 512 ? 256 : 128; }
 
 int launch_moe_gemm(const MoeGemmArgs& a, int f32, hipStream_t stream) {
     if (f32) {
@@ -554,11 +597,13 @@ int launch_moe_gemm(const MoeGemmArgs& a, int f32, hipStream_t stream) {
         else if (split) moe_small_kernel<false, true><<<grid, 256, 0, stream>>>(a);
         else moe_small_kernel<false, false><<<grid, 256, 0, stream>>>(a);
     } else {
-        constexpr size_t lds = 2 * (TM + TN) * TK * 2;
-        const int outs = a.glu ? TN / 2 : TN;
-        const dim3 grid((a.n + outs - 1) / outs, a.max_tiles);
-        if (a.glu) moe_gemm_kernel<true><<<grid, 256, lds, stream>>>(a);
-        else moe_gemm_kernel<false><<<grid, 256, lds, stream>>>(a);
+        if (a.tile_rows == 256) {
+            if (a.glu) gemm_shape<true, 2, 4, 8, 4>(a, stream);
+            else gemm_shape<false, 2, 4, 8, 4>(a, stream);
+        } else {
+            if (a.glu) gemm_shape<true, 2, 2, 4, 4>(a, stream);
+            else gemm_shape<false, 2, 2, 4, 4>(a, stream);
+        }
     }
     return check_launch("moe_gemm");
 }

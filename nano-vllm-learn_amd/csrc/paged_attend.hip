@@ -3,6 +3,8 @@
 //   rows      one query row at a time (decoding): a workgroup streams the visible keys of one (row, key/value head, split)
 // A sink is an entry of the softmax with score sink[head], no key and no value: it starts the running maximum and sum.
 // Keys a window hides are not read: the walk covers the tiles of the kept first tokens, then those of the window.
+#include <type_traits>
+
 #include "mixers.h"
 
 namespace nvh {
@@ -17,6 +19,12 @@ __global__ __launch_bounds__(256) void attn_prep_kernel(const AttnPrepArgs a) {
     const int64_t row = blockIdx.x;
     T* x = reinterpret_cast<T*>(a.qkv) + row * a.qkv_stride;
     const int nq = a.heads * a.dk, nk = a.kv_heads * a.dk, total = nq + nk + a.kv_heads * a.dv;
+    int64_t pos = a.positions[row];
+    if (pos >= a.max_position) pos = a.max_position - 1;
+    const float* cs = a.cos_sin + pos * a.rot;
+    const int slot = a.slots[row];
+    const int page = slot >= 0 ? slot / a.block_size : 0, off = slot >= 0 ? slot - page * a.block_size : 0;
+    T* cache = reinterpret_cast<T*>(a.cache) + (int64_t)page * a.kv_heads * a.block_size * (a.dk + a.dv);
     f32x8 v[CH];
     float sq = 0.f, sk = 0.f;
 #pragma unroll
@@ -37,12 +45,6 @@ __global__ __launch_bounds__(256) void attn_prep_kernel(const AttnPrepArgs a) {
         sq = 1.f / sqrtf(sq / a.q_n + a.eps);
         sk = 1.f / sqrtf(sk / a.k_n + a.eps);
     }
-    int64_t pos = a.positions[row];
-    if (pos >= a.max_position) pos = a.max_position - 1;
-    const float* cs = a.cos_sin + pos * a.rot;
-    const int slot = a.slots[row];
-    const int page = slot >= 0 ? slot / a.block_size : 0, off = slot >= 0 ? slot - page * a.block_size : 0;
-    T* cache = reinterpret_cast<T*>(a.cache) + (int64_t)page * a.kv_heads * a.block_size * (a.dk + a.dv);
 #pragma unroll
     for (int i = 0; i < CH; ++i) {
         const int c = (threadIdx.x + i * 256) * 8;
@@ -58,14 +60,29 @@ __global__ __launch_bounds__(256) void attn_prep_kernel(const AttnPrepArgs a) {
                 r.b *= inv * *reinterpret_cast<const f32x4*>(w + 4);
             }
             float e[8] = {r.a[0], r.a[1], r.a[2], r.a[3], r.b[0], r.b[1], r.b[2], r.b[3]};
+            float co[4], si[4];
+            if ((a.rot & 7) == 0) {                  // (whole pieces turn or pass)
+                const bool turns = d < a.rot;
+                const f32x4 cv = turns ? *reinterpret_cast<const f32x4*>(cs + d / 2) : f32x4{1.f, 1.f, 1.f, 1.f};
+                const f32x4 sv = turns ? *reinterpret_cast<const f32x4*>(cs + a.rot / 2 + d / 2) : f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+                for (int p = 0; p < 4; ++p) {
+                    co[p] = cv[p];
+                    si[p] = sv[p];
+                }
+            } else {
+#pragma unroll
+                for (int p = 0; p < 4; ++p) {
+                    const bool turns = d / 2 + p < a.rot / 2;
+                    co[p] = turns ? cs[d / 2 + p] : 1.f;
+                    si[p] = turns ? cs[a.rot / 2 + d / 2 + p] : 0.f;
+                }
+            }
 #pragma unroll
             for (int p = 0; p < 4; ++p) {
-                const int pair = d / 2 + p;
-                if (pair < a.rot / 2) {
-                    const float co = cs[pair], si = cs[a.rot / 2 + pair], u = e[2 * p], w = e[2 * p + 1];
-                    e[2 * p] = u * co - w * si;
-                    e[2 * p + 1] = w * co + u * si;
-                }
+                const float u = e[2 * p], w = e[2 * p + 1];
+                e[2 * p] = u * co[p] - w * si[p];
+                e[2 * p + 1] = w * co[p] + u * si[p];
             }
             r = {f32x4{e[0], e[1], e[2], e[3]}, f32x4{e[4], e[5], e[6], e[7]}};
             if (is_q) act_st8(x + c, r);
@@ -187,14 +204,11 @@ struct LanePiece {
         }
     }
 };
-template <int LPR>
-__device__ __forceinline__ float lanes_sum(float x) { return group_sum<LPR>(x); }
-
 constexpr int kRowsHeads = 8;                        // query heads a pass holds at most
 
 template <int DK, int DV, int R>
 __global__ __launch_bounds__(256) void paged_rows_kernel(const PagedAttendArgs a) {
-    constexpr int LPR = DK == 64 && DV == 64 ? 8 : 16, SLOTS = 64 / LPR, NI = DK + DV > 256 ? 4 : 8, UK = NI * SLOTS;
+    constexpr int LPR = DK == 64 && DV == 64 ? 8 : 16, SLOTS = 64 / LPR, NI = (DK + DV > 256 ? 4 : 8) / (R == 8 ? 2 : 1), UK = NI * SLOTS;
     using KL = LanePiece<DK, LPR>;
     using VL = LanePiece<DV, LPR>;
     constexpr int RECW = DV + 4;                     // floats of one head's record in LDS: sums, max, sum
@@ -248,41 +262,30 @@ __global__ __launch_bounds__(256) void paged_rows_kernel(const PagedAttendArgs a
     };
     // a unit that starts past the query's position (the second half of its tile) holds nothing to see
     auto live = [&](int u) { return u < units && unit_key(u) <= pos; };
-    int u = wave;
-    int page = live(u) ? table[unit_key(u) / a.block_size] : 0;
-    if (live(u)) {
-        load_k(unit_key(u), page);
-        load_v(unit_key(u), page);
-    }
-    int next_page = live(u + 4) ? table[unit_key(u + 4) / a.block_size] : 0;
-    for (; live(u); u += 4) {
-        const int k0 = unit_key(u);
+    auto page_of = [&](int u) { return table[unit_key(u < units ? u : 0) / a.block_size]; };
+    // one unit: scores, (the next unit's keys asked for,) softmax, sums, (its values asked for)
+    auto take = [&](auto morec, int k0, int next_key, int next_page) {
+        constexpr bool MORE = decltype(morec)::value;
         float s[R][NI];
-#pragma unroll
-        for (int r = 0; r < R; ++r)
-#pragma unroll
-            for (int i = 0; i < NI; ++i) {
-                float acc = 0.f;
-#pragma unroll
-                for (int d = 0; d < KL::DW; ++d) acc = dot2_bf16(kd[i][d], q[r][d], acc);
-                s[r][i] = acc;
-            }
-        const bool more = live(u + 4);
-        if (more) load_k(unit_key(u + 4), next_page);
-        bool sees[NI];
 #pragma unroll
         for (int i = 0; i < NI; ++i) {
             const int key = k0 + i * SLOTS + ls;
-            sees[i] = key <= pos && (a.window <= 0 || pos - key < a.window || key < a.keep_first);
+            // (added, not selected: a select would turn the sums into branches)
+            const float unseen = key <= pos && (a.window <= 0 || pos - key < a.window || key < a.keep_first) ? 0.f : -INFINITY;
+#pragma unroll
+            for (int r = 0; r < R; ++r) {
+                float acc = 0.f;
+#pragma unroll
+                for (int d = 0; d < KL::DW; ++d) acc = dot2_bf16(kd[i][d], q[r][d], acc);
+                s[r][i] = group_sum<LPR>(acc) * sc + unseen;
+            }
         }
+        if constexpr (MORE) load_k(next_key, next_page);
 #pragma unroll
         for (int r = 0; r < R; ++r) {
             float mx = m[r];
 #pragma unroll
-            for (int i = 0; i < NI; ++i) {
-                s[r][i] = sees[i] ? lanes_sum<LPR>(s[r][i]) * sc : -INFINITY;
-                mx = max2(mx, s[r][i]);
-            }
+            for (int i = 0; i < NI; ++i) mx = max2(mx, s[r][i]);
             const float m_use = mx == -INFINITY ? 0.f : mx, alpha = fast_exp2(m[r] - m_use);
             float sum = 0.f;
 #pragma unroll
@@ -306,10 +309,23 @@ __global__ __launch_bounds__(256) void paged_rows_kernel(const PagedAttendArgs a
                     o[r][2 * d + 1] += s[r][i] * v1;
                 }
             }
-        if (more) {
-            load_v(unit_key(u + 4), next_page);
-            next_page = live(u + 8) ? table[unit_key(u + 8) / a.block_size] : 0;
+        if constexpr (MORE) load_v(next_key, next_page);
+    };
+    int u = wave;
+    if (live(u)) {
+        {
+            const int k0 = unit_key(u), page = page_of(u);
+            load_k(k0, page);
+            load_v(k0, page);
         }
+        int next_page = page_of(u + 4);
+        while (live(u + 4)) {
+            const int page = next_page;
+            next_page = page_of(u + 8);
+            take(std::integral_constant<bool, true>{}, unit_key(u), unit_key(u + 4), page);
+            u += 4;
+        }
+        take(std::integral_constant<bool, false>{}, unit_key(u), 0, 0);
     }
     // ---- merge the lane groups of the wave, then the waves
 #pragma unroll

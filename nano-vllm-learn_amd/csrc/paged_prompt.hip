@@ -10,9 +10,9 @@ namespace nvh {
 namespace {
 
 template <int DK, int DV, int QT>
-__global__ __launch_bounds__(256) void paged_prompt_kernel(const PagedAttendArgs a) {
-    using Tile = AttendTile<DK, DV, QT>;
-    constexpr int BM = Tile::BM, WR = Tile::WR, BN = Tile::BN, KP = Tile::KP, VP = Tile::VP, NK = Tile::NK, NV = Tile::NV, STEPS = Tile::STEPS;
+__global__ __launch_bounds__(256, DK + DV <= 320 ? 2 : 1) void paged_prompt_kernel(const PagedAttendArgs a) {
+    using Images = TileImages<DK, DV>;
+    constexpr int BM = 64 * QT, WR = 16 * QT, BN = Images::BN, KP = Images::KP, VP = Images::VP, NK = Images::NK, NV = Images::NV;
     extern __shared__ __attribute__((aligned(16))) unsigned char lds[];
     int qt, head, b;
     attend_unit(a.heads, qt, head, b);
@@ -26,16 +26,6 @@ __global__ __launch_bounds__(256) void paged_prompt_kernel(const PagedAttendArgs
     const VisibleTiles vis = visible_tiles(q0 + shift, q0 + rows - 1 + shift, a.window, a.keep_first);
     const int n_tiles = vis.count, window = a.window > 0 ? a.window : 0x40000000;
     const int wave_first = q0 + wave * WR + shift, wave_last = wave_first + WR - 1;       // positions of this wave's rows
-
-    Tile tile;
-    tile.init(lds, lq, lg);
-    if (a.sink) {
-#pragma unroll
-        for (int qs = 0; qs < QT; ++qs) {
-            tile.m[qs] = a.sink[head] * kLog2e;
-            tile.l[qs] = lg == 0 ? 1.f : 0.f;        // (the four lane groups' sums are added at the end)
-        }
-    }
 
     // ---- staging: this lane's piece of each DMA instruction: row of the tile and offset inside it
     const uint16_t* cache = reinterpret_cast<const uint16_t*>(a.cache) + (int64_t)g * a.block_size * (DK + DV);
@@ -54,9 +44,11 @@ __global__ __launch_bounds__(256) void paged_prompt_kernel(const PagedAttendArgs
         vr[j] = R;
         vc[j] = ((s - R * VP) ^ swz_v<DV>(R)) * 8;
     }
-    auto stage = [&](int it, int page, int buf) {
-        unsigned char* kimg = Tile::k_image(lds, buf);
-        unsigned char* vimg = Tile::v_image(lds, buf);
+    auto page_of = [&](int it) { return it < n_tiles ? table[vis.tile(it) * BN / a.block_size] : 0; };
+    int page = page_of(0);                           // of the tile that is staged next
+    auto stage = [&](int it, int buf) {
+        unsigned char* kimg = Images::k(lds, buf);
+        unsigned char* vimg = Images::v(lds, buf);
         const int kv0 = vis.tile(it) * BN, off = kv0 % a.block_size, live = sk - kv0 < BN ? sk - kv0 : BN;
         const uint16_t* kb = cache + page * page_elems + (int64_t)off * DK;
         const uint16_t* vb = cache + page * page_elems + (int64_t)a.block_size * DK + (int64_t)off * DV;
@@ -64,61 +56,32 @@ __global__ __launch_bounds__(256) void paged_prompt_kernel(const PagedAttendArgs
         for (int j = 0; j < NK; ++j) dma16(kb + (kr[j] < live ? kr[j] : live - 1) * DK + kc[j], kimg + (wave * NK + j) * 1024);   // rows past the end repeat the last key: masked
 #pragma unroll
         for (int j = 0; j < NV; ++j) dma16(vb + (vr[j] < live ? vr[j] : live - 1) * DV + vc[j], vimg + (wave * NV + j) * 1024);
+        page = page_of(it + 1);
     };
-    auto page_of = [&](int it) { return it < n_tiles ? table[vis.tile(it) * BN / a.block_size] : 0; };
-    stage(0, page_of(0), 0);
-    int next_page = page_of(1);
-
     int my_q[QT];
     bool q_ok[QT];
+    const uint16_t* qp[QT];
 #pragma unroll
     for (int qs = 0; qs < QT; ++qs) {
         my_q[qs] = q0 + wave * WR + 16 * qs + lq;
         q_ok[qs] = my_q[qs] < sq;
-        const uint16_t* qp = reinterpret_cast<const uint16_t*>(a.q) + (int64_t)(q_beg + (q_ok[qs] ? my_q[qs] : sq - 1)) * a.q_stride + (int64_t)head * DK + lg * 8;
-#pragma unroll
-        for (int st = 0; st < STEPS; ++st) tile.qf[qs][st] = *reinterpret_cast<const bf16x8*>(qp + st * 32);
+        qp[qs] = reinterpret_cast<const uint16_t*>(a.q) + (int64_t)(q_beg + (q_ok[qs] ? my_q[qs] : sq - 1)) * a.q_stride + (int64_t)head * DK + lg * 8;
     }
-    const float scale_log2 = a.scale * kLog2e;
-    auto tile_body = [&](auto bufc, const int it) {
-        constexpr int buf = decltype(bufc)::value;
-        if (it + 1 < n_tiles) {
-            stage(it + 1, next_page, buf ^ 1);
-            next_page = page_of(it + 2);
-            asm volatile("s_waitcnt vmcnt(%0)" ::"n"(NK + NV) : "memory");     // tile `it` has landed, tile it + 1 is in flight
-        } else {
-            asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
-        }
-        __builtin_amdgcn_s_barrier();
-        asm volatile("" ::: "memory");
-        const int kv0 = vis.tile(it) * BN;
-        const bool in_window = kv0 + BN - 1 > wave_first - window;             // some key of the tile is near enough for the wave's first row
-        if (kv0 <= wave_last && (in_window || kv0 < a.keep_first)) {
-            int hi[QT], lo[QT];
-            const int kept = a.keep_first - kv0 - 4 * lg;
-#pragma unroll
-            for (int qs = 0; qs < QT; ++qs) {
-                const int pos = my_q[qs] + shift;
-                hi[qs] = (pos < sk - 1 ? pos : sk - 1) - kv0 - 4 * lg;
-                lo[qs] = pos - window - kv0 - 4 * lg;
-            }
-            const bool mask = kv0 + BN - 1 > wave_first || kv0 + BN > sk || (kv0 <= wave_last - window && kv0 + BN > a.keep_first);
-            tile.template attend<buf>(lds, scale_log2, mask, lq, lg, [&](int qs, int off) { return off <= hi[qs] && (off > lo[qs] || off < kept); });
-        }
-        lds_only_barrier();                                                    // everyone's reads of this buffer are done
-    };
-    for (int it = 0; it < n_tiles; it += 2) {
-        tile_body(std::integral_constant<int, 0>{}, it);
-        if (it + 1 < n_tiles) tile_body(std::integral_constant<int, 1>{}, it + 1);
-    }
-#pragma unroll
-    for (int qs = 0; qs < QT; ++qs)
-        tile.store(qs, reinterpret_cast<uint16_t*>(a.out) + (int64_t)(q_beg + my_q[qs]) * a.out_stride + head * DV, lg, q_ok[qs]);
+    attend_walk<DK, DV, QT>(
+        lds, n_tiles, a.scale * kLog2e, a.sink ? a.sink[head] * kLog2e : -INFINITY, lane, stage,
+        [&](int qs, int st) { return *reinterpret_cast<const bf16x8*>(qp[qs] + st * 32); }, [&](int it) { return vis.tile(it) * BN; },
+        [&](int kv0) { return kv0 <= wave_last && (kv0 + BN - 1 > wave_first - window || kv0 < a.keep_first); },
+        [&](int kv0) { return kv0 + BN - 1 > wave_first || kv0 + BN > sk || (kv0 <= wave_last - window && kv0 + BN > a.keep_first); },
+        [&](int kv0, int qs, int off) {
+            const int pos = my_q[qs] + shift, at = kv0 + 4 * lg + off;
+            return at <= (pos < sk - 1 ? pos : sk - 1) && (at > pos - window || at < a.keep_first);
+        },
+        [&](int qs) { return q_ok[qs] ? reinterpret_cast<uint16_t*>(a.out) + (int64_t)(q_beg + my_q[qs]) * a.out_stride + head * DV : nullptr; });
 }
 
 template <int DK, int DV, int QT>
 int launch_one(const PagedAttendArgs& a, hipStream_t stream) {
-    constexpr size_t lds = AttendTile<DK, DV, QT>::LDS;
+    constexpr size_t lds = TileImages<DK, DV>::BYTES;
     if (lds > 64 * 1024) (void)hipFuncSetAttribute(reinterpret_cast<const void*>(paged_prompt_kernel<DK, DV, QT>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
     paged_prompt_kernel<DK, DV, QT><<<dim3(a.heads, a.batch, (a.max_q + 64 * QT - 1) / (64 * QT)), 256, lds, stream>>>(a);
     return check_launch("paged_attend_prompt");

@@ -122,7 +122,7 @@ class MoeGemmDesc(ctypes.Structure):
     _fields_ = [("out", ctypes.c_void_p), ("x", ctypes.c_void_p), ("x_stride", ctypes.c_int64), ("w", ctypes.c_void_p),
                 ("pairs", ctypes.c_int32), ("top", ctypes.c_int32), ("experts", ctypes.c_int32), ("n", ctypes.c_int32),
                 ("k", ctypes.c_int32), ("glu", ctypes.c_int32), ("ids", ctypes.c_void_p), ("slot_pair", ctypes.c_void_p),
-                ("tiles", ctypes.c_void_p), ("max_tiles", ctypes.c_int32)]
+                ("tiles", ctypes.c_void_p), ("max_tiles", ctypes.c_int32), ("tile_rows", ctypes.c_int32)]
 
 
 class ResidualNormDesc(ctypes.Structure):
@@ -228,7 +228,7 @@ _SIGS = {
     "nvh_moe_route": (ctypes.c_int, [ctypes.POINTER(MoeRouteDesc), ctypes.c_int, ctypes.c_void_p]),
     "nvh_moe_dispatch_blocks": (ctypes.c_int, [ctypes.c_int]),
     "nvh_moe_dispatch": (ctypes.c_int, [ctypes.c_void_p] * 4 + [ctypes.c_int] * 4 + [ctypes.c_void_p]),
-    "nvh_moe_tile_rows": (ctypes.c_int, [ctypes.c_int]),
+    "nvh_moe_tile_rows": (ctypes.c_int, [ctypes.c_int] * 3),
     "nvh_moe_gemm": (ctypes.c_int, [ctypes.POINTER(MoeGemmDesc), ctypes.c_int, ctypes.c_void_p]),
     "nvh_residual_norm": (ctypes.c_int, [ctypes.POINTER(ResidualNormDesc), ctypes.c_int, ctypes.c_void_p]),
     "nvh_softcap": (ctypes.c_int, [ctypes.c_void_p, ctypes.c_float, ctypes.c_int, ctypes.c_int, ctypes.c_int64, ctypes.c_int, ctypes.c_void_p]),

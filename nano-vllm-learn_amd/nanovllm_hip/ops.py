@@ -876,11 +876,11 @@ def paged_attend_supported(dk, dv, block_size) -> bool:
 
 
 def paged_attend_splits(rows, kv_heads, heads, max_context, window=0, keep_first=0) -> int:
-    """Context splits of one launch over single rows: about two workgroups per CU, none with fewer than four 64-key tiles' worth of work."""
+    """Context splits of one launch over single rows: about two workgroups per CU, none with fewer than two 64-key tiles."""
     seen = min(max_context, window + keep_first + 126) if window else max_context
     tiles = (seen + 63) // 64
     groups = rows * kv_heads * ((heads // kv_heads + 7) // 8)
-    splits = max(1, min(512 // max(1, groups), (tiles + 3) // 4, 64))
+    splits = max(1, min(512 // max(1, groups), (tiles + 1) // 2, 64))
     per = -(-tiles // splits)
     return -(-tiles // per)
 
@@ -1035,19 +1035,19 @@ def moe_route(x, router, correction, top, groups, keep, scale):
     return ids, weights
 
 
-def moe_dispatch(ids, experts, dtype):
-    """(slot_pair, tiles): the pairs row * top + k sorted by expert, cut into tiles of one expert each; nothing comes back to the host."""
+def moe_dispatch(ids, experts, dtype, tile_rows=None):
+    """(slot_pair, tiles, rows per tile): the pairs row * top + k sorted by expert, cut into tiles of one expert each; nothing comes back to the host."""
     _require_i32(ids=ids)
     assert ids.is_contiguous()
     lib, pairs = _lib.load(), ids.numel()
-    tile_rows = int(lib.nvh_moe_tile_rows(_out_code(dtype)))
+    tile_rows = tile_rows or int(lib.nvh_moe_tile_rows(pairs, experts, _out_code(dtype)))
     max_tiles = pairs // tile_rows + min(experts, pairs)
     slots = torch.empty(pairs, dtype=torch.int32, device=ids.device)
     tiles = torch.empty((pairs // tile_rows + experts, 4), dtype=torch.int32, device=ids.device)
     counts = torch.empty((lib.nvh_moe_dispatch_blocks(pairs), experts), dtype=torch.int32, device=ids.device)
     _lib.check(lib.nvh_moe_dispatch(slots.data_ptr(), tiles.data_ptr(), counts.data_ptr(), ids.data_ptr(), pairs, experts, tile_rows, tiles.shape[0], _stream()),
                "nvh_moe_dispatch")
-    return slots, tiles[:max_tiles]
+    return slots, tiles[:max_tiles], tile_rows
 
 
 def moe_gemm(x, weight, ids, glu, dispatch=None):
@@ -1067,7 +1067,7 @@ def moe_gemm(x, weight, ids, glu, dispatch=None):
         assert ids.is_contiguous()
         d.ids = ids.data_ptr()
     else:
-        slots, tiles = dispatch
+        slots, tiles, d.tile_rows = dispatch
         assert slots.numel() == pairs and tiles.is_contiguous()
         d.slot_pair, d.tiles, d.max_tiles = slots.data_ptr(), tiles.data_ptr(), tiles.shape[0]
     _lib.check(_lib.load().nvh_moe_gemm(ctypes.byref(d), code, _stream()), "nvh_moe_gemm")

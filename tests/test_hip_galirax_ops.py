@@ -397,7 +397,7 @@ def test_dispatch(pairs_shape, experts, dtype):
     from nanovllm_hip import ops
     g = torch.Generator().manual_seed(1)
     ids = torch.stack([torch.randperm(max(experts - 1, pairs_shape[1]), generator=g)[:pairs_shape[1]] for _ in range(pairs_shape[0])]).int()
-    slots, tiles = ops.moe_dispatch(ids.cuda(), experts, dtype)
+    slots, tiles, _ = ops.moe_dispatch(ids.cuda(), experts, dtype)
     slots, tiles, flat = slots.cpu(), tiles.cpu(), ids.flatten()
     assert sorted(slots.tolist()) == list(range(ids.numel()))
     seen = torch.zeros(ids.numel(), dtype=torch.bool)
@@ -421,7 +421,7 @@ def test_expert_products(rows, top, experts, n, k, dtype):
         ids[1:rows // 2] = ids[0]                                                  # one expert with many rows
     x = randn(rows, k, seed=1, dtype=dtype)
     gu, dn = randn(experts, 2 * n, k, seed=2, scale=k ** -0.5, dtype=dtype), randn(experts, k, n, seed=3, scale=n ** -0.5, dtype=dtype)
-    forms = [ops.moe_dispatch(ids.cuda(), experts, dtype)] + ([None] if dtype == BF16 and rows <= 64 else [])
+    forms = [ops.moe_dispatch(ids.cuda(), experts, dtype, r) for r in ([64] if dtype == F32 else [None, 128, 256])] + ([None] if dtype == BF16 and rows <= 64 else [])
     flat = ids.flatten().long()
     xr = f64(x).repeat_interleave(top, dim=0)
     for dispatch in forms:
