@@ -611,8 +611,7 @@ typedef struct nvh_paged_attend_desc {
     int32_t window, keep_first;
     const float* sink;           /* nullable: [heads] */
     int32_t splits;
-    float* part_o;               /* splits > 1: [rows, heads, splits, dv] scratch */
-    float* part_ml;              /* [rows, heads, splits, 2] */
+    float* part;                 /* splits > 1: [rows, heads, splits, dv + 4] scratch */
     uint32_t* tickets;           /* zero before the launch, left zero: nvh_paged_attend_ticket_bytes(rows, kv_heads, heads) */
     void* out;                   /* nullable: [rows, heads * dv], row stride out_stride */
     int64_t out_stride;

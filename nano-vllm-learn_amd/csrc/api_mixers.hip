@@ -60,7 +60,7 @@ int nvh_paged_attend_rows(const nvh_paged_attend_desc* d, int generic, int dtype
     if (d->rows == 0) return 0;
     const int rc = check_attend("paged_attend_rows", d, dtype);
     if (rc) return rc;
-    REQUIRE(d->positions && d->rows > 0 && d->splits >= 1 && d->splits <= 64 && (d->splits == 1 || (d->part_o && d->part_ml && d->tickets)), NVH_E_NULL,
+    REQUIRE(d->positions && d->rows > 0 && d->splits >= 1 && d->splits <= 64 && (d->splits == 1 || (d->part && aligned16(d->part) && d->tickets)), NVH_E_NULL,
             "paged_attend_rows: rows %d splits %d or null pointer", d->rows, d->splits);
     REQUIRE(!d->out_packed || (dtype == NVH_BF16 && (d->heads * d->dv) % 32 == 0), NVH_E_SHAPE, "paged_attend_rows: packed output is bf16, width %% 32 == 0");
     return launch_paged_attend_rows(*d, dtype == NVH_F32, generic, (hipStream_t)stream);

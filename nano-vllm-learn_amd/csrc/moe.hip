@@ -277,21 +277,22 @@ __global__ __launch_bounds__(256) void moe_scatter_kernel(int32_t* __restrict__ 
 }
 
 // ------------------------------------------------------------------------------------------------ products, large batches (bf16)
-// MW x NW waves of MT x NT tiles of 16 x 16: TM pairs by TN weight rows per workgroup, 64 of the contraction at a time, both operands by LDS-DMA,
-// double-buffered.  GLU: weight rows alternate 16 of gate, 16 of up, so a lane holds both halves of its outputs.
-constexpr int TK = 64;
+// MW x NW waves of MT x NT tiles of 16 x 16: TM pairs by TN weight rows per workgroup, 32 of the contraction at a time, both operands by LDS-DMA through a
+// ring of four images: three are on their way while the fourth is read into registers, and the one before it is multiplied from there.
+// GLU: weight rows alternate 16 of gate, 16 of up, so a lane holds both halves of its outputs.
+constexpr int TK = 32, kRing = 4;
 template <int MW, int NW, int MT, int NT>
 struct GemmShape {
-    static constexpr int WAVES = MW * NW, TM = MW * MT * 16, TN = NW * NT * 16, ROWS = TM + TN, DMA = ROWS / 8 / WAVES;
-    static constexpr size_t LDS = (size_t)2 * ROWS * TK * 2;
-    static_assert(ROWS % (8 * WAVES) == 0 && NT % 2 == 0, "DMA instructions and gate/up tiles divide evenly");
+    static constexpr int WAVES = MW * NW, TM = MW * MT * 16, TN = NW * NT * 16, ROWS = TM + TN, IMG = ROWS * TK * 2, DMA = IMG / 1024 / WAVES;
+    static constexpr size_t LDS = (size_t)kRing * IMG;
+    static_assert(IMG % (1024 * WAVES) == 0 && NT % 2 == 0, "DMA instructions and gate/up tiles divide evenly");
 };
 
 template <bool GLU, int MW, int NW, int MT, int NT>
 __global__ __launch_bounds__(64 * MW * NW) void moe_gemm_kernel(const MoeGemmArgs a) {
     using G = GemmShape<MW, NW, MT, NT>;
     constexpr int TN = G::TN, DMA = G::DMA, OUTS = GLU ? TN / 2 : TN;
-    extern __shared__ __attribute__((aligned(16))) unsigned char lds[];        // [2][TN weight rows | TM pairs][128 bytes]
+    extern __shared__ __attribute__((aligned(16))) unsigned char lds[];        // [ring][TN weight rows | TM pairs][64 bytes]
     int nt, mt;
     {
         // one XCD takes a run of column tiles of the same pairs: the gathered rows and the expert's weights are shared in its L2
@@ -304,11 +305,12 @@ __global__ __launch_bounds__(64 * MW * NW) void moe_gemm_kernel(const MoeGemmArg
     const int expert = a.tiles[4 * mt], first = a.tiles[4 * mt + 1], live = a.tiles[4 * mt + 2];
     const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lq = lane & 15, lg = lane >> 4, wm = wave / NW, wn = wave % NW;
     const uint16_t* w = reinterpret_cast<const uint16_t*>(a.w) + (int64_t)expert * (GLU ? 2 : 1) * a.n * a.k;
-    // this lane's piece of each DMA instruction: 8 rows of 128 bytes, 16-byte pieces xor-ed with the row
+    auto swz = [](int r) { return (r >> 2) & 3; };   // 16-byte pieces of a row are xor-ed: 16 rows read at one column spread over all banks
+    // this lane's piece of each DMA instruction: 16 rows of 64 bytes
     const uint16_t* src[DMA];
 #pragma unroll
     for (int j = 0; j < DMA; ++j) {
-        const int R = (wave * DMA + j) * 8 + (lane >> 3), piece = ((lane & 7) ^ (R & 7)) * 8;
+        const int R = (wave * DMA + j) * 16 + (lane >> 2), piece = ((lane & 3) ^ swz(R)) * 8;
         if (R < TN) {
             int col = nt * OUTS + (GLU ? (R >> 5) * 16 + (R & 15) : R);
             if (col >= a.n) col = a.n - 1;
@@ -320,46 +322,71 @@ __global__ __launch_bounds__(64 * MW * NW) void moe_gemm_kernel(const MoeGemmArg
     }
     auto stage = [&](int it, int buf) {
 #pragma unroll
-        for (int j = 0; j < DMA; ++j) dma16(src[j] + it * TK, lds + buf * G::ROWS * 128 + (wave * DMA + j) * 1024);
+        for (int j = 0; j < DMA; ++j) dma16(src[j] + it * TK, lds + buf * G::IMG + (wave * DMA + j) * 1024);
     };
     f32x4 acc[NT][MT];                               // D[weight row 16 i + 4 lg + r][pair 16 j + lq]
 #pragma unroll
     for (int i = 0; i < NT; ++i)
 #pragma unroll
         for (int j = 0; j < MT; ++j) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
-    const int iters = a.k / TK;
-    stage(0, 0);
-    auto body = [&](auto bufc, const int it) {
-        constexpr int buf = decltype(bufc)::value;
-        if (it + 1 < iters) {
-            stage(it + 1, buf ^ 1);
-            asm volatile("s_waitcnt vmcnt(%0)" ::"n"(DMA) : "memory");
-        } else {
-            asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
-        }
-        __builtin_amdgcn_s_barrier();
-        asm volatile("" ::: "memory");
-        const unsigned char* wimg = lds + buf * G::ROWS * 128 + wn * NT * 16 * 128;
-        const unsigned char* ximg = lds + buf * G::ROWS * 128 + (TN + wm * MT * 16) * 128;
+    const int iters = a.k / TK;                      // (k is a multiple of 64: even)
+    // (images past the last one are asked for again: every iteration leaves the same number of loads in flight, without a branch)
+    auto stage_next = [&](int it) { stage(it < iters ? it : iters - 1, it % kRing); };
 #pragma unroll
-        for (int st = 0; st < 2; ++st) {
-            const int at = lq * 128 + ((4 * st + lg) ^ (lq & 7)) * 16;
-            bf16x8 wf[NT], xf[MT];
-#pragma unroll
-            for (int t = 0; t < NT; ++t) wf[t] = *reinterpret_cast<const bf16x8*>(wimg + t * 16 * 128 + at);
-#pragma unroll
-            for (int t = 0; t < MT; ++t) xf[t] = *reinterpret_cast<const bf16x8*>(ximg + t * 16 * 128 + at);
-#pragma unroll
-            for (int j = 0; j < MT; ++j)
-#pragma unroll
-                for (int i = 0; i < NT; ++i) acc[i][j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf[i], xf[j], acc[i][j], 0, 0, 0);
-        }
-        lds_only_barrier();                          // everyone's reads of this buffer are done
+    for (int it = 0; it < kRing; ++it) stage_next(it);
+    struct Operands {
+        bf16x8 w[NT], x[MT];
     };
+    Operands even, odd;                              // of the image being multiplied and of the next one, read meanwhile
+    auto read = [&](int it, Operands& f) {
+        const int at = (it % kRing) * G::IMG + lq * 64 + (lg ^ swz(lq)) * 16;
+        const unsigned char* wimg = lds + at + wn * NT * 16 * 64;
+        const unsigned char* ximg = lds + at + (TN + wm * MT * 16) * 64;
+#pragma unroll
+        for (int t = 0; t < NT; ++t) f.w[t] = *reinterpret_cast<const bf16x8*>(wimg + t * 16 * 64);
+#pragma unroll
+        for (int t = 0; t < MT; ++t) f.x[t] = *reinterpret_cast<const bf16x8*>(ximg + t * 16 * 64);
+    };
+    // the oldest image in flight has landed (`younger` behind it), and everyone has read the one before it
+    auto arrive = [&](auto younger) {
+        asm volatile("s_waitcnt vmcnt(%0)" ::"n"(decltype(younger)::value * DMA) : "memory");
+        lds_only_barrier();
+    };
+    // reads and loads spread between the products
+    auto spread = [] {
+#pragma unroll
+        for (int k = 0; k < NT + MT; ++k) {
+            __builtin_amdgcn_sched_group_barrier(0x100, 1, 0);                 // LDS read
+            __builtin_amdgcn_sched_group_barrier(0x008, 1, 0);                 // MFMA
+        }
+#pragma unroll
+        for (int k = 0; k < DMA; ++k) {
+            __builtin_amdgcn_sched_group_barrier(0x010, 1, 0);                 // load
+            __builtin_amdgcn_sched_group_barrier(0x008, 2, 0);
+        }
+    };
+    auto multiply = [&](const Operands& f) {
+#pragma unroll
+        for (int j = 0; j < MT; ++j)
+#pragma unroll
+            for (int i = 0; i < NT; ++i) acc[i][j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(f.w[i], f.x[j], acc[i][j], 0, 0, 0);
+    };
+    arrive(std::integral_constant<int, kRing - 1>{});
+    read(0, even);
+    constexpr std::integral_constant<int, kRing - 2> in_flight{};
     for (int it = 0; it < iters; it += 2) {
-        body(std::integral_constant<int, 0>{}, it);
-        if (it + 1 < iters) body(std::integral_constant<int, 1>{}, it + 1);
+        arrive(in_flight);
+        read(it + 1, odd);
+        stage_next(it + kRing);
+        multiply(even);
+        spread();
+        arrive(in_flight);
+        read(it + 2, even);                          // (behind the last image: read and not used)
+        stage_next(it + 1 + kRing);
+        multiply(odd);
+        spread();
     }
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
 #pragma unroll
     for (int j = 0; j < MT; ++j) {
         const int R = (wm * MT + j) * 16 + lq;

@@ -174,12 +174,16 @@ __global__ __launch_bounds__(256) void paged_rows_generic_kernel(const PagedAtte
 // 64 / LPR rows and the lanes that scored a key also weigh its value: no exchange until the end.  Every group of LPR lanes keeps its own running maximum,
 // sum and output; groups, waves and splits are merged once.  Loads of the next unit's keys are issued behind the scores of this one, its values behind
 // the sums, so about a unit per wave is always in flight.
-// Split partials: write-through stores, drained by every storing wave, a ticket per (row, key/value head, pass); the last workgroup to arrive merges.
-__device__ __forceinline__ void st_through(float* p, float v) {
-    __hip_atomic_store(reinterpret_cast<unsigned*>(p), __builtin_bit_cast(unsigned, v), __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+// Split records (sums, maximum, sum of weights per head): 16-byte write-through stores, drained by every storing wave, then a ticket per (row, key/value
+// head, pass); the last workgroup to arrive reads all records past the L1 and merges them in split order.
+constexpr int kThroughAux = 16;                      // cache policy of the buffer accesses: sc1
+typedef __amdgpu_buffer_rsrc_t RecordBuf;
+__device__ __forceinline__ RecordBuf record_buffer(float* base, uint32_t bytes) { return __builtin_amdgcn_make_buffer_rsrc(base, 0, (int)bytes, 0x00020000); }
+__device__ __forceinline__ void st16_through(RecordBuf rb, uint32_t byte_off, f32x4 v) {
+    __builtin_amdgcn_raw_buffer_store_b128(__builtin_bit_cast(u32x4, v), rb, (int)byte_off, 0, kThroughAux);
 }
-__device__ __forceinline__ float ld_through(const float* p) {
-    return __builtin_bit_cast(float, __hip_atomic_load(reinterpret_cast<const unsigned*>(p), __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT));
+__device__ __forceinline__ f32x4 ld16_through(RecordBuf rb, uint32_t byte_off) {
+    return __builtin_bit_cast(f32x4, __builtin_amdgcn_raw_buffer_load_b128(rb, (int)byte_off, 0, kThroughAux));
 }
 
 // this lane's share of a row of W elements: W / LPR of them, in pieces of 8 (and one of 4)
@@ -354,12 +358,13 @@ __global__ __launch_bounds__(256) void paged_rows_kernel(const PagedAttendArgs a
         }
     }
     __syncthreads();
-    constexpr int PIECES = DV / 4;
+    constexpr int PIECES = DV / 4, RECB = (DV + 4) * 4;                        // 4-column pieces of a head; bytes of a split record
     auto finish = [&](int r, int c, f32x4 v) {       // 4 normalised columns of head h0 + r
         const int col = (h0 + r) * DV + c;
         if (a.out) act_st4(reinterpret_cast<uint16_t*>(a.out) + (int64_t)row * a.out_stride + col, v);
         if (a.out_packed) act_st4(reinterpret_cast<uint16_t*>(a.out_packed) + pack_index(row, col, a.heads * DV), v);
     };
+    const RecordBuf records = record_buffer(a.splits > 1 ? a.part + ((int64_t)row * a.heads + h0) * a.splits * (DV + 4) : nullptr, a.splits > 1 ? (uint32_t)nh * a.splits * RECB : 0u);
     for (int e = tid; e < nh * PIECES; e += 256) {
         const int r = e / PIECES, c = (e - r * PIECES) * 4;
         float mw[4], mx = -INFINITY, sum = 0.f;
@@ -382,41 +387,47 @@ __global__ __launch_bounds__(256) void paged_rows_kernel(const PagedAttendArgs a
             sum += fast_exp2(sink - m_use);
             finish(r, c, v * (sum > 0.f ? 1.f / sum : 0.f));
         } else {
-            const int64_t at = ((int64_t)row * a.heads + h0 + r) * a.splits + split;
-#pragma unroll
-            for (int k = 0; k < 4; ++k) st_through(a.part_o + at * DV + c + k, v[k]);
-            if (c == 0) {
-                st_through(a.part_ml + at * 2, mx);
-                st_through(a.part_ml + at * 2 + 1, sum);
-            }
+            const uint32_t at = (uint32_t)(r * a.splits + split) * RECB;
+            st16_through(records, at + c * 4, v);
+            if (c == 0) st16_through(records, at + DV * 4, f32x4{mx, sum, 0.f, 0.f});
         }
     }
     if (a.splits == 1) return;
     asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
     __syncthreads();
-    if (tid == 0) {
-        uint32_t* ticket = a.tickets + ((int64_t)row * gridDim.y + blockIdx.y) * kAttendTicketWords;
-        const uint32_t seen = __hip_atomic_fetch_add(ticket, 1u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
-        last_flag = seen == (uint32_t)a.splits - 1;
-        if (last_flag) __hip_atomic_store(ticket, 0u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
-    }
+    uint32_t* ticket = a.tickets + ((int64_t)row * gridDim.y + blockIdx.y) * kAttendTicketWords;
+    if (tid == 0) last_flag = __hip_atomic_fetch_add(ticket, 1u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT) == (uint32_t)a.splits - 1;
     __syncthreads();
     if (!last_flag) return;
+    if (tid == 0) __hip_atomic_store(ticket, 0u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+    constexpr int SB = 4;                            // records asked for at a time
     for (int e = tid; e < nh * PIECES; e += 256) {
         const int r = e / PIECES, c = (e - r * PIECES) * 4;
-        const int64_t at = ((int64_t)row * a.heads + h0 + r) * a.splits;
-        const float sink = a.sink ? a.sink[h0 + r] * kLog2e : -INFINITY;
-        float mx = sink;
-        for (int s = 0; s < a.splits; ++s) mx = fmaxf(mx, ld_through(a.part_ml + (at + s) * 2));
-        const float m_use = mx == -INFINITY ? 0.f : mx;
-        float sum = fast_exp2(sink - m_use);
+        float mx = a.sink ? a.sink[h0 + r] * kLog2e : -INFINITY, sum = mx > -INFINITY ? 1.f : 0.f;
         f32x4 v = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll 4
-        for (int s = 0; s < a.splits; ++s) {
-            const float f = fast_exp2(ld_through(a.part_ml + (at + s) * 2) - m_use);
-            sum += f * ld_through(a.part_ml + (at + s) * 2 + 1);
+        for (int s0 = 0; s0 < a.splits; s0 += SB) {
+            f32x4 ml[SB], o4[SB];
 #pragma unroll
-            for (int k = 0; k < 4; ++k) v[k] += f * ld_through(a.part_o + (at + s) * DV + c + k);
+            for (int s = 0; s < SB; ++s) {
+                const uint32_t at = (uint32_t)(r * a.splits + (s0 + s < a.splits ? s0 + s : a.splits - 1)) * RECB;
+                ml[s] = ld16_through(records, at + DV * 4);
+                o4[s] = ld16_through(records, at + c * 4);
+            }
+            float top = mx;
+#pragma unroll
+            for (int s = 0; s < SB; ++s)
+                if (s0 + s < a.splits) top = fmaxf(top, ml[s][0]);
+            const float m_use = top == -INFINITY ? 0.f : top, old = fast_exp2(mx - m_use);
+            v *= old;
+            sum *= old;
+            mx = top;
+#pragma unroll
+            for (int s = 0; s < SB; ++s)
+                if (s0 + s < a.splits) {
+                    const float f = fast_exp2(ml[s][0] - m_use);
+                    v += o4[s] * f;
+                    sum += ml[s][1] * f;
+                }
         }
         finish(r, c, v * (sum > 0.f ? 1.f / sum : 0.f));
     }

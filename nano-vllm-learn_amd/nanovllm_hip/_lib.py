@@ -96,8 +96,8 @@ class PagedAttendDesc(ctypes.Structure):
                 ("block_size", ctypes.c_int32), ("block_tables", ctypes.c_void_p), ("bt_stride", ctypes.c_int64),
                 ("row_seq", ctypes.c_void_p), ("positions", ctypes.c_void_p), ("cu_q", ctypes.c_void_p), ("cu_k", ctypes.c_void_p),
                 ("batch", ctypes.c_int32), ("max_q", ctypes.c_int32), ("scale", ctypes.c_float), ("window", ctypes.c_int32),
-                ("keep_first", ctypes.c_int32), ("sink", ctypes.c_void_p), ("splits", ctypes.c_int32), ("part_o", ctypes.c_void_p),
-                ("part_ml", ctypes.c_void_p), ("tickets", ctypes.c_void_p), ("out", ctypes.c_void_p), ("out_stride", ctypes.c_int64),
+                ("keep_first", ctypes.c_int32), ("sink", ctypes.c_void_p), ("splits", ctypes.c_int32), ("part", ctypes.c_void_p),
+                ("tickets", ctypes.c_void_p), ("out", ctypes.c_void_p), ("out_stride", ctypes.c_int64),
                 ("out_packed", ctypes.c_void_p)]
 
 

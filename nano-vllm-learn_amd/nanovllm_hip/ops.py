@@ -925,10 +925,9 @@ def paged_attend_rows(q, cache, block_tables, positions, heads, kv_heads, dk, dv
     if code == NVH_BF16 and row_seq is None and not generic and paged_attend_supported(dk, dv, cache.shape[1]):
         d.splits = splits or paged_attend_splits(rows, kv_heads, heads, max_context, window, keep_first)
     if d.splits > 1:
-        part_o = torch.empty((rows, heads, d.splits, dv), dtype=torch.float32, device=q.device)
-        part_ml = torch.empty((rows, heads, d.splits, 2), dtype=torch.float32, device=q.device)
+        part = torch.empty((rows, heads, d.splits, dv + 4), dtype=torch.float32, device=q.device)
         tickets = reserve_workspace(q.device, paged_attend_ticket_bytes(rows, kv_heads, heads), "paged_attend")
-        d.part_o, d.part_ml, d.tickets = part_o.data_ptr(), part_ml.data_ptr(), tickets.data_ptr()
+        d.part, d.tickets = part.data_ptr(), tickets.data_ptr()
     if out_packed is not None:
         _packed_ok(out_packed, rows, heads * dv)
         d.out_packed = out_packed.data_ptr()
