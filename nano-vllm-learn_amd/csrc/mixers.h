@@ -76,6 +76,12 @@ __device__ __forceinline__ void block_sum256x2(float& u, float& v, float* lds) {
     v = lds[4] + lds[5] + lds[6] + lds[7];
 }
 
+__device__ __forceinline__ void wave_lds_sync() {    // LDS written by other lanes of this wave is visible behind it
+    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+    __builtin_amdgcn_wave_barrier();
+}
+
 __device__ __forceinline__ float silu_f(float z) { return z / (1.f + __expf(-z)); }
 
 // ---- keys a query at position `pos` sees, as 64-key tiles: the tiles of the kept first tokens, then those of the window

@@ -11,12 +11,6 @@ namespace nvh {
 
 namespace {
 
-__device__ __forceinline__ void wave_lds_sync() {    // LDS written by other lanes of this wave is visible behind it
-    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
-    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
-    __builtin_amdgcn_wave_barrier();
-}
-
 // ------------------------------------------------------------------------------------------------ choice (one wave per row)
 __device__ __forceinline__ float wave_max64(float v) {
     v = fmaxf(v, pair_in_row<1>(v));

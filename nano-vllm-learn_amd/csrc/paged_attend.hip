@@ -11,6 +11,8 @@ namespace nvh {
 
 namespace {
 
+typedef __bf16 bf16x8_t __attribute__((ext_vector_type(8)));
+
 // ------------------------------------------------------------------------------------------------ prep
 // one workgroup per row; a thread keeps its 8-element pieces of [q | k | v] in registers between the sums and the second pass
 template <typename T, int CH>
@@ -170,10 +172,10 @@ __global__ __launch_bounds__(256) void paged_rows_generic_kernel(const PagedAtte
 }
 
 // ------------------------------------------------------------------------------------------------ rows, streaming (bf16)
-// grid (splits, kv heads x passes, rows), 4 waves.  A wave takes units of UK keys: LPR lanes hold a row of keys or values, so one load instruction covers
-// 64 / LPR rows and the lanes that scored a key also weigh its value: no exchange until the end.  Every group of LPR lanes keeps its own running maximum,
-// sum and output; groups, waves and splits are merged once.  Loads of the next unit's keys are issued behind the scores of this one, its values behind
-// the sums, so about a unit per wave is always in flight.
+// grid (splits, kv heads x passes, rows), 4 waves.  A wave takes units of 32 keys: its keys come as MFMA fragments straight from the page (16 rows x 64 bytes
+// per load), scores of all the pass's heads in one product (lane = head, 8 keys); weights go through a few LDS words to the lanes that hold the values'
+// rows (16 bytes per lane), which sum them on the vector pipe.  Loads of the next unit's keys are issued behind the scores of this one, its values behind the
+// sums, so about a unit per wave is always in flight.  Waves and splits are merged once.
 // Split records (sums, maximum, sum of weights per head): 16-byte write-through stores, drained by every storing wave, then a ticket per (row, key/value
 // head, pass); the last workgroup to arrive reads all records past the L1 and merges them in split order.
 constexpr int kThroughAux = 16;                      // cache policy of the buffer accesses: sc1
@@ -186,39 +188,16 @@ __device__ __forceinline__ f32x4 ld16_through(RecordBuf rb, uint32_t byte_off) {
     return __builtin_bit_cast(f32x4, __builtin_amdgcn_raw_buffer_load_b128(rb, (int)byte_off, 0, kThroughAux));
 }
 
-// this lane's share of a row of W elements: W / LPR of them, in pieces of 8 (and one of 4)
-template <int W, int LPR>
-struct LanePiece {
-    static constexpr int E = W / LPR, P8 = E / 8, P4 = (E % 8) / 4, DW = E / 2;
-    static_assert(E % 4 == 0, "a lane holds whole pieces");
-    static __device__ __forceinline__ int column(int lane, int e) {            // of element e of lane `lane`
-        return e < 8 * P8 ? (e / 8) * 8 * LPR + lane * 8 + (e & 7) : P8 * 8 * LPR + lane * 4 + (e & 3);
-    }
-    static __device__ __forceinline__ void load(const uint16_t* row, int lane, uint32_t (&d)[DW]) {
-#pragma unroll
-        for (int p = 0; p < P8; ++p) {
-            const u32x4 r = __builtin_nontemporal_load(reinterpret_cast<const u32x4*>(row + p * 8 * LPR + lane * 8));
-#pragma unroll
-            for (int k = 0; k < 4; ++k) d[4 * p + k] = r[k];
-        }
-        if constexpr (P4) {
-            const u32x2 r = __builtin_nontemporal_load(reinterpret_cast<const u32x2*>(row + P8 * 8 * LPR + lane * 4));
-            d[4 * P8] = r[0];
-            d[4 * P8 + 1] = r[1];
-        }
-    }
-};
 constexpr int kRowsHeads = 8;                        // query heads a pass holds at most
 
 template <int DK, int DV, int R>
 __global__ __launch_bounds__(256) void paged_rows_kernel(const PagedAttendArgs a) {
-    constexpr int LPR = DK == 64 && DV == 64 ? 8 : 16, SLOTS = 64 / LPR, NI = (DK + DV > 256 ? 4 : 8) / (R == 8 ? 2 : 1), UK = NI * SLOTS;
-    using KL = LanePiece<DK, LPR>;
-    using VL = LanePiece<DV, LPR>;
+    constexpr int UK = 32, STEPS = DK / 32, LPR = DV / 8, SLOTS = 64 / LPR, NV = UK / SLOTS;      // lanes per row of values, rows per load, loads
     constexpr int RECW = DV + 4;                     // floats of one head's record in LDS: sums, max, sum
     __shared__ __attribute__((aligned(16))) float rec[4 * R * RECW];
+    __shared__ __attribute__((aligned(16))) float weights[4][UK * R + R];      // per wave: [key][head], then the factors of the old sums
     __shared__ int last_flag;
-    const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), ll = lane % LPR, ls = lane / LPR;
+    const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lq = lane & 15, lg = lane >> 4, ll = lane % LPR, ls = lane / LPR;
     const int split = blockIdx.x, row = blockIdx.z, ratio = a.heads / a.kv_heads, passes = (ratio + kRowsHeads - 1) / kRowsHeads;
     const int g = blockIdx.y / passes, h0 = g * ratio + (blockIdx.y - g * passes) * kRowsHeads;
     const int nh = (g + 1) * ratio - h0 < R ? (g + 1) * ratio - h0 : R;
@@ -227,92 +206,111 @@ __global__ __launch_bounds__(256) void paged_rows_kernel(const PagedAttendArgs a
     const int per = (vis.count + a.splits - 1) / a.splits, t_beg = split * per, t_end = t_beg + per < vis.count ? t_beg + per : vis.count;
     const int units = t_end > t_beg ? (t_end - t_beg) * (64 / UK) : 0;
 
-    uint32_t q[R][KL::DW];
+    bf16x8_s q[STEPS];                               // B operand: column = head lq (past the last one: that one again, not used)
+    {
+        const uint16_t* qr = reinterpret_cast<const uint16_t*>(a.q) + (int64_t)row * a.q_stride + (int64_t)(h0 + (lq < nh ? lq : nh - 1)) * DK + 8 * lg;
 #pragma unroll
-    for (int r = 0; r < R; ++r) {
-        const uint16_t* qr = reinterpret_cast<const uint16_t*>(a.q) + (int64_t)row * a.q_stride + (int64_t)(h0 + (r < nh ? r : nh - 1)) * DK;
-        KL::load(qr, ll, q[r]);
+        for (int st = 0; st < STEPS; ++st) q[st] = *reinterpret_cast<const bf16x8_s*>(qr + 32 * st);
     }
-    float m[R], l[R], o[R][VL::E];
+    float m = -INFINITY, l = 0.f, o[R][8];           // maximum of head lq; this lane's share of its sum; columns 8 ll .. of every head, keys of slot ls
 #pragma unroll
-    for (int r = 0; r < R; ++r) {
-        m[r] = -INFINITY;
-        l[r] = 0.f;
+    for (int r = 0; r < R; ++r)
 #pragma unroll
-        for (int e = 0; e < VL::E; ++e) o[r][e] = 0.f;
-    }
+        for (int e = 0; e < 8; ++e) o[r][e] = 0.f;
     const float sc = a.scale * kLog2e;
     const int64_t head_elems = (int64_t)a.block_size * (DK + DV);
     const int32_t* table = a.block_tables + (int64_t)row * a.bt_stride;
     auto unit_key = [&](int u) { return vis.tile(t_beg + u / (64 / UK)) * 64 + (u % (64 / UK)) * UK; };
-    uint32_t kd[NI][KL::DW], vd[NI][VL::DW];
+    bf16x8_s kd[2][STEPS];
+    u32x4 vd[NV];
     auto load_k = [&](int k0, int page) {            // rows past the query's own position repeat it: not seen
         const uint16_t* base = reinterpret_cast<const uint16_t*>(a.cache) + ((int64_t)page * a.kv_heads + g) * head_elems;
         const int o0 = k0 % a.block_size - k0;
 #pragma unroll
-        for (int i = 0; i < NI; ++i) {
-            const int key = k0 + i * SLOTS + ls;
-            KL::load(base + (int64_t)((key < pos ? key : pos) + o0) * DK, ll, kd[i]);
+        for (int t = 0; t < 2; ++t) {
+            const int key = k0 + 16 * t + lq;
+            const uint16_t* p = base + (int64_t)((key < pos ? key : pos) + o0) * DK + 8 * lg;
+#pragma unroll
+            for (int st = 0; st < STEPS; ++st) kd[t][st] = *reinterpret_cast<const bf16x8_s*>(p + 32 * st);
         }
     };
     auto load_v = [&](int k0, int page) {
-        const uint16_t* base = reinterpret_cast<const uint16_t*>(a.cache) + ((int64_t)page * a.kv_heads + g) * head_elems + (int64_t)a.block_size * DK;
+        const uint16_t* base = reinterpret_cast<const uint16_t*>(a.cache) + ((int64_t)page * a.kv_heads + g) * head_elems + (int64_t)a.block_size * DK + 8 * ll;
         const int o0 = k0 % a.block_size - k0;
 #pragma unroll
-        for (int i = 0; i < NI; ++i) {
+        for (int i = 0; i < NV; ++i) {
             const int key = k0 + i * SLOTS + ls;
-            VL::load(base + (int64_t)((key < pos ? key : pos) + o0) * DV, ll, vd[i]);
+            vd[i] = __builtin_nontemporal_load(reinterpret_cast<const u32x4*>(base + (int64_t)((key < pos ? key : pos) + o0) * DV));
         }
     };
     // a unit that starts past the query's position (the second half of its tile) holds nothing to see
     auto live = [&](int u) { return u < units && unit_key(u) <= pos; };
     auto page_of = [&](int u) { return table[unit_key(u < units ? u : 0) / a.block_size]; };
+    float* wl = weights[wave];
     // one unit: scores, (the next unit's keys asked for,) softmax, sums, (its values asked for)
     auto take = [&](auto morec, int k0, int next_key, int next_page) {
         constexpr bool MORE = decltype(morec)::value;
-        float s[R][NI];
+        f32x4 s[2] = {f32x4{0.f, 0.f, 0.f, 0.f}, f32x4{0.f, 0.f, 0.f, 0.f}};
 #pragma unroll
-        for (int i = 0; i < NI; ++i) {
-            const int key = k0 + i * SLOTS + ls;
-            // (added, not selected: a select would turn the sums into branches)
-            const float unseen = key <= pos && (a.window <= 0 || pos - key < a.window || key < a.keep_first) ? 0.f : -INFINITY;
+        for (int st = 0; st < STEPS; ++st)
 #pragma unroll
-            for (int r = 0; r < R; ++r) {
-                float acc = 0.f;
-#pragma unroll
-                for (int d = 0; d < KL::DW; ++d) acc = dot2_bf16(kd[i][d], q[r][d], acc);
-                s[r][i] = group_sum<LPR>(acc) * sc + unseen;
-            }
-        }
+            for (int t = 0; t < 2; ++t)
+                s[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, kd[t][st]), __builtin_bit_cast(bf16x8_t, q[st]), s[t], 0, 0, 0);
         if constexpr (MORE) load_k(next_key, next_page);
+        float mx = m;
+#pragma unroll
+        for (int t = 0; t < 2; ++t)
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+                const int key = k0 + 16 * t + 4 * lg + r;
+                const float unseen = key <= pos && (a.window <= 0 || pos - key < a.window || key < a.keep_first) ? 0.f : -INFINITY;
+                s[t][r] = s[t][r] * sc + unseen;
+                mx = fmaxf(mx, s[t][r]);
+            }
+        mx = max_xor16(mx);
+        mx = max_xor32(mx);
+        const float m_use = mx == -INFINITY ? 0.f : mx, alpha = fast_exp2(m - m_use);
+        float sum = 0.f;
+#pragma unroll
+        for (int t = 0; t < 2; ++t)
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+                s[t][r] = fast_exp2(s[t][r] - m_use);
+                sum += s[t][r];
+            }
+        l = l * alpha + sum;
+        m = mx;
+        if (lq < R) {
+#pragma unroll
+            for (int t = 0; t < 2; ++t)
+#pragma unroll
+                for (int r = 0; r < 4; ++r) wl[(16 * t + 4 * lg + r) * R + lq] = s[t][r];
+            if (lg == 0) wl[UK * R + lq] = alpha;
+        }
+        wave_lds_sync();
+        float p[NV][R];
 #pragma unroll
         for (int r = 0; r < R; ++r) {
-            float mx = m[r];
+            const float f = wl[UK * R + r];
 #pragma unroll
-            for (int i = 0; i < NI; ++i) mx = max2(mx, s[r][i]);
-            const float m_use = mx == -INFINITY ? 0.f : mx, alpha = fast_exp2(m[r] - m_use);
-            float sum = 0.f;
-#pragma unroll
-            for (int i = 0; i < NI; ++i) {
-                s[r][i] = fast_exp2(s[r][i] - m_use);
-                sum += s[r][i];
-            }
-            l[r] = l[r] * alpha + sum;
-            m[r] = mx;
-#pragma unroll
-            for (int e = 0; e < VL::E; ++e) o[r][e] *= alpha;
+            for (int e = 0; e < 8; ++e) o[r][e] *= f;
         }
 #pragma unroll
-        for (int i = 0; i < NI; ++i)
+        for (int i = 0; i < NV; ++i)
 #pragma unroll
-            for (int d = 0; d < VL::DW; ++d) {
+            for (int r = 0; r < R; ++r) p[i][r] = wl[(i * SLOTS + ls) * R + r];
+#pragma unroll
+        for (int i = 0; i < NV; ++i)
+#pragma unroll
+            for (int d = 0; d < 4; ++d) {
                 const float v0 = bf16_lo(vd[i][d]), v1 = bf16_hi(vd[i][d]);
 #pragma unroll
                 for (int r = 0; r < R; ++r) {
-                    o[r][2 * d] += s[r][i] * v0;
-                    o[r][2 * d + 1] += s[r][i] * v1;
+                    o[r][2 * d] += p[i][r] * v0;
+                    o[r][2 * d + 1] += p[i][r] * v1;
                 }
             }
+        wave_lds_sync();                             // (the next unit's weights go to the same words)
         if constexpr (MORE) load_v(next_key, next_page);
     };
     int u = wave;
@@ -331,30 +329,23 @@ __global__ __launch_bounds__(256) void paged_rows_kernel(const PagedAttendArgs a
         }
         take(std::integral_constant<bool, false>{}, unit_key(u), 0, 0);
     }
-    // ---- merge the lane groups of the wave, then the waves
+    // ---- merge the value slots of the wave, then the waves
+    l = sum_xor16(l);
+    l = sum_xor32(l);
 #pragma unroll
     for (int r = 0; r < R; ++r) {
-        float mx = m[r];
-        if constexpr (LPR == 8) mx = max2(mx, __shfl_xor(mx, 8));
-        mx = max_xor16(mx);
-        mx = max_xor32(mx);
-        const float f = mx == -INFINITY ? 0.f : fast_exp2(m[r] - mx);
-        float sum = l[r] * f;
-        if constexpr (LPR == 8) sum += __shfl_xor(sum, 8);
-        sum = sum_xor16(sum);
-        sum = sum_xor32(sum);
         float* dst = rec + (wave * R + r) * RECW;
 #pragma unroll
-        for (int e = 0; e < VL::E; ++e) {
-            float v = o[r][e] * f;
-            if constexpr (LPR == 8) v += __shfl_xor(v, 8);
-            v = sum_xor16(v);
+        for (int e = 0; e < 8; ++e) {
+            float v = o[r][e];
+            if constexpr (SLOTS >= 8) v += __shfl_xor(v, 8);
+            if constexpr (SLOTS >= 4) v = sum_xor16(v);
             v = sum_xor32(v);
-            if (ls == 0) dst[VL::column(ll, e)] = v;
+            if (ls == 0) dst[8 * ll + e] = v;
         }
-        if (lane == 0) {
-            dst[DV] = mx;
-            dst[DV + 1] = sum;
+        if (lane == r) {                             // (lane lq = r, lg = 0 holds head r's maximum and sum)
+            dst[DV] = m;
+            dst[DV + 1] = l;
         }
     }
     __syncthreads();

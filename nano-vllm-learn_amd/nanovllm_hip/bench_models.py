@@ -139,14 +139,16 @@ def qwen_attention(size, batch, ctx, seqs, prompt):
     for name, form in (("qwen_prefill_attention", None), ("qwen_prefill_attention_exact", False)):
         us = _time([lambda x=x: old_prefill(x, form) for x in qkv] * 2)
         out[name] = _line(us, 4 * rows * (h + hk) * 128, 4 * 128 * h * pairs)
-    opages = -(-ctx // 256)
-    n = max(2, int(3e8 // (4 * batch * opages * 256 * hk * 128)) + 1)
-    caches = [_randn(2, batch * opages, 256, hk, 128) for _ in range(n)]
-    obt = torch.randperm(batch * opages).view(batch, opages).int().cuda()
-    cl = torch.full((batch,), ctx, dtype=torch.int32, device="cuda")
     oq = _randn(batch, h, 128)
-    us = _time([lambda c=c: ops.flash_attn_with_kvcache(oq, c[0], c[1], cl, obt) for c in caches] * 3)
-    out["qwen_decode_attention"] = _line(us, batch * (4 * ctx * hk * 128 + 4 * h * 128))
+    for name, c in (("qwen_decode_attention", ctx), (f"qwen_decode_attention, context {WINDOW + KEEP}", WINDOW + KEEP)):
+        opages = -(-c // 256)
+        n = max(2, int(3e8 // (4 * batch * opages * 256 * hk * 128)) + 1)
+        caches = [_randn(2, batch * opages, 256, hk, 128) for _ in range(n)]
+        obt = torch.randperm(batch * opages).view(batch, opages).int().cuda()
+        cl = torch.full((batch,), c, dtype=torch.int32, device="cuda")
+        us = _time([lambda kv=kv: ops.flash_attn_with_kvcache(oq, kv[0], kv[1], cl, obt) for kv in caches] * 3)
+        out[name] = _line(us, batch * (4 * c * hk * 128 + 4 * h * 128))
+        del caches
     return out
 
 
