@@ -289,12 +289,13 @@ __global__ __launch_bounds__(64 * MW * NW) void moe_gemm_kernel(const MoeGemmArg
     extern __shared__ __attribute__((aligned(16))) unsigned char lds[];        // [ring][TN weight rows | TM pairs][64 bytes]
     int nt, mt;
     {
-        // one XCD takes a run of column tiles of the same pairs: the gathered rows and the expert's weights are shared in its L2
-        const int total = (int)gridDim.x * a.tiles[3], lin = (int)(blockIdx.x + gridDim.x * blockIdx.y), per = total >> 3;
+        // one XCD takes a run of the tiles, eight row tiles times the columns at a time, rows first: what runs at once shares rows and weights in its L2
+        const int nx = gridDim.x, tiles = a.tiles[3], total = nx * tiles, lin = (int)(blockIdx.x + gridDim.x * blockIdx.y), per = total >> 3;
         if (lin >= total) return;
         const int idx = lin < per * 8 ? (lin & 7) * per + (lin >> 3) : lin;
-        mt = idx / (int)gridDim.x;
-        nt = idx - mt * (int)gridDim.x;
+        const int g = idx / (8 * nx), in = idx - g * 8 * nx, gm = tiles - 8 * g < 8 ? tiles - 8 * g : 8;
+        nt = in / gm;
+        mt = 8 * g + in - nt * gm;
     }
     const int expert = a.tiles[4 * mt], first = a.tiles[4 * mt + 1], live = a.tiles[4 * mt + 2];
     const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lq = lane & 15, lg = lane >> 4, wm = wave / NW, wn = wave % NW;
@@ -381,26 +382,37 @@ __global__ __launch_bounds__(64 * MW * NW) void moe_gemm_kernel(const MoeGemmArg
         spread();
     }
     asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+    // ---- results through LDS (the images are done with): a wave's MT * 16 pairs by CW columns, then whole rows of them to memory
+    lds_only_barrier();
+    constexpr int CW = GLU ? NT * 8 : NT * 16, CP = CW / 8;                    // columns of a wave, 16-byte pieces of a row
+    unsigned char* tile = lds + wave * MT * 16 * CW * 2;
+    auto put = [&](int r, int col, f32x4 v) {        // columns col .. + 3 of row r
+        act_st4(reinterpret_cast<uint16_t*>(tile + r * CW * 2 + (((col >> 3) ^ (r & (CP - 1))) * 16 + (col & 4) * 2)), v);
+    };
 #pragma unroll
     for (int j = 0; j < MT; ++j) {
-        const int R = (wm * MT + j) * 16 + lq;
-        if (R >= live) continue;
-        uint16_t* out = reinterpret_cast<uint16_t*>(a.out) + (int64_t)a.slot_pair[first + R] * a.n;
         if constexpr (GLU) {
 #pragma unroll
             for (int i = 0; i < NT / 2; ++i) {
-                const int col = nt * OUTS + (wn * NT / 2 + i) * 16 + 4 * lg;
                 f32x4 v;
 #pragma unroll
                 for (int r = 0; r < 4; ++r) v[r] = silu_f(acc[2 * i][j][r]) * acc[2 * i + 1][j][r];
-                if (col < a.n) act_st4(out + col, v);
+                put(16 * j + lq, 16 * i + 4 * lg, v);
             }
         } else {
 #pragma unroll
-            for (int i = 0; i < NT; ++i) {
-                const int col = nt * OUTS + (wn * NT + i) * 16 + 4 * lg;
-                if (col < a.n) act_st4(out + col, acc[i][j]);
-            }
+            for (int i = 0; i < NT; ++i) put(16 * j + lq, 16 * i + 4 * lg, acc[i][j]);
+        }
+    }
+    wave_lds_sync();
+    const int col = nt * OUTS + wn * CW + (lane % CP) * 8;
+    if (col < a.n) {                                 // (n is a multiple of 64: whole pieces)
+#pragma unroll
+        for (int k = 0; k < MT * 16 * CP / 64; ++k) {
+            const int r = (k * 64 + lane) / CP, R = wm * MT * 16 + r;
+            if (R < live)
+                *reinterpret_cast<u32x4*>(reinterpret_cast<uint16_t*>(a.out) + (int64_t)a.slot_pair[first + R] * a.n + col) =
+                    *reinterpret_cast<const u32x4*>(tile + r * CW * 2 + ((lane % CP) ^ (r & (CP - 1))) * 16);
         }
     }
 }
@@ -602,7 +614,7 @@ int launch_moe_dispatch(int32_t* slot_pair, int32_t* tiles, int32_t* counts, con
     return check_launch("moe_scatter");
 }
 
-int moe_tile_rows(int pairs, int experts, int f32) { return f32 ? FM : pairs / experts >= 512 ? 256 : 128; }
+int moe_tile_rows(int pairs, int experts, int f32) { return f32 ? FM : pairs / experts >= 256 ? 256 : 128; }
 
 int launch_moe_gemm(const MoeGemmArgs& a, int f32, hipStream_t stream) {
     if (f32) {
