@@ -449,8 +449,8 @@ __device__ __forceinline__ void moe_small_tile(const MoeGemmArgs& a, int expert,
         bf16x8 wg[UN], wu[UN], xf[UN][MT];
 #pragma unroll
         for (int i = 0; i < UN; ++i) {
-            wg[i] = __builtin_nontemporal_load(reinterpret_cast<const bf16x8*>(w + 32 * (s + i)));
-            if constexpr (GLU) wu[i] = __builtin_nontemporal_load(reinterpret_cast<const bf16x8*>(w + up + 32 * (s + i)));
+            wg[i] = *reinterpret_cast<const bf16x8*>(w + 32 * (s + i));    // (half of a 128-byte line: a streaming hint would drop the other half)
+            if constexpr (GLU) wu[i] = *reinterpret_cast<const bf16x8*>(w + up + 32 * (s + i));
         }
 #pragma unroll
         for (int i = 0; i < UN; ++i)
@@ -623,7 +623,7 @@ int launch_moe_gemm(const MoeGemmArgs& a, int f32, hipStream_t stream) {
         else moe_gemm_f32_kernel<false><<<grid, 256, 0, stream>>>(a);
     } else if (!a.tiles) {
         const int tiles = a.n / 16, busy = a.pairs < a.experts ? a.pairs : a.experts;
-        const bool split = (int64_t)busy * tiles < 4 * 512;                    // too few waves with a tile each: four share one
+        const bool split = a.k >= 2048 || (int64_t)busy * tiles < 4 * 512;     // a long contraction, or too few waves with a tile each: four share one
         const dim3 grid(split ? tiles : (tiles + 3) / 4, a.experts);
         if (a.glu && split) moe_small_kernel<true, true><<<grid, 256, 0, stream>>>(a);
         else if (a.glu) moe_small_kernel<true, false><<<grid, 256, 0, stream>>>(a);
