@@ -442,8 +442,10 @@ int nvh_allreduce_oneshot(void* out, const void* x, void* packed, void* const* s
  * cache row and matrix operand is then float).  Widths ("cols") may be padded with zeros; the counts a mean runs over are given apart.
  */
 /* x[rows, cols] (fp32) = embed[token] * scale; xb (nullable): the same in the activation type; packed
- * (nullable, bf16, cols % 32 == 0): in fragment order.  Tokens outside [0, vocab) are clamped. */
-int nvh_embed_rows(float* x, void* xb, void* packed, const int64_t* tokens, const void* embed, float scale, int rows, int cols, int vocab, int dtype, void* stream);
+ * (nullable, bf16, cols % 32 == 0): in fragment order.  Tokens outside [0, vocab) are clamped.  table (nullable, fp32 [max_position, cols]): row
+ * positions[row] of it is added; copy (nullable): the fp32 rows a second time. */
+int nvh_embed_rows(float* x, void* xb, void* packed, const int64_t* tokens, const void* embed, float scale, int rows, int cols, int vocab, float* copy,
+                   const int64_t* positions, const float* table, int max_position, int dtype, void* stream);
 /* x += rmsnorm(y) * w (y given), or the result = rmsnorm(x) * w with x unchanged (y NULL). */
 typedef struct nvh_norm_residual_desc {
     float* x;                    /* [rows, cols] fp32 residual stream */
@@ -587,6 +589,7 @@ typedef struct nvh_attn_prep_desc {
     void* cache;
     const int32_t* slots;        /* [rows] page * block_size + offset; < 0: not stored */
     int32_t block_size;
+    int32_t head_norm;           /* != 0: the norms run over every head by itself; q_w and k_w are [dk], shared by the heads, q_n and k_n the columns of a head */
 } nvh_attn_prep_desc;
 int nvh_attn_prep(const nvh_attn_prep_desc* d, int dtype, void* stream);
 /* softmax(scale q . k) v over the keys a query sees: position j of its sequence if j <= its own and (window == 0 or nearer than `window` or
@@ -616,11 +619,24 @@ typedef struct nvh_paged_attend_desc {
     void* out;                   /* nullable: [rows, heads * dv], row stride out_stride */
     int64_t out_stride;
     void* out_packed;            /* nullable (bf16, rows form): the same in MFMA-fragment order */
+    const float* talk;           /* nvh_talk_*: [heads, heads]; NULL otherwise */
+    float softcap;               /* nvh_talk_*: 0 or the cap */
+    float* scores;               /* nvh_talk_rows: [rows, span, nvh_talk_score_cols(heads)] scratch */
+    int32_t span;                /* 64 times the most 64-key tiles a row sees */
 } nvh_paged_attend_desc;
 int nvh_paged_attend_supported(int dk, int dv, int block_size);
 size_t nvh_paged_attend_ticket_bytes(int rows, int kv_heads, int heads);
 int nvh_paged_attend_rows(const nvh_paged_attend_desc* d, int generic, int dtype, void* stream);
 int nvh_paged_attend_prompt(const nvh_paged_attend_desc* d, int dtype, void* stream);
+
+/* The same attention with scores capped, softcap tanh(scale q . k / softcap), and then mixed across the heads, score_h <- sum_g talk[h][g] score_g, before the
+ * softmax.  nvh_talk_rows is two launches (scores to memory, then the rest); nvh_talk_prompt is one, all heads of 16 rows in a workgroup. */
+int nvh_talk_rows_supported(int heads, int dk, int dv, int block_size);
+int nvh_talk_score_cols(int heads);
+size_t nvh_talk_ticket_bytes(int rows, int kv_heads, int heads);
+int nvh_talk_rows(const nvh_paged_attend_desc* d, int generic, int dtype, void* stream);
+int nvh_talk_prompt_supported(int heads, int dk, int dv, int block_size);
+int nvh_talk_prompt(const nvh_paged_attend_desc* d, int dtype, void* stream);
 
 /* Lightning attention: per head S = decay S + k v^T, o = S^T q with q, k, v = silu of the projection's columns (rounded to the activation type);
  * the state is fp32.  nvh_lightning_chunks: portions cut into segments as for nvh_rglru_chunks; nvh_lightning_step: row i is one new token of
@@ -650,7 +666,8 @@ int nvh_norm_gate(void* out, void* packed, const void* x, const void* gate, cons
 
 /* Mixture of experts.  Route: s = sigmoid(h . router_e) in 32-bit; choice scores s + correction; the experts form `groups` equal groups of neighbours,
  * a group counts the sum of its two largest choice scores, the best `keep` groups stay open, the `top` largest choice scores among them win;
- * weights s / (sum + 1e-20) * scale.  Pair p = row * top + k. */
+ * weights s / (sum + 1e-20) * scale.  softmax != 0: the scores are the logits themselves, `correction` a bias on them (choice and weights), groups 1, the weights
+ * the softmax over the chosen scores, times scale.  Pair p = row * top + k. */
 typedef struct nvh_moe_route_desc {
     const void* x;               /* [rows, cols], row stride x_stride */
     int64_t x_stride;
@@ -660,6 +677,7 @@ typedef struct nvh_moe_route_desc {
     float scale;
     int32_t* ids;                /* [rows, top] */
     float* weights;              /* [rows, top] */
+    int32_t softmax;
 } nvh_moe_route_desc;
 int nvh_moe_route(const nvh_moe_route_desc* d, int dtype, void* stream);
 /* Pairs sorted by expert: slot_pair[slot], tiles [max_tiles][4] = (expert, first slot, slots, tiles in use), unused ones with
@@ -667,7 +685,8 @@ int nvh_moe_route(const nvh_moe_route_desc* d, int dtype, void* stream);
  * counts: [nvh_moe_dispatch_blocks(pairs), experts] scratch.  max_tiles >= pairs / tile_rows + experts. */
 int nvh_moe_dispatch_blocks(int pairs);
 int nvh_moe_dispatch(int32_t* slot_pair, int32_t* tiles, int32_t* counts, const int32_t* ids, int pairs, int experts, int tile_rows, int max_tiles, void* stream);
-/* Expert products.  glu: act[p] = silu(x[p / top] . gate_e) * (x . up_e), w = [experts, 2 * n, k] (gate rows, then up rows); otherwise
+/* Expert products.  glu: act[p] = silu(x[p / top] . gate_e) * (x . up_e), w = [experts, 2 * n, k] (gate rows, then up rows), or with alpha != 0 the clamped unit
+ * g sigmoid(alpha g) (u + 1), g = min(gate, limit), u = clamp(up, -limit, limit); otherwise
  * out[p] = x[p] . w_e, w = [experts, n, k].
  * tiles == NULL: small batches (bf16, at most 64 rows), the pairs of an expert found from ids; otherwise tiles of tile_rows from
  * nvh_moe_dispatch (bf16: 128 or 256, f32: 64; nvh_moe_tile_rows picks).  n and k multiples of 64. */
@@ -681,12 +700,13 @@ typedef struct nvh_moe_gemm_desc {
     const int32_t* slot_pair;    /* [pairs] */
     const int32_t* tiles;
     int32_t max_tiles, tile_rows;
+    float limit, alpha;
 } nvh_moe_gemm_desc;
 int nvh_moe_tile_rows(int pairs, int experts, int dtype);
 int nvh_moe_gemm(const nvh_moe_gemm_desc* d, int dtype, void* stream);
 
-/* x (fp32 stream) += y + sum_k ew[row, k] * e[row * top + k]  (each part nullable), then, with w given, the layer norm of the new row:
- * (x - mean) / sqrt(var + eps) * w + b. */
+/* x (fp32 stream) += mult * P(y + sum_k ew[row, k] * e[row * top + k])  (each part nullable; P: the layer norm with post_w and post_b where given, nothing
+ * otherwise), x += base, x += shift, then, with w given, the layer norm of the new row: (x - mean) / sqrt(var + eps) * w + b. */
 typedef struct nvh_residual_norm_desc {
     float* x;                    /* [rows, cols] */
     const void* y;               /* nullable: [rows, cols], row stride y_stride */
@@ -700,8 +720,15 @@ typedef struct nvh_residual_norm_desc {
     int32_t rows, cols, n;       /* n: elements mean and variance run over */
     void* xb;                    /* nullable: the normed rows in the activation type */
     void* packed;                /* nullable (bf16): the same in MFMA-fragment order */
+    const float* post_w;         /* nullable: [cols] */
+    const float* post_b;
+    float mult;
+    const float* base;           /* nullable: [rows, cols] */
+    const float* shift;          /* nullable: [cols] */
 } nvh_residual_norm_desc;
 int nvh_residual_norm(const nvh_residual_norm_desc* d, int dtype, void* stream);
+/* out = coef[0] N(z) + coef[1] N(z^2) + coef[2] N(z^3) + coef[3], powers by element, N(v) = v / sqrt(mean over n columns of v^2 + eps); zero past n. */
+int nvh_poly_norm(void* out, void* packed, const void* z, const float* coef, float eps, int rows, int cols, int n, int64_t z_stride, int64_t out_stride, int dtype, void* stream);
 /* x = cap * tanh(x / cap) in place, rows of `cols` elements. */
 int nvh_softcap(void* x, float cap, int rows, int cols, int64_t stride, int dtype, void* stream);
 

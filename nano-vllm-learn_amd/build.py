@@ -22,11 +22,12 @@ LIB = os.path.join(OUT_DIR, "libnvh_attn.so")
 LINEAR_SOURCES = ["api_layers.hip", "api_rows.hip", "layer_ops.hip", "skinny_gemm.hip", "linear_stream.hip", "hybrid_ops.hip"]
 MODEL_SOURCES = {
     "Zobasun": ["api_hybrid.hip", "rglru.hip", "latent_attention.hip", "latent_prefill.hip"],
-    "Galirax": ["api_mixers.hip", "paged_attend.hip", "paged_prompt.hip", "lightning.hip", "moe.hip"],
+    "Galirax": ["api_paged.hip", "attn_prep.hip", "paged_attend.hip", "paged_prompt.hip", "api_lightning.hip", "lightning.hip", "api_moe.hip", "moe.hip"],
+    "Kekapel": ["api_talk.hip", "attn_prep.hip", "talk_rows.hip", "talk_prompt.hip", "api_moe.hip", "moe.hip"],
 }
 SOURCES = ["api.hip", "store_kvcache.hip", "paged_decode.hip", "prefill_mfma.hip", "rope_store.hip", "allreduce_oneshot.hip", "qkv_attend.hip", *LINEAR_SOURCES,
-           *[s for sources in MODEL_SOURCES.values() for s in sources]]
-HEADERS = ["common.h", "kernels.h", "hybrid.h", "mixers.h", "attend_tile.h", "api_common.h", "decode_chunked.h", os.path.join("..", "..", "include", "nvh_attn.h")]
+           *dict.fromkeys(s for sources in MODEL_SOURCES.values() for s in sources)]
+HEADERS = ["common.h", "kernels.h", "hybrid.h", "mixers.h", "attend_tile.h", "paged_rows.h", "talk.h", "api_common.h", "decode_chunked.h", os.path.join("..", "..", "include", "nvh_attn.h")]
 HIPCC = os.environ.get("HIPCC", "/opt/rocm/bin/hipcc")
 # -amdgpu-mfma-vgpr-form: MFMA results stay in the architectural VGPRs.  By default hipcc parks accumulators in the AGPR file
 # and pays a v_accvgpr_read/write per element wherever VALU code touches them (softmax on S, rescale of O): 159 such moves in

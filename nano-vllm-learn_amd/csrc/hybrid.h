@@ -40,7 +40,8 @@ __device__ __forceinline__ float block_sum256(float v, float* lds) {
 }
 
 // ---- row-wise ops (hybrid_ops.hip)
-int launch_embed_rows(float* x, void* xb, void* packed, const int64_t* tokens, const void* embed, float scale, int rows, int cols, int vocab, int f32, hipStream_t stream);
+int launch_embed_rows(float* x, void* xb, void* packed, const int64_t* tokens, const void* embed, float scale, int rows, int cols, int vocab, float* copy,
+                      const int64_t* positions, const float* table, int max_position, int f32, hipStream_t stream);
 using NormResidualArgs = nvh_norm_residual_desc;
 int launch_norm_residual(const NormResidualArgs& a, int f32, hipStream_t stream);
 int launch_clamped_glu(void* out, const void* gate_up, int rows, int inter, int64_t gu_stride, int64_t out_stride, float limit, float alpha, int f32, hipStream_t stream);

@@ -15,14 +15,21 @@ using ResidualNormArgs = nvh_residual_norm_desc;
 constexpr int kRowPieces = 16;                       // 8-element pieces a thread of a row kernel holds at most: rows of up to 256 * 16 * 8 elements
 constexpr int kMaxRowCols = 256 * kRowPieces * 8;
 constexpr int kAttendTicketWords = 32;               // one arrival ticket per 128-byte line
+constexpr int kRowsHeads = 8;                        // query heads of one key/value head a pass over single rows holds at most
 constexpr int kLightningChunk = 64;                  // tokens a workgroup takes at a time
 constexpr int kMoeMaxExperts = 1024;
 
 int launch_attn_prep(const AttnPrepArgs& a, int f32, hipStream_t stream);
 bool paged_attend_supported(int dk, int dv, int block_size);
-int paged_attend_groups(int heads, int kv_heads);    // passes over the query heads of one key/value head
+inline int paged_attend_groups(int heads, int kv_heads) { return (heads / kv_heads + kRowsHeads - 1) / kRowsHeads; }      // passes per key/value head
 int launch_paged_attend_rows(const PagedAttendArgs& a, int f32, int generic, hipStream_t stream);
 int launch_paged_attend_prompt(const PagedAttendArgs& a, hipStream_t stream);
+
+__host__ __device__ constexpr int score_cols(int heads) { return (heads + 3) / 4 * 4; }          // row length of PagedAttendArgs::scores
+bool talk_rows_supported(int heads, int dk, int dv, int block_size);
+int launch_talk_rows(const PagedAttendArgs& a, int f32, int generic, hipStream_t stream);
+bool talk_prompt_supported(int heads, int dk, int dv, int block_size);
+int launch_talk_prompt(const PagedAttendArgs& a, hipStream_t stream);
 
 bool lightning_supported(int dk, int dv);
 int launch_lightning_chunks(const LightningArgs& a, int f32, int generic, hipStream_t stream);
@@ -38,6 +45,8 @@ int moe_tile_rows(int pairs, int experts, int f32);
 int launch_moe_gemm(const MoeGemmArgs& a, int f32, hipStream_t stream);
 
 int launch_residual_norm(const ResidualNormArgs& a, int f32, hipStream_t stream);
+int launch_poly_norm(void* out, void* packed, const void* z, const float* coef, float eps, int rows, int cols, int n, int64_t z_stride, int64_t out_stride, int f32,
+                     hipStream_t stream);
 int launch_softcap(void* x, float cap, int rows, int cols, int64_t stride, int f32, hipStream_t stream);
 
 // ---- 8 elements of an activation row
@@ -74,6 +83,20 @@ __device__ __forceinline__ void block_sum256x2(float& u, float& v, float* lds) {
     __syncthreads();
     u = lds[0] + lds[1] + lds[2] + lds[3];
     v = lds[4] + lds[5] + lds[6] + lds[7];
+}
+
+// sums of N values over a 256-thread workgroup; `lds` holds 4 * N floats and is free again after the next barrier
+template <int N>
+__device__ __forceinline__ void block_sums256(float (&v)[N], float* lds) {
+#pragma unroll
+    for (int i = 0; i < N; ++i) v[i] = wave_sum64(v[i]);
+    if ((threadIdx.x & 63) == 0) {
+#pragma unroll
+        for (int i = 0; i < N; ++i) lds[4 * i + (threadIdx.x >> 6)] = v[i];
+    }
+    __syncthreads();
+#pragma unroll
+    for (int i = 0; i < N; ++i) v[i] = lds[4 * i] + lds[4 * i + 1] + lds[4 * i + 2] + lds[4 * i + 3];
 }
 
 __device__ __forceinline__ void wave_lds_sync() {    // LDS written by other lanes of this wave is visible behind it

@@ -1,7 +1,7 @@
-// Mixture of experts with a sigmoid router, choice corrections and expert groups.
-//   route     32-bit logits of a row tile against every expert (MFMA for bf16), sigmoid, group and expert choice, weights: one launch
+// Mixture of experts; the router's scores are sigmoids with choice corrections and expert groups, or a softmax over the chosen logits.
+//   route     32-bit logits of a row tile against every expert (MFMA for bf16), group and expert choice, weights: one launch
 //   dispatch  pairs (row, chosen expert) sorted by expert and cut into tiles of one expert each: two launches, no host round trip
-//   gemm      expert products: gate | up with the SiLU product in the epilogue, and down.  Large batches: 128 x 128 or 256 x 256 MFMA tiles over the
+//   gemm      expert products: gate | up with the gated unit in the epilogue, and down.  Large batches: 128 x 128 or 256 x 256 MFMA tiles over the
 //             sorted pairs, the rows gathered by the DMA that fills LDS.  At most 64 rows: every wave streams 16 weight rows once for all the rows that chose the expert.
 // Outputs stay per pair; the weighted sum over a row's experts belongs to the residual add (hybrid_ops.hip).
 #include "attend_tile.h"
@@ -44,15 +44,20 @@ __device__ __forceinline__ void store_choice(const MoeRouteArgs& a, int row, int
     }
 }
 
+// score of an expert from its logit
+__device__ __forceinline__ float expert_score(const MoeRouteArgs& a, float z, int e) { return a.softmax ? z + a.correction[e] : 1.f / (1.f + expf(-z)); }
+// its part of the weights, with `top` the score of the first choice (a softmax is taken relative to its largest entry)
+__device__ __forceinline__ float expert_part(const MoeRouteArgs& a, float score, float top) { return a.softmax ? expf(score - top) : score; }
+
 // z [E]: logits in, scores out; choice [E], gs [groups]: scratch in LDS.  Up to 64 experts: one per lane, LDS for the group scores only.
 __device__ __forceinline__ void choose_experts(const MoeRouteArgs& a, int row, int lane, float* z, float* choice, float* gs) {
     const int size = a.experts / a.groups;
-    float total = 0.f, mine = 0.f;
+    float total = 0.f, mine = 0.f, top = 0.f;
     int my_id = 0;
     if (a.experts <= 64) {
         const bool ok = lane < a.experts;
-        const float s = ok ? 1.f / (1.f + expf(-z[lane])) : 0.f;
-        float c = ok ? s + a.correction[lane] : -INFINITY;
+        const float s = ok ? expert_score(a, z[lane], lane) : 0.f;
+        float c = ok ? (a.softmax ? s : s + a.correction[lane]) : -INFINITY;
         if (a.keep < a.groups) {
             choice[lane] = c;
             wave_lds_sync();
@@ -67,7 +72,9 @@ __device__ __forceinline__ void choose_experts(const MoeRouteArgs& a, int row, i
         }
         for (int k = 0; k < a.top; ++k) {
             const int w = wave_winner(c);
-            const float sw = lane_value(s, w);
+            const float score = lane_value(s, w);
+            if (k == 0) top = score;
+            const float sw = expert_part(a, score, top);
             total += sw;
             if (lane == k) {
                 mine = sw;
@@ -79,9 +86,9 @@ __device__ __forceinline__ void choose_experts(const MoeRouteArgs& a, int row, i
         return;
     }
     for (int e = lane; e < a.experts; e += 64) {
-        const float s = 1.f / (1.f + expf(-z[e]));
+        const float s = expert_score(a, z[e], e);
         z[e] = s;
-        choice[e] = s + a.correction[e];
+        choice[e] = a.softmax ? s : s + a.correction[e];
     }
     wave_lds_sync();
     auto best = [&](const float* list, int n) {      // index of the list's largest value
@@ -110,7 +117,8 @@ __device__ __forceinline__ void choose_experts(const MoeRouteArgs& a, int row, i
     }
     for (int k = 0; k < a.top; ++k) {
         const int e = best(choice, a.experts);
-        const float s = z[e];
+        if (k == 0) top = z[e];
+        const float s = expert_part(a, z[e], top);
         total += s;
         if (lane == k) {
             mine = s;
@@ -275,6 +283,8 @@ __global__ __launch_bounds__(256) void moe_scatter_kernel(int32_t* __restrict__ 
 // ring of four images: three are on their way while the fourth is read into registers, and the one before it is multiplied from there.
 // GLU: weight rows alternate 16 of gate, 16 of up, so a lane holds both halves of its outputs.
 constexpr int TK = 32, kRing = 4;
+// SiLU(g) u, or the clamped unit where the launch names an alpha
+__device__ __forceinline__ float expert_unit(const MoeGemmArgs& a, float g, float u) { return a.alpha != 0.f ? clamped_glu(g, u, a.limit, a.alpha) : silu_f(g) * u; }
 template <int MW, int NW, int MT, int NT>
 struct GemmShape {
     static constexpr int WAVES = MW * NW, TM = MW * MT * 16, TN = NW * NT * 16, ROWS = TM + TN, IMG = ROWS * TK * 2, DMA = IMG / 1024 / WAVES;
@@ -396,7 +406,7 @@ __global__ __launch_bounds__(64 * MW * NW) void moe_gemm_kernel(const MoeGemmArg
             for (int i = 0; i < NT / 2; ++i) {
                 f32x4 v;
 #pragma unroll
-                for (int r = 0; r < 4; ++r) v[r] = silu_f(acc[2 * i][j][r]) * acc[2 * i + 1][j][r];
+                for (int r = 0; r < 4; ++r) v[r] = expert_unit(a, acc[2 * i][j][r], acc[2 * i + 1][j][r]);
                 put(16 * j + lq, 16 * i + 4 * lg, v);
             }
         } else {
@@ -498,7 +508,7 @@ __device__ __forceinline__ void moe_small_tile(const MoeGemmArgs& a, int expert,
         f32x4 v = g[m];
         if constexpr (GLU) {
 #pragma unroll
-            for (int r = 0; r < 4; ++r) v[r] = silu_f(g[m][r]) * u[m][r];
+            for (int r = 0; r < 4; ++r) v[r] = expert_unit(a, g[m][r], u[m][r]);
         }
         act_st4(reinterpret_cast<uint16_t*>(a.out) + (int64_t)list[16 * m + lq] * a.n + n0 + 4 * lg, v);
     }
@@ -580,7 +590,17 @@ __global__ __launch_bounds__(256) void moe_gemm_f32_kernel(const MoeGemmArgs a) 
         if (tm + i >= live) continue;
         f32x4 v;
 #pragma unroll
-        for (int j = 0; j < 4; ++j) v[j] = GLU ? g[i][j] / (1.f + expf(-g[i][j])) * u[i][j] : g[i][j];
+        for (int j = 0; j < 4; ++j) {
+            v[j] = g[i][j];
+            if constexpr (GLU) {
+                if (a.alpha != 0.f) {
+                    const float gate = fminf(g[i][j], a.limit);
+                    v[j] = gate / (1.f + expf(-a.alpha * gate)) * (fminf(fmaxf(u[i][j], -a.limit), a.limit) + 1.f);
+                } else {
+                    v[j] = g[i][j] / (1.f + expf(-g[i][j])) * u[i][j];
+                }
+            }
+        }
         *reinterpret_cast<f32x4*>(reinterpret_cast<float*>(a.out) + (int64_t)a.slot_pair[first + tm + i] * a.n + n0 + tn) = v;
     }
 }

@@ -86,7 +86,7 @@ class AttnPrepDesc(ctypes.Structure):
                 ("kv_heads", ctypes.c_int32), ("dk", ctypes.c_int32), ("dv", ctypes.c_int32), ("q_w", ctypes.c_void_p),
                 ("k_w", ctypes.c_void_p), ("q_n", ctypes.c_int32), ("k_n", ctypes.c_int32), ("eps", ctypes.c_float),
                 ("positions", ctypes.c_void_p), ("cos_sin", ctypes.c_void_p), ("max_position", ctypes.c_int32), ("rot", ctypes.c_int32),
-                ("cache", ctypes.c_void_p), ("slots", ctypes.c_void_p), ("block_size", ctypes.c_int32)]
+                ("cache", ctypes.c_void_p), ("slots", ctypes.c_void_p), ("block_size", ctypes.c_int32), ("head_norm", ctypes.c_int32)]
 
 
 class PagedAttendDesc(ctypes.Structure):
@@ -98,7 +98,8 @@ class PagedAttendDesc(ctypes.Structure):
                 ("batch", ctypes.c_int32), ("max_q", ctypes.c_int32), ("scale", ctypes.c_float), ("window", ctypes.c_int32),
                 ("keep_first", ctypes.c_int32), ("sink", ctypes.c_void_p), ("splits", ctypes.c_int32), ("part", ctypes.c_void_p),
                 ("tickets", ctypes.c_void_p), ("out", ctypes.c_void_p), ("out_stride", ctypes.c_int64),
-                ("out_packed", ctypes.c_void_p)]
+                ("out_packed", ctypes.c_void_p), ("talk", ctypes.c_void_p), ("softcap", ctypes.c_float), ("scores", ctypes.c_void_p),
+                ("span", ctypes.c_int32)]
 
 
 class LightningDesc(ctypes.Structure):
@@ -114,7 +115,7 @@ class MoeRouteDesc(ctypes.Structure):
     _fields_ = [("x", ctypes.c_void_p), ("x_stride", ctypes.c_int64), ("router", ctypes.c_void_p), ("correction", ctypes.c_void_p),
                 ("rows", ctypes.c_int32), ("cols", ctypes.c_int32), ("experts", ctypes.c_int32), ("top", ctypes.c_int32),
                 ("groups", ctypes.c_int32), ("keep", ctypes.c_int32), ("scale", ctypes.c_float), ("ids", ctypes.c_void_p),
-                ("weights", ctypes.c_void_p)]
+                ("weights", ctypes.c_void_p), ("softmax", ctypes.c_int32)]
 
 
 class MoeGemmDesc(ctypes.Structure):
@@ -122,7 +123,8 @@ class MoeGemmDesc(ctypes.Structure):
     _fields_ = [("out", ctypes.c_void_p), ("x", ctypes.c_void_p), ("x_stride", ctypes.c_int64), ("w", ctypes.c_void_p),
                 ("pairs", ctypes.c_int32), ("top", ctypes.c_int32), ("experts", ctypes.c_int32), ("n", ctypes.c_int32),
                 ("k", ctypes.c_int32), ("glu", ctypes.c_int32), ("ids", ctypes.c_void_p), ("slot_pair", ctypes.c_void_p),
-                ("tiles", ctypes.c_void_p), ("max_tiles", ctypes.c_int32), ("tile_rows", ctypes.c_int32)]
+                ("tiles", ctypes.c_void_p), ("max_tiles", ctypes.c_int32), ("tile_rows", ctypes.c_int32),
+                ("limit", ctypes.c_float), ("alpha", ctypes.c_float)]
 
 
 class ResidualNormDesc(ctypes.Structure):
@@ -130,7 +132,8 @@ class ResidualNormDesc(ctypes.Structure):
     _fields_ = [("x", ctypes.c_void_p), ("y", ctypes.c_void_p), ("y_stride", ctypes.c_int64), ("e", ctypes.c_void_p),
                 ("ew", ctypes.c_void_p), ("top", ctypes.c_int32), ("w", ctypes.c_void_p), ("b", ctypes.c_void_p), ("eps", ctypes.c_float),
                 ("rows", ctypes.c_int32), ("cols", ctypes.c_int32), ("n", ctypes.c_int32), ("xb", ctypes.c_void_p),
-                ("packed", ctypes.c_void_p)]
+                ("packed", ctypes.c_void_p), ("post_w", ctypes.c_void_p), ("post_b", ctypes.c_void_p), ("mult", ctypes.c_float),
+                ("base", ctypes.c_void_p), ("shift", ctypes.c_void_p)]
 
 
 EPI_NONE, EPI_SILU_MUL, EPI_RESIDUAL_ADD, EPI_ROPE_STORE = 0, 1, 2, 3
@@ -203,7 +206,7 @@ _SIGS = {
                                                                       ctypes.c_void_p] +
                                             [ctypes.c_void_p, ctypes.c_int, ctypes.c_int, ctypes.c_void_p, ctypes.c_int64, ctypes.c_void_p, ctypes.c_int,
                                              ctypes.c_void_p]),
-    "nvh_embed_rows": (ctypes.c_int, [ctypes.c_void_p] * 5 + [ctypes.c_float] + [ctypes.c_int] * 4 + [ctypes.c_void_p]),
+    "nvh_embed_rows": (ctypes.c_int, [ctypes.c_void_p] * 5 + [ctypes.c_float] + [ctypes.c_int] * 3 + [ctypes.c_void_p] * 3 + [ctypes.c_int] * 2 + [ctypes.c_void_p]),
     "nvh_norm_residual": (ctypes.c_int, [ctypes.POINTER(NormResidualDesc), ctypes.c_int, ctypes.c_void_p]),
     "nvh_clamped_glu": (ctypes.c_int, [ctypes.c_void_p] * 2 + [ctypes.c_int] * 2 + [ctypes.c_int64] * 2 + [ctypes.c_float] * 2 + [ctypes.c_int, ctypes.c_void_p]),
     "nvh_rglru_chunk_tokens": (ctypes.c_int, []),
@@ -221,6 +224,12 @@ _SIGS = {
     "nvh_paged_attend_ticket_bytes": (ctypes.c_size_t, [ctypes.c_int] * 3),
     "nvh_paged_attend_rows": (ctypes.c_int, [ctypes.POINTER(PagedAttendDesc), ctypes.c_int, ctypes.c_int, ctypes.c_void_p]),
     "nvh_paged_attend_prompt": (ctypes.c_int, [ctypes.POINTER(PagedAttendDesc), ctypes.c_int, ctypes.c_void_p]),
+    "nvh_talk_rows_supported": (ctypes.c_int, [ctypes.c_int] * 4),
+    "nvh_talk_score_cols": (ctypes.c_int, [ctypes.c_int]),
+    "nvh_talk_ticket_bytes": (ctypes.c_size_t, [ctypes.c_int] * 3),
+    "nvh_talk_rows": (ctypes.c_int, [ctypes.POINTER(PagedAttendDesc), ctypes.c_int, ctypes.c_int, ctypes.c_void_p]),
+    "nvh_talk_prompt_supported": (ctypes.c_int, [ctypes.c_int] * 4),
+    "nvh_talk_prompt": (ctypes.c_int, [ctypes.POINTER(PagedAttendDesc), ctypes.c_int, ctypes.c_void_p]),
     "nvh_lightning_supported": (ctypes.c_int, [ctypes.c_int] * 2),
     "nvh_lightning_chunks": (ctypes.c_int, [ctypes.POINTER(LightningDesc), ctypes.c_int, ctypes.c_int, ctypes.c_void_p]),
     "nvh_lightning_step": (ctypes.c_int, [ctypes.POINTER(LightningDesc), ctypes.c_int, ctypes.c_void_p]),
@@ -231,6 +240,7 @@ _SIGS = {
     "nvh_moe_tile_rows": (ctypes.c_int, [ctypes.c_int] * 3),
     "nvh_moe_gemm": (ctypes.c_int, [ctypes.POINTER(MoeGemmDesc), ctypes.c_int, ctypes.c_void_p]),
     "nvh_residual_norm": (ctypes.c_int, [ctypes.POINTER(ResidualNormDesc), ctypes.c_int, ctypes.c_void_p]),
+    "nvh_poly_norm": (ctypes.c_int, [ctypes.c_void_p] * 4 + [ctypes.c_float] + [ctypes.c_int] * 3 + [ctypes.c_int64] * 2 + [ctypes.c_int, ctypes.c_void_p]),
     "nvh_softcap": (ctypes.c_int, [ctypes.c_void_p, ctypes.c_float, ctypes.c_int, ctypes.c_int, ctypes.c_int64, ctypes.c_int, ctypes.c_void_p]),
 }
 EXPORTS = tuple(_SIGS)

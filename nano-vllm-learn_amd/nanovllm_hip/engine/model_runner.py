@@ -136,7 +136,7 @@ class ModelRunner:
         self.world_size = dist.get_world_size() if dist.is_initialized() else 1
         self.device = torch.device(device if device is not None else f"cuda:{torch.cuda.current_device()}")
         if hasattr(cfg, "dtype"):
-            assert max_model_len <= cfg.max_position_embeddings, "max_model_len exceeds the rotation table"
+            assert max_model_len <= cfg.max_position_embeddings, "max_model_len exceeds the model's positions"
             assert self.world_size == 1, f"{cfg.name} runs on one GPU"
             if cfg.dtype == torch.float32:
                 torch.set_float32_matmul_precision("highest")                     # true 32-bit products

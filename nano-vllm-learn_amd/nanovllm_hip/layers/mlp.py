@@ -1,4 +1,6 @@
-"""Dense feed-forward with a clamped gated unit: down(g sigmoid(alpha g) (u + 1)), g = min(gate, limit), u = clamp(up, -limit, limit)."""
+"""Dense feed-forwards.
+ClampedGLU: down(g sigmoid(alpha g) (u + 1)), g = min(gate, limit), u = clamp(up, -limit, limit).
+PolyNormMLP: down(a N(z) + b N(z^2) + c N(z^3) + e), z = up(x), powers by element, N(v) = v / sqrt(mean(v^2) + eps) over a token's values."""
 import torch
 import torch.nn.functional as F
 from torch import nn
@@ -33,3 +35,28 @@ class ClampedGLU(nn.Module):
 
     def linears(self):
         return [(self.w_gate_up, "silu_mul"), (self.w_down, "none")]
+
+
+class PolyNormMLP(nn.Module):
+    def __init__(self, in_width, in_cols, ff, eps, dtype):
+        super().__init__()
+        self.in_width, self.in_cols, self.ff, self.eps, self.dtype = in_width, in_cols, ff, eps, dtype
+        self.cols = round_up(ff, 64)
+
+    def load(self, get):
+        assert get("up").shape == (self.ff, self.in_width) and get("act").numel() == 4
+        self.register_buffer("w_up", padded(get("up"), self.cols, self.in_cols).to(self.dtype).contiguous())
+        self.register_buffer("w_down", padded(get("down"), self.in_cols, self.cols).to(self.dtype).contiguous())
+        self.register_buffer("coef", get("act").float().contiguous())
+
+    def forward(self, x):
+        return linear(ops.poly_norm(linear(x, self.w_up), self.coef, self.eps, self.ff), self.w_down)
+
+    def decode(self, xp, rows, bufs):
+        z = ops.fused_linear(xp, self.w_up, x_packed_rows=rows, workspace=bufs.workspace)
+        mid = bufs.packed(self.cols)
+        ops.poly_norm(z, self.coef, self.eps, self.ff, packed=mid)
+        return ops.fused_linear(mid, self.w_down, x_packed_rows=rows, workspace=bufs.workspace)
+
+    def linears(self):
+        return [(self.w_up, "none"), (self.w_down, "none")]

@@ -1,5 +1,5 @@
-"""Softmax attention with grouped heads over its own pages: optional projection biases, RMS norm over the whole query and key projections, rotation of the
-leading dimensions, a sliding window with kept first tokens, a learned sink per head.  Every pass over the layer (a looped layer has several) has its own
+"""Softmax attention with grouped heads over its own pages: optional projection biases, RMS norm over the whole query and key projections or over every head,
+rotation of the leading dimensions, a sliding window with kept first tokens, a learned sink per head, scores capped and mixed across the heads.  Every pass over the layer (a looped layer has several) has its own
 cache, bound by the runner (`page_cache` [passes, pages, block_size, kv_heads * (dk + dv)], inside a page [kv head][keys | values]).
 
 Single rows (decode) stream the visible keys; prompt portions run the MFMA kernel over the pages.  Widths those kernels do not take, and fp32 models, use
@@ -24,8 +24,11 @@ class PagedAttention(nn.Module):
     cache_name = "page_cache"
 
     def __init__(self, in_width, in_cols, heads, kv_heads, dim, vdim, scale, rope, dtype, eps, bias=False, qk_norm=False, sink=False, window=0, keep_first=0, passes=1,
-                 block_size=64):
+                 block_size=64, talk=False, softcap=0.0):
+        """rope: device -> rotation table, or None.  qk_norm: True (whole projections) or "heads" (one weight for all heads).  talk: scores, capped by softcap
+        tanh(score / softcap) if that is not 0, are mixed across the heads before the softmax."""
         super().__init__()
+        assert talk or not softcap, "capped scores come with mixed heads"
         assert heads % kv_heads == 0, f"{heads} query heads must share {kv_heads} key/value heads evenly"
         self.in_width, self.in_cols, self.dtype, self.eps, self.rope = in_width, in_cols, dtype, eps, rope
         self.heads, self.kv_heads, self.dim, self.vdim, self.scale = heads, kv_heads, dim, vdim, float(scale)
@@ -35,8 +38,13 @@ class PagedAttention(nn.Module):
         self.out_cols = round_up(heads * self.dv, 64)
         self.proj_cols = round_up(self.q_cols + self.k_cols + self.v_cols, 64)
         self.page_cache = torch.tensor([])
-        # the MFMA prompt kernel takes the maximum before the scale
-        self.fast = dtype == torch.bfloat16 and self.scale > 0 and heads * self.dv == self.out_cols and ops.paged_attend_supported(self.dk, self.dv, block_size)
+        self.talking, self.softcap = talk, float(softcap)
+        self.fast = self.fast_prompt = dtype == torch.bfloat16 and heads * self.dv == self.out_cols
+        if talk:
+            self.fast = self.fast and ops.talk_rows_supported(heads, self.dk, self.dv, block_size)
+            self.fast_prompt = self.fast_prompt and ops.talk_prompt_supported(heads, self.dk, self.dv, block_size)
+        else:                                                # (the MFMA prompt kernel takes the maximum before the scale)
+            self.fast = self.fast_prompt = self.fast and self.scale > 0 and ops.paged_attend_supported(self.dk, self.dv, block_size)
 
     def cache_row(self):
         """Elements and type of one token's cache row."""
@@ -55,21 +63,28 @@ class PagedAttention(nn.Module):
         reg("w_qkv", padded(w, self.proj_cols, c).to(self.dtype).contiguous())
         reg("b_qkv", padded(torch.cat([head_rows(get(n + ".b"), *s).reshape(-1) for n, *s in parts]), self.proj_cols).to(self.dtype).contiguous() if self.bias else None)
         for n, heads in (("q", h), ("k", g)):
-            reg(n + "_norm", head_rows(get(n + ".norm").float(), heads, self.dim, self.dk).reshape(-1).contiguous() if self.qk_norm else None)
+            shared = self.qk_norm == "heads"
+            reg(n + "_norm", head_rows(get(n + ".norm").float(), 1 if shared else heads, self.dim, self.dk).reshape(-1).contiguous() if self.qk_norm else None)
         reg("sink", get("sink").float().contiguous() if self.has_sink else None)
+        reg("talk", get("talk").float().contiguous() if self.talking else None)
         o = padded(get("o").reshape(self.in_width, h, self.vdim), self.in_width, h, self.dv).reshape(self.in_width, h * self.dv)
         reg("w_o", padded(o, c, self.out_cols).to(self.dtype).contiguous())
 
     def _prep(self, qkv, positions, step, cache):
-        norm = dict(q_weight=self.q_norm, k_weight=self.k_norm, q_n=self.heads * self.dim, k_n=self.kv_heads * self.dim, eps=self.eps) if self.qk_norm else {}
-        ops.attn_prep(qkv, self.heads, self.kv_heads, self.dk, self.dv, positions, self.rope(qkv.device), cache, step.slot_mapping, **norm)
+        each = self.qk_norm == "heads"
+        norm = dict(q_weight=self.q_norm, k_weight=self.k_norm, q_n=self.dim if each else self.heads * self.dim, k_n=self.dim if each else self.kv_heads * self.dim,
+                    eps=self.eps, head_norm=each) if self.qk_norm else {}
+        table = self.rope(qkv.device) if self.rope is not None else None
+        ops.attn_prep(qkv, self.heads, self.kv_heads, self.dk, self.dv, positions, table, cache, step.slot_mapping, **norm)
 
     def _mask(self):
-        return dict(window=self.window, keep_first=self.keep_first, sink=self.sink)
+        mask = dict(window=self.window, keep_first=self.keep_first, sink=self.sink)
+        return dict(mask, talk=self.talk, softcap=self.softcap) if self.talking else mask
 
     def _rows(self, q, positions, step, cache, row_seq=None, **kw):
-        return ops.paged_attend_rows(q, cache, step.block_tables, positions, self.heads, self.kv_heads, self.dk, self.dv, self.scale, step.max_context,
-                                     row_seq=row_seq, **self._mask(), **kw)
+        attend = ops.talk_rows if self.talking else ops.paged_attend_rows
+        return attend(q, cache, step.block_tables, positions, self.heads, self.kv_heads, self.dk, self.dv, self.scale, step.max_context,
+                      row_seq=row_seq, **self._mask(), **kw)
 
     def forward(self, x, positions, step, run=0):
         """x [rows, in_cols] in the activation type -> the mixer's output, same shape; run: which pass over the layer this is."""
@@ -81,9 +96,9 @@ class PagedAttention(nn.Module):
         o = out[:, :self.heads * self.dv]
         if n:
             self._rows(qkv[:n], positions[:n], step, cache, out=o[:n])
-        if n < rows and self.fast:
-            ops.paged_attend_prompt(qkv[n:], cache, step.block_tables[n:], step.cu_q, step.cu_k, step.max_q, self.heads, self.kv_heads, self.dk, self.dv, self.scale,
-                                    out=o[n:], **self._mask())
+        if n < rows and self.fast_prompt:
+            attend = ops.talk_prompt if self.talking else ops.paged_attend_prompt
+            attend(qkv[n:], cache, step.block_tables[n:], step.cu_q, step.cu_k, step.max_q, self.heads, self.kv_heads, self.dk, self.dv, self.scale, out=o[n:], **self._mask())
         elif n < rows:
             self._rows(qkv[n:], positions[n:], step, cache, row_seq=step.row_seq[n:], out=o[n:])
         return linear(out, self.w_o)

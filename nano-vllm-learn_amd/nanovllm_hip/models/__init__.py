@@ -14,12 +14,17 @@ def _galirax():
     return GaliraxConfig.from_json, GaliraxForCausalLM
 
 
+def _kekapel():
+    from .kekapel import KekapelConfig, KekapelForCausalLM
+    return KekapelConfig.from_json, KekapelForCausalLM
+
+
 def _qwen():
     from .qwen import ModelConfig, QwenForCausalLM
     return ModelConfig.from_json, QwenForCausalLM
 
 
-REGISTRY = {"Zobasun": _zobasun, "Galirax": _galirax, "Qwen2ForCausalLM": _qwen, "Qwen3ForCausalLM": _qwen}
+REGISTRY = {"Zobasun": _zobasun, "Galirax": _galirax, "Kekapel": _kekapel, "Qwen2ForCausalLM": _qwen, "Qwen3ForCausalLM": _qwen}
 
 
 def architecture(config_json):
@@ -37,9 +42,11 @@ def load_config(path, **overrides):
 
 def model_class(cfg):
     from .galirax import GaliraxConfig, GaliraxForCausalLM
+    from .kekapel import KekapelConfig, KekapelForCausalLM
     from .qwen import ModelConfig, QwenForCausalLM
     from .zobasun import ZobasunConfig, ZobasunForCausalLM
-    return {ModelConfig: QwenForCausalLM, ZobasunConfig: ZobasunForCausalLM, GaliraxConfig: GaliraxForCausalLM}[type(cfg)]
+    return {ModelConfig: QwenForCausalLM, ZobasunConfig: ZobasunForCausalLM, GaliraxConfig: GaliraxForCausalLM,
+            KekapelConfig: KekapelForCausalLM}[type(cfg)]
 
 
 def build_model(cfg, path=None, seed=0):

@@ -19,12 +19,13 @@ from ..layers.moe import MixtureOfExperts
 from ..layers.paged_attention import PagedAttention
 from ..layers.rglru import choose_segment
 from ..layers.rotary import rotation_table
+from .looped import LoopedLayers
 
 FUSED_DECODE = True          # tests flip this to compare the fused decode path with the plain one
 
 
 @dataclass
-class GaliraxConfig:
+class GaliraxConfig(LoopedLayers):
     hidden_size: int
     vocab_size: int
     layers: list                                    # entries of config.json: type, mixer, mlp
@@ -62,25 +63,8 @@ class GaliraxConfig:
                 g = r["groups"]
                 if r["experts"] % g["count"] or not 0 < g["keep"] <= g["count"] or not 0 < r["top"] <= g["keep"] * (r["experts"] // g["count"]):
                     raise ValueError(f"layer {i}: top {r['top']} of {r['experts']} experts in {g['count']} groups, {g['keep']} kept")
-        if cfg.loop is not None and not 0 <= cfg.loop["start"] <= cfg.loop["stop"] <= len(cfg.layers) or cfg.loop is not None and cfg.loop["times"] < 1:
-            raise ValueError(f"loop {cfg.loop} over {len(cfg.layers)} layers")
+        cfg.check_loop()
         return cfg
-
-    @property
-    def num_hidden_layers(self):
-        return len(self.layers)
-
-    def passes(self, index):
-        """How often layer `index` runs."""
-        return self.loop["times"] if self.loop is not None and self.loop["start"] <= index < self.loop["stop"] else 1
-
-    def runs(self):
-        """(layer, pass) in the order they run."""
-        n = len(self.layers)
-        if self.loop is None:
-            return [(i, 0) for i in range(n)]
-        a, b = self.loop["start"], self.loop["stop"]
-        return [(i, 0) for i in range(a)] + [(i, t) for t in range(self.loop["times"]) for i in range(a, b)] + [(i, 0) for i in range(b, n)]
 
 
 class GaliraxLayer(nn.Module):

@@ -588,25 +588,35 @@ def _act_code(*tensors):
     return _out_code(dtype)
 
 
+def _ptr(t):
+    return t.data_ptr() if t is not None else None
+
+
 def _require_f32(**tensors):
     for name, t in tensors.items():
         if not t.is_cuda or t.dtype != torch.float32 or not t.is_contiguous():
             raise TypeError(f"{name} must be a contiguous fp32 GPU tensor, got {t.dtype} on {t.device}")
 
 
-def embed_rows(tokens, embed, scale, packed=None):
-    """(fp32 stream [rows, cols], the same in the activation type — the stream itself for fp32) = embed[tokens] * scale.  packed (bf16): the second
-    form in fragment order into this buffer instead."""
+def embed_rows(tokens, embed, scale, packed=None, positions=None, table=None, copy=None, want_rows=True):
+    """(fp32 stream [rows, cols], the same in the activation type — the stream itself for fp32) = embed[tokens] * scale (+ table[positions], fp32).
+    packed (bf16): the second form in fragment order into this buffer instead; want_rows=False: no second form.  copy (fp32): the stream a second time."""
     code = _act_code(embed)
     assert tokens.dtype == torch.int64 and tokens.is_cuda and tokens.is_contiguous() and embed.is_contiguous()
     rows, cols = tokens.numel(), embed.shape[1]
     x = torch.empty((rows, cols), dtype=torch.float32, device=embed.device)
-    xb = torch.empty((rows, cols), dtype=embed.dtype, device=embed.device) if embed.dtype != torch.float32 and packed is None else None
+    xb = torch.empty((rows, cols), dtype=embed.dtype, device=embed.device) if embed.dtype != torch.float32 and packed is None and want_rows else None
+    if table is not None:
+        _require_f32(table=table)
+        assert positions.dtype == torch.int64 and positions.is_contiguous() and positions.numel() == rows and table.shape[1] == cols
+    if copy is not None:
+        _require_f32(copy=copy)
+        assert copy.shape == x.shape
     if packed is not None:
         _require_gpu_bf16(embed=embed, packed=packed)
         assert packed.is_contiguous() and packed.numel() >= ((rows + 15) // 16) * 16 * cols
-    rc = _lib.load().nvh_embed_rows(x.data_ptr(), xb.data_ptr() if xb is not None else None, packed.data_ptr() if packed is not None else None, tokens.data_ptr(), embed.data_ptr(), float(scale), rows, cols,
-                                    embed.shape[0], code, _stream())
+    rc = _lib.load().nvh_embed_rows(x.data_ptr(), _ptr(xb), _ptr(packed), tokens.data_ptr(), embed.data_ptr(), float(scale), rows, cols, embed.shape[0], _ptr(copy),
+                                    _ptr(positions) if table is not None else None, _ptr(table), table.shape[0] if table is not None else 0, code, _stream())
     _lib.check(rc, "nvh_embed_rows")
     return x, xb if xb is not None else x
 
@@ -849,13 +859,12 @@ def _packed_ok(packed, rows, cols):
     assert packed.is_contiguous() and packed.numel() >= ((rows + 15) // 16) * 16 * cols
 
 
-def attn_prep(qkv, heads, kv_heads, dk, dv, positions, cos_sin, cache, slots, q_weight=None, k_weight=None, q_n=0, k_n=0, eps=0.0):
-    """Row ops behind a q | k | v projection: optional RMS norm over all query and all key columns (means over q_n / k_n of them), rotation of
-    interleaved pairs of the first cos_sin.shape[1] dimensions of every head, keys and values into the cache [pages, block_size, kv_heads * (dk + dv)]
+def attn_prep(qkv, heads, kv_heads, dk, dv, positions, cos_sin, cache, slots, q_weight=None, k_weight=None, q_n=0, k_n=0, eps=0.0, head_norm=False):
+    """Row ops behind a q | k | v projection: optional RMS norm over all query and all key columns (means over q_n / k_n of them; head_norm: over every head
+    by itself, weights [dk] shared by the heads), rotation of interleaved pairs of the first cos_sin.shape[1] dimensions of every head (None: no rotation), keys and values into the cache [pages, block_size, kv_heads * (dk + dv)]
     (inside a page: [kv head][keys | values]).  The queries are rewritten in place."""
     code = _act_code(qkv, cache)
     rows = qkv.shape[0]
-    _require_f32(cos_sin=cos_sin)
     _require_i32(slots=slots)
     assert qkv.dim() == 2 and qkv.stride(1) == 1 and qkv.shape[1] >= heads * dk + kv_heads * (dk + dv)
     assert cache.dim() == 3 and cache.is_contiguous() and cache.shape[2] == kv_heads * (dk + dv)
@@ -864,9 +873,13 @@ def attn_prep(qkv, heads, kv_heads, dk, dv, positions, cos_sin, cache, slots, q_
     d.qkv, d.qkv_stride, d.rows, d.heads, d.kv_heads, d.dk, d.dv = qkv.data_ptr(), qkv.stride(0), rows, heads, kv_heads, dk, dv
     if q_weight is not None:
         _require_f32(q_weight=q_weight, k_weight=k_weight)
-        assert q_weight.numel() == heads * dk and k_weight.numel() == kv_heads * dk
+        assert (q_weight.numel(), k_weight.numel()) == ((dk, dk) if head_norm else (heads * dk, kv_heads * dk))
+        d.head_norm = int(head_norm)
         d.q_w, d.k_w, d.q_n, d.k_n, d.eps = q_weight.data_ptr(), k_weight.data_ptr(), int(q_n), int(k_n), float(eps)
-    d.positions, d.cos_sin, d.max_position, d.rot = positions.data_ptr(), cos_sin.data_ptr(), cos_sin.shape[0], cos_sin.shape[1]
+    d.positions = positions.data_ptr()
+    if cos_sin is not None:
+        _require_f32(cos_sin=cos_sin)
+        d.cos_sin, d.max_position, d.rot = cos_sin.data_ptr(), cos_sin.shape[0], cos_sin.shape[1]
     d.cache, d.slots, d.block_size = cache.data_ptr(), slots.data_ptr(), cache.shape[1]
     _lib.check(_lib.load().nvh_attn_prep(ctypes.byref(d), code, _stream()), "nvh_attn_prep")
 
@@ -903,6 +916,80 @@ def _paged_desc(q, cache, block_tables, heads, kv_heads, dk, dv, scale, window, 
         assert out.shape == (rows, heads * dv) and out.stride(1) == 1 and out.dtype == q.dtype
         d.out, d.out_stride = out.data_ptr(), out.stride(0)
     return d, code
+
+
+SCORE_BYTES = 256 << 20        # scores talk_rows keeps in memory at a time: more rows run in several launches
+
+
+def talk_rows_supported(heads, dk, dv, block_size) -> bool:
+    return bool(_lib.load().nvh_talk_rows_supported(int(heads), int(dk), int(dv), int(block_size)))
+
+
+def talk_prompt_supported(heads, dk, dv, block_size) -> bool:
+    return bool(_lib.load().nvh_talk_prompt_supported(int(heads), int(dk), int(dv), int(block_size)))
+
+
+def _set_talk(d, talk, softcap, heads):
+    _require_f32(talk=talk)
+    assert talk.shape == (heads, heads)
+    d.talk, d.softcap = talk.data_ptr(), float(softcap)
+
+
+def talk_rows(q, cache, block_tables, positions, heads, kv_heads, dk, dv, scale, max_context, talk, softcap=0.0, window=0, keep_first=0, sink=None, row_seq=None, out=None,
+              out_packed=None, want_out=True, splits=None, generic=False):
+    """paged_attend_rows with scores capped (softcap tanh(scale q . k / softcap); 0: not) and mixed across the heads by talk [heads, heads] before the softmax."""
+    rows = q.shape[0]
+    if out is None and want_out:
+        out = torch.empty((rows, heads * dv), dtype=q.dtype, device=q.device)
+    assert positions.dtype == torch.int64 and positions.is_contiguous() and positions.numel() == rows
+    if row_seq is not None:
+        _require_i32(row_seq=row_seq)
+        assert row_seq.numel() == rows and row_seq.is_contiguous()
+    else:
+        assert block_tables.shape[0] >= rows
+    lib = _lib.load()
+    # 64-key tiles a row sees at most: all of its context, or those a window and the kept first tokens touch
+    tiles = (max_context + 63) // 64
+    if window:
+        tiles = min(tiles, (window + 126) // 64 + (keep_first + 63) // 64)
+    cols = int(lib.nvh_talk_score_cols(heads))
+    step = max(1, SCORE_BYTES // (tiles * 64 * cols * 4))
+    fast = q.dtype == torch.bfloat16 and row_seq is None and not generic and talk_rows_supported(heads, dk, dv, cache.shape[1])
+    assert out_packed is None or step >= rows, "packed rows are few"
+    for r in range(0, rows, step):
+        n = min(step, rows - r)
+        d, code = _paged_desc(q[r:r + n], cache, block_tables if row_seq is not None else block_tables[r:], heads, kv_heads, dk, dv, scale, window, keep_first, sink,
+                              out[r:r + n] if out is not None else None)
+        _set_talk(d, talk, softcap, heads)
+        d.positions = positions[r:].data_ptr()
+        d.row_seq = row_seq[r:].data_ptr() if row_seq is not None else None
+        scores = torch.empty((n, tiles * 64, cols), dtype=torch.float32, device=q.device)
+        d.scores, d.span = scores.data_ptr(), tiles * 64
+        if fast:
+            d.splits = splits or paged_attend_splits(n, kv_heads, heads, max_context, window, keep_first)
+        if d.splits > 1:
+            part = torch.empty((n, heads, d.splits, dv + 4), dtype=torch.float32, device=q.device)
+            tickets = reserve_workspace(q.device, int(lib.nvh_talk_ticket_bytes(n, kv_heads, heads)), "paged_attend")
+            d.part, d.tickets = part.data_ptr(), tickets.data_ptr()
+        if out_packed is not None:
+            _packed_ok(out_packed, rows, heads * dv)
+            d.out_packed = out_packed.data_ptr()
+        _lib.check(lib.nvh_talk_rows(ctypes.byref(d), int(generic), code, _stream()), "nvh_talk_rows")
+    return out
+
+
+def talk_prompt(q, cache, block_tables, cu_q, cu_k, max_q, heads, kv_heads, dk, dv, scale, talk, softcap=0.0, window=0, keep_first=0, sink=None, out=None):
+    """paged_attend_prompt with capped scores mixed across the heads (see talk_rows)."""
+    _require_gpu_bf16(q=q)
+    _require_i32(cu_q=cu_q, cu_k=cu_k)
+    if out is None:
+        out = torch.empty((q.shape[0], heads * dv), dtype=q.dtype, device=q.device)
+    d, code = _paged_desc(q, cache, block_tables, heads, kv_heads, dk, dv, scale, window, keep_first, sink, out)
+    assert cu_q.numel() == cu_k.numel() and cu_q.is_contiguous() and cu_k.is_contiguous() and block_tables.shape[0] >= cu_q.numel() - 1
+    d.cu_q, d.cu_k, d.batch, d.max_q = cu_q.data_ptr(), cu_k.data_ptr(), cu_q.numel() - 1, int(max_q)
+    _set_talk(d, talk, softcap, heads)
+    _lib.check(_lib.load().nvh_talk_prompt(ctypes.byref(d), code, _stream()), "nvh_talk_prompt")
+    return out
 
 
 def paged_attend_rows(q, cache, block_tables, positions, heads, kv_heads, dk, dv, scale, max_context, window=0, keep_first=0, sink=None, row_seq=None, out=None,
@@ -1017,8 +1104,9 @@ def norm_gate(x, gate, weight, eps, n, packed=None):
 
 
 # --------------------------------------------------------------------------------------- mixture of experts
-def moe_route(x, router, correction, top, groups, keep, scale):
-    """(chosen experts int32 [rows, top], weights fp32 [rows, top]) of rows x against router [experts, cols]."""
+def moe_route(x, router, correction, top, groups=1, keep=1, scale=1.0, softmax=False):
+    """(chosen experts int32 [rows, top], weights fp32 [rows, top]) of rows x against router [experts, cols].  softmax: the choice goes by the logits with
+    `correction` as their bias, the weights are the softmax over the chosen ones; otherwise sigmoid scores, corrections for the choice only, groups."""
     code = _act_code(x, router)
     _require_f32(correction=correction)
     rows, cols = x.shape
@@ -1029,7 +1117,7 @@ def moe_route(x, router, correction, top, groups, keep, scale):
     d = _lib.MoeRouteDesc()
     d.x, d.x_stride, d.router, d.correction = x.data_ptr(), x.stride(0), router.data_ptr(), correction.data_ptr()
     d.rows, d.cols, d.experts, d.top, d.groups, d.keep, d.scale = rows, cols, experts, int(top), int(groups), int(keep), float(scale)
-    d.ids, d.weights = ids.data_ptr(), weights.data_ptr()
+    d.ids, d.weights, d.softmax = ids.data_ptr(), weights.data_ptr(), int(softmax)
     _lib.check(_lib.load().nvh_moe_route(ctypes.byref(d), code, _stream()), "nvh_moe_route")
     return ids, weights
 
@@ -1049,8 +1137,9 @@ def moe_dispatch(ids, experts, dtype, tile_rows=None):
     return slots, tiles[:max_tiles], tile_rows
 
 
-def moe_gemm(x, weight, ids, glu, dispatch=None):
-    """Expert products per pair p = row * top + k: glu: silu(x[row] . gate_e) * (x[row] . up_e) with weight [experts, 2 * n, k]; otherwise x[p] . w_e with
+def moe_gemm(x, weight, ids, glu, dispatch=None, unit=None):
+    """Expert products per pair p = row * top + k: glu: silu(x[row] . gate_e) * (x[row] . up_e) with weight [experts, 2 * n, k], or with unit = (limit, alpha)
+    the clamped unit g sigmoid(alpha g) (u + 1), g = min(gate, limit), u = clamp(up, -limit, limit); otherwise x[p] . w_e with
     weight [experts, n, k].  dispatch: what moe_dispatch returned; None: the form for at most 64 rows (bf16)."""
     code = _act_code(x, weight)
     experts, n, k = weight.shape
@@ -1061,6 +1150,9 @@ def moe_gemm(x, weight, ids, glu, dispatch=None):
     d = _lib.MoeGemmDesc()
     d.out, d.x, d.x_stride, d.w = out.data_ptr(), x.data_ptr(), x.stride(0), weight.data_ptr()
     d.pairs, d.top, d.experts, d.n, d.k, d.glu = pairs, top, experts, n, k, int(glu)
+    if unit is not None:
+        assert glu and unit[1] != 0.0
+        d.limit, d.alpha = float(unit[0]), float(unit[1])
     if dispatch is None:
         _require_i32(ids=ids)
         assert ids.is_contiguous()
@@ -1074,8 +1166,9 @@ def moe_gemm(x, weight, ids, glu, dispatch=None):
 
 
 # --------------------------------------------------------------------------------------- residual and output of models with one norm per layer
-def residual_norm(x, dtype, y=None, experts=None, weight=None, bias=None, eps=0.0, n=0, packed=None, want_rows=True):
-    """x (fp32 stream, in place) += y + the weighted sum of experts = (outputs [rows * top, cols], weights [rows, top]); with weight given returns the layer norm
+def residual_norm(x, dtype, y=None, experts=None, weight=None, bias=None, eps=0.0, n=0, packed=None, want_rows=True, post=None, mult=1.0, base=None, shift=None):
+    """x (fp32 stream, in place) += y + the weighted sum of experts = (outputs [rows * top, cols], weights [rows, top]), or mult times the layer norm of that sum
+    with post = (weight, bias); += base [rows, cols], += shift [cols] (fp32) where given; with weight given returns the layer norm
     of the new rows (mean and variance over n columns) in `dtype`, and in fragment order into `packed` (bf16)."""
     _require_f32(x=x)
     rows, cols = x.shape
@@ -1090,6 +1183,19 @@ def residual_norm(x, dtype, y=None, experts=None, weight=None, bias=None, eps=0.
         _require_f32(ew=ew)
         assert ew.shape[0] == rows and e.shape == (ew.numel(), cols) and e.is_contiguous() and e.dtype == dtype and e.is_cuda
         d.e, d.ew, d.top = e.data_ptr(), ew.data_ptr(), ew.shape[1]
+    d.mult = float(mult)
+    if post is not None:
+        _require_f32(post_weight=post[0], post_bias=post[1])
+        assert post[0].numel() == cols and post[1].numel() == cols
+        d.post_w, d.post_b = post[0].data_ptr(), post[1].data_ptr()
+    if base is not None:
+        _require_f32(base=base)
+        assert base.shape == x.shape
+        d.base = base.data_ptr()
+    if shift is not None:
+        _require_f32(shift=shift)
+        assert shift.numel() == cols
+        d.shift = shift.data_ptr()
     out = None
     if weight is not None:
         _require_f32(weight=weight, bias=bias)
@@ -1102,6 +1208,22 @@ def residual_norm(x, dtype, y=None, experts=None, weight=None, bias=None, eps=0.
             _packed_ok(packed, rows, cols)
             d.packed = packed.data_ptr()
     _lib.check(_lib.load().nvh_residual_norm(ctypes.byref(d), code, _stream()), "nvh_residual_norm")
+    return out
+
+
+def poly_norm(z, coef, eps, n, packed=None):
+    """coef[0] N(z) + coef[1] N(z^2) + coef[2] N(z^3) + coef[3] with N(v) = v / sqrt(mean over n columns of v^2 + eps), zero past n; packed (bf16): in fragment
+    order into this buffer, returns None."""
+    code = _act_code(z)
+    _require_f32(coef=coef)
+    rows, cols = z.shape
+    assert z.stride(1) == 1 and coef.numel() == 4
+    out = None
+    if packed is None:
+        out = torch.empty((rows, cols), dtype=z.dtype, device=z.device)
+    else:
+        _packed_ok(packed, rows, cols)
+    _lib.check(_lib.load().nvh_poly_norm(_ptr(out), _ptr(packed), z.data_ptr(), coef.data_ptr(), float(eps), rows, cols, int(n), z.stride(0), cols, code, _stream()), "nvh_poly_norm")
     return out
 
 

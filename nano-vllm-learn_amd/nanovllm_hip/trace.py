@@ -13,16 +13,18 @@ import sys
 import torch
 
 from .engine.llm_engine import LLMEngine
+from .models import load_config
 
 LIVE_REQUESTS = 4
 
 
 class TraceRunner:
     def __init__(self, model, dtype, max_tokens):
-        overrides = {"dtype": dtype, "max_position_embeddings": max(max_tokens, 1)}
         block = 64
-        self.engine = LLMEngine.from_folder(model, {**overrides, "kvcache_block_size": block}, num_kvcache_blocks=-(-max_tokens // block),
-                                            max_num_seqs=LIVE_REQUESTS, max_model_len=max_tokens)
+        cfg = load_config(model, dtype=dtype, max_position_embeddings=max(max_tokens, 1), kvcache_block_size=block)
+        # the pool is for all live requests; one of them may have fewer positions (a learned table is as long as it is)
+        self.engine = LLMEngine(cfg, num_kvcache_blocks=-(-max_tokens // block), weights=model, max_num_seqs=LIVE_REQUESTS,
+                                max_model_len=min(max_tokens, cfg.max_position_embeddings))
         if not self.engine.runner.mixed_batches:
             raise SystemExit(f"{self.engine.cfg.name}: trace replay needs a model that takes mixed batches")
         self.live = {}
