@@ -303,7 +303,7 @@ def main():
     ap.add_argument("--eager", action="store_true", help="no HIP graph (debug)")
     ap.add_argument("--graph-steps", type=int, default=0, help="A/B: decode steps captured per replayed graph (0 = the session's default)")
     ap.add_argument("--kv-ahead", default=None, choices=["o_k+gu_v", "o_v+gu_k", "o_k", "gu_k"],
-                    help="A/B: the o_proj / gate_up launches of a layer touch the NEXT layer's K / V cache regions (Infinity-Cache prefetch experiment, DESIGN.md 12.1)")
+                    help="A/B: the o_proj / gate_up launches of a layer touch the NEXT layer's K / V cache regions (Infinity-Cache prefetch experiment)")
     ap.add_argument("--no-prefetch", action="store_true", help="A/B: the qkv / down launches do not prefetch the next small projection's weights")
     ap.add_argument("--qkv-attend", default=None, choices=["two_launches", "one_launch", "two_launches_kv_prefetch", "auto"],
                     help="A/B: how the qkv projection + decode attention front of a layer runs (nvh_qkv_rope_attend_variant)")
@@ -313,7 +313,7 @@ def main():
     ap.add_argument("--prefill-leg", action="store_true", help="time the prefill attention op for models other than the headline one too")
     ap.add_argument("--beside", choices=["1k", "2k", "4k"], help="instead of the default workload: another model beside a Qwen2-shaped one of this size "
                     "(engine throughput and kernels against their rooflines), one JSON line")
-    ap.add_argument("--beside-model", choices=["zobasun", "galirax"], default="zobasun")
+    ap.add_argument("--beside-model", choices=["zobasun", "galirax", "kekapel"], default="zobasun")
     ap.add_argument("--beside-only", choices=["kernels", "engine"])
     args = ap.parse_args()
     if args.beside:

@@ -1,5 +1,5 @@
-"""Zobasun or Galirax beside the closest other model (a Qwen2-shaped stack) at equal size, on random weights: prefill and decode throughput through the
-engine, and each hot kernel against its roofline.  bench.py --beside SIZE [--beside-model NAME] prints the result as one JSON line."""
+"""Zobasun, Galirax or Kekapel beside the closest other model (a Qwen2-shaped stack; for Kekapel also Galirax with windows in every layer) at equal size, on
+random weights: prefill and decode throughput through the engine, and each hot kernel against its roofline.  bench.py --beside SIZE [--beside-model NAME] prints the result as one JSON line."""
 from __future__ import annotations
 
 import time
@@ -14,10 +14,11 @@ from .engine.model_runner import recurrence_chunks
 from .layers.rglru import choose_segment
 from .layers.rotary import rotation_table
 from .models.galirax import GaliraxConfig
+from .models.kekapel import KekapelConfig
 from .models.qwen import ModelConfig
 from .models.zobasun import ZobasunConfig
 
-HBM_GBPS, MFMA_TFLOPS = 8000.0, 2500.0          # MI355X peaks (dense bf16)
+HBM_GBPS, MFMA_TFLOPS, MFMA32_TFLOPS = 8000.0, 2500.0, 157.3      # MI355X peaks (dense bf16, fp32 matrix)
 
 # width, feed-forward, layers; attention heads (128 wide); latent ranks and widths; recurrence width, blocks; experts (each ff / top wide)
 SIZES = {
@@ -26,7 +27,7 @@ SIZES = {
     "4k": dict(width=4096, ff=12288, layers=6, heads=32, kv_heads=8, q_rank=1536, kv_rank=512, dim=128, rot=64, vdim=128, rec=4096, blocks=16, experts=32, top=4),
 }
 VOCAB = 32000
-WINDOW, KEEP = 512, 4                           # Galirax's windowed layers
+WINDOW, KEEP = 512, 4                           # Galirax's windowed layers; Kekapel's window
 
 
 def qwen_config(size):
@@ -36,15 +37,27 @@ def qwen_config(size):
                        qk_norm=False)
 
 
-def galirax_config(size):
-    """Windowed attention, lightning attention, full attention in turn; the experts a token uses are together as wide as the Qwen stack's feed-forward."""
+def galirax_config(size, windows_only=False):
+    """Windowed attention, lightning attention, full attention in turn (windows_only: windowed attention in every layer); the experts a token uses are together
+    as wide as the Qwen stack's feed-forward."""
     s = SIZES[size]
     mlp = {"kind": "moe", "expert": {"ff": s["ff"] // s["top"]}, "router": {"experts": s["experts"], "top": s["top"], "groups": {"count": 8, "keep": 4}, "scale": 2.5}}
     att = dict(heads=s["heads"], kv_heads=s["kv_heads"], dim=128, vdim=128, scale=128 ** -0.5, rot={"base": 10000.0, "dims": 128})
     kinds = [("attention_2", {**att, "mask": {"size": WINDOW, "keep_first": KEEP}}),
              ("lightning", dict(heads=s["heads"], dim=128, vdim=128, decay=[1 - 2.0 ** -(3 + 6 * i / s["heads"]) for i in range(s["heads"])])), ("attention", att)]
+    if windows_only:
+        kinds = kinds[:1] * 3
     return GaliraxConfig.from_json({"width": s["width"], "vocab": VOCAB, "norm": {"eps": 1e-6}, "logit_softcap": 15.0,
                                     "layers": [dict(type=kinds[i % 3][0], mixer=kinds[i % 3][1], mlp=mlp) for i in range(s["layers"])]})
+
+
+def kekapel_config(size):
+    """Windowed attention with mixed heads in every layer, dense feed-forwards and experts in turn."""
+    s = SIZES[size]
+    att = dict(heads=s["heads"], kv_heads=s["kv_heads"], dim=128, vdim=128, scale=128 ** -0.5, softcap=20.0, mask={"size": WINDOW})
+    mlps = ({"kind": "dense", "ff": s["ff"]}, {"kind": "moe", "expert": {"ff": s["ff"] // s["top"], "limit": 7.0}, "router": {"experts": s["experts"], "top": s["top"]}})
+    return KekapelConfig.from_json({"width": s["width"], "vocab": VOCAB, "norm": {"eps": 1e-6}, "embedding": {"scale": 1.0}, "residual_mult": 0.7, "max_positions": 16384,
+                                    "layers": [dict(type="attention", mixer=att, mlp=mlps[i % 2]) for i in range(s["layers"])]})
 
 
 def zobasun_config(size):
@@ -115,10 +128,11 @@ def _time(calls, iters=10):
     return a.elapsed_time(b) * 1e3 / (iters * len(calls))
 
 
-def _line(us, nbytes=0, flops=0):
-    floor = max(nbytes / (HBM_GBPS * 1e3), flops / (MFMA_TFLOPS * 1e6))
-    return {"us": round(us, 2), "bound": "hbm" if nbytes / HBM_GBPS * 1e3 >= flops / MFMA_TFLOPS else "mfma", "GBps": round(nbytes / us / 1e3, 1),
-            "TFLOPs": round(flops / us / 1e6, 1), "roofline": round(floor / us, 4)}
+def _line(us, nbytes=0, flops=0, flops32=0):
+    """flops: bf16 matrix products; flops32: those of the fp32 matrix pipe, which is the same pipe: their times add up"""
+    hbm, mfma = nbytes / (HBM_GBPS * 1e3), flops / (MFMA_TFLOPS * 1e6) + flops32 / (MFMA32_TFLOPS * 1e6)
+    return {"us": round(us, 2), "bound": "hbm" if hbm >= mfma else "mfma", "GBps": round(nbytes / us / 1e3, 1),
+            "TFLOPs": round((flops + flops32) / us / 1e6, 1), "roofline": round(max(hbm, mfma) / us, 4)}
 
 
 def _randn(*shape, dtype=torch.bfloat16):
@@ -328,20 +342,107 @@ def zobasun_kernels(size, batch=32, ctx=1536, seqs=16, prompt=1024):
     return out
 
 
-MODELS = {"zobasun": (zobasun_config, zobasun_kernels), "galirax": (galirax_config, galirax_kernels)}
+@torch.inference_mode()
+def kekapel_kernels(size, batch=32, ctx=1536, seqs=16, prompt=1024):
+    """Each hot kernel of Kekapel alone, and on the same operands the like kernels of Galirax (paged attention, prep, residual, experts) and of the Qwen stack."""
+    s, out, rows = SIZES[size], {}, seqs * prompt
+    h, g, d, width, experts, top = s["heads"], s["kv_heads"], 128, s["width"], s["experts"], s["top"]
+    ff, cap, scale = s["ff"] // top, 20.0, d ** -0.5
+    cu = torch.arange(0, rows + 1, prompt, dtype=torch.int32, device="cuda")
+    pos = torch.arange(prompt, device="cuda").repeat(seqs)
+    talk = torch.eye(h, device="cuda") + 0.1 * _randn(h, h, dtype=torch.float32)
+    # ---- attention over prompts, row ops in front
+    cols = (h + 2 * g) * d
+    qkv = [_randn(rows, cols) for _ in range(3)]
+    cache = torch.zeros(rows // 64, 64, 2 * g * d, dtype=torch.bfloat16, device="cuda")
+    slot = torch.arange(rows, dtype=torch.int32, device="cuda")
+    one, qw, kw = torch.ones(d, device="cuda"), torch.ones(h * d, device="cuda"), torch.ones(g * d, device="cuda")
+    us = _time([lambda x=x: ops.attn_prep(x, h, g, d, d, pos, None, cache, slot, one, one, d, d, 1e-6, head_norm=True) for x in qkv])
+    out["attn_prep, norm per head"] = _line(us, rows * 4 * cols)
+    us = _time([lambda x=x: ops.attn_prep(x, h, g, d, d, pos, None, cache, slot, qw, kw, h * d, g * d, 1e-6) for x in qkv])
+    out["galirax attn_prep"] = _line(us, rows * 4 * cols)
+    bt = torch.arange(rows // 64, dtype=torch.int32, device="cuda").view(seqs, -1)
+    o = torch.empty(rows, h * d, device="cuda", dtype=torch.bfloat16)
+    nbytes = 4 * rows * (h + g) * d
+    for name, window in (("prompt", 0), (f"prompt, window {WINDOW}", WINDOW)):
+        seen = seqs * (sum(min(t + 1, window) for t in range(prompt)) if window else prompt * (prompt + 1) / 2)
+        us = _time([lambda x=x: ops.talk_prompt(x, cache, bt, cu, cu, prompt, h, g, d, d, scale, talk, cap, window=window, out=o) for x in qkv] * 2)
+        out[f"talk_{name}"] = _line(us, nbytes, 4 * d * h * seen, 2 * h * h * seen)
+        us = _time([lambda x=x: ops.paged_attend_prompt(x, cache, bt, cu, cu, prompt, h, g, d, d, scale, window=window, out=o) for x in qkv] * 2)
+        out[f"galirax paged_{name}"] = _line(us, nbytes, 4 * d * h * seen)
+    del qkv, o, cache
+    # ---- decode attention
+    pages = -(-ctx // 64)
+    n = max(2, int(3e8 // (batch * pages * 64 * 4 * g * d)) + 1)
+    caches = [_randn(batch * pages, 64, 2 * g * d) for _ in range(n)]
+    bt = torch.randperm(batch * pages).view(batch, pages).int().cuda()
+    dpos = torch.full((batch,), ctx - 1, device="cuda")
+    q, o = _randn(batch, h * d), torch.empty(batch, h * d, device="cuda", dtype=torch.bfloat16)
+    for name, window in (("rows", 0), (f"rows, window {WINDOW}", WINDOW)):
+        nbytes = batch * (4 * (window or ctx) * g * d + 4 * h * d)
+        us = _time([lambda c=c: ops.talk_rows(q, c, bt, dpos, h, g, d, d, scale, ctx, talk, cap, window=window, out=o) for c in caches] * 3)
+        out[f"talk_{name} (scores + rows)"] = _line(us, nbytes)
+        us = _time([lambda c=c: ops.paged_attend_rows(q, c, bt, dpos, h, g, d, d, scale, ctx, window=window, out=o) for c in caches] * 3)
+        out[f"galirax paged_{name}"] = _line(us, nbytes)
+    del caches
+    # ---- feed-forwards
+    xs, router, bias = [_randn(rows, width) for _ in range(2)], _randn(experts, width) * width ** -0.5, torch.zeros(experts, device="cuda")
+    z, coef = [_randn(rows, s["ff"]) for _ in range(2)], torch.ones(4, device="cuda")
+    out["poly_norm"] = _line(_time([lambda t=t: ops.poly_norm(t, coef, 1e-6, s["ff"]) for t in z] * 2), rows * s["ff"] * 4)
+    gu = [_randn(rows, 2 * s["ff"]) for _ in range(2)]
+    out["qwen_silu_mul"] = _line(_time([lambda t=t: ops.silu_mul(t) for t in gu]), rows * s["ff"] * 6)
+    del z, gu
+    us = _time([lambda a=a: ops.moe_route(a, router, bias, top, softmax=True) for a in xs] * 2)
+    out["moe_route, softmax"] = _line(us, 2 * rows * width, 2 * rows * width * experts)
+    us = _time([lambda a=a: ops.moe_route(a, router, bias, top, 8, 4, 2.5) for a in xs] * 2)
+    out["galirax moe_route"] = _line(us, 2 * rows * width, 2 * rows * width * experts)
+    ids, ew = ops.moe_route(xs[0], router, bias, top, softmax=True)
+    dispatch, unit = ops.moe_dispatch(ids, experts, torch.bfloat16), (7.0, 1.702)
+    wgu = [_randn(experts, 2 * ff, width) * 0.02 for _ in range(2)]
+    for name, u in (("moe_gate_up, clamped unit", unit), ("galirax moe_gate_up", None)):
+        out[name] = _line(_time([lambda w=w: ops.moe_gemm(xs[0], w, ids, True, dispatch, u) for w in wgu]), 0, 4 * rows * top * ff * width)
+    e, st, w32 = _randn(rows * top, width), _randn(rows, width, dtype=torch.float32), torch.ones(width, device="cuda")
+    norm = dict(weight=w32, bias=w32, eps=1e-6)
+    for name, kw in (("residual_norm, both sides", dict(post=(w32, w32), mult=0.7)), ("galirax residual_norm", {})):
+        us = _time([lambda a=a: ops.residual_norm(st, torch.bfloat16, y=a, **norm, **kw) for a in xs])
+        out[f"{name}, attention"] = _line(us, rows * width * (8 + 2 + 2))
+        us = _time([lambda: ops.residual_norm(st, torch.bfloat16, experts=(e, ew), **norm, **kw)] * 2)
+        out[f"{name}, experts"] = _line(us, rows * width * (8 + 2 * top + 2))
+    del e, st, xs
+    # ---- decode batch
+    x1 = _randn(batch, width)
+    ids, _ = ops.moe_route(x1, router, bias, top, softmax=True)
+    used = ids.unique().numel()
+    wgu += [_randn(experts, 2 * ff, width) * 0.02 for _ in range(max(0, int(3e8 // (4 * experts * ff * width)) - 1))]
+    for name, u in (("moe_gate_up_decode, clamped unit", unit), ("galirax moe_gate_up_decode", None)):
+        out[name] = _line(_time([lambda w=w: ops.moe_gemm(x1, w, ids, True, None, u) for w in wgu] * 3), used * 4 * ff * width)
+    del wgu
+    for name, kw in (("moe_route_decode, softmax", dict(softmax=True)), ("galirax moe_route_decode", dict(groups=8, keep=4, scale=2.5))):
+        out[name] = _line(_time([lambda: ops.moe_route(x1, router, bias, top, **kw)] * 20), 2 * (batch + experts) * width)
+    z = _randn(batch, s["ff"])
+    packed = torch.zeros((batch + 15) // 16 * 16 * s["ff"], dtype=torch.bfloat16, device="cuda")
+    out["poly_norm_decode"] = _line(_time([lambda: ops.poly_norm(z, coef, 1e-6, s["ff"], packed=packed)] * 20), batch * s["ff"] * 4)
+    torch.cuda.empty_cache()
+    return out
+
+
+MODELS = {"zobasun": (zobasun_config, zobasun_kernels), "galirax": (galirax_config, galirax_kernels), "kekapel": (kekapel_config, kekapel_kernels)}
 
 
 def run(size, only=None, model="zobasun"):
     torch.manual_seed(0)
     config, kernels = MODELS[model]
-    new, old = config(size), qwen_config(size)
-    res = {"metric": f"{new.name} beside a Qwen2-shaped stack of equal width, depth and feed-forward (random weights)", "size": size, "shape": SIZES[size], "dtype": "bf16"}
+    beside = [("qwen", qwen_config(size))]
+    if model == "kekapel":
+        beside.append(("galirax", galirax_config(size, windows_only=True)))
+    stacks = [(model, config(size)), *beside]
+    res = {"metric": f"{stacks[0][1].name} beside a Qwen2-shaped stack of equal width, depth and feed-forward (random weights)", "size": size, "shape": SIZES[size], "dtype": "bf16"}
     if only in (None, "kernels"):
         res["kernels"] = kernels(size)
     if only in (None, "engine"):
         for batch, prompt in ((16, 1024), (2, 8192)):
-            for name, cfg in ((model, new), ("qwen", old)):
+            for name, cfg in stacks:
                 res[f"{name}_{batch}x{prompt}"] = _engine_throughput(cfg, batch, prompt, 64)
-        for name, cfg in ((model, new), ("qwen", old)):
+        for name, cfg in stacks:
             res[f"{name}_32x1024"] = _engine_throughput(cfg, 32, 1024, 256, repeats=1)
     return res
