@@ -630,12 +630,13 @@ int nvh_paged_attend_rows(const nvh_paged_attend_desc* d, int generic, int dtype
 int nvh_paged_attend_prompt(const nvh_paged_attend_desc* d, int dtype, void* stream);
 
 /* The same attention with scores capped, softcap tanh(scale q . k / softcap), and then mixed across the heads, score_h <- sum_g talk[h][g] score_g, before the
- * softmax.  nvh_talk_rows is two launches (scores to memory, then the rest); nvh_talk_prompt is one, all heads of 16 rows in a workgroup. */
+ * softmax.  nvh_talk_rows is two launches (scores to memory, then the rest); nvh_talk_prompt is one, all heads of 16 rows in a workgroup: it takes caps in
+ * (0, 1e4] and mixing matrices with entries of at most 2000 (both pass through pairs of fp16 numbers). */
 int nvh_talk_rows_supported(int heads, int dk, int dv, int block_size);
 int nvh_talk_score_cols(int heads);
 size_t nvh_talk_ticket_bytes(int rows, int kv_heads, int heads);
 int nvh_talk_rows(const nvh_paged_attend_desc* d, int generic, int dtype, void* stream);
-int nvh_talk_prompt_supported(int heads, int dk, int dv, int block_size);
+int nvh_talk_prompt_supported(int heads, int kv_heads, int dk, int dv, int block_size, float softcap);
 int nvh_talk_prompt(const nvh_paged_attend_desc* d, int dtype, void* stream);
 
 /* Lightning attention: per head S = decay S + k v^T, o = S^T q with q, k, v = silu of the projection's columns (rounded to the activation type);

@@ -28,7 +28,8 @@ int launch_paged_attend_prompt(const PagedAttendArgs& a, hipStream_t stream);
 __host__ __device__ constexpr int score_cols(int heads) { return (heads + 3) / 4 * 4; }          // row length of PagedAttendArgs::scores
 bool talk_rows_supported(int heads, int dk, int dv, int block_size);
 int launch_talk_rows(const PagedAttendArgs& a, int f32, int generic, hipStream_t stream);
-bool talk_prompt_supported(int heads, int dk, int dv, int block_size);
+bool talk_prompt_supported(int heads, int kv_heads, int dk, int dv, int block_size);
+constexpr float kTalkPromptCap = 1e4f;               // it takes capped scores only
 int launch_talk_prompt(const PagedAttendArgs& a, hipStream_t stream);
 
 bool lightning_supported(int dk, int dv);

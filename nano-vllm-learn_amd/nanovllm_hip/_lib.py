@@ -228,7 +228,7 @@ _SIGS = {
     "nvh_talk_score_cols": (ctypes.c_int, [ctypes.c_int]),
     "nvh_talk_ticket_bytes": (ctypes.c_size_t, [ctypes.c_int] * 3),
     "nvh_talk_rows": (ctypes.c_int, [ctypes.POINTER(PagedAttendDesc), ctypes.c_int, ctypes.c_int, ctypes.c_void_p]),
-    "nvh_talk_prompt_supported": (ctypes.c_int, [ctypes.c_int] * 4),
+    "nvh_talk_prompt_supported": (ctypes.c_int, [ctypes.c_int] * 5 + [ctypes.c_float]),
     "nvh_talk_prompt": (ctypes.c_int, [ctypes.POINTER(PagedAttendDesc), ctypes.c_int, ctypes.c_void_p]),
     "nvh_lightning_supported": (ctypes.c_int, [ctypes.c_int] * 2),
     "nvh_lightning_chunks": (ctypes.c_int, [ctypes.POINTER(LightningDesc), ctypes.c_int, ctypes.c_int, ctypes.c_void_p]),

@@ -42,7 +42,7 @@ class PagedAttention(nn.Module):
         self.fast = self.fast_prompt = dtype == torch.bfloat16 and heads * self.dv == self.out_cols
         if talk:
             self.fast = self.fast and ops.talk_rows_supported(heads, self.dk, self.dv, block_size)
-            self.fast_prompt = self.fast_prompt and ops.talk_prompt_supported(heads, self.dk, self.dv, block_size)
+            self.fast_prompt = self.fast_prompt and ops.talk_prompt_supported(heads, kv_heads, self.dk, self.dv, block_size, self.softcap)
         else:                                                # (the MFMA prompt kernel takes the maximum before the scale)
             self.fast = self.fast_prompt = self.fast and self.scale > 0 and ops.paged_attend_supported(self.dk, self.dv, block_size)
 
@@ -67,6 +67,8 @@ class PagedAttention(nn.Module):
             reg(n + "_norm", head_rows(get(n + ".norm").float(), 1 if shared else heads, self.dim, self.dk).reshape(-1).contiguous() if self.qk_norm else None)
         reg("sink", get("sink").float().contiguous() if self.has_sink else None)
         reg("talk", get("talk").float().contiguous() if self.talking else None)
+        if self.talking:
+            self.fast_prompt = self.fast_prompt and self.talk.abs().max().item() <= ops.TALK_PROMPT_MAX
         o = padded(get("o").reshape(self.in_width, h, self.vdim), self.in_width, h, self.dv).reshape(self.in_width, h * self.dv)
         reg("w_o", padded(o, c, self.out_cols).to(self.dtype).contiguous())
 

@@ -925,8 +925,11 @@ def talk_rows_supported(heads, dk, dv, block_size) -> bool:
     return bool(_lib.load().nvh_talk_rows_supported(int(heads), int(dk), int(dv), int(block_size)))
 
 
-def talk_prompt_supported(heads, dk, dv, block_size) -> bool:
-    return bool(_lib.load().nvh_talk_prompt_supported(int(heads), int(dk), int(dv), int(block_size)))
+TALK_PROMPT_MAX = 2000.0       # largest entry of a mixing matrix talk_prompt takes
+
+
+def talk_prompt_supported(heads, kv_heads, dk, dv, block_size, softcap) -> bool:
+    return bool(_lib.load().nvh_talk_prompt_supported(int(heads), int(kv_heads), int(dk), int(dv), int(block_size), float(softcap)))
 
 
 def _set_talk(d, talk, softcap, heads):

@@ -30,7 +30,7 @@ CONFIGS = {
                             attention(2, 1, 64, 64, 300, 30.0, 0.4, mlp=dense(70))], loop=(0, 3, 3)),
     # more query heads per key head than a pass takes, more heads than a tile of the mixing product, windows at page borders, wide heads, many experts
     "wide": config(192, 160, [attention(20, 2, 64, 128, 64, 8.0, 0.2, mlp=experts(64, 1.5, 32, 6)), attention(4, 1, 128, 64, 129, 15.0, 0.1, mlp=dense(192)),
-                              attention(12, 3, 192, 64, 65, 4.0, 0.1, mlp=experts(128, 0.4, 70, 5)), attention(8, 8, 70, 200, 128, 6.0, 0.15, mlp=dense(320))],
+                              attention(12, 3, 192, 64, 65, 4.0, 0.1, mlp=experts(128, 0.4, 70, 5)), attention(8, 4, 70, 200, 128, 6.0, 0.15, mlp=dense(320))],
                    eps=1e-6, scale=1.0, mult=1.0, positions=1024, loop=(1, 3, 2)),
     # beyond the fast kernels: wide keys, wide values, many heads; in bf16 too these layers, or their prompts, run on the plain kernels
     "plain": config(136, 90, [attention(2, 1, 270, 40, 30, 3.0, 0.1, mlp=experts(40, 2.0, 4, 2)), attention(40, 8, 16, 24, 90, 4.0, 0.3, mlp=dense(100)),

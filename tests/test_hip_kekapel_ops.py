@@ -29,9 +29,9 @@ def attend_ref(q, k, v, talk, pos, scale, cap, window=0, keep=0, sink=None):
     return torch.stack([p[h] @ f64(v)[:, h // ratio] for h in range(heads)], dim=1)
 
 
-SHAPES = [(6, 2, 20, 12), (20, 2, 64, 128), (3, 3, 40, 100), (12, 3, 128, 128), (4, 1, 192, 128), (8, 8, 70, 200), (16, 1, 64, 64), (32, 4, 128, 120), (1, 1, 64, 64),
-          (17, 17, 60, 64)]
-ROWS_ONLY = [(40, 8, 16, 24), (64, 4, 64, 64)]                           # more heads than the prompt kernel holds
+SHAPES = [(6, 2, 20, 12), (20, 2, 64, 128), (3, 3, 40, 100), (12, 3, 128, 128), (4, 1, 192, 128), (8, 4, 70, 200), (16, 1, 64, 64), (32, 4, 128, 120), (1, 1, 64, 64),
+          (17, 17, 60, 64), (12, 12, 128, 128), (32, 8, 128, 128), (9, 3, 256, 250)]
+ROWS_ONLY = [(40, 8, 16, 24), (64, 4, 64, 64), (14, 14, 128, 128)]     # more heads, or values of more heads, than the prompt kernel holds
 PLAIN = [(2, 1, 270, 300), (70, 10, 8, 8)]
 MASKS = [(0, 0), (1, 0), (64, 0), (65, 0), (100, 70), (7, 130)]
 
@@ -40,8 +40,10 @@ def test_supported_shapes():
     from nanovllm_hip import ops
     from nanovllm_hip.layers.paged_attention import padded_widths
     for shapes, rows, prompt in ((SHAPES, True, True), (ROWS_ONLY, True, False), (PLAIN, False, False)):
-        for h, _, *w in shapes:
-            assert (ops.talk_rows_supported(h, *padded_widths(*w), 64), ops.talk_prompt_supported(h, *padded_widths(*w), 64)) == (rows, prompt), (h, w)
+        for h, g, *w in shapes:
+            assert (ops.talk_rows_supported(h, *padded_widths(*w), 64), ops.talk_prompt_supported(h, g, *padded_widths(*w), 64, 5.0)) == (rows, prompt), (h, w)
+    for cap in (0.0, 2e4):
+        assert not ops.talk_prompt_supported(4, 2, 64, 64, 64, cap)
 
 
 @pytest.mark.parametrize("dtype,generic", [(BF16, False), (BF16, True), (F32, False)])
@@ -122,7 +124,7 @@ def test_prompt(heads, kvh, dim, vdim, window, keep):
     """Portions of several sequences (rows, keys) in one launch."""
     from nanovllm_hip import ops
     sink, talk = randn(heads, seed=6, dtype=F32) if keep else None, mixing(heads)
-    for cap, portions in ((3.0, PORTIONS[:5]), (0.0, PORTIONS[3:])) if heads <= 12 and dim <= 128 else ((15.0, PORTIONS[2:6]),):
+    for cap, portions in ((3.0, PORTIONS[:5]), (50.0, PORTIONS[3:])) if heads <= 12 and dim <= 128 else ((15.0, PORTIONS[2:6]),):
         pg = Pages([k for _, k in portions], kvh, dim, vdim, BF16, seed=3)
         q = randn(sum(r for r, _ in portions), heads, dim, seed=8)
         cu_q = torch.tensor([0] + [r for r, _ in portions]).cumsum(0).int().cuda()
