@@ -1,15 +1,14 @@
 // Attention with mixed heads over prompt portions (gfx950 MFMA): scores are capped (tanh) and mixed across the heads before the softmax, so one workgroup holds all
 // heads of 16 query rows and walks the visible keys 32 at a time:
-//   1  S^T = K Q^T with the keys as fragments straight from the page, capped, to LDS: a wave takes its own heads, or (one head per wave) the heads of a pair of
-//      waves over half of the keys
-//   2  the mixing matrix times the heads' scores, 16 (query, key) pairs per product, in place: a wave takes whole pairs, all heads of them.  Scores and matrix
-//      enter as the sum of two fp16 numbers each (22 bits; both scaled by powers of two so that the second one is a normal number), the sums are fp32
+//   1  S^T = K Q^T with the keys as fragments straight from the page, capped, to LDS: a wave takes its own heads, or the two heads of a pair of waves (they have the
+//      same keys) over half of the keys.  cap tanh(t) = cap - 2 cap / (1 + exp(2 t)): the first term mixes to a constant per head, which a softmax does not see, so only
+//      1 / (1 + exp(2 t)) is kept
+//   2  the mixing matrix times these, 16 (query, key) pairs per product, in place: a wave takes whole pairs, all heads of them.  Both factors enter as the sum of two
+//      fp16 numbers (22 bits; scaled by powers of two so that the second one is a normal number), the sums are fp32
 //   3  every wave, for its own heads: online softmax (log2 domain: the matrix carries log2 e), O^T = V^T P^T with the weights as bf16 hi + lo
 // Two barriers per 32 keys.  Values reach LDS by DMA, an image per key/value head that all waves read; with room for two images they are a step ahead.  The keys
 // of the next step are on their way into registers meanwhile.  What no query of the tile sees is not read.  A sink starts the running maximum and sum.
 // Algorithmic flops per launch: sum over sequences of (2 (DK + DV) + 2 heads) heads (visible pairs).
-#include <math.h>
-
 #include "attend_tile.h"
 #include "talk.h"
 
@@ -21,10 +20,10 @@ typedef _Float16 f16x8 __attribute__((ext_vector_type(8)));
 typedef __fp16 f16x2 __attribute__((ext_vector_type(2)));
 
 constexpr int kTile = 512;                           // scores of a head: 16 queries x 32 keys
-constexpr float kMixGain = 16.f;                     // of the mixing matrix
+constexpr float kMixGain = 16.f, kScoreGain = 4096.f;          // of the mixing matrix, of what step 1 keeps
 constexpr size_t kLdsBytes = 160 * 1024;
 
-// rows of scores in LDS (twice where a wave writes rows another one reads: one head per wave)
+// rows of scores in LDS (twice where a wave writes rows another one reads: PAIRS)
 __host__ __device__ constexpr int rows_held(int heads, int hpw) { return hpw == 1 ? (heads + 3) / 4 * 4 : (heads + 15) / 16 * 16; }
 // place of score i of head h: four groups of four heads read or written together lie in different banks
 __device__ __forceinline__ int score_at(int h, int i) { return h * kTile + (i ^ (((h >> 2) & 3) * 16)); }
@@ -44,6 +43,8 @@ __device__ __forceinline__ void read_v2(bf16x8& v0, bf16x8& v1, uint32_t at0, ui
     v0 = __builtin_bit_cast(bf16x8, u32x4{a[0], a[1], b[0], b[1]});
     v1 = __builtin_bit_cast(bf16x8, u32x4{c[0], c[1], d[0], d[1]});
 }
+// products that the vector pipe may read behind this: hipcc counts the wait states in between along one path into a join only
+__device__ __forceinline__ void settle(f32x4& u, f32x4& v) { asm volatile("s_nop 7" : "+v"(u), "+v"(v)); }
 // four numbers as their fp16 parts: hi of all four, then lo
 __device__ __forceinline__ f16x8 split4(const float (&x)[4]) {
     u32x4 r;
@@ -54,12 +55,13 @@ __device__ __forceinline__ f16x8 split4(const float (&x)[4]) {
     return __builtin_bit_cast(f16x8, r);
 }
 
-// waves of HPW heads each; MT: tiles of 16 heads.  gain: power of two the capped scores carry; images: of a key/value head's values, 1 or 2
-template <int DK, int DV, int HPW, int MT>
-__global__ __launch_bounds__(HPW == 1 ? 1024 : 512) void talk_prompt_kernel(const PagedAttendArgs a, const int q_tiles, const float gain, const int images) {
+// waves of HPW heads each; MT: tiles of 16 heads; PAIRS: step 1 in pairs of waves (HPW == 1, an even number of heads per key/value head).  images: of a key/value head's values, 1 or 2; rate: 2 log2(e) scale / cap; unscale: of a mixed score as step 2
+// leaves it (log2 domain); slack: 8 of that domain, unscaled
+template <int DK, int DV, int HPW, int MT, bool PAIRS>
+__global__ __launch_bounds__(HPW == 1 ? 1024 : 512) void talk_prompt_kernel(const PagedAttendArgs a, const int q_tiles, const int images, const float rate, const float unscale, const float slack) {
     constexpr int STEPS = DK / 32, DT = DV / 16, KB = 32, VROW = DV * 2, VIMG = KB * VROW, VP = DV / 8, NV = VIMG / 1024;
-    constexpr int SH = HPW == 1 ? 2 : HPW, HALVES = HPW == 1 ? 1 : 2;          // step 1: heads of a wave, halves of the keys
-    constexpr int PB = 2;                            // step 2: products at a time
+    constexpr int SH = PAIRS ? 2 : HPW, HALVES = PAIRS ? 1 : 2;                // step 1: heads of a wave, halves of the keys
+    constexpr int PB = HPW == 1 ? 1 : 2;                            // step 2: products at a time
     extern __shared__ __attribute__((aligned(16))) unsigned char lds[];        // [1 or 2][rows_held][kTile] scores, [images][kv heads] values, the mixing matrix
     int b, qt;
     {
@@ -72,16 +74,16 @@ __global__ __launch_bounds__(HPW == 1 ? 1024 : 512) void talk_prompt_kernel(cons
     if (q0 >= sq || sk < sq) return;
     const int shift = sk - sq;                       // query row r has position r + shift
     const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), waves = blockDim.x >> 6, lq = lane & 15, lg = lane >> 4;
-    const int heads = a.heads, ratio = heads / a.kv_heads, h0 = wave * HPW, s0 = HPW == 1 ? wave & ~1 : h0;
+    const int heads = a.heads, ratio = heads / a.kv_heads, h0 = wave * HPW, s0 = PAIRS ? wave & ~1 : h0;
     const int rows = sq - q0 < 16 ? sq - q0 : 16, first_pos = q0 + shift, last_pos = first_pos + rows - 1;
     const int window = a.window > 0 ? a.window : 0x40000000;
     const VisibleTiles vis = visible_tiles(first_pos, last_pos, a.window, a.keep_first);
     float* const scores_lds = reinterpret_cast<float*>(lds);
     const int score_rows = rows_held(heads, HPW), score_tile = score_rows * kTile;
-    unsigned char* vimg = lds + (HPW == 1 ? 2 : 1) * score_tile * 4;
+    unsigned char* vimg = lds + (PAIRS ? 2 : 1) * score_tile * 4;
     for (int i = heads * kTile + tid; i < score_tile; i += blockDim.x) {                                      // heads that do not exist
         scores_lds[i] = 0.f;
-        if (HPW == 1) scores_lds[score_tile + i] = 0.f;
+        if (PAIRS) scores_lds[score_tile + i] = 0.f;
     }
 
     // steps of 32 keys: the halves of the visible tiles, without those nobody sees
@@ -120,31 +122,30 @@ __global__ __launch_bounds__(HPW == 1 ? 1024 : 512) void talk_prompt_kernel(cons
     // (rows past the last key repeat it: not seen)
     auto load_k = [&](bf16x8 (&kf)[STEPS], int k0, const Place& at, int g, int half) {
         const int live = sk - k0, r = 16 * half + lq;
-        const uint16_t* p = at.keys + g * head_elems;
-        const uint32_t off = (r < live ? r : live - 1) * DK + 8 * lg;
+        const char* p = reinterpret_cast<const char*>(at.keys + g * head_elems);                              // (uniform base, 32-bit offset: one address register)
+        const uint32_t off = ((r < live ? r : live - 1) * DK + 8 * lg) * 2;
 #pragma unroll
-        for (int st = 0; st < STEPS; ++st) kf[st] = *reinterpret_cast<const bf16x8*>(p + (off + 32 * st));
+        for (int st = 0; st < STEPS; ++st) kf[st] = *reinterpret_cast<const bf16x8*>(p + off + 64 * st);
     };
     auto stage_v = [&](int k0, const Place& at, int image) {
         const int live = sk - k0;
-        const uint16_t* p = at.keys + (a.block_size * DK + at.row * (DV - DK));
+        const char* p = reinterpret_cast<const char*>(at.keys + (a.block_size * DK + at.row * (DV - DK)));
         unsigned char* to = vimg + image * a.kv_heads * VIMG;
         for (int i = wave; i < a.kv_heads * NV; i += waves) {
-            const int g = i / NV, s = (i - g * NV) * 64 + lane, r = s / VP, c = ((s - r * VP) ^ swz_v<DV>(r)) * 8;
-            dma16(p + (uint32_t)(g * head_elems + (r < live ? r : live - 1) * DV + c), to + i * 1024);
+            const int g = (unsigned)i / NV, r = (unsigned)((i - g * NV) * 64 + lane) / VP, c = ((lane & (VP - 1)) ^ swz_v<DV>(r)) * 8;
+            dma16(p + (uint32_t)(g * head_elems + (r < live ? r : live - 1) * DV + c) * 2u, to + i * 1024);
         }
     };
     const int end = 2 * vis.count;
     int it = next_step(-1);
     fetch(it >> 1);
     Place at = place(it);
-    const int g0 = (s0 < heads ? s0 : heads - 1) / ratio, half0 = HPW == 1 ? wave & 1 : 0;
+    const int g0 = (s0 < heads ? s0 : heads - 1) / ratio, half0 = PAIRS ? wave & 1 : 0;
     bf16x8 ka[STEPS], kb[HALVES == 2 ? STEPS : 1];
     load_k(ka, step_key(it), at, g0, half0);
     if (images == 2) stage_v(step_key(it), at, 0);
 
     const int my_q = q0 + lq, q_row = q_beg + (my_q < sq ? my_q : sq - 1), my_pos = my_q + shift;
-    const float unscale = 1.f / (gain * kMixGain), slack = 8.f / unscale;
     bf16x8 qf[SH][STEPS];
 #pragma unroll
     for (int j = 0; j < SH; ++j) {
@@ -159,8 +160,15 @@ __global__ __launch_bounds__(HPW == 1 ? 1024 : 512) void talk_prompt_kernel(cons
     for (int j = 0; j < HPW; ++j) {
 #pragma unroll
         for (int t = 0; t < DT; ++t) o[j][t] = f32x4{0.f, 0.f, 0.f, 0.f};
-        m[j] = a.sink ? a.sink[h0 + j < heads ? h0 + j : heads - 1] * (kLog2e / unscale) : -INFINITY;
-        l[j] = a.sink && lg == 0 ? 1.f : 0.f;
+        m[j] = -INFINITY;
+        l[j] = 0.f;
+        if (a.sink) {
+            const int h = h0 + j < heads ? h0 + j : heads - 1;
+            float row_sum = 0.f;
+            for (int g = 0; g < heads; ++g) row_sum += a.talk[h * heads + g];
+            m[j] = (a.sink[h] - a.softcap * row_sum) * (kLog2e / unscale);
+            l[j] = lg == 0 ? 1.f : 0.f;
+        }
     }
     // A operands: T[16 i + lq][16 c + 4 lg + (e & 3)], the parts of it, behind the images of values
     f16x8* mix = reinterpret_cast<f16x8*>(vimg + images * a.kv_heads * VIMG) + lane;
@@ -169,7 +177,7 @@ __global__ __launch_bounds__(HPW == 1 ? 1024 : 512) void talk_prompt_kernel(cons
 #pragma unroll
         for (int e = 0; e < 4; ++e) {
             const int r = 16 * (ic / MT) + lq, h = 16 * (ic % MT) + 4 * lg + e;
-            const float x = r < heads && h < heads ? a.talk[r * heads + h] * (kLog2e * kMixGain) : 0.f;
+            const float x = r < heads && h < heads ? a.talk[r * heads + h] * (-kLog2e * kMixGain) : 0.f;
             hi[e] = hi[e + 4] = (_Float16)x;
             lo[e] = lo[e + 4] = (_Float16)(x - (float)hi[e]);
         }
@@ -178,7 +186,6 @@ __global__ __launch_bounds__(HPW == 1 ? 1024 : 512) void talk_prompt_kernel(cons
     }
     // place in an image of value tile 0 (rows R0 and R0 + 16 share a swizzle); the swizzle is even, so tile t lies at this ^ 32 t
     const int R0 = 4 * lg + (lq >> 2), vplace = R0 * VROW + (lq & 1) * 8 + ((lq & 2) >> 1) * 16 + swz_v<DV>(R0) * 16;
-    const ScoreCap cap(a.scale, a.softcap, gain);
     int key_head[SH];
 #pragma unroll
     for (int j = 0; j < SH; ++j) key_head[j] = (s0 + j < heads ? s0 + j : heads - 1) / ratio;
@@ -191,40 +198,45 @@ __global__ __launch_bounds__(HPW == 1 ? 1024 : 512) void talk_prompt_kernel(cons
         const int k0 = step_key(it), next = next_step(it);
         const bool more = next < end;
         if (more) fetch(next >> 1);
-        const int next_k0 = step_key(next);
-        const Place next_at = place(next);
+        const int next_k0 = step_key(more ? next : it);                        // (behind the last step: that one again, not used)
+        const Place next_at = place(more ? next : it);
         // ---- 1: scores
         if constexpr (HALVES == 2) load_k(kb, k0, at, g0, 1);
-        // (what a product leaves is used in its own branch: hipcc counts the wait states between the two along one path into a join only)
+        auto product = [&](const auto& kf, int j) {
+            f32x4 s = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int st = 0; st < STEPS; ++st) s = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[st], qf[j][st], s, 0, 0, 0);
+            return s;
+        };
+        auto keep = [&](f32x4 s, int j, int half) {  // (heads that do not exist fill rows the matrix has zeros for)
+#pragma unroll
+            for (int i = 0; i < 4; ++i) s[i] = fast_rcp(fmaf(fast_exp2(s[i] * rate), 1.f / kScoreGain, 1.f / kScoreGain));
+            *reinterpret_cast<f32x4*>(ex + at1 + j * kTile + 256 * half) = s;
+        };
         auto scores = [&](auto& kf, int half) {
             int g = g0;
-            auto product = [&](int j) {
-                f32x4 s = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-                for (int st = 0; st < STEPS; ++st) s = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[st], qf[j][st], s, 0, 0, 0);
-                return s;
-            };
-            // (heads that do not exist fill rows the matrix has zeros for)
-            auto keep = [&](int j, f32x4 s) { *reinterpret_cast<f32x4*>(ex + at1 + j * kTile + 256 * half) = cap.capped(s); };
 #pragma unroll
             for (int j = 0; j < SH; j += 2) {
-                if (key_head[j] != g) load_k(kf, k0, at, key_head[j], half);
-                if (key_head[j] == key_head[j + 1]) {
-                    const f32x4 u = product(j), v = product(j + 1);
-                    keep(j, u);
-                    keep(j + 1, v);
+                if (!PAIRS && key_head[j] != g) load_k(kf, k0, at, key_head[j], half);
+                f32x4 u = product(kf, j);
+                g = key_head[j];
+                if constexpr (SH > 1) {
+                    if (!PAIRS && key_head[j + 1] != g) load_k(kf, k0, at, key_head[j + 1], half);
+                    f32x4 v = product(kf, j + 1);
+                    g = key_head[j + 1];
+                    settle(u, v);
+                    keep(u, j, half);
+                    keep(v, j + 1, half);
                 } else {
-                    keep(j, product(j));
-                    load_k(kf, k0, at, key_head[j + 1], half);
-                    keep(j + 1, product(j + 1));
+                    settle(u, u);
+                    keep(u, j, half);
                 }
-                g = key_head[j + 1];
             }
         };
         scores(ka, half0);
         if constexpr (HALVES == 2) scores(kb, 1);
         if (images == 2) asm volatile("s_waitcnt vmcnt(0)" ::: "memory");      // this step's values have landed
-        if (more) load_k(ka, next_k0, next_at, g0, half0);
+        load_k(ka, next_k0, next_at, g0, half0);
         lds_only_barrier();
         if (images == 1) stage_v(k0, at, 0);
         else if (more) stage_v(next_k0, next_at, image ^ 1);
@@ -329,7 +341,7 @@ __global__ __launch_bounds__(HPW == 1 ? 1024 : 512) void talk_prompt_kernel(cons
             }
         }
         image ^= images - 1;
-        if (HPW == 1) ex = scores_lds + (ex == scores_lds ? score_tile : 0);   // (a wave of the pair may be ahead)
+        if (PAIRS) ex = scores_lds + (ex == scores_lds ? score_tile : 0);   // (a wave of the pair may be ahead)
         it = next;
         at = next_at;
     }
@@ -350,27 +362,33 @@ int heads_per_wave(int heads, int dk, int dv) {
     const bool narrow = dk <= 128 && dv <= 128;
     return heads <= 16 ? (narrow ? 1 : 2) : heads <= 32 && narrow ? 4 : 0;
 }
+bool in_pairs(int heads, int kv_heads, int hpw) { return hpw == 1 && heads / kv_heads % 2 == 0; }
 size_t lds_bytes(int heads, int kv_heads, int hpw, int dv, int images) {
     const size_t mt = (heads + 15) / 16;
-    return (size_t)(hpw == 1 ? 2 : 1) * rows_held(heads, hpw) * kTile * 4 + (size_t)images * kv_heads * 64 * dv + mt * mt * 2048;
+    return (size_t)(in_pairs(heads, kv_heads, hpw) ? 2 : 1) * rows_held(heads, hpw) * kTile * 4 + (size_t)images * kv_heads * 64 * dv + mt * mt * 2048;
 }
 
-template <int DK, int DV, int HPW, int MT>
+template <int DK, int DV, int HPW, int MT, bool PAIRS>
 int launch_one(const PagedAttendArgs& a, hipStream_t stream) {
-    const int waves = HPW == 1 ? (a.heads + 1) / 2 * 2 : (a.heads + HPW - 1) / HPW, q_tiles = (a.max_q + 15) / 16;
+    const int waves = (a.heads + HPW - 1) / HPW, q_tiles = (a.max_q + 15) / 16;
     // two images where they take no workgroup's place
     const size_t one = lds_bytes(a.heads, a.kv_heads, HPW, DV, 1), two = lds_bytes(a.heads, a.kv_heads, HPW, DV, 2);
     const int images = two <= kLdsBytes && (two <= kLdsBytes / 2 || one > kLdsBytes / 2 || waves > 8) ? 2 : 1;
     const size_t lds = images == 2 ? two : one;
-    const float gain = exp2f(12.f - ceilf(log2f(a.softcap)));                  // (capped scores stay below 2^12)
-    if (lds > 64 * 1024) (void)hipFuncSetAttribute(reinterpret_cast<const void*>(talk_prompt_kernel<DK, DV, HPW, MT>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
-    talk_prompt_kernel<DK, DV, HPW, MT><<<a.batch * q_tiles, 64 * waves, lds, stream>>>(a, q_tiles, gain, images);
+    const float rate = 2.f * kLog2e * a.scale / a.softcap, unscale = 2.f * a.softcap / (kScoreGain * kMixGain);
+    const auto kernel = talk_prompt_kernel<DK, DV, HPW, MT, PAIRS>;
+    if (lds > 64 * 1024) (void)hipFuncSetAttribute(reinterpret_cast<const void*>(kernel), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+    kernel<<<a.batch * q_tiles, 64 * waves, lds, stream>>>(a, q_tiles, images, rate, unscale, 8.f / unscale);
     return check_launch("talk_prompt");
 }
 template <int DK, int DV>
 int launch_dims(const PagedAttendArgs& a, hipStream_t stream) {
-    if constexpr (DK <= 128 && DV <= 128) return a.heads > 16 ? launch_one<DK, DV, 4, 2>(a, stream) : launch_one<DK, DV, 1, 1>(a, stream);
-    else return launch_one<DK, DV, 2, 1>(a, stream);
+    if constexpr (DK <= 128 && DV <= 128) {
+        if (a.heads > 16) return launch_one<DK, DV, 4, 2, false>(a, stream);
+        return in_pairs(a.heads, a.kv_heads, 1) ? launch_one<DK, DV, 1, 1, true>(a, stream) : launch_one<DK, DV, 1, 1, false>(a, stream);
+    } else {
+        return launch_one<DK, DV, 2, 1, false>(a, stream);
+    }
 }
 template <int DK>
 int launch_key(const PagedAttendArgs& a, hipStream_t stream) {

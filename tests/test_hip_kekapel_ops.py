@@ -30,8 +30,8 @@ def attend_ref(q, k, v, talk, pos, scale, cap, window=0, keep=0, sink=None):
 
 
 SHAPES = [(6, 2, 20, 12), (20, 2, 64, 128), (3, 3, 40, 100), (12, 3, 128, 128), (4, 1, 192, 128), (8, 4, 70, 200), (16, 1, 64, 64), (32, 4, 128, 120), (1, 1, 64, 64),
-          (17, 17, 60, 64), (12, 12, 128, 128), (32, 8, 128, 128), (9, 3, 256, 250)]
-ROWS_ONLY = [(40, 8, 16, 24), (64, 4, 64, 64), (14, 14, 128, 128)]     # more heads, or values of more heads, than the prompt kernel holds
+          (17, 17, 60, 64), (14, 14, 128, 128), (32, 8, 128, 128), (9, 3, 256, 250)]
+ROWS_ONLY = [(40, 8, 16, 24), (64, 4, 64, 64), (16, 16, 128, 128)]     # more heads, or values of more heads, than the prompt kernel holds
 PLAIN = [(2, 1, 270, 300), (70, 10, 8, 8)]
 MASKS = [(0, 0), (1, 0), (64, 0), (65, 0), (100, 70), (7, 130)]
 
