@@ -47,7 +47,8 @@ int nvh_residual_norm(const nvh_residual_norm_desc* d, int dtype, void* stream) 
     REQUIRE(d, NVH_E_NULL, "residual_norm: null descriptor");
     if (d->rows == 0) return 0;
     DTYPE("residual_norm");
-    REQUIRE(d->x && (d->y || d->e || d->w || d->base || d->shift) && (!d->post_w || (d->post_b && (d->y || d->e))) && (!d->e || d->ew) && (!d->w || (d->b && (d->xb || d->packed))), NVH_E_NULL, "residual_norm: null pointer");
+    REQUIRE(d->x && (d->y || d->e || d->w || d->base || d->shift) && (!d->post_w || (d->post_b && (d->y || d->e))) && (!d->e || d->ew) &&
+            (!d->w || (d->b && (d->xb || d->packed))), NVH_E_NULL, "residual_norm: null pointer");
     REQUIRE(d->rows > 0 && d->cols > 0 && d->cols % 8 == 0 && d->cols <= 16384 && d->n > 0 && d->n <= d->cols && (!d->e || d->top > 0), NVH_E_SHAPE,
             "residual_norm: cols %d (%%8, <= 16384), mean over %d, top %d", d->cols, d->n, d->top);
     REQUIRE(!d->packed || (dtype == NVH_BF16 && d->cols % 32 == 0), NVH_E_SHAPE, "residual_norm: packed rows are bf16, cols %% 32 == 0");

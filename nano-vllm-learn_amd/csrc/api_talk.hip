@@ -48,7 +48,8 @@ int nvh_talk_prompt(const nvh_paged_attend_desc* d, int dtype, void* stream) {
     if (rc) return rc;
     REQUIRE(dtype == NVH_BF16, NVH_E_DTYPE, "talk_prompt: bf16 only");
     REQUIRE(d->cu_q && d->cu_k && d->out && !d->out_packed, NVH_E_NULL, "talk_prompt: null pointer or packed output");
-    REQUIRE(nvh_talk_prompt_supported(d->heads, d->kv_heads, d->dk, d->dv, d->block_size, d->softcap) && d->batch > 0 && d->max_q > 0 && (int64_t)d->batch * ((d->max_q + 15) / 16) <= 0x7fffffff, NVH_E_SHAPE,
+    REQUIRE(nvh_talk_prompt_supported(d->heads, d->kv_heads, d->dk, d->dv, d->block_size, d->softcap) && d->batch > 0 &&
+            d->max_q > 0 && (int64_t)d->batch * ((d->max_q + 15) / 16) <= 0x7fffffff, NVH_E_SHAPE,
             "talk_prompt: heads %d/%d, widths %d/%d page %d cap %g", d->heads, d->kv_heads, d->dk, d->dv, d->block_size, (double)d->softcap);
     return launch_talk_prompt(*d, (hipStream_t)stream);
 }

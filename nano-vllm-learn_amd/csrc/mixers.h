@@ -1,4 +1,4 @@
-// Launcher interface of the paged sink/window attention, lightning attention and mixture-of-experts kernels (api_mixers.hip validates), and the pieces
+// Launcher interface of the paged sink/window attention, lightning attention and mixture-of-experts kernels (the api_*.hip files validate), and the pieces
 // their kernels share.
 #pragma once
 #include "hybrid.h"

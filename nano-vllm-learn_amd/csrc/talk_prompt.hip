@@ -55,10 +55,12 @@ __device__ __forceinline__ f16x8 split4(const float (&x)[4]) {
     return __builtin_bit_cast(f16x8, r);
 }
 
-// waves of HPW heads each; MT: tiles of 16 heads; PAIRS: step 1 in pairs of waves (HPW == 1, an even number of heads per key/value head).  images: of a key/value head's values, 1 or 2; rate: 2 log2(e) scale / cap; unscale: of a mixed score as step 2
-// leaves it (log2 domain); slack: 8 of that domain, unscaled
+// waves of HPW heads each; MT: tiles of 16 heads; PAIRS: step 1 in pairs of waves (HPW == 1, an even number of heads per key/value head).
+// images: of a key/value head's values, 1 or 2; rate: 2 log2(e) scale / cap; unscale: what turns a mixed score as step 2 leaves it into the log2 domain; slack: 8 of
+// that domain, as step 2 leaves it
 template <int DK, int DV, int HPW, int MT, bool PAIRS>
-__global__ __launch_bounds__(HPW == 1 ? 1024 : 512) void talk_prompt_kernel(const PagedAttendArgs a, const int q_tiles, const int images, const float rate, const float unscale, const float slack) {
+__global__ __launch_bounds__(HPW == 1 ? 1024 : 512) void talk_prompt_kernel(const PagedAttendArgs a, const int q_tiles, const int images, const float rate,
+                                                                                const float unscale, const float slack) {
     constexpr int STEPS = DK / 32, DT = DV / 16, KB = 32, VROW = DV * 2, VIMG = KB * VROW, VP = DV / 8, NV = VIMG / 1024;
     constexpr int SH = PAIRS ? 2 : HPW, HALVES = PAIRS ? 1 : 2;                // step 1: heads of a wave, halves of the keys
     constexpr int PB = HPW == 1 ? 1 : 2;                            // step 2: products at a time

@@ -1,5 +1,6 @@
 """Zobasun, Galirax or Kekapel beside the closest other model (a Qwen2-shaped stack; for Kekapel also Galirax with windows in every layer) at equal size, on
-random weights: prefill and decode throughput through the engine, and each hot kernel against its roofline.  bench.py --beside SIZE [--beside-model NAME] prints the result as one JSON line."""
+random weights: prefill and decode throughput through the engine, and each hot kernel against its roofline.
+bench.py --beside SIZE [--beside-model NAME] prints the result as one JSON line."""
 from __future__ import annotations
 
 import time
@@ -18,7 +19,7 @@ from .models.kekapel import KekapelConfig
 from .models.qwen import ModelConfig
 from .models.zobasun import ZobasunConfig
 
-HBM_GBPS, MFMA_TFLOPS, MFMA32_TFLOPS = 8000.0, 2500.0, 157.3      # MI355X peaks (dense bf16, fp32 matrix)
+HBM_GBPS, MFMA_TFLOPS = 8000.0, 2500.0          # MI355X peaks (dense bf16)
 
 # width, feed-forward, layers; attention heads (128 wide); latent ranks and widths; recurrence width, blocks; experts (each ff / top wide)
 SIZES = {
@@ -128,11 +129,10 @@ def _time(calls, iters=10):
     return a.elapsed_time(b) * 1e3 / (iters * len(calls))
 
 
-def _line(us, nbytes=0, flops=0, flops32=0):
-    """flops: bf16 matrix products; flops32: those of the fp32 matrix pipe, which is the same pipe: their times add up"""
-    hbm, mfma = nbytes / (HBM_GBPS * 1e3), flops / (MFMA_TFLOPS * 1e6) + flops32 / (MFMA32_TFLOPS * 1e6)
-    return {"us": round(us, 2), "bound": "hbm" if hbm >= mfma else "mfma", "GBps": round(nbytes / us / 1e3, 1),
-            "TFLOPs": round((flops + flops32) / us / 1e6, 1), "roofline": round(max(hbm, mfma) / us, 4)}
+def _line(us, nbytes=0, flops=0):
+    floor = max(nbytes / (HBM_GBPS * 1e3), flops / (MFMA_TFLOPS * 1e6))
+    return {"us": round(us, 2), "bound": "hbm" if nbytes / HBM_GBPS * 1e3 >= flops / MFMA_TFLOPS else "mfma", "GBps": round(nbytes / us / 1e3, 1),
+            "TFLOPs": round(flops / us / 1e6, 1), "roofline": round(floor / us, 4)}
 
 
 def _randn(*shape, dtype=torch.bfloat16):
@@ -367,7 +367,7 @@ def kekapel_kernels(size, batch=32, ctx=1536, seqs=16, prompt=1024):
     for name, window in (("prompt", 0), (f"prompt, window {WINDOW}", WINDOW)):
         seen = seqs * (sum(min(t + 1, window) for t in range(prompt)) if window else prompt * (prompt + 1) / 2)
         us = _time([lambda x=x: ops.talk_prompt(x, cache, bt, cu, cu, prompt, h, g, d, d, scale, talk, cap, window=window, out=o) for x in qkv] * 2)
-        out[f"talk_{name}"] = _line(us, nbytes, 4 * d * h * seen, 2 * h * h * seen)
+        out[f"talk_{name}"] = _line(us, nbytes, (4 * d + 2 * h) * h * seen)
         us = _time([lambda x=x: ops.paged_attend_prompt(x, cache, bt, cu, cu, prompt, h, g, d, d, scale, window=window, out=o) for x in qkv] * 2)
         out[f"galirax paged_{name}"] = _line(us, nbytes, 4 * d * h * seen)
     del qkv, o, cache

@@ -34,7 +34,8 @@ def main(argv=None):
         ap.error(f"{cfg.name} runs in bfloat16 only")
     bs = cfg.kvcache_block_size
     blocks = -(-a.kvcache_tokens // bs) or sum(-(-(len(p) + a.max_tokens) // bs) for p in prompts)
-    engine = LLMEngine(cfg, blocks, weights=None if a.random_weights else a.model, max_model_len=min(a.max_model_len, getattr(cfg, "max_position_embeddings", a.max_model_len)), max_num_seqs=a.max_num_seqs,
+    longest = min(a.max_model_len, getattr(cfg, "max_position_embeddings", a.max_model_len))
+    engine = LLMEngine(cfg, blocks, weights=None if a.random_weights else a.model, max_model_len=longest, max_num_seqs=a.max_num_seqs,
                        max_num_batched_tokens=a.max_num_batched_tokens, enforce_eager=a.enforce_eager)
     for p, c in zip(prompts, engine.generate(prompts, a.max_tokens)):
         print(json.dumps({"prompt": p, "completion": c}))

@@ -1,6 +1,6 @@
 """Softmax attention with grouped heads over its own pages: optional projection biases, RMS norm over the whole query and key projections or over every head,
-rotation of the leading dimensions, a sliding window with kept first tokens, a learned sink per head, scores capped and mixed across the heads.  Every pass over the layer (a looped layer has several) has its own
-cache, bound by the runner (`page_cache` [passes, pages, block_size, kv_heads * (dk + dv)], inside a page [kv head][keys | values]).
+rotation of the leading dimensions, a sliding window with kept first tokens, a learned sink per head, scores capped and mixed across the heads.  Every pass
+over the layer (a looped layer has several) has its own cache, bound by the runner (`page_cache` [passes, pages, block_size, kv_heads * (dk + dv)], inside a page [kv head][keys | values]).
 
 Single rows (decode) stream the visible keys; prompt portions run the MFMA kernel over the pages.  Widths those kernels do not take, and fp32 models, use
 the plain kernel for both.  Padded widths (zeros): keys to 64 / 128 / 192 / 256, values to 64 / 128 / 256.

@@ -861,8 +861,8 @@ def _packed_ok(packed, rows, cols):
 
 def attn_prep(qkv, heads, kv_heads, dk, dv, positions, cos_sin, cache, slots, q_weight=None, k_weight=None, q_n=0, k_n=0, eps=0.0, head_norm=False):
     """Row ops behind a q | k | v projection: optional RMS norm over all query and all key columns (means over q_n / k_n of them; head_norm: over every head
-    by itself, weights [dk] shared by the heads), rotation of interleaved pairs of the first cos_sin.shape[1] dimensions of every head (None: no rotation), keys and values into the cache [pages, block_size, kv_heads * (dk + dv)]
-    (inside a page: [kv head][keys | values]).  The queries are rewritten in place."""
+    by itself, weights [dk] shared by the heads), rotation of interleaved pairs of the first cos_sin.shape[1] dimensions of every head (None: no rotation), keys
+    and values into the cache [pages, block_size, kv_heads * (dk + dv)] (inside a page: [kv head][keys | values]).  The queries are rewritten in place."""
     code = _act_code(qkv, cache)
     rows = qkv.shape[0]
     _require_i32(slots=slots)
