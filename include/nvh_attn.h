@@ -332,6 +332,11 @@ typedef struct nvh_linear_desc {
     size_t prefetch_bytes;
     /* SILU_MUL with glu_alpha != 0: the clamped gated unit of nvh_clamped_glu (limit glu_limit) instead of SiLU(g) * u */
     float glu_limit, glu_alpha;
+    /* SILU_MUL with glu_gelu != 0: gelu_tanh(g) * u (nvh_gelu_glu) instead */
+    int32_t glu_gelu;
+    /* NONE with x_packed, x_groups > 1: weight rows come in groups of x_group_rows (a multiple of 16; the last group may have any multiple of 16), group g is
+       applied to the activations at x + g * x_group_stride elements */
+    int32_t x_groups, x_group_rows, x_group_stride;
 } nvh_linear_desc;
 int nvh_linear_small_m_ex(const nvh_linear_desc* desc, int dtype, void* stream);
 /* residual[n_rows, hidden] += y (bf16, one rounding — the add of add_rms_forward, layers/layernorm.py:35-36) and, if `packed` is
@@ -461,6 +466,8 @@ int nvh_norm_residual(const nvh_norm_residual_desc* d, int dtype, void* stream);
 /* out[rows, inter] = g sigmoid(alpha g) (u + 1), g = min(gate, limit), u = clamp(up, -limit, limit); gate_up rows hold gate | up. */
 int nvh_clamped_glu(void* out, const void* gate_up, int rows, int inter, int64_t gate_up_row_stride, int64_t out_row_stride, float limit, float alpha,
                     int dtype, void* stream);
+/* gelu(gate) * up, the tanh form of gelu. */
+int nvh_gelu_glu(void* out, const void* gate_up, int rows, int inter, int64_t gate_up_row_stride, int64_t out_row_stride, int dtype, void* stream);
 /* Real-gated linear recurrent unit behind a causal depthwise convolution: log a = -rate sigmoid(ra u), S = a S + sqrt(1 - a^2) sigmoid(ri u) u,
  * out = S gelu(y).  nvh_rglru_chunks: portions of prompts (and single tokens), cut by the caller into segments that are
  * scanned side by side; segments of one portion are consecutive.  nvh_rglru_step: row i is one new token of sequence i (bf16; nvh_rglru_step_supported(block)).
@@ -590,10 +597,13 @@ typedef struct nvh_attn_prep_desc {
     const int32_t* slots;        /* [rows] page * block_size + offset; < 0: not stored */
     int32_t block_size;
     int32_t head_norm;           /* != 0: the norms run over every head by itself; q_w and k_w are [dk], shared by the heads, q_n and k_n the columns of a head */
+    const float* v_cos_sin;      /* nullable: values turn too, [max_position, v_rot] as cos_sin, the first v_rot <= dv dimensions of every head */
+    int32_t v_rot;
 } nvh_attn_prep_desc;
 int nvh_attn_prep(const nvh_attn_prep_desc* d, int dtype, void* stream);
 /* softmax(scale q . k) v over the keys a query sees: position j of its sequence if j <= its own and (window == 0 or nearer than `window` or
- * j < keep_first).  sink (nullable): exp(sink[head]) joins the denominator.  Query head h reads key/value head h / (heads / kv_heads).
+ * j < keep_first); with chunk > 0 (window 0) instead of a window: j / chunk == its own / chunk, or j < keep_first.  o_cos_sin (nullable): a head's output at
+ * position p is turned back, interleaved pairs of its first o_rot dimensions by minus the angles of row p (values stored turned, see nvh_attn_prep).  sink (nullable): exp(sink[head]) joins the denominator.  Query head h reads key/value head h / (heads / kv_heads).
  *   rows form   (nvh_paged_attend_rows): row i belongs to sequence row_seq[i] (or i); splits > 1: context splits, merged by the last workgroup to arrive
  *   portions    (nvh_paged_attend_prompt, bf16): rows cu_q[b] .. of sequence b are its last ones, cu_k[b + 1] - cu_k[b] keys in all
  * MFMA / streaming forms for the widths nvh_paged_attend_supported names; `generic` (rows form): the plain kernel, any width up to 2048. */
@@ -623,6 +633,9 @@ typedef struct nvh_paged_attend_desc {
     float softcap;               /* nvh_talk_*: 0 or the cap */
     float* scores;               /* nvh_talk_rows: [rows, span, nvh_talk_score_cols(heads)] scratch */
     int32_t span;                /* 64 times the most 64-key tiles a row sees */
+    int32_t chunk;               /* not for nvh_talk_* */
+    const float* o_cos_sin;      /* nullable: [max_position, o_rot]; not for nvh_talk_* */
+    int32_t max_position, o_rot;
 } nvh_paged_attend_desc;
 int nvh_paged_attend_supported(int dk, int dv, int block_size);
 size_t nvh_paged_attend_ticket_bytes(int rows, int kv_heads, int heads);
@@ -732,6 +745,164 @@ int nvh_residual_norm(const nvh_residual_norm_desc* d, int dtype, void* stream);
 int nvh_poly_norm(void* out, void* packed, const void* z, const float* coef, float eps, int rows, int cols, int n, int64_t z_stride, int64_t out_stride, int dtype, void* stream);
 /* x = cap * tanh(x / cap) in place, rows of `cols` elements. */
 int nvh_softcap(void* x, float cap, int rows, int cols, int64_t stride, int dtype, void* stream);
+
+/* ---- several residual streams, and what looks at the token before (csrc/streams.hip).
+ * Portions: row_seq [rows] and cu_rows [sequences + 1] give every row's sequence and the rows of a sequence's portion; both NULL: row i is the one new token of
+ * sequence i.  Rings hold a sequence's last rows, [slots, depth, cols] in the activation type, the row of position p at entry p % depth.  state_slots < 0: nothing
+ * is read or kept; nothing is read before position 0. */
+/* x = embed[token] + bigram[b], b = (previous token * mul_prev + token * mul_cur) mod buckets, or row `buckets` for a sequence's first token. */
+typedef struct nvh_bigram_embed_desc {
+    float* x;                    /* [rows, cols] */
+    const int64_t* tokens;       /* [rows] */
+    const int64_t* positions;    /* [rows] */
+    const int32_t* row_seq;
+    const int32_t* cu_rows;
+    const int32_t* state_slots;  /* [sequences] */
+    int64_t* last_token;         /* [slots] */
+    const void* embed;           /* [vocab, cols] */
+    const void* bigram;          /* [buckets + 1, cols] */
+    int64_t buckets, mul_prev, mul_cur;
+    int32_t rows, cols, vocab;
+} nvh_bigram_embed_desc;
+int nvh_bigram_embed(const nvh_bigram_embed_desc* d, int dtype, void* stream);
+
+/* Hyper-connections: with y given, x_t <- sum_s mix[s][t] x_s + out[t] y for all streams at once (to xout, if given); y2 given: y is first replaced by
+ * y_scale (rms(y) y_w + rms(y2) y2_w), means over n columns.  u = sum_s in[s] x_s (in NULL: plain sum) of the new streams goes to `sum`, and, with w given, its RMS
+ * norm in `groups` equal parts of the n columns, times w, to h and / or `packed`. */
+typedef struct nvh_stream_mix_desc {
+    const float* xin;            /* stream s of row r at xin + r * xin_row + s * xin_stream (xin_stream 0: all streams alike) */
+    int64_t xin_row, xin_stream;
+    float* xout;                 /* nullable: [rows, streams, cols]; may be xin */
+    int32_t rows, cols, n, streams;
+    const void* y;               /* nullable: [rows, cols] */
+    int64_t y_stride;
+    const void* y2;              /* nullable */
+    int64_t y2_stride;
+    const float* y_w;
+    const float* y2_w;
+    float y_scale;
+    const float* mix;            /* [streams, streams], [from][to] */
+    const float* out;            /* [streams] */
+    const float* in;             /* nullable: [streams] */
+    float* sum;                  /* nullable: [rows, cols] */
+    const float* w;              /* nullable: [cols], zero past n */
+    int32_t groups;
+    float eps;
+    void* h;                     /* nullable: [rows, cols] in the activation type */
+    void* packed;                /* nullable (bf16): the same in MFMA-fragment order */
+} nvh_stream_mix_desc;
+int nvh_stream_mix(const nvh_stream_mix_desc* d, int dtype, void* stream);
+
+/* s = h + (h' - h) shift with h' the previous token's h; mixes == 0: out = s; otherwise out[k] = s + (s' - s) mu[k] with s' the previous token's s (zeros before the
+ * first token).  Depth of the ring: 2 without mixes, 3 with. */
+typedef struct nvh_token_shift_desc {
+    const void* h;               /* [rows, cols], row stride h_stride */
+    int64_t h_stride;
+    int32_t rows, cols;
+    const float* shift;          /* [cols] */
+    const float* mu;             /* [mixes, cols] */
+    int32_t mixes;
+    void* out;                   /* [max(mixes, 1)][rows, cols], out_mix elements apart; packed != 0 (bf16): each in MFMA-fragment order */
+    int64_t out_mix;
+    int32_t packed;
+    void* ring;
+    int32_t depth;
+    const int64_t* positions;
+    const int32_t* row_seq;
+    const int32_t* cu_rows;
+    const int32_t* state_slots;
+    int32_t sequences;
+} nvh_token_shift_desc;
+int nvh_token_shift(const nvh_token_shift_desc* d, int dtype, void* stream);
+
+/* silu(b + sum over taps of w[tap] x), the last tap on the current token; ring of `taps` rows. */
+typedef struct nvh_causal_conv_desc {
+    const void* x;               /* [rows, cols], row stride x_stride */
+    int64_t x_stride;
+    int32_t rows, cols, taps;
+    const float* w;              /* [taps, cols] */
+    const float* b;              /* [cols] */
+    void* out;                   /* nullable: [rows, cols] */
+    void* packed;                /* nullable (bf16): the same in MFMA-fragment order */
+    void* ring;
+    const int64_t* positions;
+    const int32_t* row_seq;
+    const int32_t* cu_rows;
+    const int32_t* state_slots;
+    int32_t sequences;
+} nvh_causal_conv_desc;
+int nvh_causal_conv(const nvh_causal_conv_desc* d, int dtype, void* stream);
+
+/* Selective scan: S[c][n] <- exp(dt_c A[c][n]) S[c][n] + dt_c x_c B[n], y_c = sum_n S[c][n] C[n] + d_c x_c, out = y silu(z), dt = softplus(. + dt_bias).  The state is
+ * fp32; a token at position 0 takes it as zero.  nvh_scan_states(n): the number of states kept for n of them (0: too many).
+ *   portions (nvh_scan_chunks)  dt [rows, inner]; cut into segments as for nvh_rglru_chunks
+ *   single   (nvh_scan_step)    bf16; row i is one new token of sequence i; dt [rows, rank] is multiplied by w_dt [inner, rank] first */
+typedef struct nvh_scan_desc {
+    const void* x;               /* [rows, inner] */
+    int64_t x_stride;
+    const void* dt;
+    int64_t dt_stride;
+    const float* dt_bias;        /* [inner] */
+    const void* bc;              /* [rows, n | n]: B | C */
+    int64_t bc_stride;
+    const void* z;               /* [rows, inner] */
+    int64_t z_stride;
+    const float* a_log2;         /* [inner, n]: A log2(e) */
+    const float* d;              /* [inner] */
+    int32_t rows, inner, n;
+    const int64_t* positions;    /* [rows] */
+    const int32_t* state_slots;  /* [sequences]; < 0: nothing is read or kept */
+    float* state;                /* [slots, inner, n] */
+    const int32_t* chunks;       /* [n_chunks, 4]: first row, rows, sequence, index of the segment in its sequence's portion */
+    int32_t n_chunks;
+    int32_t summaries;           /* != 0: some portion has more than one segment */
+    float* seg_state;            /* summaries: [n_chunks, inner, n] scratch */
+    float* seg_dt;               /* summaries: [n_chunks, inner] scratch */
+    const void* w_dt;
+    int32_t rank;
+    void* out;                   /* [rows, inner], row stride out_stride (single tokens: nullable) */
+    int64_t out_stride;
+    void* out_packed;            /* nullable (single tokens): the same in MFMA-fragment order */
+} nvh_scan_desc;
+int nvh_scan_states(int n);
+int nvh_scan_chunks(const nvh_scan_desc* d, int dtype, void* stream);
+int nvh_scan_step(const nvh_scan_desc* d, int dtype, void* stream);
+
+/* Time mixing: per head o = (S + diag(u) k v^T)^T r, S <- diag(w) S + k v^T with w = exp(-exp(z + w0)) per token and key channel, then
+ * out = o / sqrt(mean over n columns of o^2 + eps) * norm * silu(g).  The state is fp32; a token at position 0 takes it as zero.
+ *   portions (nvh_wkv_chunks)  z [rows, heads * dim]; cut into segments as for nvh_rglru_chunks; generic: the plain token-by-token kernel, any width
+ *   single   (nvh_wkv_step)    bf16; row i is one new token of sequence i; z [rows, rank]: w2 tanh(z) is computed first; nvh_wkv_supported(dim) */
+typedef struct nvh_wkv_desc {
+    const void* r;               /* r, k, v, g: [rows, heads * dim], one row stride */
+    const void* k;
+    const void* v;
+    const void* g;
+    int64_t stride;
+    const void* z;
+    int64_t z_stride;
+    const float* w0;             /* [heads * dim] */
+    const float* u;              /* [heads * dim] */
+    const float* norm;           /* [heads * dim] */
+    float eps;
+    int32_t n;                   /* columns of a head that count (the rest is zero padding) */
+    int32_t rows, heads, dim;
+    const void* w2;              /* [heads * dim, rank] */
+    int32_t rank;
+    const int64_t* positions;    /* [rows] */
+    const int32_t* state_slots;  /* [sequences]; < 0: nothing is read or kept */
+    float* state;                /* [slots, heads, dim, dim]: [key][value] */
+    const int32_t* chunks;       /* [n_chunks, 4]: first row, rows, sequence, index of the segment in its sequence's portion */
+    int32_t n_chunks;
+    int32_t summaries;           /* != 0: some portion has more than one segment */
+    float* seg_state;            /* summaries: [n_chunks, heads, dim, dim] scratch */
+    float* seg_decay;            /* summaries: [n_chunks, heads * dim] scratch */
+    void* out;                   /* [rows, heads * dim], row stride out_stride (single tokens: nullable) */
+    int64_t out_stride;
+    void* out_packed;            /* nullable (single tokens): the same in MFMA-fragment order */
+} nvh_wkv_desc;
+int nvh_wkv_supported(int dim);
+int nvh_wkv_chunks(const nvh_wkv_desc* d, int generic, int dtype, void* stream);
+int nvh_wkv_step(const nvh_wkv_desc* d, int dtype, void* stream);
 
 #ifdef __cplusplus
 }

@@ -23,6 +23,7 @@ LINEAR_SOURCES = ["api_layers.hip", "api_rows.hip", "layer_ops.hip", "skinny_gem
 MODEL_SOURCES = {
     "Zobasun": ["api_hybrid.hip", "rglru.hip", "latent_attention.hip", "latent_prefill.hip"],
     "Galirax": ["api_paged.hip", "attn_prep.hip", "paged_attend.hip", "paged_prompt.hip", "api_lightning.hip", "lightning.hip", "api_moe.hip", "moe.hip"],
+    "Zaposun": ["api_paged.hip", "attn_prep.hip", "paged_attend.hip", "paged_prompt.hip", "streams.hip", "mamba.hip", "wkv.hip"],
     "Kekapel": ["api_talk.hip", "attn_prep.hip", "talk_rows.hip", "talk_prompt.hip", "api_moe.hip", "moe.hip"],
 }
 SOURCES = ["api.hip", "store_kvcache.hip", "paged_decode.hip", "prefill_mfma.hip", "rope_store.hip", "allreduce_oneshot.hip", "qkv_attend.hip", *LINEAR_SOURCES,

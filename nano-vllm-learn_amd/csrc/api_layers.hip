@@ -168,10 +168,20 @@ int nvh::linear_args(LinearArgs& a, const nvh_linear_desc* d, int dtype) {
     a.M = d->m; a.N = d->n; a.K = d->k; a.inter = d->silu_inter; a.x_stride = d->x_row_stride; a.out_stride = d->out_row_stride;
     if (d->norm_folded && d->norm_weight) { set_error("linear_small_m_ex: norm_folded excludes norm_weight"); return NVH_E_NULL; }
     a.norm_w = (const uint16_t*)d->norm_weight; a.norm_eps = d->norm_eps; a.epi = d->epilogue;
-    a.glu_limit = d->glu_limit; a.glu_alpha = d->glu_alpha;
+    a.glu_limit = d->glu_limit; a.glu_alpha = d->glu_alpha; a.glu_gelu = d->glu_gelu;
+    a.x_groups = 0;
     a.norm_mode = d->norm_folded ? 2 : (d->norm_weight ? 1 : 0);
     a.positions = d->positions; a.cos_sin = d->cos_sin; a.k_cache = (uint16_t*)d->k_cache; a.v_cache = (uint16_t*)d->v_cache;
     a.slots = d->slot_mapping; a.h = d->h; a.kvh = d->kvh; a.hd = d->hd;
+    if (d->epilogue == NVH_EPI_NONE) a.inter = a.hd = 0;
+    if (d->x_groups > 1) {
+        if (d->epilogue != NVH_EPI_NONE || !d->x_packed || d->candidate_val || d->x_group_rows <= 0 || d->x_group_rows % 16 ||
+            (int64_t)d->x_group_rows * (d->x_groups - 1) >= d->n || d->x_group_stride < (d->m + 15) / 16 * 16 * d->k || d->x_group_stride % 8) {
+            set_error("linear_small_m_ex: x groups need packed activations, the NONE epilogue, rows %% 16 == 0 and a stride of whole packed rows");
+            return NVH_E_SHAPE;
+        }
+        a.x_groups = d->x_groups; a.inter = d->x_group_rows; a.hd = d->x_group_stride;
+    }
     a.stamps = g_stamps;
     a.x_packed = d->x_packed; a.out_packed = (uint16_t*)d->out_packed; a.ws_raw = d->workspace; a.ws_bytes = d->workspace_bytes;
     a.ws = nullptr; a.counters = nullptr; a.ksplit = 1; a.tiles = 0;

@@ -32,15 +32,30 @@ int nvh_norm_residual(const nvh_norm_residual_desc* d, int dtype, void* stream) 
     return launch_norm_residual(*d, dtype == NVH_F32, (hipStream_t)stream);
 }
 
+namespace {
+
+int check_glu(const char* fn, void* out, const void* gate_up, int rows, int inter, int64_t gate_up_row_stride, int64_t out_row_stride, int dtype) {
+    DTYPE(fn);
+    REQUIRE(out && gate_up, NVH_E_NULL, "%s: null pointer", fn);
+    REQUIRE(rows > 0 && inter > 0 && inter % 8 == 0 && gate_up_row_stride >= 2 * (int64_t)inter && gate_up_row_stride % 8 == 0 && out_row_stride >= inter && out_row_stride % 8 == 0,
+            NVH_E_SHAPE, "%s: inter %d (%%8) / row strides", fn, inter);
+    REQUIRE(aligned16(out) && aligned16(gate_up), NVH_E_ALIGN, "%s: pointers must be 16-byte aligned", fn);
+    return 0;
+}
+
+}  // namespace
+
 int nvh_clamped_glu(void* out, const void* gate_up, int rows, int inter, int64_t gate_up_row_stride, int64_t out_row_stride, float limit, float alpha,
                     int dtype, void* stream) {
     if (rows == 0) return 0;
-    DTYPE("clamped_glu");
-    REQUIRE(out && gate_up, NVH_E_NULL, "clamped_glu: null pointer");
-    REQUIRE(rows > 0 && inter > 0 && inter % 8 == 0 && gate_up_row_stride >= 2 * (int64_t)inter && gate_up_row_stride % 8 == 0 && out_row_stride >= inter && out_row_stride % 8 == 0,
-            NVH_E_SHAPE, "clamped_glu: inter %d (%%8) / row strides", inter);
-    REQUIRE(aligned16(out) && aligned16(gate_up), NVH_E_ALIGN, "clamped_glu: pointers must be 16-byte aligned");
-    return launch_clamped_glu(out, gate_up, rows, inter, gate_up_row_stride, out_row_stride, limit, alpha, dtype == NVH_F32, (hipStream_t)stream);
+    const int rc = check_glu("clamped_glu", out, gate_up, rows, inter, gate_up_row_stride, out_row_stride, dtype);
+    return rc ? rc : launch_clamped_glu(out, gate_up, rows, inter, gate_up_row_stride, out_row_stride, limit, alpha, dtype == NVH_F32, (hipStream_t)stream);
+}
+
+int nvh_gelu_glu(void* out, const void* gate_up, int rows, int inter, int64_t gate_up_row_stride, int64_t out_row_stride, int dtype, void* stream) {
+    if (rows == 0) return 0;
+    const int rc = check_glu("gelu_glu", out, gate_up, rows, inter, gate_up_row_stride, out_row_stride, dtype);
+    return rc ? rc : launch_gelu_glu(out, gate_up, rows, inter, gate_up_row_stride, out_row_stride, dtype == NVH_F32, (hipStream_t)stream);
 }
 
 int nvh_residual_norm(const nvh_residual_norm_desc* d, int dtype, void* stream) {

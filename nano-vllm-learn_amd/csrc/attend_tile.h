@@ -55,12 +55,12 @@ struct TileImages {
 //   query(qs, st)        query fragment: row lq of sub-tile qs, columns 32 st + 8 lg .. (B operand of S^T)
 //   first_key(it)        key of the tile's first row; covers(kv0): this wave sees something of that tile; masked(kv0): but not all of it:
 //   sees(kv0, qs, off)   key kv0 + 4 lg + off counts for the lane's query of sub-tile qs
-//   row(qs)              where the lane's query of sub-tile qs goes, or null
+//   row(qs)              where the lane's query of sub-tile qs goes, or null; last(qs, d, v): what becomes of its 4 output columns from d on
 // start: score (log2 domain) of a softmax entry without key and value, -inf for none.
 // (The sums, the fragments and the tile loop live in ONE function: split up, the same code takes 32 registers more.)
-template <int DK, int DV, int QT, typename Stage, typename Query, typename FirstKey, typename Covers, typename Masked, typename Sees, typename Row>
+template <int DK, int DV, int QT, typename Stage, typename Query, typename FirstKey, typename Covers, typename Masked, typename Sees, typename Row, typename Last>
 __device__ __forceinline__ void attend_walk(unsigned char* lds, int n_tiles, float scale_log2, float start, int lane, Stage stage, Query query, FirstKey first_key, Covers covers,
-                                            Masked need_mask, Sees sees, Row row) {
+                                            Masked need_mask, Sees sees, Row row, Last last) {
     using Images = TileImages<DK, DV>;
     constexpr int BN = Images::BN, KROW = Images::KROW, VROW = Images::VROW, KIMG = Images::KIMG, VIMG = Images::VIMG, NK = Images::NK, NV = Images::NV;
     constexpr int STEPS = DK / 32, DT = DV / 16, NT = BN / 16;
@@ -216,7 +216,7 @@ __device__ __forceinline__ void attend_walk(unsigned char* lds, int n_tiles, flo
         if (!out) continue;
         const float inv = sum > 0.f ? 1.f / sum : 0.f;
 #pragma unroll
-        for (int t = 0; t < DT; ++t) act_st4(out + 16 * t + 4 * lg, o[qs][t] * inv);
+        for (int t = 0; t < DT; ++t) act_st4(out + 16 * t + 4 * lg, last(qs, 16 * t + 4 * lg, o[qs][t] * inv));
     }
 }
 

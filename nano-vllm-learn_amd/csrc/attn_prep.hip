@@ -1,5 +1,5 @@
 // Row ops between a q | k | v projection and attention over pages: norm of queries and keys (over all columns of the projection at once, or per head with one
-// weight for all heads), rotation of interleaved pairs, store of keys and values: one launch over the projection's rows.
+// weight for all heads), rotation of interleaved pairs (of values too, where they are stored turned), store of keys and values: one launch over the projection's rows.
 #include <type_traits>
 
 #include "api_common.h"
@@ -8,6 +8,36 @@
 namespace nvh {
 
 namespace {
+
+// interleaved pairs of 8 elements from dimension d on, turned by a table row (cos | sin of `rot` / 2 angles); dimensions past `rot` pass
+__device__ __forceinline__ f32x8 turn8(const f32x8& r, const float* cs, int rot, int d) {
+    float e[8] = {r.a[0], r.a[1], r.a[2], r.a[3], r.b[0], r.b[1], r.b[2], r.b[3]};
+    float co[4], si[4];
+    if ((rot & 7) == 0) {                            // (whole pieces turn or pass)
+        const bool turns = d < rot;
+        const f32x4 cv = turns ? *reinterpret_cast<const f32x4*>(cs + d / 2) : f32x4{1.f, 1.f, 1.f, 1.f};
+        const f32x4 sv = turns ? *reinterpret_cast<const f32x4*>(cs + rot / 2 + d / 2) : f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int p = 0; p < 4; ++p) {
+            co[p] = cv[p];
+            si[p] = sv[p];
+        }
+    } else {
+#pragma unroll
+        for (int p = 0; p < 4; ++p) {
+            const bool turns = d / 2 + p < rot / 2;
+            co[p] = turns ? cs[d / 2 + p] : 1.f;
+            si[p] = turns ? cs[rot / 2 + d / 2 + p] : 0.f;
+        }
+    }
+#pragma unroll
+    for (int p = 0; p < 4; ++p) {
+        const float u = e[2 * p], w = e[2 * p + 1];
+        e[2 * p] = u * co[p] - w * si[p];
+        e[2 * p + 1] = w * co[p] + u * si[p];
+    }
+    return {f32x4{e[0], e[1], e[2], e[3]}, f32x4{e[4], e[5], e[6], e[7]}};
+}
 
 // one workgroup per row; a thread keeps its 8-element pieces of [q | k | v] in registers between the sums and the second pass
 // HEADS: the norm runs over every head of queries and keys by itself
@@ -18,7 +48,7 @@ __global__ __launch_bounds__(256) void attn_prep_kernel(const AttnPrepArgs a) {
     T* x = reinterpret_cast<T*>(a.qkv) + row * a.qkv_stride;
     const int nq = a.heads * a.dk, nk = a.kv_heads * a.dk, total = nq + nk + a.kv_heads * a.dv;
     int64_t pos = a.positions[row];
-    if (a.rot > 0 && pos >= a.max_position) pos = a.max_position - 1;
+    if ((a.rot > 0 || a.v_cos_sin) && pos >= a.max_position) pos = a.max_position - 1;
     const float* cs = a.cos_sin + pos * a.rot;
     const int slot = a.slots[row];
     const int page = slot >= 0 ? slot / a.block_size : 0, off = slot >= 0 ? slot - page * a.block_size : 0;
@@ -83,38 +113,12 @@ __global__ __launch_bounds__(256) void attn_prep_kernel(const AttnPrepArgs a) {
                 r.a *= inv * *reinterpret_cast<const f32x4*>(w);
                 r.b *= inv * *reinterpret_cast<const f32x4*>(w + 4);
             }
-            if (a.rot > 0) {
-                float e[8] = {r.a[0], r.a[1], r.a[2], r.a[3], r.b[0], r.b[1], r.b[2], r.b[3]};
-                float co[4], si[4];
-                if ((a.rot & 7) == 0) {                  // (whole pieces turn or pass)
-                    const bool turns = d < a.rot;
-                    const f32x4 cv = turns ? *reinterpret_cast<const f32x4*>(cs + d / 2) : f32x4{1.f, 1.f, 1.f, 1.f};
-                    const f32x4 sv = turns ? *reinterpret_cast<const f32x4*>(cs + a.rot / 2 + d / 2) : f32x4{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-                    for (int p = 0; p < 4; ++p) {
-                        co[p] = cv[p];
-                        si[p] = sv[p];
-                    }
-                } else {
-#pragma unroll
-                    for (int p = 0; p < 4; ++p) {
-                        const bool turns = d / 2 + p < a.rot / 2;
-                        co[p] = turns ? cs[d / 2 + p] : 1.f;
-                        si[p] = turns ? cs[a.rot / 2 + d / 2 + p] : 0.f;
-                    }
-                }
-#pragma unroll
-                for (int p = 0; p < 4; ++p) {
-                    const float u = e[2 * p], w = e[2 * p + 1];
-                    e[2 * p] = u * co[p] - w * si[p];
-                    e[2 * p + 1] = w * co[p] + u * si[p];
-                }
-                r = {f32x4{e[0], e[1], e[2], e[3]}, f32x4{e[4], e[5], e[6], e[7]}};
-            }
+            if (a.rot > 0) r = turn8(r, cs, a.rot, d);
             if (is_q) act_st8(x + c, r);
             else if (slot >= 0) act_st8(cache + (int64_t)h * a.block_size * (a.dk + a.dv) + off * a.dk + d, r);
         } else if (slot >= 0) {
             const int h = (c - nq - nk) / a.dv, d = c - nq - nk - h * a.dv;
+            if (a.v_cos_sin) r = turn8(r, a.v_cos_sin + pos * a.v_rot, a.v_rot, d);
             act_st8(cache + (int64_t)h * a.block_size * (a.dk + a.dv) + (int64_t)a.block_size * a.dk + (int64_t)off * a.dv + d, r);
         }
     }
@@ -154,7 +158,7 @@ extern "C" int nvh_attn_prep(const nvh_attn_prep_desc* d, int dtype, void* strea
     REQUIRE(d->qkv && d->positions && (d->cos_sin || d->rot == 0) && d->cache && d->slots && (!d->q_w == !d->k_w), NVH_E_NULL, "attn_prep: null pointer");
     const int64_t cols = (int64_t)d->heads * d->dk + (int64_t)d->kv_heads * (d->dk + d->dv);
     REQUIRE(d->rows > 0 && d->heads > 0 && d->kv_heads > 0 && d->dk > 0 && d->dk % 8 == 0 && d->dv > 0 && d->dv % 8 == 0 && cols <= kMaxRowCols && d->rot >= 0 && d->rot % 2 == 0 &&
-            d->rot <= d->dk && (d->rot == 0 || d->max_position > 0) && d->block_size > 0 && (!d->q_w || (d->q_n > 0 && d->k_n > 0)) && (!d->head_norm || d->q_w), NVH_E_SHAPE,
+            d->rot <= d->dk && ((d->rot == 0 && !d->v_cos_sin) || d->max_position > 0) && (!d->v_cos_sin || (d->v_rot > 0 && d->v_rot % 2 == 0 && d->v_rot <= d->dv)) && d->block_size > 0 && (!d->q_w || (d->q_n > 0 && d->k_n > 0)) && (!d->head_norm || d->q_w), NVH_E_SHAPE,
             "attn_prep: heads %d/%d widths %d/%d rot %d (row of at most %d)", d->heads, d->kv_heads, d->dk, d->dv, d->rot, kMaxRowCols);
     REQUIRE(d->qkv_stride % 8 == 0 && d->qkv_stride >= cols, NVH_E_STRIDE, "attn_prep: row stride");
     REQUIRE(aligned16(d->qkv) && aligned16(d->cache) && aligned16(d->q_w) && aligned16(d->k_w), NVH_E_ALIGN, "attn_prep: pointers must be 16-byte aligned");

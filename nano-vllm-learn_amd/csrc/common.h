@@ -126,8 +126,14 @@ __device__ __forceinline__ float clamped_glu(float gate, float up, float limit, 
     return g / (1.f + __expf(-alpha * g)) * (u + 1.f);
 }
 
-// the gated unit of a gate_up projection: the clamped one when alpha != 0, SiLU(g) u with the gate rounded to bf16 first otherwise
-__device__ __forceinline__ float gated_unit(float g, float u, float limit, float alpha) {
+__device__ __forceinline__ float gelu_tanh_f(float z) {          // 0.5 z (1 + tanh(k (z + 0.044715 z^3))) with tanh(t) = 1 - 2 / (1 + exp(2t))
+    const float t = 0.7978845608028654f * (z + 0.044715f * z * z * z);
+    return z - z / (1.f + __expf(2.f * t));
+}
+
+// the gated unit of a gate_up projection: gelu(g) u, the clamped one when alpha != 0, SiLU(g) u with the gate rounded to bf16 first otherwise
+__device__ __forceinline__ float gated_unit(float g, float u, float limit, float alpha, int gelu) {
+    if (gelu) return gelu_tanh_f(g) * u;
     if (alpha != 0.f) return clamped_glu(g, u, limit, alpha);
     return (float)(__bf16)(g / (1.f + __expf(-g))) * u;
 }

@@ -24,10 +24,6 @@ __device__ __forceinline__ float act_round(float v, const uint16_t*) { return (f
 __device__ __forceinline__ float act_round(float v, const float*) { return v; }
 
 __device__ __forceinline__ float sigmoid_f(float x) { return 1.f / (1.f + __expf(-x)); }
-__device__ __forceinline__ float gelu_tanh_f(float z) {          // 0.5 z (1 + tanh(k (z + 0.044715 z^3))) with tanh(t) = 1 - 2 / (1 + exp(2t))
-    const float t = 0.7978845608028654f * (z + 0.044715f * z * z * z);
-    return z - z / (1.f + __expf(2.f * t));
-}
 
 // sum over a 256-thread workgroup; `lds` holds at least 4 floats and is free again after the next barrier
 __device__ __forceinline__ float block_sum256(float v, float* lds) {
@@ -45,6 +41,7 @@ int launch_embed_rows(float* x, void* xb, void* packed, const int64_t* tokens, c
 using NormResidualArgs = nvh_norm_residual_desc;
 int launch_norm_residual(const NormResidualArgs& a, int f32, hipStream_t stream);
 int launch_clamped_glu(void* out, const void* gate_up, int rows, int inter, int64_t gu_stride, int64_t out_stride, float limit, float alpha, int f32, hipStream_t stream);
+int launch_gelu_glu(void* out, const void* gate_up, int rows, int inter, int64_t gu_stride, int64_t out_stride, int f32, hipStream_t stream);
 
 // ---- gated linear recurrence (rglru.hip)
 constexpr int kRglruChunk = 64;  // tokens a workgroup scans at a time

@@ -5,7 +5,7 @@
 //                  norm of the new row (what the next sublayers read)
 //   poly_norm      a N(z) + b N(z^2) + c N(z^3) + e, powers by element, N(v) = v / sqrt(mean(v^2) + eps) over the row
 //   softcap        cap * tanh(x / cap)
-//   clamped_glu    g * sigmoid(alpha g) * (u + 1) with g = min(gate, limit), u = clamp(up, -limit, limit)
+//   clamped_glu    g * sigmoid(alpha g) * (u + 1) with g = min(gate, limit), u = clamp(up, -limit, limit);  gelu_glu  gelu_tanh(gate) * up
 // HBM-bound row streams; one workgroup per row where a norm needs the whole row.  Every op exists for bf16 and for fp32 activations.
 #include <type_traits>
 
@@ -67,7 +67,7 @@ __global__ __launch_bounds__(256) void norm_residual_kernel(const NormResidualAr
     }
 }
 
-template <typename T>
+template <typename T, bool GELU>
 __global__ __launch_bounds__(256) void clamped_glu_kernel(T* __restrict__ out, const T* __restrict__ gu, int rows, int inter, int64_t gu_stride,
                                                            int64_t out_stride, float limit, float alpha) {
     const int pieces = inter / 4;
@@ -78,7 +78,7 @@ __global__ __launch_bounds__(256) void clamped_glu_kernel(T* __restrict__ out, c
         const f32x4 g = act_ld4(gu + row * gu_stride + c), u = act_ld4(gu + row * gu_stride + inter + c);
         f32x4 r;
 #pragma unroll
-        for (int k = 0; k < 4; ++k) r[k] = clamped_glu(g[k], u[k], limit, alpha);
+        for (int k = 0; k < 4; ++k) r[k] = GELU ? gelu_tanh_f(g[k]) * u[k] : clamped_glu(g[k], u[k], limit, alpha);
         act_st4(out + row * out_stride + c, r);
     }
 }
@@ -253,13 +253,23 @@ int launch_norm_residual(const NormResidualArgs& a, int f32, hipStream_t stream)
     return check_launch("norm_residual");
 }
 
-int launch_clamped_glu(void* out, const void* gate_up, int rows, int inter, int64_t gu_stride, int64_t out_stride, float limit, float alpha, int f32,
-                       hipStream_t stream) {
+template <bool GELU>
+static void glu_go(void* out, const void* gate_up, int rows, int inter, int64_t gu_stride, int64_t out_stride, float limit, float alpha, int f32, hipStream_t stream) {
     const int64_t work = ((int64_t)rows * (inter / 4) + 255) / 256;
     const int grid = (int)(work < 8192 ? (work < 1 ? 1 : work) : 8192);
-    if (f32) clamped_glu_kernel<float><<<grid, 256, 0, stream>>>((float*)out, (const float*)gate_up, rows, inter, gu_stride, out_stride, limit, alpha);
-    else clamped_glu_kernel<uint16_t><<<grid, 256, 0, stream>>>((uint16_t*)out, (const uint16_t*)gate_up, rows, inter, gu_stride, out_stride, limit, alpha);
+    if (f32) clamped_glu_kernel<float, GELU><<<grid, 256, 0, stream>>>((float*)out, (const float*)gate_up, rows, inter, gu_stride, out_stride, limit, alpha);
+    else clamped_glu_kernel<uint16_t, GELU><<<grid, 256, 0, stream>>>((uint16_t*)out, (const uint16_t*)gate_up, rows, inter, gu_stride, out_stride, limit, alpha);
+}
+
+int launch_clamped_glu(void* out, const void* gate_up, int rows, int inter, int64_t gu_stride, int64_t out_stride, float limit, float alpha, int f32,
+                       hipStream_t stream) {
+    glu_go<false>(out, gate_up, rows, inter, gu_stride, out_stride, limit, alpha, f32, stream);
     return check_launch("clamped_glu");
+}
+
+int launch_gelu_glu(void* out, const void* gate_up, int rows, int inter, int64_t gu_stride, int64_t out_stride, int f32, hipStream_t stream) {
+    glu_go<true>(out, gate_up, rows, inter, gu_stride, out_stride, 0.f, 0.f, f32, stream);
+    return check_launch("gelu_glu");
 }
 
 template <typename T>

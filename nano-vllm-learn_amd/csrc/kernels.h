@@ -101,6 +101,8 @@ struct LinearArgs {
     int norm_mode;               // 0 none; 1 exact RMSNorm prologue; 2 folded RMSNorm (w already multiplied by the norm weight)
     int epi;
     float glu_limit, glu_alpha;  // SILU epilogue with glu_alpha != 0: the clamped gated unit of common.h instead of SiLU(g) * u
+    int glu_gelu;                // SILU epilogue: gelu_tanh(g) * u
+    int x_groups;                // NONE, x_packed: > 1: `inter` weight rows read the activations at x, the next ones those at x + hd, ...
     const int64_t* positions;    // ROPE: [M]
     const float* cos_sin;        // ROPE: [max_position, D]
     uint16_t* k_cache;           // ROPE: paged caches and slots of this step's rows

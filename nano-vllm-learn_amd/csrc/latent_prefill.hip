@@ -93,7 +93,7 @@ __global__ __launch_bounds__(256, DK + DV <= 320 ? 2 : 1) void latent_prefill_ke
         lds, n_tiles, a.scale_log2, -INFINITY, lane, stage, query, [&](int it) { return it * BN; }, [&](int kv0) { return kv0 <= wave_last_key; },
         [&](int kv0) { return kv0 + BN - 1 > wave_first_key || kv0 + BN > sk; },
         [&](int kv0, int qs, int off) { return off <= (my_q[qs] + shift < sk - 1 ? my_q[qs] + shift : sk - 1) - kv0 - 4 * lg; },
-        [&](int qs) { return q_ok[qs] ? a.out + (int64_t)(q_beg + my_q[qs]) * a.out_stride + head * DV : nullptr; });
+        [&](int qs) { return q_ok[qs] ? a.out + (int64_t)(q_beg + my_q[qs]) * a.out_stride + head * DV : nullptr; }, [](int, int, f32x4 v) { return v; });
 }
 
 template <int DK, int DV, int QT>

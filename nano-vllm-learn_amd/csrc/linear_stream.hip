@@ -311,6 +311,11 @@ __global__ __launch_bounds__(NWV * 64) void linear_stream_kernel(
         }
     }
 
+    // grouped activations (p_inter weight rows per group, p_hd elements between the groups' activations: LS_FLAT)
+    const uint16_t* x_base = p_x;
+    if constexpr (EPI == EPI_NONE && XPACK && !MULTI) {
+        if (p_inter > 0) x_base += (int64_t)min(tile_first * 16 / p_inter, a.x_groups - 1) * p_hd;
+    }
     // ---- x fragments of this wave's K range, kept in registers for every tile of the workgroup
     u32x4 araw[2 * PMAX][MT];
 #pragma unroll
@@ -322,7 +327,7 @@ __global__ __launch_bounds__(NWV * 64) void linear_stream_kernel(
 #pragma unroll
                 for (int m = 0; m < MT; ++m) {
                     if constexpr (XPACK) {
-                        araw[2 * pi + j][m] = *reinterpret_cast<const u32x4*>(p_x + (((int64_t)m * KS + ks) * 64 + lane) * 8);
+                        araw[2 * pi + j][m] = *reinterpret_cast<const u32x4*>(x_base + (((int64_t)m * KS + ks) * 64 + lane) * 8);
                     } else {
                         const int r = 16 * m + lq;                   // rows past M repeat the last row; discarded
                         araw[2 * pi + j][m] = *reinterpret_cast<const u32x4*>(p_x + (int64_t)(r < a.M ? r : a.M - 1) * a.x_stride + ks * 32 + lg * 8);
@@ -547,13 +552,13 @@ __global__ __launch_bounds__(NWV * 64) void linear_stream_kernel(
                     const int col = 24 * tile + 16 * hb + c;
                     if ((hb == 1 && c >= 8) || col >= p_inter) continue;
                     const float g = (float)(__bf16)y[hb], u = (float)(__bf16)y[2 + hb];
-                    const __bf16 o = (__bf16)gated_unit(g, u, a.glu_limit, a.glu_alpha);
+                    const __bf16 o = (__bf16)gated_unit(g, u, a.glu_limit, a.glu_alpha, a.glu_gelu);
                     if (out) out[(int64_t)row * e_out_stride + col] = o;
                     if (e_out_packed) e_out_packed[pack_index(row, col, p_inter)] = __builtin_bit_cast(uint16_t, o);
                 }
             } else if constexpr (EPI == EPI_SILU) {
                 const float g = (float)(__bf16)y[0], u = (float)(__bf16)y[1];          // the projection output is bf16 in the reference
-                const __bf16 o = (__bf16)gated_unit(g, u, a.glu_limit, a.glu_alpha);
+                const __bf16 o = (__bf16)gated_unit(g, u, a.glu_limit, a.glu_alpha, a.glu_gelu);
                 if (out) out[(int64_t)row * e_out_stride + n0 + c] = o;
                 if (e_out_packed) e_out_packed[pack_index(row, n0 + c, p_inter)] = __builtin_bit_cast(uint16_t, o);
             } else if constexpr (EPI == EPI_RESADD) {
@@ -647,7 +652,7 @@ static dim3 grid_of(const LinearArgs& a) {
 template <int MT, int EPI, int NORM, bool XPACK>
 int launch_x(const LinearArgs& a_in, hipStream_t stream) {
     LinearArgs a = a_in;
-    const bool multi = EPI == EPI_NONE && a.ksplit == 1 && a.tiles > 1024;
+    const bool multi = EPI == EPI_NONE && a.ksplit == 1 && a.tiles > 1024 && a.x_groups <= 1;
     if (multi) {
         if constexpr (EPI == EPI_NONE) {
             // (eight waves per workgroup measured slower here: 72 vs 49 us for the LM head)

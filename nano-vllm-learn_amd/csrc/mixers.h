@@ -113,14 +113,36 @@ struct VisibleTiles {
     int kept, first, count;                          // tiles [0, kept), then [first, first + count - kept)
     __device__ __forceinline__ int tile(int i) const { return i < kept ? i : first + i - kept; }
 };
-// first_pos .. last_pos: positions of the queries that walk together
-__device__ __forceinline__ VisibleTiles visible_tiles(int first_pos, int last_pos, int window, int keep_first) {
+// the first key, kept ones aside, that a query at `pos` sees through a window (the last `window` tokens; 0: all) or in its chunk (chunk > 0)
+__device__ __forceinline__ int first_seen(int pos, int window, int chunk) {
+    if (chunk > 0) return pos - pos % chunk;
+    return window > 0 && pos >= window ? pos - window + 1 : 0;
+}
+// lo: first_seen of the first query that walks along, last_pos: position of the last one
+__device__ __forceinline__ VisibleTiles visible_from(int lo, int last_pos, int keep_first) {
     VisibleTiles v;
-    const int lo = window > 0 && first_pos >= window ? first_pos - window + 1 : 0;
     v.first = lo >> 6;
     const int k = (keep_first + 63) >> 6;
     v.kept = k < v.first ? k : v.first;
     v.count = v.kept + ((last_pos + 64) >> 6) - v.first;
+    return v;
+}
+// first_pos .. last_pos: positions of the queries that walk together
+__device__ __forceinline__ VisibleTiles visible_tiles(int first_pos, int last_pos, int window, int keep_first) {
+    return visible_from(first_seen(first_pos, window, 0), last_pos, keep_first);
+}
+
+// 4 columns of a head's output at `pos`, from dimension d on (a multiple of 4), turned back: interleaved pairs of the first `rot` dimensions, table rows cos | sin
+__device__ __forceinline__ f32x4 turn_back(f32x4 v, const float* table, int64_t pos, int max_position, int rot, int d) {
+    if (d >= rot) return v;
+    const float* cs = table + (pos < max_position ? pos : max_position - 1) * rot;
+#pragma unroll
+    for (int p = 0; p < 2; ++p) {
+        if (d + 2 * p >= rot) continue;
+        const float c = cs[d / 2 + p], s = cs[rot / 2 + d / 2 + p], x = v[2 * p], y = v[2 * p + 1];
+        v[2 * p] = x * c + y * s;
+        v[2 * p + 1] = y * c - x * s;
+    }
     return v;
 }
 

@@ -23,9 +23,10 @@ __global__ __launch_bounds__(256, DK + DV <= 320 ? 2 : 1) void paged_prompt_kern
     const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lq = lane & 15, lg = lane >> 4;
     const int g = head / (a.heads / a.kv_heads);
     const int rows = sq - q0 < BM ? sq - q0 : BM;
-    const VisibleTiles vis = visible_tiles(q0 + shift, q0 + rows - 1 + shift, a.window, a.keep_first);
-    const int n_tiles = vis.count, window = a.window > 0 ? a.window : 0x40000000;
+    const VisibleTiles vis = visible_from(first_seen(q0 + shift, a.window, a.chunk), q0 + rows - 1 + shift, a.keep_first);
+    const int n_tiles = vis.count;
     const int wave_first = q0 + wave * WR + shift, wave_last = wave_first + WR - 1;       // positions of this wave's rows
+    const int lo_first = first_seen(wave_first, a.window, a.chunk), lo_last = first_seen(wave_last, a.window, a.chunk);
 
     // ---- staging: this lane's piece of each DMA instruction: row of the tile and offset inside it
     const uint16_t* cache = reinterpret_cast<const uint16_t*>(a.cache) + (int64_t)g * a.block_size * (DK + DV);
@@ -58,25 +59,27 @@ __global__ __launch_bounds__(256, DK + DV <= 320 ? 2 : 1) void paged_prompt_kern
         for (int j = 0; j < NV; ++j) dma16(vb + (vr[j] < live ? vr[j] : live - 1) * DV + vc[j], vimg + (wave * NV + j) * 1024);
         page = page_of(it + 1);
     };
-    int my_q[QT];
+    int my_q[QT], lo[QT];
     bool q_ok[QT];
     const uint16_t* qp[QT];
 #pragma unroll
     for (int qs = 0; qs < QT; ++qs) {
         my_q[qs] = q0 + wave * WR + 16 * qs + lq;
         q_ok[qs] = my_q[qs] < sq;
+        lo[qs] = first_seen(my_q[qs] + shift, a.window, a.chunk);
         qp[qs] = reinterpret_cast<const uint16_t*>(a.q) + (int64_t)(q_beg + (q_ok[qs] ? my_q[qs] : sq - 1)) * a.q_stride + (int64_t)head * DK + lg * 8;
     }
     attend_walk<DK, DV, QT>(
         lds, n_tiles, a.scale * kLog2e, a.sink ? a.sink[head] * kLog2e : -INFINITY, lane, stage,
         [&](int qs, int st) { return *reinterpret_cast<const bf16x8*>(qp[qs] + st * 32); }, [&](int it) { return vis.tile(it) * BN; },
-        [&](int kv0) { return kv0 <= wave_last && (kv0 + BN - 1 > wave_first - window || kv0 < a.keep_first); },
-        [&](int kv0) { return kv0 + BN - 1 > wave_first || kv0 + BN > sk || (kv0 <= wave_last - window && kv0 + BN > a.keep_first); },
+        [&](int kv0) { return kv0 <= wave_last && (kv0 + BN > lo_first || kv0 < a.keep_first); },
+        [&](int kv0) { return kv0 + BN - 1 > wave_first || kv0 + BN > sk || (kv0 < lo_last && kv0 + BN > a.keep_first); },
         [&](int kv0, int qs, int off) {
             const int pos = my_q[qs] + shift, at = kv0 + 4 * lg + off;
-            return at <= (pos < sk - 1 ? pos : sk - 1) && (at > pos - window || at < a.keep_first);
+            return at <= (pos < sk - 1 ? pos : sk - 1) && (at >= lo[qs] || at < a.keep_first);
         },
-        [&](int qs) { return q_ok[qs] ? reinterpret_cast<uint16_t*>(a.out) + (int64_t)(q_beg + my_q[qs]) * a.out_stride + head * DV : nullptr; });
+        [&](int qs) { return q_ok[qs] ? reinterpret_cast<uint16_t*>(a.out) + (int64_t)(q_beg + my_q[qs]) * a.out_stride + head * DV : nullptr; },
+        [&](int qs, int d, f32x4 v) { return a.o_cos_sin ? turn_back(v, a.o_cos_sin, my_q[qs] + shift, a.max_position, a.o_rot, d) : v; });
 }
 
 template <int DK, int DV, int QT>

@@ -42,10 +42,11 @@ __global__ __launch_bounds__(256) void paged_rows_generic_kernel(const PagedAtte
         const int64_t page = a.block_tables[seq * a.bt_stride + key / a.block_size];
         return reinterpret_cast<const T*>(a.cache) + (page * a.kv_heads + g) * head_elems;
     };
-    const VisibleTiles vis = visible_tiles(pos, pos, a.window, a.keep_first);
+    const int lo = first_seen(pos, a.window, a.chunk);
+    const VisibleTiles vis = visible_from(lo, pos, a.keep_first);
     for (int it = 0; it < vis.count; ++it) {
         const int t0 = vis.tile(it) * 64, key = t0 + (tid >> 2);
-        const bool sees = key <= pos && (a.window <= 0 || pos - key < a.window || key < a.keep_first);
+        const bool sees = key <= pos && (key >= lo || key < a.keep_first);
         float s = 0.f;
         if (TALK && sees && it * 64 < a.span) {
             const int cols = score_cols(a.heads);
@@ -89,6 +90,15 @@ __global__ __launch_bounds__(256) void paged_rows_generic_kernel(const PagedAtte
 #pragma unroll
     for (int j = 0; j < OC; ++j) {
         const int c = tid + 256 * j;
+        if (256 * j >= a.dv) continue;
+        if (a.o_cos_sin) {                           // (pairs of columns lie in neighbouring lanes)
+            const float other = __shfl_xor(o[j], 1);
+            if (c < a.o_rot) {
+                const float* cs = a.o_cos_sin + (int64_t)(pos < a.max_position ? pos : a.max_position - 1) * a.o_rot;
+                const float co = cs[c / 2], si = cs[a.o_rot / 2 + c / 2];
+                o[j] = c & 1 ? o[j] * co - other * si : o[j] * co + other * si;
+            }
+        }
         if (c >= a.dv) continue;
         if (a.out) act_st(reinterpret_cast<T*>(a.out) + (int64_t)row * a.out_stride + head * a.dv + c, o[j] * inv);
         if (a.out_packed) act_st(reinterpret_cast<uint16_t*>(a.out_packed) + pack_index(row, head * a.dv + c, a.heads * a.dv), o[j] * inv);
@@ -158,7 +168,8 @@ __global__ __launch_bounds__(256) void paged_rows_kernel(const PagedAttendArgs a
     const int g = blockIdx.y / passes, h0 = g * ratio + (blockIdx.y - g * passes) * kRowsHeads;
     const int nh = (g + 1) * ratio - h0 < R ? (g + 1) * ratio - h0 : R;
     const int pos = (int)a.positions[row];
-    const VisibleTiles vis = visible_tiles(pos, pos, a.window, a.keep_first);
+    const int lo = first_seen(pos, a.window, a.chunk);
+    const VisibleTiles vis = visible_from(lo, pos, a.keep_first);
     const int per = (vis.count + a.splits - 1) / a.splits, t_beg = split * per, t_end = t_beg + per < vis.count ? t_beg + per : vis.count;
     const int units = t_end > t_beg ? (t_end - t_beg) * (64 / UK) : 0;
 
@@ -202,7 +213,7 @@ __global__ __launch_bounds__(256) void paged_rows_kernel(const PagedAttendArgs a
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
                 const int key = k0 + 16 * t + 4 * lg + r;
-                const float unseen = key <= pos && (a.window <= 0 || pos - key < a.window || key < a.keep_first) ? 0.f : -INFINITY;
+                const float unseen = key <= pos && (key >= lo || key < a.keep_first) ? 0.f : -INFINITY;
                 s[t][r] = s[t][r] * sc + unseen;
                 mx = fmaxf(mx, s[t][r]);
             }
@@ -290,6 +301,7 @@ __global__ __launch_bounds__(256) void paged_rows_kernel(const PagedAttendArgs a
     __syncthreads();
     constexpr int PIECES = DV / 4, RECB = (DV + 4) * 4;                        // 4-column pieces of a head; bytes of a split record
     auto finish = [&](int r, int c, f32x4 v) {       // 4 normalised columns of head h0 + r
+        if (a.o_cos_sin) v = turn_back(v, a.o_cos_sin, pos, a.max_position, a.o_rot, c);
         const int col = (h0 + r) * DV + c;
         if (a.out) act_st4(reinterpret_cast<uint16_t*>(a.out) + (int64_t)row * a.out_stride + col, v);
         if (a.out_packed) act_st4(reinterpret_cast<uint16_t*>(a.out_packed) + pack_index(row, col, a.heads * DV), v);

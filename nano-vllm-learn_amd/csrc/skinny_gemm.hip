@@ -257,7 +257,7 @@ __global__ __launch_bounds__(WAVES * 64) void linear_small_m_kernel(const Linear
         __bf16* const out = reinterpret_cast<__bf16*>(a.out);
         if constexpr (EPI == EPI_SILU) {
             const float g = (float)(__bf16)s[0], u = (float)(__bf16)s[1];          // the projection output is bf16 in the reference
-            out[(int64_t)row * a.out_stride + n0 + c] = (__bf16)gated_unit(g, u, a.glu_limit, a.glu_alpha);
+            out[(int64_t)row * a.out_stride + n0 + c] = (__bf16)gated_unit(g, u, a.glu_limit, a.glu_alpha, a.glu_gelu);
         } else if constexpr (EPI == EPI_RESADD) {
             __bf16* p = out + (int64_t)row * a.out_stride + n0 + c;
             *p = (__bf16)(s[0] + (float)*p);

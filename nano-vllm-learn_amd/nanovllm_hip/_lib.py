@@ -29,7 +29,8 @@ class LinearDesc(ctypes.Structure):
                 ("workspace", ctypes.c_void_p), ("workspace_bytes", ctypes.c_size_t),
                 ("candidate_val", ctypes.c_void_p), ("candidate_idx", ctypes.c_void_p), ("candidate_stride", ctypes.c_int64),
                 ("prefetch", ctypes.c_void_p), ("prefetch_bytes", ctypes.c_size_t),
-                ("glu_limit", ctypes.c_float), ("glu_alpha", ctypes.c_float)]
+                ("glu_limit", ctypes.c_float), ("glu_alpha", ctypes.c_float), ("glu_gelu", ctypes.c_int32),
+                ("x_groups", ctypes.c_int32), ("x_group_rows", ctypes.c_int32), ("x_group_stride", ctypes.c_int32)]
 
 
 class NormResidualDesc(ctypes.Structure):
@@ -86,7 +87,8 @@ class AttnPrepDesc(ctypes.Structure):
                 ("kv_heads", ctypes.c_int32), ("dk", ctypes.c_int32), ("dv", ctypes.c_int32), ("q_w", ctypes.c_void_p),
                 ("k_w", ctypes.c_void_p), ("q_n", ctypes.c_int32), ("k_n", ctypes.c_int32), ("eps", ctypes.c_float),
                 ("positions", ctypes.c_void_p), ("cos_sin", ctypes.c_void_p), ("max_position", ctypes.c_int32), ("rot", ctypes.c_int32),
-                ("cache", ctypes.c_void_p), ("slots", ctypes.c_void_p), ("block_size", ctypes.c_int32), ("head_norm", ctypes.c_int32)]
+                ("cache", ctypes.c_void_p), ("slots", ctypes.c_void_p), ("block_size", ctypes.c_int32), ("head_norm", ctypes.c_int32),
+                ("v_cos_sin", ctypes.c_void_p), ("v_rot", ctypes.c_int32)]
 
 
 class PagedAttendDesc(ctypes.Structure):
@@ -99,7 +101,7 @@ class PagedAttendDesc(ctypes.Structure):
                 ("keep_first", ctypes.c_int32), ("sink", ctypes.c_void_p), ("splits", ctypes.c_int32), ("part", ctypes.c_void_p),
                 ("tickets", ctypes.c_void_p), ("out", ctypes.c_void_p), ("out_stride", ctypes.c_int64),
                 ("out_packed", ctypes.c_void_p), ("talk", ctypes.c_void_p), ("softcap", ctypes.c_float), ("scores", ctypes.c_void_p),
-                ("span", ctypes.c_int32)]
+                ("span", ctypes.c_int32), ("chunk", ctypes.c_int32), ("o_cos_sin", ctypes.c_void_p), ("max_position", ctypes.c_int32), ("o_rot", ctypes.c_int32)]
 
 
 class LightningDesc(ctypes.Structure):
@@ -134,6 +136,63 @@ class ResidualNormDesc(ctypes.Structure):
                 ("rows", ctypes.c_int32), ("cols", ctypes.c_int32), ("n", ctypes.c_int32), ("xb", ctypes.c_void_p),
                 ("packed", ctypes.c_void_p), ("post_w", ctypes.c_void_p), ("post_b", ctypes.c_void_p), ("mult", ctypes.c_float),
                 ("base", ctypes.c_void_p), ("shift", ctypes.c_void_p)]
+
+
+class BigramEmbedDesc(ctypes.Structure):
+    """nvh_bigram_embed_desc (include/nvh_attn.h)."""
+    _fields_ = [("x", ctypes.c_void_p), ("tokens", ctypes.c_void_p), ("positions", ctypes.c_void_p), ("row_seq", ctypes.c_void_p),
+                ("cu_rows", ctypes.c_void_p), ("state_slots", ctypes.c_void_p), ("last_token", ctypes.c_void_p),
+                ("embed", ctypes.c_void_p), ("bigram", ctypes.c_void_p), ("buckets", ctypes.c_int64), ("mul_prev", ctypes.c_int64),
+                ("mul_cur", ctypes.c_int64), ("rows", ctypes.c_int32), ("cols", ctypes.c_int32), ("vocab", ctypes.c_int32)]
+
+
+class StreamMixDesc(ctypes.Structure):
+    """nvh_stream_mix_desc (include/nvh_attn.h)."""
+    _fields_ = [("xin", ctypes.c_void_p), ("xin_row", ctypes.c_int64), ("xin_stream", ctypes.c_int64), ("xout", ctypes.c_void_p),
+                ("rows", ctypes.c_int32), ("cols", ctypes.c_int32), ("n", ctypes.c_int32), ("streams", ctypes.c_int32),
+                ("y", ctypes.c_void_p), ("y_stride", ctypes.c_int64), ("y2", ctypes.c_void_p), ("y2_stride", ctypes.c_int64),
+                ("y_w", ctypes.c_void_p), ("y2_w", ctypes.c_void_p), ("y_scale", ctypes.c_float), ("mix", ctypes.c_void_p),
+                ("out", ctypes.c_void_p), ("in", ctypes.c_void_p), ("sum", ctypes.c_void_p), ("w", ctypes.c_void_p),
+                ("groups", ctypes.c_int32), ("eps", ctypes.c_float), ("h", ctypes.c_void_p), ("packed", ctypes.c_void_p)]
+
+
+class TokenShiftDesc(ctypes.Structure):
+    """nvh_token_shift_desc (include/nvh_attn.h)."""
+    _fields_ = [("h", ctypes.c_void_p), ("h_stride", ctypes.c_int64), ("rows", ctypes.c_int32), ("cols", ctypes.c_int32),
+                ("shift", ctypes.c_void_p), ("mu", ctypes.c_void_p), ("mixes", ctypes.c_int32), ("out", ctypes.c_void_p),
+                ("out_mix", ctypes.c_int64), ("packed", ctypes.c_int32), ("ring", ctypes.c_void_p), ("depth", ctypes.c_int32),
+                ("positions", ctypes.c_void_p), ("row_seq", ctypes.c_void_p), ("cu_rows", ctypes.c_void_p),
+                ("state_slots", ctypes.c_void_p), ("sequences", ctypes.c_int32)]
+
+
+class CausalConvDesc(ctypes.Structure):
+    """nvh_causal_conv_desc (include/nvh_attn.h)."""
+    _fields_ = [("x", ctypes.c_void_p), ("x_stride", ctypes.c_int64), ("rows", ctypes.c_int32), ("cols", ctypes.c_int32),
+                ("taps", ctypes.c_int32), ("w", ctypes.c_void_p), ("b", ctypes.c_void_p), ("out", ctypes.c_void_p),
+                ("packed", ctypes.c_void_p), ("ring", ctypes.c_void_p), ("positions", ctypes.c_void_p), ("row_seq", ctypes.c_void_p),
+                ("cu_rows", ctypes.c_void_p), ("state_slots", ctypes.c_void_p), ("sequences", ctypes.c_int32)]
+
+
+class ScanDesc(ctypes.Structure):
+    """nvh_scan_desc (include/nvh_attn.h)."""
+    _fields_ = [("x", ctypes.c_void_p), ("x_stride", ctypes.c_int64), ("dt", ctypes.c_void_p), ("dt_stride", ctypes.c_int64),
+                ("dt_bias", ctypes.c_void_p), ("bc", ctypes.c_void_p), ("bc_stride", ctypes.c_int64), ("z", ctypes.c_void_p),
+                ("z_stride", ctypes.c_int64), ("a_log2", ctypes.c_void_p), ("d", ctypes.c_void_p), ("rows", ctypes.c_int32),
+                ("inner", ctypes.c_int32), ("n", ctypes.c_int32), ("positions", ctypes.c_void_p), ("state_slots", ctypes.c_void_p),
+                ("state", ctypes.c_void_p), ("chunks", ctypes.c_void_p), ("n_chunks", ctypes.c_int32), ("summaries", ctypes.c_int32),
+                ("seg_state", ctypes.c_void_p), ("seg_dt", ctypes.c_void_p), ("w_dt", ctypes.c_void_p), ("rank", ctypes.c_int32),
+                ("out", ctypes.c_void_p), ("out_stride", ctypes.c_int64), ("out_packed", ctypes.c_void_p)]
+
+
+class WkvDesc(ctypes.Structure):
+    """nvh_wkv_desc (include/nvh_attn.h)."""
+    _fields_ = [("r", ctypes.c_void_p), ("k", ctypes.c_void_p), ("v", ctypes.c_void_p), ("g", ctypes.c_void_p), ("stride", ctypes.c_int64),
+                ("z", ctypes.c_void_p), ("z_stride", ctypes.c_int64), ("w0", ctypes.c_void_p), ("u", ctypes.c_void_p),
+                ("norm", ctypes.c_void_p), ("eps", ctypes.c_float), ("n", ctypes.c_int32), ("rows", ctypes.c_int32),
+                ("heads", ctypes.c_int32), ("dim", ctypes.c_int32), ("w2", ctypes.c_void_p), ("rank", ctypes.c_int32),
+                ("positions", ctypes.c_void_p), ("state_slots", ctypes.c_void_p), ("state", ctypes.c_void_p), ("chunks", ctypes.c_void_p),
+                ("n_chunks", ctypes.c_int32), ("summaries", ctypes.c_int32), ("seg_state", ctypes.c_void_p),
+                ("seg_decay", ctypes.c_void_p), ("out", ctypes.c_void_p), ("out_stride", ctypes.c_int64), ("out_packed", ctypes.c_void_p)]
 
 
 EPI_NONE, EPI_SILU_MUL, EPI_RESIDUAL_ADD, EPI_ROPE_STORE = 0, 1, 2, 3
@@ -209,6 +268,7 @@ _SIGS = {
     "nvh_embed_rows": (ctypes.c_int, [ctypes.c_void_p] * 5 + [ctypes.c_float] + [ctypes.c_int] * 3 + [ctypes.c_void_p] * 3 + [ctypes.c_int] * 2 + [ctypes.c_void_p]),
     "nvh_norm_residual": (ctypes.c_int, [ctypes.POINTER(NormResidualDesc), ctypes.c_int, ctypes.c_void_p]),
     "nvh_clamped_glu": (ctypes.c_int, [ctypes.c_void_p] * 2 + [ctypes.c_int] * 2 + [ctypes.c_int64] * 2 + [ctypes.c_float] * 2 + [ctypes.c_int, ctypes.c_void_p]),
+    "nvh_gelu_glu": (ctypes.c_int, [ctypes.c_void_p] * 2 + [ctypes.c_int] * 2 + [ctypes.c_int64] * 2 + [ctypes.c_int, ctypes.c_void_p]),
     "nvh_rglru_chunk_tokens": (ctypes.c_int, []),
     "nvh_rglru_step_supported": (ctypes.c_int, [ctypes.c_int]),
     "nvh_rglru_chunks": (ctypes.c_int, [ctypes.POINTER(RglruDesc), ctypes.c_int, ctypes.c_int, ctypes.c_void_p]),
@@ -242,6 +302,16 @@ _SIGS = {
     "nvh_residual_norm": (ctypes.c_int, [ctypes.POINTER(ResidualNormDesc), ctypes.c_int, ctypes.c_void_p]),
     "nvh_poly_norm": (ctypes.c_int, [ctypes.c_void_p] * 4 + [ctypes.c_float] + [ctypes.c_int] * 3 + [ctypes.c_int64] * 2 + [ctypes.c_int, ctypes.c_void_p]),
     "nvh_softcap": (ctypes.c_int, [ctypes.c_void_p, ctypes.c_float, ctypes.c_int, ctypes.c_int, ctypes.c_int64, ctypes.c_int, ctypes.c_void_p]),
+    "nvh_bigram_embed": (ctypes.c_int, [ctypes.POINTER(BigramEmbedDesc), ctypes.c_int, ctypes.c_void_p]),
+    "nvh_stream_mix": (ctypes.c_int, [ctypes.POINTER(StreamMixDesc), ctypes.c_int, ctypes.c_void_p]),
+    "nvh_token_shift": (ctypes.c_int, [ctypes.POINTER(TokenShiftDesc), ctypes.c_int, ctypes.c_void_p]),
+    "nvh_causal_conv": (ctypes.c_int, [ctypes.POINTER(CausalConvDesc), ctypes.c_int, ctypes.c_void_p]),
+    "nvh_scan_states": (ctypes.c_int, [ctypes.c_int]),
+    "nvh_scan_chunks": (ctypes.c_int, [ctypes.POINTER(ScanDesc), ctypes.c_int, ctypes.c_void_p]),
+    "nvh_scan_step": (ctypes.c_int, [ctypes.POINTER(ScanDesc), ctypes.c_int, ctypes.c_void_p]),
+    "nvh_wkv_supported": (ctypes.c_int, [ctypes.c_int]),
+    "nvh_wkv_chunks": (ctypes.c_int, [ctypes.POINTER(WkvDesc), ctypes.c_int, ctypes.c_int, ctypes.c_void_p]),
+    "nvh_wkv_step": (ctypes.c_int, [ctypes.POINTER(WkvDesc), ctypes.c_int, ctypes.c_void_p]),
 }
 EXPORTS = tuple(_SIGS)
 

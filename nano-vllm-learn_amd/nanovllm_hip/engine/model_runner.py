@@ -98,7 +98,7 @@ def build_step_meta(portions, block_size, segment=64):
     _check_block_size([s for s, _ in portions], block_size)
     order = sorted(range(len(portions)), key=lambda i: portions[i][1] > 1)
     input_ids, positions, slots, row_seq, chunks = [], [], [], [], []
-    cu_q, cu_k, max_q, num_decode = [0], [0], 0, 0
+    cu_rows, cu_q, cu_k, max_q, num_decode = [0], [0], [0], 0, 0
     for j, i in enumerate(order):
         seq, n = portions[i]
         lo, hi = seq.num_cached_tokens, seq.num_cached_tokens + n
@@ -108,6 +108,7 @@ def build_step_meta(portions, block_size, segment=64):
         positions += range(lo, hi)
         slots += [seq.block_table[p // block_size] * block_size + p % block_size for p in range(lo, hi)]
         row_seq += [j] * n
+        cu_rows.append(len(input_ids))
         if n == 1:
             num_decode += 1
         else:
@@ -121,7 +122,7 @@ def build_step_meta(portions, block_size, segment=64):
     return dict(order=order, input_ids=torch.tensor(input_ids, dtype=torch.int64), positions=torch.tensor(positions, dtype=torch.int64), num_decode=num_decode,
                 slot_mapping=i32(slots), block_tables=build_block_tables(seqs, pad=0), state_slots=i32([s.state_slot for s in seqs]), chunks=i32(chunks), segment=segment,
                 summaries=any(k for *_, k in chunks),
-                row_seq=i32(row_seq), cu_q=i32(cu_q), cu_k=i32(cu_k), max_q=max_q, total_k=cu_k[-1], max_context=max(positions) + 1)
+                row_seq=i32(row_seq), cu_rows=i32(cu_rows), cu_q=i32(cu_q), cu_k=i32(cu_k), max_q=max_q, total_k=cu_k[-1], max_context=max(positions) + 1)
 
 
 # ----------------------------------------------------------------------------- runner
@@ -207,7 +208,7 @@ class ModelRunner:
         assert all(0 <= p < portions[i][1] for i, places in enumerate(want) for p in places), "a wanted place is outside its portion"
         decode_only = m["num_decode"] == row
         step = StepMeta(m["num_decode"], self._dev(m["slot_mapping"]), self._dev(m["block_tables"]), self._dev(m["state_slots"]), self._dev(m["chunks"]),
-                        m["segment"], m["summaries"], m["max_context"], *([] if decode_only else [self._dev(m["row_seq"]), self._dev(m["cu_q"]), self._dev(m["cu_k"]), m["max_q"], m["total_k"]]))
+                        m["segment"], m["summaries"], m["max_context"], *([] if decode_only else [self._dev(m["row_seq"]), self._dev(m["cu_rows"]), self._dev(m["cu_q"]), self._dev(m["cu_k"]), m["max_q"], m["total_k"]]))
         hidden = self.model(self._dev(m["input_ids"]), self._dev(m["positions"]), step)
         for seq, n in portions:
             seq.num_cached_tokens += n

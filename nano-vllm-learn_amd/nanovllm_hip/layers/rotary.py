@@ -26,3 +26,9 @@ def rotation_table(dims, base, max_position, device, scaling=None):
         angle = torch.arange(max_position, dtype=torch.float64)[:, None] * frequencies(dims, base, scaling)[None, :]
         _TABLES[key] = torch.cat((angle.cos(), angle.sin()), dim=1).float().contiguous().to(device)
     return _TABLES[key]
+
+
+def halves_to_pairs(width, dims):
+    """Index that brings the pairs (i, i + dims / 2) of the first `dims` of `width` dimensions next to each other, as the kernels turn them."""
+    half = torch.arange(dims // 2)
+    return torch.cat((torch.stack((half, half + dims // 2), dim=1).reshape(-1), torch.arange(dims, width)))

@@ -19,12 +19,17 @@ def _kekapel():
     return KekapelConfig.from_json, KekapelForCausalLM
 
 
+def _zaposun():
+    from .zaposun import ZaposunConfig, ZaposunForCausalLM
+    return ZaposunConfig.from_json, ZaposunForCausalLM
+
+
 def _qwen():
     from .qwen import ModelConfig, QwenForCausalLM
     return ModelConfig.from_json, QwenForCausalLM
 
 
-REGISTRY = {"Zobasun": _zobasun, "Galirax": _galirax, "Kekapel": _kekapel, "Qwen2ForCausalLM": _qwen, "Qwen3ForCausalLM": _qwen}
+REGISTRY = {"Zobasun": _zobasun, "Galirax": _galirax, "Kekapel": _kekapel, "Zaposun": _zaposun, "Qwen2ForCausalLM": _qwen, "Qwen3ForCausalLM": _qwen}
 
 
 def architecture(config_json):
@@ -44,9 +49,10 @@ def model_class(cfg):
     from .galirax import GaliraxConfig, GaliraxForCausalLM
     from .kekapel import KekapelConfig, KekapelForCausalLM
     from .qwen import ModelConfig, QwenForCausalLM
+    from .zaposun import ZaposunConfig, ZaposunForCausalLM
     from .zobasun import ZobasunConfig, ZobasunForCausalLM
     return {ModelConfig: QwenForCausalLM, ZobasunConfig: ZobasunForCausalLM, GaliraxConfig: GaliraxForCausalLM,
-            KekapelConfig: KekapelForCausalLM}[type(cfg)]
+            KekapelConfig: KekapelForCausalLM, ZaposunConfig: ZaposunForCausalLM}[type(cfg)]
 
 
 def build_model(cfg, path=None, seed=0):

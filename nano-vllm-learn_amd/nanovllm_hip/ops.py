@@ -378,7 +378,7 @@ _EPI_CODES = {"none": _lib.EPI_NONE, "silu_mul": _lib.EPI_SILU_MUL, "residual_ad
 
 
 def fused_linear(x, weight, *, bias=None, norm_weight=None, norm_eps=1e-6, norm_folded=False, epilogue="none", out=None, rope=None,
-                 x_packed_rows=None, out_packed=None, workspace=None, want_out=True, candidates=None, prefetch=None, glu=None):
+                 x_packed_rows=None, out_packed=None, workspace=None, want_out=True, candidates=None, prefetch=None, glu=None, x_groups=None):
     """nvh_linear_small_m_ex: x [M<=64, K] . weight[N, K]^T with an optional RMSNorm prologue and one of the epilogues
     "none" (+bias) | "silu_mul" | "residual_add" (out = the residual stream, updated in place) | "rope_store"
     (rope = dict(positions, cos_sin, k_cache, v_cache, slot_mapping, num_heads, num_kv_heads, head_dim); returns q [M, H*D]).
@@ -390,12 +390,19 @@ def fused_linear(x, weight, *, bias=None, norm_weight=None, norm_eps=1e-6, norm_
     never written (LM head + greedy arg-max in one pass; finish with greedy_advance_candidates).
     prefetch = a contiguous CUDA tensor the NEXT launch will stream (the following projection's weights): the CUs this launch
     leaves idle read it into the caches first (a hint; results do not depend on it).
-    glu = (limit, alpha): "silu_mul" applies the clamped gated unit of clamped_glu() instead of SiLU(g) * u."""
+    glu = (limit, alpha): "silu_mul" applies the clamped gated unit of clamped_glu() instead of SiLU(g) * u; "gelu": gelu_tanh(g) * u.
+    x_groups = (count, weight rows): `x` holds `count` packed buffers of equal size, each group of weight rows is applied to its own ("none" only)."""
     d, out = _linear_desc(x, weight, bias=bias, norm_weight=norm_weight, norm_eps=norm_eps, norm_folded=norm_folded, epilogue=epilogue, out=out,
                           rope=rope, x_packed_rows=x_packed_rows, out_packed=out_packed, workspace=workspace, want_out=want_out,
                           candidates=candidates, prefetch=prefetch)
-    if glu is not None:
+    if glu == "gelu":
+        d.glu_gelu = 1
+    elif glu is not None:
         d.glu_limit, d.glu_alpha = float(glu[0]), float(glu[1])
+    if x_groups is not None:
+        d.x_groups, d.x_group_rows = int(x_groups[0]), int(x_groups[1])
+        d.x_group_stride = x.numel() // d.x_groups
+        assert x_packed_rows is not None and x.numel() % d.x_groups == 0
     rc = _lib.load().nvh_linear_small_m_ex(ctypes.byref(d), NVH_BF16, _stream())
     _lib.check(rc, "nvh_linear_small_m_ex")
     return out
@@ -656,6 +663,17 @@ def clamped_glu(gate_up, limit, alpha):
     return out
 
 
+def gelu_glu(gate_up):
+    """gelu(gate) * up with the tanh form of gelu; rows hold gate | up."""
+    code = _act_code(gate_up)
+    inter = gate_up.shape[1] // 2
+    assert gate_up.dim() == 2 and gate_up.stride(1) == 1
+    out = torch.empty((gate_up.shape[0], inter), dtype=gate_up.dtype, device=gate_up.device)
+    rc = _lib.load().nvh_gelu_glu(out.data_ptr(), gate_up.data_ptr(), gate_up.shape[0], inter, gate_up.stride(0), out.stride(0), code, _stream())
+    _lib.check(rc, "nvh_gelu_glu")
+    return out
+
+
 def rglru_chunk_tokens() -> int:
     return int(_lib.load().nvh_rglru_chunk_tokens())
 
@@ -859,10 +877,10 @@ def _packed_ok(packed, rows, cols):
     assert packed.is_contiguous() and packed.numel() >= ((rows + 15) // 16) * 16 * cols
 
 
-def attn_prep(qkv, heads, kv_heads, dk, dv, positions, cos_sin, cache, slots, q_weight=None, k_weight=None, q_n=0, k_n=0, eps=0.0, head_norm=False):
+def attn_prep(qkv, heads, kv_heads, dk, dv, positions, cos_sin, cache, slots, q_weight=None, k_weight=None, q_n=0, k_n=0, eps=0.0, head_norm=False, v_cos_sin=None):
     """Row ops behind a q | k | v projection: optional RMS norm over all query and all key columns (means over q_n / k_n of them; head_norm: over every head
-    by itself, weights [dk] shared by the heads), rotation of interleaved pairs of the first cos_sin.shape[1] dimensions of every head (None: no rotation), keys
-    and values into the cache [pages, block_size, kv_heads * (dk + dv)] (inside a page: [kv head][keys | values]).  The queries are rewritten in place."""
+    by itself, weights [dk] shared by the heads), rotation of interleaved pairs of the first cos_sin.shape[1] dimensions of every head (None: no rotation), of
+    values by v_cos_sin, keys and values into the cache [pages, block_size, kv_heads * (dk + dv)] (inside a page: [kv head][keys | values]).  The queries are rewritten in place."""
     code = _act_code(qkv, cache)
     rows = qkv.shape[0]
     _require_i32(slots=slots)
@@ -880,6 +898,10 @@ def attn_prep(qkv, heads, kv_heads, dk, dv, positions, cos_sin, cache, slots, q_
     if cos_sin is not None:
         _require_f32(cos_sin=cos_sin)
         d.cos_sin, d.max_position, d.rot = cos_sin.data_ptr(), cos_sin.shape[0], cos_sin.shape[1]
+    if v_cos_sin is not None:
+        _require_f32(v_cos_sin=v_cos_sin)
+        assert cos_sin is None or cos_sin.shape[0] == v_cos_sin.shape[0]
+        d.v_cos_sin, d.max_position, d.v_rot = v_cos_sin.data_ptr(), v_cos_sin.shape[0], v_cos_sin.shape[1]
     d.cache, d.slots, d.block_size = cache.data_ptr(), slots.data_ptr(), cache.shape[1]
     _lib.check(_lib.load().nvh_attn_prep(ctypes.byref(d), code, _stream()), "nvh_attn_prep")
 
@@ -888,8 +910,9 @@ def paged_attend_supported(dk, dv, block_size) -> bool:
     return bool(_lib.load().nvh_paged_attend_supported(int(dk), int(dv), int(block_size)))
 
 
-def paged_attend_splits(rows, kv_heads, heads, max_context, window=0, keep_first=0) -> int:
+def paged_attend_splits(rows, kv_heads, heads, max_context, window=0, keep_first=0, chunk=0) -> int:
     """Context splits of one launch over single rows: about two workgroups per CU, none with fewer than two 64-key tiles."""
+    window = window or chunk
     seen = min(max_context, window + keep_first + 126) if window else max_context
     tiles = (seen + 63) // 64
     groups = rows * kv_heads * ((heads // kv_heads + 7) // 8)
@@ -898,7 +921,7 @@ def paged_attend_splits(rows, kv_heads, heads, max_context, window=0, keep_first
     return -(-tiles // per)
 
 
-def _paged_desc(q, cache, block_tables, heads, kv_heads, dk, dv, scale, window, keep_first, sink, out):
+def _paged_desc(q, cache, block_tables, heads, kv_heads, dk, dv, scale, window, keep_first, sink, out, chunk=0, turn=None):
     code = _act_code(q, cache)
     rows = q.shape[0]
     _require_i32(block_tables=block_tables)
@@ -907,7 +930,10 @@ def _paged_desc(q, cache, block_tables, heads, kv_heads, dk, dv, scale, window, 
     d = _lib.PagedAttendDesc()
     d.q, d.q_stride, d.rows, d.heads, d.kv_heads, d.dk, d.dv = q.data_ptr(), q.stride(0), rows, heads, kv_heads, dk, dv
     d.cache, d.block_size, d.block_tables, d.bt_stride = cache.data_ptr(), cache.shape[1], block_tables.data_ptr(), block_tables.stride(0)
-    d.scale, d.window, d.keep_first, d.splits = float(scale), int(window), int(keep_first), 1
+    d.scale, d.window, d.keep_first, d.splits, d.chunk = float(scale), int(window), int(keep_first), 1, int(chunk)
+    if turn is not None:
+        _require_f32(turn=turn)
+        d.o_cos_sin, d.max_position, d.o_rot = turn.data_ptr(), turn.shape[0], turn.shape[1]
     if sink is not None:
         _require_f32(sink=sink)
         assert sink.numel() == heads
@@ -996,14 +1022,15 @@ def talk_prompt(q, cache, block_tables, cu_q, cu_k, max_q, heads, kv_heads, dk, 
 
 
 def paged_attend_rows(q, cache, block_tables, positions, heads, kv_heads, dk, dv, scale, max_context, window=0, keep_first=0, sink=None, row_seq=None, out=None,
-                      out_packed=None, want_out=True, splits=None, generic=False):
+                      out_packed=None, want_out=True, splits=None, generic=False, chunk=0, turn=None):
     """Attention of single query rows over the pages (row i: sequence row_seq[i], or i; sees its own position and before, with window > 0 only what is
-    nearer than `window` or among the first keep_first tokens; sink [heads] joins the softmax).  Returns [rows, heads * dv].
+    nearer than `window` or among the first keep_first tokens, with chunk > 0 only what lies in its own chunk of that many positions, or among those; sink
+    [heads] joins the softmax; turn [positions, dims]: the output is turned back by the angles of its position).  Returns [rows, heads * dv].
     generic=True forces the plain kernel (tests)."""
     rows = q.shape[0]
     if out is None and want_out:
         out = torch.empty((rows, heads * dv), dtype=q.dtype, device=q.device)
-    d, code = _paged_desc(q, cache, block_tables, heads, kv_heads, dk, dv, scale, window, keep_first, sink, out)
+    d, code = _paged_desc(q, cache, block_tables, heads, kv_heads, dk, dv, scale, window, keep_first, sink, out, chunk, turn)
     assert positions.dtype == torch.int64 and positions.is_contiguous() and positions.numel() == rows
     d.positions = positions.data_ptr()
     if row_seq is not None:
@@ -1013,7 +1040,7 @@ def paged_attend_rows(q, cache, block_tables, positions, heads, kv_heads, dk, dv
     else:
         assert block_tables.shape[0] >= rows
     if code == NVH_BF16 and row_seq is None and not generic and paged_attend_supported(dk, dv, cache.shape[1]):
-        d.splits = splits or paged_attend_splits(rows, kv_heads, heads, max_context, window, keep_first)
+        d.splits = splits or paged_attend_splits(rows, kv_heads, heads, max_context, window, keep_first, chunk)
     if d.splits > 1:
         part = torch.empty((rows, heads, d.splits, dv + 4), dtype=torch.float32, device=q.device)
         tickets = reserve_workspace(q.device, paged_attend_ticket_bytes(rows, kv_heads, heads), "paged_attend")
@@ -1029,14 +1056,14 @@ def paged_attend_ticket_bytes(rows, kv_heads, heads) -> int:
     return int(_lib.load().nvh_paged_attend_ticket_bytes(rows, kv_heads, heads))
 
 
-def paged_attend_prompt(q, cache, block_tables, cu_q, cu_k, max_q, heads, kv_heads, dk, dv, scale, window=0, keep_first=0, sink=None, out=None):
+def paged_attend_prompt(q, cache, block_tables, cu_q, cu_k, max_q, heads, kv_heads, dk, dv, scale, window=0, keep_first=0, sink=None, out=None, chunk=0, turn=None):
     """Attention of prompt portions over the pages (bf16): rows cu_q[b] .. of q are the last ones of sequence b, which has cu_k[b + 1] - cu_k[b] keys;
-    visibility and sink as in paged_attend_rows.  Returns [rows, heads * dv]."""
+    visibility, sink and turn as in paged_attend_rows.  Returns [rows, heads * dv]."""
     _require_gpu_bf16(q=q)
     _require_i32(cu_q=cu_q, cu_k=cu_k)
     if out is None:
         out = torch.empty((q.shape[0], heads * dv), dtype=q.dtype, device=q.device)
-    d, code = _paged_desc(q, cache, block_tables, heads, kv_heads, dk, dv, scale, window, keep_first, sink, out)
+    d, code = _paged_desc(q, cache, block_tables, heads, kv_heads, dk, dv, scale, window, keep_first, sink, out, chunk, turn)
     assert cu_q.numel() == cu_k.numel() and cu_q.is_contiguous() and cu_k.is_contiguous() and block_tables.shape[0] >= cu_q.numel() - 1
     d.cu_q, d.cu_k, d.batch, d.max_q = cu_q.data_ptr(), cu_k.data_ptr(), cu_q.numel() - 1, int(max_q)
     _lib.check(_lib.load().nvh_paged_attend_prompt(ctypes.byref(d), code, _stream()), "nvh_paged_attend_prompt")
@@ -1103,6 +1130,249 @@ def norm_gate(x, gate, weight, eps, n, packed=None):
     rc = _lib.load().nvh_norm_gate(out.data_ptr() if out is not None else None, packed.data_ptr() if packed is not None else None, x.data_ptr(), gate.data_ptr(),
                                    weight.data_ptr(), float(eps), rows, cols, int(n), x.stride(0), gate.stride(0), cols, code, _stream())
     _lib.check(rc, "nvh_norm_gate")
+    return out
+
+
+# --------------------------------------------------------------------------------------- several residual streams, the token before
+def _rows_desc(d, positions, rows, step):
+    """Where rows stand in their sequences (utils/step.py StepMeta)."""
+    assert positions.dtype == torch.int64 and positions.is_contiguous() and positions.numel() == rows
+    _require_i32(state_slots=step.state_slots)
+    d.positions, d.state_slots = positions.data_ptr(), step.state_slots.data_ptr()
+    if step.cu_rows is not None:
+        _require_i32(row_seq=step.row_seq, cu_rows=step.cu_rows)
+        assert step.row_seq.numel() == rows and step.state_slots.numel() >= step.cu_rows.numel() - 1
+        d.row_seq, d.cu_rows = step.row_seq.data_ptr(), step.cu_rows.data_ptr()
+        if hasattr(d, "sequences"):
+            d.sequences = step.cu_rows.numel() - 1
+    else:
+        assert step.num_decode == rows and step.state_slots.numel() >= rows
+
+
+def bigram_embed(tokens, positions, step, embed, bigram, mul_prev, mul_cur, last_token):
+    """embed[token] + bigram[(previous token * mul_prev + token * mul_cur) mod buckets] (the last of the buckets + 1 rows for a sequence's first token) as fp32
+    rows; last_token int64 [slots] carries the previous token from step to step."""
+    code, rows, cols = _act_code(embed, bigram), tokens.numel(), embed.shape[1]
+    assert tokens.dtype == torch.int64 and tokens.is_cuda and tokens.is_contiguous() and embed.is_contiguous() and bigram.is_contiguous() and bigram.shape[1] == cols
+    assert last_token.dtype == torch.int64 and last_token.is_cuda and last_token.is_contiguous()
+    x = torch.empty((rows, cols), dtype=torch.float32, device=embed.device)
+    d = _lib.BigramEmbedDesc()
+    _rows_desc(d, positions, rows, step)
+    d.x, d.tokens, d.last_token, d.embed, d.bigram = x.data_ptr(), tokens.data_ptr(), last_token.data_ptr(), embed.data_ptr(), bigram.data_ptr()
+    d.buckets, d.mul_prev, d.mul_cur, d.rows, d.cols, d.vocab = bigram.shape[0] - 1, int(mul_prev), int(mul_cur), rows, cols, embed.shape[0]
+    _lib.check(_lib.load().nvh_bigram_embed(ctypes.byref(d), code, _stream()), "nvh_bigram_embed")
+    return x
+
+
+def stream_mix(x, streams, dtype, n, update=None, read=None, norm=None, packed=None, want_rows=True, out=None):
+    """Hyper-connections between two sublayers.  x: [rows, streams, cols] (fp32), or [rows, cols] where all streams are alike.
+    update = dict(y, mix [from, to], out [to]): x_t <- sum_s mix[s, t] x_s + out[t] y (into `out`, or in place); with post = (y2, w, w2, scale) y is
+    scale (rms(y) w + rms(y2) w2) first, eps of the norm, as norm = (.., eps) or update["eps"].  Of the new streams u = sum_s read[s] x_s (None: plain sum);
+    norm = (weight, groups, eps): returns its RMS norm in `groups` equal parts of the n columns (in `dtype`; packed: in fragment order too); norm None: returns u (fp32)."""
+    alike = x.dim() == 2
+    rows, cols = x.shape[0], x.shape[-1]
+    _require_f32(x=x)
+    assert alike or x.shape[1] == streams
+    d = _lib.StreamMixDesc()
+    d.xin, d.xin_row, d.xin_stream = x.data_ptr(), cols if alike else streams * cols, 0 if alike else cols
+    d.rows, d.cols, d.n, d.streams, d.groups = rows, cols, int(n), int(streams), 1
+    if update is not None:
+        y = update["y"]
+        _require_f32(mix=update["mix"], out=update["out"])
+        assert y.shape == (rows, cols) and y.stride(1) == 1 and y.dtype == dtype and y.is_cuda and update["mix"].shape == (streams, streams) and update["out"].numel() == streams
+        d.y, d.y_stride, d.mix, d.out = y.data_ptr(), y.stride(0), update["mix"].data_ptr(), update["out"].data_ptr()
+        if update.get("post") is not None:
+            y2, w, w2, scale = update["post"]
+            _require_f32(w=w, w2=w2)
+            assert y2.shape == (rows, cols) and y2.stride(1) == 1 and y2.dtype == dtype and y2.is_cuda and w.numel() == w2.numel() == cols
+            d.y2, d.y2_stride, d.y_w, d.y2_w, d.y_scale, d.eps = y2.data_ptr(), y2.stride(0), w.data_ptr(), w2.data_ptr(), float(scale), float(update["eps"])
+        if out is None:
+            assert not alike, "streams that are all alike need somewhere to go"
+            out = x
+        _require_f32(out=out)
+        assert out.shape == (rows, streams, cols)
+        d.xout = out.data_ptr()
+    if read is not None:
+        _require_f32(read=read)
+        assert read.numel() == streams
+        setattr(d, "in", read.data_ptr())
+    if norm is None:
+        res = torch.empty((rows, cols), dtype=torch.float32, device=x.device)
+        d.sum = res.data_ptr()
+    else:
+        weight, d.groups, eps = norm
+        _require_f32(weight=weight)
+        assert weight.numel() == cols and (update is None or update.get("post") is None or update["eps"] == eps)
+        d.w, d.eps, res = weight.data_ptr(), float(eps), None
+        if want_rows:
+            res = torch.empty((rows, cols), dtype=dtype, device=x.device)
+            d.h = res.data_ptr()
+        if packed is not None:
+            _packed_ok(packed, rows, cols)
+            d.packed = packed.data_ptr()
+    _lib.check(_lib.load().nvh_stream_mix(ctypes.byref(d), _out_code(dtype), _stream()), "nvh_stream_mix")
+    return res
+
+
+def token_shift(h, positions, step, shift, ring, mu=None, packed=None):
+    """s = h + (h' - h) shift with h' the previous token's h; without mu returns s [1, rows, cols], with mu [mixes, cols] s + (s' - s) mu[k] for every k
+    [mixes, rows, cols]; packed (bf16): in fragment order into this buffer (one after the other), returns None.  ring [slots, 2 or 3 with mu, cols] carries h."""
+    code = _act_code(h, ring)
+    _require_f32(shift=shift)
+    rows, cols = h.shape
+    mixes = 0 if mu is None else mu.shape[0]
+    assert h.stride(1) == 1 and shift.numel() == cols and ring.is_contiguous() and ring.shape[1:] == (3 if mixes else 2, cols)
+    d = _lib.TokenShiftDesc()
+    _rows_desc(d, positions, rows, step)
+    d.h, d.h_stride, d.rows, d.cols, d.shift, d.mixes, d.ring, d.depth = h.data_ptr(), h.stride(0), rows, cols, shift.data_ptr(), mixes, ring.data_ptr(), ring.shape[1]
+    if mixes:
+        _require_f32(mu=mu)
+        assert mu.shape == (mixes, cols)
+        d.mu = mu.data_ptr()
+    out, count = None, max(mixes, 1)
+    if packed is None:
+        out = torch.empty((count, rows, cols), dtype=h.dtype, device=h.device)
+        d.out, d.out_mix = out.data_ptr(), rows * cols
+    else:
+        d.packed, d.out, d.out_mix = 1, packed.data_ptr(), (rows + 15) // 16 * 16 * cols
+        _require_gpu_bf16(packed=packed)
+        assert packed.is_contiguous() and packed.numel() >= count * d.out_mix
+    _lib.check(_lib.load().nvh_token_shift(ctypes.byref(d), code, _stream()), "nvh_token_shift")
+    return out
+
+
+def causal_conv(x, positions, step, weight, bias, ring, packed=None, want_rows=True):
+    """silu(bias + sum over taps of weight[tap] x), weight [taps, cols] with the last tap on the current token; ring [slots, taps, cols] carries x."""
+    code = _act_code(x, ring)
+    _require_f32(weight=weight, bias=bias)
+    rows, cols = x.shape
+    taps = weight.shape[0]
+    assert x.stride(1) == 1 and weight.shape[1] == cols and bias.numel() == cols and ring.is_contiguous() and ring.shape[1:] == (taps, cols)
+    d = _lib.CausalConvDesc()
+    _rows_desc(d, positions, rows, step)
+    d.x, d.x_stride, d.rows, d.cols, d.taps, d.w, d.b, d.ring = x.data_ptr(), x.stride(0), rows, cols, taps, weight.data_ptr(), bias.data_ptr(), ring.data_ptr()
+    out = None
+    if want_rows:
+        out = torch.empty((rows, cols), dtype=x.dtype, device=x.device)
+        d.out = out.data_ptr()
+    if packed is not None:
+        _packed_ok(packed, rows, cols)
+        d.packed = packed.data_ptr()
+    _lib.check(_lib.load().nvh_causal_conv(ctypes.byref(d), code, _stream()), "nvh_causal_conv")
+    return out
+
+
+# --------------------------------------------------------------------------------------- selective scan
+def scan_states(n) -> int:
+    """States the kernels keep for n of them (a power of two; 0: too many)."""
+    return int(_lib.load().nvh_scan_states(int(n)))
+
+
+def _scan_desc(x, dt, bc, z, p, positions, state_slots, state, out):
+    code = _act_code(x, dt, bc, z)
+    rows, (inner, n) = x.shape[0], p["a_log2"].shape
+    _require_f32(a_log2=p["a_log2"], d=p["d"], dt_bias=p["dt_bias"], state=state)
+    _require_i32(state_slots=state_slots)
+    assert x.shape[1] == z.shape[1] == p["d"].numel() == p["dt_bias"].numel() == inner and z.shape[0] == dt.shape[0] == bc.shape[0] == rows and bc.shape[1] >= 2 * n
+    assert x.stride(1) == z.stride(1) == dt.stride(1) == bc.stride(1) == 1 and state.shape[1:] == (inner, n)
+    assert positions.dtype == torch.int64 and positions.is_contiguous() and positions.numel() == rows
+    d = _lib.ScanDesc()
+    d.x, d.x_stride, d.dt, d.dt_stride, d.bc, d.bc_stride, d.z, d.z_stride = x.data_ptr(), x.stride(0), dt.data_ptr(), dt.stride(0), bc.data_ptr(), bc.stride(0), z.data_ptr(), z.stride(0)
+    d.dt_bias, d.a_log2, d.d, d.rows, d.inner, d.n = p["dt_bias"].data_ptr(), p["a_log2"].data_ptr(), p["d"].data_ptr(), rows, inner, n
+    d.positions, d.state_slots, d.state = positions.data_ptr(), state_slots.data_ptr(), state.data_ptr()
+    if out is not None:
+        assert out.shape == (rows, inner) and out.stride(1) == 1 and out.dtype == x.dtype
+        d.out, d.out_stride = out.data_ptr(), out.stride(0)
+    return d, code
+
+
+def scan_chunks(x, dt, bc, z, params, positions, state_slots, chunks, summaries, state, out=None):
+    """Selective scan over portions of sequences: x, dt (in front of bias and softplus), z [rows, inner]; bc rows B (n) | C (n); params = dict(a_log2 [inner, n], d,
+    dt_bias); chunks int32 [n, 4] = (first row, rows, sequence, index in its portion); summaries: some portion has more than one segment; state [slots, inner, n]
+    fp32 is updated.  Returns (scan + d x) silu(z); rows no segment covers are left alone in `out`."""
+    if out is None:
+        out = torch.empty((x.shape[0], x.shape[1]), dtype=x.dtype, device=x.device)
+    d, code = _scan_desc(x, dt, bc, z, params, positions, state_slots, state, out)
+    _require_i32(chunks=chunks)
+    assert dt.shape[1] == x.shape[1] and chunks.dim() == 2 and chunks.shape[1] == 4 and chunks.is_contiguous()
+    d.chunks, d.n_chunks, d.summaries = chunks.data_ptr(), chunks.shape[0], int(summaries)
+    if summaries:
+        seg, seg_dt = (torch.empty((chunks.shape[0], *s), dtype=torch.float32, device=x.device) for s in (state.shape[1:], state.shape[1:2]))
+        d.seg_state, d.seg_dt = seg.data_ptr(), seg_dt.data_ptr()
+    _lib.check(_lib.load().nvh_scan_chunks(ctypes.byref(d), code, _stream()), "nvh_scan_chunks")
+    return out
+
+
+def scan_step(x, dt, bc, z, params, positions, state_slots, state, out=None, out_packed=None, want_out=True):
+    """One new token per sequence (row i = sequence i), bf16; dt [rows, rank] is multiplied by params["w_dt"] [inner, rank] first."""
+    rows, w = x.shape[0], params["w_dt"]
+    if out is None and want_out:
+        out = torch.empty((rows, x.shape[1]), dtype=x.dtype, device=x.device)
+    d, code = _scan_desc(x, dt, bc, z, params, positions, state_slots, state, out)
+    _act_code(x, w)
+    assert w.is_contiguous() and w.shape[0] == x.shape[1] and dt.shape[1] >= w.shape[1] and state_slots.numel() >= rows
+    d.w_dt, d.rank = w.data_ptr(), w.shape[1]
+    if out_packed is not None:
+        _packed_ok(out_packed, rows, x.shape[1])
+        d.out_packed = out_packed.data_ptr()
+    _lib.check(_lib.load().nvh_scan_step(ctypes.byref(d), code, _stream()), "nvh_scan_step")
+    return out
+
+
+# --------------------------------------------------------------------------------------- time mixing with a decaying matrix state
+def wkv_supported(dim) -> bool:
+    return bool(_lib.load().nvh_wkv_supported(int(dim)))
+
+
+def _wkv_desc(r, k, v, g, z, p, eps, n, positions, state_slots, state, out):
+    code = _act_code(r, k, v, g, z)
+    slots, heads, dim, dv = state.shape
+    rows, cols = r.shape[0], heads * dim
+    _require_f32(w0=p["w0"], u=p["u"], norm=p["norm"], state=state)
+    _require_i32(state_slots=state_slots)
+    assert dv == dim and all(t.shape[0] == rows and t.shape[1] >= cols and t.stride(1) == 1 and t.stride(0) == r.stride(0) for t in (r, k, v, g))
+    assert z.shape[0] == rows and z.stride(1) == 1 and all(p[t].numel() == cols for t in ("w0", "u", "norm"))
+    assert positions.dtype == torch.int64 and positions.is_contiguous() and positions.numel() == rows
+    d = _lib.WkvDesc()
+    d.r, d.k, d.v, d.g, d.stride, d.z, d.z_stride = r.data_ptr(), k.data_ptr(), v.data_ptr(), g.data_ptr(), r.stride(0), z.data_ptr(), z.stride(0)
+    d.w0, d.u, d.norm, d.eps, d.n, d.rows, d.heads, d.dim = p["w0"].data_ptr(), p["u"].data_ptr(), p["norm"].data_ptr(), float(eps), int(n), rows, heads, dim
+    d.positions, d.state_slots, d.state = positions.data_ptr(), state_slots.data_ptr(), state.data_ptr()
+    if out is not None:
+        assert out.shape == (rows, cols) and out.stride(1) == 1 and out.dtype == r.dtype
+        d.out, d.out_stride = out.data_ptr(), out.stride(0)
+    return d, code
+
+
+def wkv_chunks(r, k, v, g, z, params, eps, n, positions, state_slots, chunks, summaries, state, out=None, generic=False):
+    """Time mixing over portions of sequences: r, k, v, g, z [rows, heads * dim]; params = dict(w0, u, norm [heads * dim]); decays exp(-exp(z + w0)); n: columns of a
+    head the norm counts; chunks int32 [n, 4] = (first row, rows, sequence, index in its portion); summaries: some portion has more than one segment; state
+    [slots, heads, dim, dim] fp32 is updated.  Rows no segment covers are left alone in `out`.  generic=True forces the plain kernel (tests)."""
+    if out is None:
+        out = torch.empty((r.shape[0], state.shape[1] * state.shape[2]), dtype=r.dtype, device=r.device)
+    d, code = _wkv_desc(r, k, v, g, z, params, eps, n, positions, state_slots, state, out)
+    _require_i32(chunks=chunks)
+    assert z.shape[1] >= state.shape[1] * state.shape[2] and chunks.dim() == 2 and chunks.shape[1] == 4 and chunks.is_contiguous()
+    d.chunks, d.n_chunks, d.summaries = chunks.data_ptr(), chunks.shape[0], int(summaries)
+    if summaries:
+        seg, dec = (torch.empty((chunks.shape[0], *s), dtype=torch.float32, device=r.device) for s in (state.shape[1:], state.shape[1:3]))
+        d.seg_state, d.seg_decay = seg.data_ptr(), dec.data_ptr()
+    _lib.check(_lib.load().nvh_wkv_chunks(ctypes.byref(d), int(generic), code, _stream()), "nvh_wkv_chunks")
+    return out
+
+
+def wkv_step(r, k, v, g, z, params, eps, n, positions, state_slots, state, out=None, out_packed=None, want_out=True):
+    """One new token per sequence (row i = sequence i), bf16; z [rows, rank]: decays of params["w2"] tanh(z) with w2 [heads * dim, rank]."""
+    rows, w2, cols = r.shape[0], params["w2"], state.shape[1] * state.shape[2]
+    if out is None and want_out:
+        out = torch.empty((rows, cols), dtype=r.dtype, device=r.device)
+    d, code = _wkv_desc(r, k, v, g, z, params, eps, n, positions, state_slots, state, out)
+    _act_code(r, w2)
+    assert w2.is_contiguous() and w2.shape[0] >= cols and z.shape[1] >= w2.shape[1] and state_slots.numel() >= rows
+    d.w2, d.rank = w2.data_ptr(), w2.shape[1]
+    if out_packed is not None:
+        _packed_ok(out_packed, rows, cols)
+        d.out_packed = out_packed.data_ptr()
+    _lib.check(_lib.load().nvh_wkv_step(ctypes.byref(d), code, _stream()), "nvh_wkv_step")
     return out
 
 

@@ -16,6 +16,7 @@ class StepMeta:
     summaries: bool                                 # some portion has more than one segment
     max_context: int                                # host bound on the context of any row
     row_seq: torch.Tensor | None = None             # int32 [rows] sequence of every row (None: decode rows only)
+    cu_rows: torch.Tensor | None = None             # int32 [sequences + 1] rows of every sequence (None: decode rows only)
     cu_q: torch.Tensor | None = None                # int32 [portions + 1] row offsets of the portions, from the first portion row
     cu_k: torch.Tensor | None = None                # int32 [portions + 1] offsets of the keys the portions see
     max_q: int = 0
