@@ -313,7 +313,7 @@ def main():
     ap.add_argument("--prefill-leg", action="store_true", help="time the prefill attention op for models other than the headline one too")
     ap.add_argument("--beside", choices=["1k", "2k", "4k"], help="instead of the default workload: another model beside a Qwen2-shaped one of this size "
                     "(engine throughput and kernels against their rooflines), one JSON line")
-    ap.add_argument("--beside-model", choices=["zobasun", "galirax", "kekapel"], default="zobasun")
+    ap.add_argument("--beside-model", choices=["zobasun", "galirax", "kekapel", "zaposun"], default="zobasun")
     ap.add_argument("--beside-only", choices=["kernels", "engine"])
     args = ap.parse_args()
     if args.beside:

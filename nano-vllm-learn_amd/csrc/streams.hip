@@ -193,68 +193,122 @@ __device__ __forceinline__ const T* earlier_row(const T* rows, int64_t stride, c
 }
 __device__ __forceinline__ f32x8 lerp8(const f32x8& h, const f32x8& before, const f32x8& mu) { return {h.a + (before.a - h.a) * mu.a, h.b + (before.b - h.b) * mu.b}; }
 
-// grid (rows, column blocks of 2048)
-template <typename T>
+// whether CNT rows from `row` on belong to one portion
+template <int CNT>
+__device__ __forceinline__ bool one_portion(const int32_t* row_seq, const int32_t* cu_rows, int row, int rows) {
+    return CNT > 1 && cu_rows && row + CNT <= rows && row_seq[row] == row_seq[row + CNT - 1];
+}
+
+// grid (CNT rows each, column blocks of 2048).  Rows of one portion share the loads of coefficients and of each other; others go one by one
+template <typename T, int CNT>
 __global__ __launch_bounds__(256) void token_shift_kernel(const TokenShiftArgs a) {
-    const int row = blockIdx.x, c = (blockIdx.y * 256 + threadIdx.x) * 8;
+    const int r0 = blockIdx.x * CNT, c = (blockIdx.y * 256 + threadIdx.x) * 8;
     if (c >= a.cols) return;
-    const RowPlace at = row_place(a.row_seq, a.cu_rows, row);
-    const int slot = a.state_slots[at.seq];
-    const int64_t pos = a.positions[row];
     const T* h = reinterpret_cast<const T*>(a.h);
     T* ring = reinterpret_cast<T*>(a.ring);
-    const T* p1 = earlier_row(h, a.h_stride, (const T*)ring, a.depth, a.cols, row, 1, at, pos, slot);
-    const T* p2 = a.mixes ? earlier_row(h, a.h_stride, (const T*)ring, a.depth, a.cols, row, 2, at, pos, slot) : nullptr;
-    const f32x8 h0 = act_ld8(h + (int64_t)row * a.h_stride + c), h1 = p1 ? act_ld8(p1 + c) : zero8(), h2 = p2 ? act_ld8(p2 + c) : zero8(), shift = act_ld8(a.shift + c);
-    const f32x8 s0 = lerp8(h0, h1, shift);
-    auto put = [&](int k, const f32x8& v) {
+    const f32x8 shift = act_ld8(a.shift + c);
+    auto put = [&](int row, int k, const f32x8& v) {
         if (a.packed) act_st8(reinterpret_cast<uint16_t*>(a.out) + k * a.out_mix + pack_index(row, c, a.cols), v);
         else act_st8(reinterpret_cast<T*>(a.out) + k * a.out_mix + (int64_t)row * a.cols + c, v);
     };
-    if (a.mixes == 0) put(0, s0);
-    else {
-        const f32x8 s1 = lerp8(h1, h2, shift);
-        for (int k = 0; k < a.mixes; ++k) put(k, lerp8(s0, s1, act_ld8(a.mu + (int64_t)k * a.cols + c)));
+    auto run = [&](auto cnt, int row0) {             // decltype(cnt)::value rows of one portion
+        constexpr int N = decltype(cnt)::value;
+        const RowPlace at = row_place(a.row_seq, a.cu_rows, row0);
+        const int slot = a.state_slots[at.seq];
+        const int64_t pos = a.positions[row0];
+        const T* p1 = earlier_row(h, a.h_stride, (const T*)ring, a.depth, a.cols, row0, 1, at, pos, slot);
+        const T* p2 = a.mixes ? earlier_row(h, a.h_stride, (const T*)ring, a.depth, a.cols, row0, 2, at, pos, slot) : nullptr;
+        f32x8 hv[N], before = p1 ? act_ld8(p1 + c) : zero8(), s1 = p2 ? act_ld8(p2 + c) : zero8();
+#pragma unroll
+        for (int i = 0; i < N; ++i) hv[i] = act_ld8(h + (int64_t)(row0 + i) * a.h_stride + c);
+        s1 = lerp8(before, s1, shift);
+        if (!a.cu_rows && slot >= 0) act_st8(ring + ((int64_t)slot * a.depth + (int)(pos % a.depth)) * a.cols + c, hv[0]);
+        f32x8 sv[N];
+#pragma unroll
+        for (int i = 0; i < N; ++i) {
+            sv[i] = lerp8(hv[i], before, shift);
+            before = hv[i];
+            if (a.mixes == 0) put(row0 + i, 0, sv[i]);
+        }
+        for (int k = 0; k < a.mixes; ++k) {
+            const f32x8 mu = act_ld8(a.mu + (int64_t)k * a.cols + c);
+#pragma unroll
+            for (int i = 0; i < N; ++i) put(row0 + i, k, lerp8(sv[i], i ? sv[i ? i - 1 : 0] : s1, mu));
+        }
+    };
+    if (one_portion<CNT>(a.row_seq, a.cu_rows, r0, a.rows)) {
+        run(std::integral_constant<int, CNT>{}, r0);
+    } else {
+        for (int r = r0; r < r0 + CNT && r < a.rows; ++r) run(std::integral_constant<int, 1>{}, r);
     }
-    if (!a.cu_rows && slot >= 0) act_st8(ring + ((int64_t)slot * a.depth + (int)(pos % a.depth)) * a.cols + c, h0);
 }
 
-// grid (rows, column blocks of 2048).  TAPS: the kernel's size, 0: any
-template <typename T, int TAPS>
+// grid (CNT rows each, column blocks of 2048).  TAPS: the kernel's size, 0: any (CNT 1)
+template <typename T, int TAPS, int CNT>
 __global__ __launch_bounds__(256) void causal_conv_kernel(const ConvArgs a) {
-    const int row = blockIdx.x, c = (blockIdx.y * 256 + threadIdx.x) * 8;
+    const int r0 = blockIdx.x * CNT, c = (blockIdx.y * 256 + threadIdx.x) * 8, taps = TAPS ? TAPS : a.taps;
     if (c >= a.cols) return;
-    const RowPlace at = row_place(a.row_seq, a.cu_rows, row);
-    const int slot = a.state_slots[at.seq], taps = TAPS ? TAPS : a.taps;
-    const int64_t pos = a.positions[row];
     const T* x = reinterpret_cast<const T*>(a.x);
     T* ring = reinterpret_cast<T*>(a.ring);
-    f32x8 acc = act_ld8(a.b + c);
-    const f32x8 own = act_ld8(x + (int64_t)row * a.x_stride + c);
-    auto tap = [&](int back) {
-        const T* p = earlier_row(x, a.x_stride, (const T*)ring, a.taps, a.cols, row, back, at, pos, slot);
-        if (!p) return;
-        const f32x8 v = act_ld8(p + c), w = act_ld8(a.w + (int64_t)(taps - 1 - back) * a.cols + c);
+    const f32x8 bias = act_ld8(a.b + c);
+    auto tap = [&](f32x8& acc, const f32x8& v, const f32x8& w) {
         acc.a += v.a * w.a;
         acc.b += v.b * w.b;
     };
-    if constexpr (TAPS > 0) {
+    auto finish = [&](int row, f32x8 acc) {
 #pragma unroll
-        for (int back = TAPS - 1; back > 0; --back) tap(back);
-    } else {
-        for (int back = taps - 1; back > 0; --back) tap(back);
-    }
-    const f32x8 w = act_ld8(a.w + (int64_t)(taps - 1) * a.cols + c);
-    acc.a += own.a * w.a;
-    acc.b += own.b * w.b;
+        for (int k = 0; k < 4; ++k) {
+            acc.a[k] = silu_f(acc.a[k]);
+            acc.b[k] = silu_f(acc.b[k]);
+        }
+        if (a.packed) act_st8(reinterpret_cast<uint16_t*>(a.packed) + pack_index(row, c, a.cols), acc);
+        if (a.out) act_st8(reinterpret_cast<T*>(a.out) + (int64_t)row * a.cols + c, acc);
+    };
+    auto before = [&](int row, int back, const RowPlace& at, int64_t pos, int slot) {
+        const T* p = earlier_row(x, a.x_stride, (const T*)ring, a.taps, a.cols, row, back, at, pos, slot);
+        return p ? act_ld8(p + c) : zero8();
+    };
+    if constexpr (TAPS > 0 && CNT > 1) {
+        if (one_portion<CNT>(a.row_seq, a.cu_rows, r0, a.rows)) {
+            const RowPlace at = row_place(a.row_seq, a.cu_rows, r0);
+            const int slot = a.state_slots[at.seq];
+            const int64_t pos = a.positions[r0];
+            f32x8 v[CNT + TAPS - 1], w[TAPS];
 #pragma unroll
-    for (int k = 0; k < 4; ++k) {
-        acc.a[k] = silu_f(acc.a[k]);
-        acc.b[k] = silu_f(acc.b[k]);
+            for (int i = 0; i < CNT; ++i) v[TAPS - 1 + i] = act_ld8(x + (int64_t)(r0 + i) * a.x_stride + c);
+#pragma unroll
+            for (int i = 0; i < TAPS - 1; ++i) v[i] = before(r0, TAPS - 1 - i, at, pos, slot);
+#pragma unroll
+            for (int j = 0; j < TAPS; ++j) w[j] = act_ld8(a.w + (int64_t)j * a.cols + c);
+#pragma unroll
+            for (int i = 0; i < CNT; ++i) {
+                f32x8 acc = bias;
+#pragma unroll
+                for (int j = 0; j < TAPS; ++j) tap(acc, v[i + j], w[j]);
+                finish(r0 + i, acc);
+            }
+            return;
+        }
     }
-    if (a.packed) act_st8(reinterpret_cast<uint16_t*>(a.packed) + pack_index(row, c, a.cols), acc);
-    if (a.out) act_st8(reinterpret_cast<T*>(a.out) + (int64_t)row * a.cols + c, acc);
-    if (!a.cu_rows && slot >= 0) act_st8(ring + ((int64_t)slot * a.taps + (int)(pos % a.taps)) * a.cols + c, own);
+    for (int row = r0; row < r0 + CNT && row < a.rows; ++row) {
+        const RowPlace at = row_place(a.row_seq, a.cu_rows, row);
+        const int slot = a.state_slots[at.seq];
+        const int64_t pos = a.positions[row];
+        f32x8 acc = bias;
+        const f32x8 own = act_ld8(x + (int64_t)row * a.x_stride + c);
+        if constexpr (TAPS > 0) {
+            f32x8 v[TAPS > 1 ? TAPS - 1 : 1];
+#pragma unroll
+            for (int j = 0; j < TAPS - 1; ++j) v[j] = before(row, TAPS - 1 - j, at, pos, slot);
+#pragma unroll
+            for (int j = 0; j < TAPS - 1; ++j) tap(acc, v[j], act_ld8(a.w + (int64_t)j * a.cols + c));
+        } else {
+            for (int j = 0; j < taps - 1; ++j) tap(acc, before(row, taps - 1 - j, at, pos, slot), act_ld8(a.w + (int64_t)j * a.cols + c));
+        }
+        tap(acc, own, act_ld8(a.w + (int64_t)(taps - 1) * a.cols + c));
+        finish(row, acc);
+        if (!a.cu_rows && slot >= 0) act_st8(ring + ((int64_t)slot * a.taps + (int)(pos % a.taps)) * a.cols + c, own);
+    }
 }
 
 // the last rows of every portion into its ring; grid (sequences, depth, column blocks)
@@ -299,16 +353,24 @@ int mix_t(const StreamMixArgs& a, hipStream_t stream) {
 
 template <typename T>
 int shift_t(const TokenShiftArgs& a, hipStream_t stream) {
-    token_shift_kernel<T><<<dim3(a.rows, (a.cols + 2047) / 2048), 256, 0, stream>>>(a);
+    const unsigned blocks = (a.cols + 2047) / 2048;
+    if (a.cu_rows && a.rows >= 1024) token_shift_kernel<T, 4><<<dim3((a.rows + 3) / 4, blocks), 256, 0, stream>>>(a);
+    else token_shift_kernel<T, 1><<<dim3(a.rows, blocks), 256, 0, stream>>>(a);
     if (a.cu_rows) ring_store<T>(a.ring, a.h, a.h_stride, a.depth, a.cols, a.sequences, a.cu_rows, a.positions, a.state_slots, stream);
     return check_launch("token_shift");
 }
 
 template <typename T>
 int conv_t(const ConvArgs& a, hipStream_t stream) {
-    const dim3 grid(a.rows, (a.cols + 2047) / 2048);
-    if (a.taps == 4) causal_conv_kernel<T, 4><<<grid, 256, 0, stream>>>(a);
-    else causal_conv_kernel<T, 0><<<grid, 256, 0, stream>>>(a);
+    const unsigned blocks = (a.cols + 2047) / 2048;
+    auto go = [&](auto taps) {
+        if (a.cu_rows && a.rows >= 1024) causal_conv_kernel<T, decltype(taps)::value, 8><<<dim3((a.rows + 7) / 8, blocks), 256, 0, stream>>>(a);
+        else causal_conv_kernel<T, decltype(taps)::value, 1><<<dim3(a.rows, blocks), 256, 0, stream>>>(a);
+    };
+    if (a.taps == 4) go(std::integral_constant<int, 4>{});
+    else if (a.taps == 3) go(std::integral_constant<int, 3>{});
+    else if (a.taps == 2) go(std::integral_constant<int, 2>{});
+    else causal_conv_kernel<T, 0, 1><<<dim3(a.rows, blocks), 256, 0, stream>>>(a);
     if (a.cu_rows) ring_store<T>(a.ring, a.x, a.x_stride, a.taps, a.cols, a.sequences, a.cu_rows, a.positions, a.state_slots, stream);
     return check_launch("causal_conv");
 }

@@ -1,5 +1,5 @@
-"""Zobasun, Galirax or Kekapel beside the closest other model (a Qwen2-shaped stack; for Kekapel also Galirax with windows in every layer) at equal size, on
-random weights: prefill and decode throughput through the engine, and each hot kernel against its roofline.
+"""Zobasun, Galirax, Kekapel or Zaposun beside the closest other model (a Qwen2-shaped stack; for Kekapel also Galirax with windows in every layer, for Zaposun also
+Zobasun) at equal size, on random weights: prefill and decode throughput through the engine, and each hot kernel against its roofline.
 bench.py --beside SIZE [--beside-model NAME] prints the result as one JSON line."""
 from __future__ import annotations
 
@@ -17,7 +17,9 @@ from .layers.rotary import rotation_table
 from .models.galirax import GaliraxConfig
 from .models.kekapel import KekapelConfig
 from .models.qwen import ModelConfig
+from .models.zaposun import ZaposunConfig
 from .models.zobasun import ZobasunConfig
+from .utils.step import StepMeta
 
 HBM_GBPS, MFMA_TFLOPS = 8000.0, 2500.0          # MI355X peaks (dense bf16)
 
@@ -28,7 +30,8 @@ SIZES = {
     "4k": dict(width=4096, ff=12288, layers=6, heads=32, kv_heads=8, q_rank=1536, kv_rank=512, dim=128, rot=64, vdim=128, rec=4096, blocks=16, experts=32, top=4),
 }
 VOCAB = 32000
-WINDOW, KEEP = 512, 4                           # Galirax's windowed layers; Kekapel's window
+WINDOW, KEEP = 512, 4                           # Galirax's windowed layers; Kekapel's window; Zaposun's chunks
+STREAMS, STATES, TAPS = 4, 16, 4                # Zaposun
 
 
 def qwen_config(size):
@@ -59,6 +62,18 @@ def kekapel_config(size):
     mlps = ({"kind": "dense", "ff": s["ff"]}, {"kind": "moe", "expert": {"ff": s["ff"] // s["top"], "limit": 7.0}, "router": {"experts": s["experts"], "top": s["top"]}})
     return KekapelConfig.from_json({"width": s["width"], "vocab": VOCAB, "norm": {"eps": 1e-6}, "embedding": {"scale": 1.0}, "residual_mult": 0.7, "max_positions": 16384,
                                     "layers": [dict(type="attention", mixer=att, mlp=mlps[i % 2]) for i in range(s["layers"])]})
+
+
+def zaposun_config(size):
+    """Time mixing (heads of 64) and attention beside a scan of twice the width in turn."""
+    s = SIZES[size]
+    mlp = {"kind": "dense", "ff": s["ff"]}
+    wkv = {"type": "wkv", "mixer": {"heads": s["width"] // 64, "dim": 64}, "mlp": mlp}
+    par = {"type": "parallel", "mlp": mlp, "mixer": {
+        "left": dict(heads=s["heads"], kv_heads=s["kv_heads"], dim=128, vdim=128, scale=128 ** -0.5, rot={"base": 10000.0, "dims": 128}, mask={"size": WINDOW}),
+        "right": dict(inner=2 * s["width"], state=STATES, dt_rank=s["width"] // 16, conv=TAPS)}}
+    return ZaposunConfig.from_json({"width": s["width"], "vocab": VOCAB, "norm": {"eps": 1e-6, "groups": 2}, "streams": STREAMS, "logit_scale": 1.0,
+                                    "embedding": {"bigram": {"buckets": 4093, "mul_prev": 31, "mul_cur": 17}}, "layers": [(wkv, par)[i % 2] for i in range(s["layers"])]})
 
 
 def zobasun_config(size):
@@ -426,7 +441,158 @@ def kekapel_kernels(size, batch=32, ctx=1536, seqs=16, prompt=1024):
     return out
 
 
-MODELS = {"zobasun": (zobasun_config, zobasun_kernels), "galirax": (galirax_config, galirax_kernels), "kekapel": (kekapel_config, kekapel_kernels)}
+@torch.inference_mode()
+def zaposun_kernels(size, batch=32, ctx=1536, seqs=16, prompt=1024):
+    """Each hot kernel of Zaposun alone, and on operands of the same size the like kernels of Galirax (lightning attention, windowed attention, prep, residual), of
+    Zobasun (recurrence) and of the Qwen stack."""
+    s, out, rows = SIZES[size], {}, seqs * prompt
+    h, g, d, width, ff = s["heads"], s["kv_heads"], 128, s["width"], s["ff"]
+    cu = torch.arange(0, rows + 1, prompt, dtype=torch.int32, device="cuda")
+    pos = torch.arange(prompt, device="cuda").repeat(seqs)
+    slots = torch.arange(max(seqs, batch), dtype=torch.int32, device="cuda")
+    row_seq = torch.arange(seqs, dtype=torch.int32, device="cuda").repeat_interleave(prompt)
+    dpos = torch.full((batch,), ctx - 1, device="cuda")
+    many = StepMeta(0, None, None, slots[:seqs], None, 64, False, prompt, row_seq, cu)
+    single = StepMeta(batch, None, None, slots[:batch], None, 64, False, ctx)
+    f32, one = torch.float32, torch.ones(width, device="cuda")
+
+    def segments(units):
+        seg = choose_segment([prompt] * seqs, units)
+        return torch.tensor([c for i in range(seqs) for c in recurrence_chunks(i * prompt, prompt, i, seg)], dtype=torch.int32, device="cuda"), seg < prompt
+    # ---- residual streams, shifts
+    ys = [_randn(rows, width) for _ in range(3)]
+    mix, vec, w32 = torch.eye(STREAMS, device="cuda"), torch.full((STREAMS,), 0.3, device="cuda"), (one, 2, 1e-6)
+    xs = [_randn(rows, STREAMS, width, dtype=f32)]
+    us = _time([lambda y=y: ops.stream_mix(xs[0], STREAMS, torch.bfloat16, width, dict(y=y, mix=mix, out=vec), vec, w32) for y in ys])
+    out["stream_mix"] = _line(us, rows * width * (8 * STREAMS + 4))
+    us = _time([lambda y=y: ops.stream_mix(xs[0], STREAMS, torch.bfloat16, width, dict(y=y, mix=mix, out=vec, eps=1e-6, post=(ys[0], one, one, 0.5)), vec, w32) for y in ys[1:]])
+    out["stream_mix, two mixers"] = _line(us, rows * width * (8 * STREAMS + 6))
+    st = xs.pop()[:, 0].contiguous()
+    us = _time([lambda y=y: ops.residual_norm(st, torch.bfloat16, y=y, weight=one, bias=one, eps=1e-6) for y in ys])
+    out["galirax residual_norm"] = _line(us, rows * width * 12)
+    ring, mu = torch.zeros(max(seqs, batch), 3, width, device="cuda", dtype=torch.bfloat16), torch.rand(5, width, device="cuda")
+    us = _time([lambda y=y: ops.token_shift(y, pos, many, one, ring, mu) for y in ys])
+    out["token_shift, five mixes"] = _line(us, rows * width * 12)
+    ring2 = torch.zeros(max(seqs, batch), 2, width, device="cuda", dtype=torch.bfloat16)
+    us = _time([lambda y=y: ops.token_shift(y, pos, many, one, ring2) for y in ys])
+    out["token_shift"] = _line(us, rows * width * 4)
+    x1 = [_randn(batch, STREAMS, width, dtype=f32) for _ in range(4)]
+    y1, pk = _randn(batch, width), torch.zeros((batch + 15) // 16 * 16 * width * 5, dtype=torch.bfloat16, device="cuda")
+    us = _time([lambda x=x: ops.stream_mix(x, STREAMS, torch.bfloat16, width, dict(y=y1, mix=mix, out=vec), vec, w32) for x in x1] * 5)
+    out["stream_mix_decode"] = _line(us, batch * width * (8 * STREAMS + 4))
+    us = _time([lambda: ops.token_shift(y1, dpos, single, one, ring, mu, packed=pk)] * 20)
+    out["token_shift_decode"] = _line(us, batch * width * 18)
+    x1 = _randn(batch, width, dtype=f32)
+    us = _time([lambda: ops.residual_norm(x1, torch.bfloat16, y=y1, weight=one, bias=one, eps=1e-6)] * 20)
+    out["galirax residual_norm_decode"] = _line(us, batch * width * 12)
+    del ys, st
+    # ---- time mixing
+    hw = width // 64
+    x = [[_randn(rows, width) for _ in range(5)] for _ in range(2)]
+    p = dict(w0=torch.rand(width, device="cuda") * 5 - 6, u=_randn(width, dtype=f32), norm=one, w2=_randn(width, 64) * 0.05)
+    o = torch.empty(rows, width, device="cuda", dtype=torch.bfloat16)
+    state = torch.zeros(max(seqs, batch), hw, 64, 64, device="cuda")
+    chunks, more = segments(hw)
+    us = _time([lambda a=a: ops.wkv_chunks(*a, p, 1e-6, 64, pos, slots, chunks, more, state, out=o) for a in x] * 2)
+    out["wkv_chunks"] = _line(us, rows * 12 * width, 4 * rows * width * 64)
+    x1 = [_randn(batch, width) for _ in range(4)]
+    z1 = _randn(batch, 64)
+    states = [torch.zeros(batch, hw, 64, 64, device="cuda") for _ in range(max(2, int(3e8 // (4 * batch * width * 64)) + 1))]
+    us = _time([lambda t=t: ops.wkv_step(*x1, z1, p, 1e-6, 64, dpos, slots, t) for t in states] * 3)
+    out["wkv_step"] = _line(us, 8 * batch * width * 64)
+    del x, states, state
+    x = [_randn(rows, 4 * h * d) for _ in range(2)]
+    decay, state = torch.linspace(0.8, 0.999, h, device="cuda"), torch.zeros(max(seqs, batch), h, d, d, device="cuda")
+    o = torch.empty(rows, h * d, device="cuda", dtype=torch.bfloat16)
+    chunks, more = segments(h * 2)
+    us = _time([lambda a=a: ops.lightning_chunks(a, decay, pos, slots, chunks, more, state, out=o) for a in x] * 2)
+    out["galirax lightning_chunks"] = _line(us, rows * 8 * h * d, 4 * rows * h * d * d)
+    x1 = _randn(batch, 4 * h * d)
+    states = [torch.zeros(batch, h, d, d, device="cuda") for _ in range(max(2, int(3e8 // (4 * batch * h * d * d)) + 1))]
+    us = _time([lambda t=t: ops.lightning_step(x1, decay, dpos, slots, t) for t in states] * 3)
+    out["galirax lightning_step"] = _line(us, 8 * batch * h * d * d)
+    del x, states, state
+    # ---- scan
+    inner, rank = 2 * width, width // 16
+    xz = [_randn(rows, 2 * inner) for _ in range(2)]
+    conv, bias, cring = _randn(TAPS, inner, dtype=f32), _randn(inner, dtype=f32), torch.zeros(max(seqs, batch), TAPS, inner, device="cuda", dtype=torch.bfloat16)
+    us = _time([lambda a=a: ops.causal_conv(a[:, :inner], pos, many, conv, bias, cring) for a in xz] * 2)
+    out["causal_conv"] = _line(us, rows * inner * 4)
+    dt, bc = _randn(rows, inner), _randn(rows, 64)
+    p = dict(a_log2=-torch.rand(inner, STATES, device="cuda") * 4, d=torch.ones(inner, device="cuda"), dt_bias=torch.rand(inner, device="cuda") * 4 - 5, w_dt=_randn(inner, (rank + 63) // 64 * 64) * 0.1)
+    o = torch.empty(rows, inner, device="cuda", dtype=torch.bfloat16)
+    state = torch.zeros(max(seqs, batch), inner, STATES, device="cuda")
+    chunks, more = segments(inner // 64)
+    us = _time([lambda a=a: ops.scan_chunks(a[:, :inner], dt, bc, a[:, inner:], p, pos, slots, chunks, more, state, out=o) for a in xz] * 2)
+    out["scan_chunks"] = _line(us, rows * inner * 8)
+    x1, low, bc1 = _randn(batch, 2 * inner), _randn(batch, p["w_dt"].shape[1]), _randn(batch, 64)
+    states = [torch.zeros(batch, inner, STATES, device="cuda") for _ in range(max(2, int(3e8 // (4 * batch * inner * STATES)) + 1))]
+    us = _time([lambda t=t: ops.scan_step(x1[:, :inner], low, bc1, x1[:, inner:], p, dpos, slots, t) for t in states] * 3)
+    out["scan_step"] = _line(us, batch * inner * (8 * STATES + 6) + 2 * p["w_dt"].numel())
+    us = _time([lambda: ops.causal_conv(x1[:, :inner], dpos, single, conv, bias, cring)] * 20)
+    out["causal_conv_decode"] = _line(us, batch * inner * 2 * (TAPS + 2))
+    del xz, dt, o, states, state
+    rec, blocks = s["rec"], s["blocks"]
+    p = dict(conv_w=_randn(4, rec, dtype=f32), conv_b=_randn(rec, dtype=f32), ra=_randn(blocks, rec // blocks, rec // blocks) * 0.05, ri=_randn(blocks, rec // blocks, rec // blocks) * 0.05,
+             ra_b=_randn(rec, dtype=f32), ri_b=_randn(rec, dtype=f32), rate=torch.rand(rec, device="cuda"))
+    state, cring = torch.zeros(max(seqs, batch), rec, device="cuda"), torch.zeros(max(seqs, batch), 4, rec, dtype=torch.bfloat16, device="cuda")
+    yx, o = [_randn(rows, 2 * rec) for _ in range(2)], torch.empty(rows, rec, device="cuda", dtype=torch.bfloat16)
+    seg = choose_segment([prompt] * seqs, blocks)
+    chunks, more = segments(blocks)
+    us = _time([lambda a=a: ops.rglru_chunks(a, p, pos, slots, chunks, seg, more, state, cring, out=o) for a in yx] * 2)
+    out["zobasun rglru_chunks"] = _line(us, rows * rec * 6, 4 * rows * rec * (rec // blocks))
+    x1 = _randn(batch, 2 * rec)
+    us = _time([lambda: ops.rglru_step(x1, p, dpos, slots, state, cring)] * 20)
+    out["zobasun rglru_step"] = _line(us, 2 * (p["ra"].numel() + p["ri"].numel()) + batch * rec * 22)
+    del yx, o, state, cring
+    # ---- attention: values turned, chunks
+    cols = (h + 2 * g) * d
+    qkv = [_randn(rows, cols) for _ in range(3)]
+    cache, slot = torch.zeros(rows // 64, 64, 2 * g * d, dtype=torch.bfloat16, device="cuda"), torch.arange(rows, dtype=torch.int32, device="cuda")
+    head, qw, kw, table = torch.ones(d, device="cuda"), torch.ones(h * d, device="cuda"), torch.ones(g * d, device="cuda"), rotation_table(d, 10000.0, 4096, "cuda")
+    us = _time([lambda a=a: ops.attn_prep(a, h, g, d, d, pos, table, cache, slot, head, head, d, d, 1e-6, head_norm=True, v_cos_sin=table) for a in qkv])
+    out["attn_prep, values turned"] = _line(us, rows * 4 * cols)
+    us = _time([lambda a=a: ops.attn_prep(a, h, g, d, d, pos, table, cache, slot, qw, kw, h * d, g * d, 1e-6) for a in qkv])
+    out["galirax attn_prep"] = _line(us, rows * 4 * cols)
+    bt, o = torch.arange(rows // 64, dtype=torch.int32, device="cuda").view(seqs, -1), torch.empty(rows, h * d, device="cuda", dtype=torch.bfloat16)
+    for name, mask, seen in (("paged_prompt, chunks, values turned", dict(chunk=WINDOW, turn=table), sum(t % WINDOW + 1 for t in range(prompt))),
+                             ("galirax paged_prompt, window", dict(window=WINDOW), sum(min(t + 1, WINDOW) for t in range(prompt)))):
+        us = _time([lambda a=a: ops.paged_attend_prompt(a, cache, bt, cu, cu, prompt, h, g, d, d, d ** -0.5, out=o, **mask) for a in qkv] * 2)
+        out[name] = _line(us, 4 * rows * (h + g) * d, 4 * d * h * seqs * seen)
+    del qkv, cache, o
+    pages = -(-ctx // 64)
+    n = max(2, int(3e8 // (batch * pages * 64 * 4 * g * d)) + 1)
+    caches, bt = [_randn(batch * pages, 64, 2 * g * d) for _ in range(n)], torch.randperm(batch * pages).view(batch, pages).int().cuda()
+    q, o = _randn(batch, h * d), torch.empty(batch, h * d, device="cuda", dtype=torch.bfloat16)
+    for name, mask in (("paged_rows, chunks, values turned", dict(chunk=WINDOW, turn=table)), ("galirax paged_rows, window", dict(window=WINDOW))):      # (a full chunk)
+        us = _time([lambda c=c: ops.paged_attend_rows(q, c, bt, dpos, h, g, d, d, d ** -0.5, ctx, out=o, **mask) for c in caches] * 3)
+        out[name] = _line(us, batch * (4 * WINDOW * g * d + 4 * h * d))
+    del caches
+    # ---- feed-forward, grouped projection
+    gu = [_randn(rows, 2 * ff) for _ in range(2)]
+    out["gelu_glu"] = _line(_time([lambda t=t: ops.gelu_glu(t) for t in gu]), rows * ff * 6)
+    out["qwen silu_mul"] = _line(_time([lambda t=t: ops.silu_mul(t) for t in gu]), rows * ff * 6)
+    del gu
+    xp = ops.pack_rows(_randn(batch, width))
+    for name, glu, n in (("gate_up_decode, gelu", "gelu", 2 * ff), ("qwen gate_up_decode", None, 2 * ff)):
+        ws = torch.zeros(max(16, ops.linear_workspace_bytes(batch, n, width, "silu_mul")), dtype=torch.uint8, device="cuda")
+        mid = torch.zeros((batch + 15) // 16 * 16 * ff, dtype=torch.bfloat16, device="cuda")
+        ww = [_randn(n, width) for _ in range(int(3e8 // (2 * n * width)) + 2)]
+        us = _time([lambda w=w: ops.fused_linear(xp, w, x_packed_rows=batch, epilogue="silu_mul", out_packed=mid, want_out=False, workspace=ws, glu=glu) for w in ww] * 2)
+        out[name] = _line(us, 2 * n * width)
+    n = 4 * width + 64
+    ws = torch.zeros(max(16, ops.linear_workspace_bytes(batch, n, width)), dtype=torch.uint8, device="cuda")
+    ww = [_randn(n, width) for _ in range(int(3e8 // (2 * n * width)) + 2)]
+    us = _time([lambda w=w: ops.fused_linear(pk, w, x_packed_rows=batch, workspace=ws, x_groups=(5, width)) for w in ww] * 2)
+    out["projection of five inputs, decode"] = _line(us, 2 * n * width)
+    us = _time([lambda w=w: ops.fused_linear(xp, w, x_packed_rows=batch, workspace=ws) for w in ww] * 2)
+    out["projection of one input, decode"] = _line(us, 2 * n * width)
+    torch.cuda.empty_cache()
+    return out
+
+
+MODELS = {"zobasun": (zobasun_config, zobasun_kernels), "galirax": (galirax_config, galirax_kernels), "kekapel": (kekapel_config, kekapel_kernels),
+          "zaposun": (zaposun_config, zaposun_kernels)}
 
 
 def run(size, only=None, model="zobasun"):
@@ -435,6 +601,8 @@ def run(size, only=None, model="zobasun"):
     beside = [("qwen", qwen_config(size))]
     if model == "kekapel":
         beside.append(("galirax", galirax_config(size, windows_only=True)))
+    if model == "zaposun":
+        beside.append(("zobasun", zobasun_config(size)))
     stacks = [(model, config(size)), *beside]
     res = {"metric": f"{stacks[0][1].name} beside a Qwen2-shaped stack of equal width, depth and feed-forward (random weights)", "size": size, "shape": SIZES[size], "dtype": "bf16"}
     if only in (None, "kernels"):
