@@ -768,7 +768,8 @@ int nvh_bigram_embed(const nvh_bigram_embed_desc* d, int dtype, void* stream);
 
 /* Hyper-connections: with y given, x_t <- sum_s mix[s][t] x_s + out[t] y for all streams at once (to xout, if given); y2 given: y is first replaced by
  * y_scale (rms(y) y_w + rms(y2) y2_w), means over n columns.  u = sum_s in[s] x_s (in NULL: plain sum) of the new streams goes to `sum`, and, with w given, its RMS
- * norm in `groups` equal parts of the n columns, times w, to h and / or `packed`. */
+ * norm in `groups` equal parts of the n columns, times w, to h and / or `packed`.  shift given (bf16, row i is one new token of sequence i): nvh_token_shift of the
+ * normed rows in the same launch, in fragment order to `shifted`. */
 typedef struct nvh_stream_mix_desc {
     const float* xin;            /* stream s of row r at xin + r * xin_row + s * xin_stream (xin_stream 0: all streams alike) */
     int64_t xin_row, xin_stream;
@@ -790,6 +791,14 @@ typedef struct nvh_stream_mix_desc {
     float eps;
     void* h;                     /* nullable: [rows, cols] in the activation type */
     void* packed;                /* nullable (bf16): the same in MFMA-fragment order */
+    const float* shift;          /* nullable: [cols]; the following as in nvh_token_shift_desc */
+    const float* mu;
+    int32_t mixes, depth;
+    void* ring;
+    void* shifted;
+    int64_t shifted_mix;
+    const int64_t* positions;
+    const int32_t* state_slots;
 } nvh_stream_mix_desc;
 int nvh_stream_mix(const nvh_stream_mix_desc* d, int dtype, void* stream);
 

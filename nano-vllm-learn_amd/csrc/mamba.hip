@@ -31,6 +31,8 @@ __device__ __forceinline__ float softplus_f(float z) {
     return z > 20.f ? z : e < 0.0625f ? small : __logf(1.f + e);
 }
 
+__device__ __forceinline__ float gate_f(float z) { return z * fast_rcp(1.f + fast_exp2(-kLog2e * z)); }         // silu
+
 template <int LANES>
 __device__ __forceinline__ float sum_lanes(float v) {        // over aligned groups of LANES lanes
     if constexpr (LANES >= 2) v += pair_in_row<1>(v);
@@ -149,8 +151,8 @@ __global__ __launch_bounds__(256) void scan_walk_kernel(const ScanArgs a) {
                 y.b += D.b * xk.b;
 #pragma unroll
                 for (int k = 0; k < 4; ++k) {
-                    y.a[k] *= silu_f(zk.a[k]);
-                    y.b[k] *= silu_f(zk.b[k]);
+                    y.a[k] *= gate_f(zk.a[k]);
+                    y.b[k] *= gate_f(zk.b[k]);
                 }
                 act_st8(reinterpret_cast<T*>(a.out) + (int64_t)(row0 + t0 + pt) * a.out_stride + pc, y);
             }
@@ -238,7 +240,7 @@ __global__ __launch_bounds__(256) void scan_step_kernel(const ScanArgs a) {
         }
         const int64_t slot = a.state_slots[row];
         if (ok && slot >= 0) *reinterpret_cast<f32x4*>(a.state + (slot * a.inner + my) * NP + 4 * sl) = n;
-        y = (sum_lanes<LN>(y) + D * xv[i]) * silu_f(zv[i]);
+        y = (sum_lanes<LN>(y) + D * xv[i]) * gate_f(zv[i]);
         if (ok && sl == 0) {
             if (a.out) act_st(reinterpret_cast<uint16_t*>(a.out) + (int64_t)row * a.out_stride + c, y);
             if (a.out_packed) act_st(reinterpret_cast<uint16_t*>(a.out_packed) + pack_index(row, c, a.inner), y);

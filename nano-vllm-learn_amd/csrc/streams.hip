@@ -2,7 +2,7 @@
 //   bigram_embed   x = embed[token] + bigram[row of (previous token, token)]
 //   stream_mix     x_t <- sum_s mix[s][t] x_s + out[t] y, all streams at once from the old ones; u = sum_s in[s] x_s; RMS norm of u in equal groups of columns.
 //                  y is a sublayer's output, or a scaled sum of two, each RMS-normed over the row first
-//   token_shift    h + (h' - h) shift with h' the previous token's h, and mixes of that and ITS previous value, one per coefficient row
+//   token_shift    h + (h' - h) shift with h' the previous token's h, and mixes of that and ITS previous value, one per coefficient row (single tokens: inside stream_mix)
 //   causal_conv    depthwise convolution over a sequence's last tokens, bias, silu
 // Streams and sums are fp32.  HBM-bound row streams; one workgroup per row where a norm needs the whole row.
 // What a later step needs of earlier rows lives in rings per state slot: row of position p at entry p % depth, one entry more than a step looks back, so the
@@ -77,6 +77,15 @@ __device__ __forceinline__ void block_sum2(float& u, float& v, float* lds) {
         v += lds[16 + w];
     }
 }
+
+// row `back` tokens before `row` of a sequence (null: before position 0): this step's rows, or the ring
+template <typename T>
+__device__ __forceinline__ const T* earlier_row(const T* rows, int64_t stride, const T* ring, int depth, int cols, int row, int back, const RowPlace& at, int64_t pos, int slot) {
+    if (row - back >= at.first) return rows + (int64_t)(row - back) * stride;
+    if (pos < back || slot < 0) return nullptr;
+    return ring + ((int64_t)slot * depth + (int)((pos - back) % depth)) * cols;
+}
+__device__ __forceinline__ f32x8 lerp8(const f32x8& h, const f32x8& before, const f32x8& mu) { return {h.a + (before.a - h.a) * mu.a, h.b + (before.b - h.b) * mu.b}; }
 
 // a thread's 8-column pieces of all streams stay in registers from the update to the normed store.  S: streams held (the model's or the next size), CH: pieces
 template <typename T, int S, int CH>
@@ -181,17 +190,27 @@ __global__ __launch_bounds__(1024) void stream_mix_kernel(const StreamMixArgs a)
         }
         if (a.h) act_st8(reinterpret_cast<T*>(a.h) + row * a.cols + c, r);
         if (a.packed) act_st8(reinterpret_cast<uint16_t*>(a.packed) + pack_index((int)row, c, a.cols), r);
+        if (a.shift) {                               // single tokens: shift and mixes on the spot, the normed row goes to the ring
+            const int slot = a.state_slots[row];
+            const int64_t pos = a.positions[row];
+            T* ring = reinterpret_cast<T*>(a.ring);
+            const RowPlace at = {(int)row, (int)row, (int)row};
+            const T* p1 = earlier_row((const T*)nullptr, 0, (const T*)ring, a.depth, a.cols, (int)row, 1, at, pos, slot);
+            const T* p2 = a.mixes ? earlier_row((const T*)nullptr, 0, (const T*)ring, a.depth, a.cols, (int)row, 2, at, pos, slot) : nullptr;
+#pragma unroll
+            for (int k = 0; k < 4; ++k) {            // (the value the ring holds)
+                r.a[k] = act_round(r.a[k], (const T*)nullptr);
+                r.b[k] = act_round(r.b[k], (const T*)nullptr);
+            }
+            const f32x8 h1 = p1 ? act_ld8(p1 + c) : zero8(), h2 = p2 ? act_ld8(p2 + c) : zero8(), shift = act_ld8(a.shift + c);
+            const f32x8 s0 = lerp8(r, h1, shift), s1 = lerp8(h1, h2, shift);
+            uint16_t* dst = reinterpret_cast<uint16_t*>(a.shifted) + pack_index((int)row, c, a.cols);
+            if (a.mixes == 0) act_st8(dst, s0);
+            for (int k = 0; k < a.mixes; ++k) act_st8(dst + k * a.shifted_mix, lerp8(s0, s1, act_ld8(a.mu + (int64_t)k * a.cols + c)));
+            if (slot >= 0) act_st8(ring + ((int64_t)slot * a.depth + (int)(pos % a.depth)) * a.cols + c, r);
+        }
     }
 }
-
-// row `back` tokens before `row` of a sequence (null: before position 0): this step's rows, or the ring
-template <typename T>
-__device__ __forceinline__ const T* earlier_row(const T* rows, int64_t stride, const T* ring, int depth, int cols, int row, int back, const RowPlace& at, int64_t pos, int slot) {
-    if (row - back >= at.first) return rows + (int64_t)(row - back) * stride;
-    if (pos < back || slot < 0) return nullptr;
-    return ring + ((int64_t)slot * depth + (int)((pos - back) % depth)) * cols;
-}
-__device__ __forceinline__ f32x8 lerp8(const f32x8& h, const f32x8& before, const f32x8& mu) { return {h.a + (before.a - h.a) * mu.a, h.b + (before.b - h.b) * mu.b}; }
 
 // whether CNT rows from `row` on belong to one portion
 template <int CNT>
@@ -400,11 +419,14 @@ int nvh_stream_mix(const nvh_stream_mix_desc* d, int dtype, void* stream) {
     REQUIRE(d, NVH_E_NULL, "stream_mix: null descriptor");
     if (d->rows == 0) return 0;
     DTYPE("stream_mix");
-    REQUIRE(d->xin && (!d->y || (d->mix && d->out)) && (!d->y2 || (d->y && d->y_w && d->y2_w)) && (!d->xout || d->y) && (!d->w || d->h || d->packed) && (d->w || d->sum || d->xout), NVH_E_NULL,
+    REQUIRE(d->xin && (!d->y || (d->mix && d->out)) && (!d->y2 || (d->y && d->y_w && d->y2_w)) && (!d->xout || d->y) && (!d->w || d->h || d->packed || d->shift) && (d->w || d->sum || d->xout), NVH_E_NULL,
             "stream_mix: null pointer");
     REQUIRE(d->rows > 0 && d->cols > 0 && d->cols % 8 == 0 && d->cols <= 16384 && d->n > 0 && d->n <= d->cols && d->streams > 0 && d->streams <= 16 && d->groups > 0 &&
             d->n % d->groups == 0, NVH_E_SHAPE, "stream_mix: cols %d (%%8, <= 16384), %d columns in %d groups, %d streams (<= 16)", d->cols, d->n, d->groups, d->streams);
-    REQUIRE(!d->packed || (dtype == NVH_BF16 && d->cols % 32 == 0), NVH_E_SHAPE, "stream_mix: packed rows are bf16, cols %% 32 == 0");
+    REQUIRE((!d->packed && !d->shift) || (dtype == NVH_BF16 && d->cols % 32 == 0), NVH_E_SHAPE, "stream_mix: packed rows are bf16, cols %% 32 == 0");
+    REQUIRE(!d->shift || (d->w && d->ring && d->shifted && d->positions && d->state_slots && d->mixes >= 0 && d->mixes <= 64 && (!d->mixes || d->mu) && d->depth == (d->mixes ? 3 : 2) &&
+            d->shifted_mix % 8 == 0 && aligned16(d->shift) && aligned16(d->mu) && aligned16(d->ring) && aligned16(d->shifted)), NVH_E_SHAPE, "stream_mix: shift of %d mixes, ring of %d",
+            d->mixes, d->depth);
     REQUIRE(d->xin_row % 8 == 0 && d->xin_stream % 8 == 0 && (!d->y || (d->y_stride % 8 == 0 && d->y_stride >= d->cols)) && (!d->y2 || (d->y2_stride % 8 == 0 && d->y2_stride >= d->cols)),
             NVH_E_STRIDE, "stream_mix: row strides");
     REQUIRE(aligned16(d->xin) && aligned16(d->xout) && aligned16(d->y) && aligned16(d->y2) && aligned16(d->y_w) && aligned16(d->y2_w) && aligned16(d->w) && aligned16(d->sum) && aligned16(d->h) &&

@@ -183,7 +183,7 @@ __global__ __launch_bounds__(DIM * 4) void wkv_walk_kernel(const WkvArgs a) {
 #pragma unroll
             for (int i = 0; i < 8; ++i) {
                 const int t = 8 * tg + i;
-                *reinterpret_cast<f32x2*>(w_f + t * DIM + 2 * cp) = f32x2{fast_exp2(la[i] - (i ? la[i ? i - 1 : 0] : 0.f)), fast_exp2(lb[i] - (i ? lb[i ? i - 1 : 0] : 0.f))};
+                *reinterpret_cast<f32x2*>(w_f + t * DIM + 2 * cp) = f32x2{fast_exp2(log2_decay(bf16_lo(zz[i]) + w0a)), fast_exp2(log2_decay(bf16_hi(zz[i]) + w0b))};
                 *reinterpret_cast<uint32_t*>(lds.k_hi + t * ROW + 4 * cp) = kk[i];
                 if constexpr (!SUMMARY) *reinterpret_cast<uint32_t*>(lds.k_lo + t * ROW + 4 * cp) = rr[i];
             }

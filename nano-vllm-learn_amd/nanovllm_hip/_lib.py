@@ -153,7 +153,9 @@ class StreamMixDesc(ctypes.Structure):
                 ("y", ctypes.c_void_p), ("y_stride", ctypes.c_int64), ("y2", ctypes.c_void_p), ("y2_stride", ctypes.c_int64),
                 ("y_w", ctypes.c_void_p), ("y2_w", ctypes.c_void_p), ("y_scale", ctypes.c_float), ("mix", ctypes.c_void_p),
                 ("out", ctypes.c_void_p), ("in", ctypes.c_void_p), ("sum", ctypes.c_void_p), ("w", ctypes.c_void_p),
-                ("groups", ctypes.c_int32), ("eps", ctypes.c_float), ("h", ctypes.c_void_p), ("packed", ctypes.c_void_p)]
+                ("groups", ctypes.c_int32), ("eps", ctypes.c_float), ("h", ctypes.c_void_p), ("packed", ctypes.c_void_p), ("shift", ctypes.c_void_p),
+                ("mu", ctypes.c_void_p), ("mixes", ctypes.c_int32), ("depth", ctypes.c_int32), ("ring", ctypes.c_void_p),
+                ("shifted", ctypes.c_void_p), ("shifted_mix", ctypes.c_int64), ("positions", ctypes.c_void_p), ("state_slots", ctypes.c_void_p)]
 
 
 class TokenShiftDesc(ctypes.Structure):

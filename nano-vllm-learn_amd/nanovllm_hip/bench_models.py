@@ -73,7 +73,7 @@ def zaposun_config(size):
         "left": dict(heads=s["heads"], kv_heads=s["kv_heads"], dim=128, vdim=128, scale=128 ** -0.5, rot={"base": 10000.0, "dims": 128}, mask={"size": WINDOW}),
         "right": dict(inner=2 * s["width"], state=STATES, dt_rank=s["width"] // 16, conv=TAPS)}}
     return ZaposunConfig.from_json({"width": s["width"], "vocab": VOCAB, "norm": {"eps": 1e-6, "groups": 2}, "streams": STREAMS, "logit_scale": 1.0,
-                                    "embedding": {"bigram": {"buckets": 4093, "mul_prev": 31, "mul_cur": 17}}, "layers": [(wkv, par)[i % 2] for i in range(s["layers"])]})
+                                    "embedding": {"bigram": {"buckets": 4093, "mul_prev": 29, "mul_cur": 13}}, "layers": [(wkv, par)[i % 2] for i in range(s["layers"])]})
 
 
 def zobasun_config(size):
@@ -480,8 +480,9 @@ def zaposun_kernels(size, batch=32, ctx=1536, seqs=16, prompt=1024):
     y1, pk = _randn(batch, width), torch.zeros((batch + 15) // 16 * 16 * width * 5, dtype=torch.bfloat16, device="cuda")
     us = _time([lambda x=x: ops.stream_mix(x, STREAMS, torch.bfloat16, width, dict(y=y1, mix=mix, out=vec), vec, w32) for x in x1] * 5)
     out["stream_mix_decode"] = _line(us, batch * width * (8 * STREAMS + 4))
-    us = _time([lambda: ops.token_shift(y1, dpos, single, one, ring, mu, packed=pk)] * 20)
-    out["token_shift_decode"] = _line(us, batch * width * 18)
+    sh = dict(positions=dpos, step=single, shift=one, ring=ring, mu=mu, packed=pk)
+    us = _time([lambda x=x: ops.stream_mix(x, STREAMS, torch.bfloat16, width, dict(y=y1, mix=mix, out=vec), vec, w32, want_rows=False, shift=sh) for x in x1] * 5)
+    out["stream_mix_decode with five shifted mixes"] = _line(us, batch * width * (8 * STREAMS + 2 + 16))
     x1 = _randn(batch, width, dtype=f32)
     us = _time([lambda: ops.residual_norm(x1, torch.bfloat16, y=y1, weight=one, bias=one, eps=1e-6)] * 20)
     out["galirax residual_norm_decode"] = _line(us, batch * width * 12)
@@ -522,7 +523,7 @@ def zaposun_kernels(size, batch=32, ctx=1536, seqs=16, prompt=1024):
     p = dict(a_log2=-torch.rand(inner, STATES, device="cuda") * 4, d=torch.ones(inner, device="cuda"), dt_bias=torch.rand(inner, device="cuda") * 4 - 5, w_dt=_randn(inner, (rank + 63) // 64 * 64) * 0.1)
     o = torch.empty(rows, inner, device="cuda", dtype=torch.bfloat16)
     state = torch.zeros(max(seqs, batch), inner, STATES, device="cuda")
-    chunks, more = segments(inner // 64)
+    chunks, more = segments(inner // 192)
     us = _time([lambda a=a: ops.scan_chunks(a[:, :inner], dt, bc, a[:, inner:], p, pos, slots, chunks, more, state, out=o) for a in xz] * 2)
     out["scan_chunks"] = _line(us, rows * inner * 8)
     x1, low, bc1 = _randn(batch, 2 * inner), _randn(batch, p["w_dt"].shape[1]), _randn(batch, 64)

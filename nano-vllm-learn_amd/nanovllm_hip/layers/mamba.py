@@ -12,7 +12,8 @@ from .linear import linear, padded, round_up
 
 
 class SelectiveScan(nn.Module):
-    segment_units = property(lambda self: self.inner_cols // 64)     # workgroups that walk one segment
+    # what choose_segment takes for workgroups that walk one segment: it counts one per CU, the scan's small ones want company (three per CU)
+    segment_units = property(lambda self: max(1, self.inner_cols // 192))
 
     def __init__(self, in_width, in_cols, inner, states, rank, taps, dtype):
         super().__init__()

@@ -38,10 +38,14 @@ class TokenShift(nn.Module):
         self.register_buffer("shift", padded(shift.float(), self.cols))
         self.register_buffer("mu", torch.stack([padded(m.float(), self.cols) for m in mu]) if self.mixes else None)
 
-    def forward(self, h, positions, step, packed=None):
-        """[rows, cols] -> the shifted rows, or [mixes, rows, cols]; packed: in fragment order into this buffer."""
-        s = ops.token_shift(h, positions, step, self.shift, self.ring, self.mu, packed)
-        return s if self.mixes or s is None else s[0]
+    def forward(self, h, positions, step):
+        """[rows, cols] -> the shifted rows, or [mixes, rows, cols]."""
+        s = ops.token_shift(h, positions, step, self.shift, self.ring, self.mu)
+        return s if self.mixes else s[0]
+
+    def fused(self, positions, step, packed):
+        """What ops.stream_mix needs to do this to single tokens in the launch that norms them; packed: where the rows go in fragment order."""
+        return dict(positions=positions, step=step, shift=self.shift, ring=self.ring, mu=self.mu, packed=packed)
 
 
 class BigramEmbedding(nn.Module):

@@ -157,13 +157,12 @@ class ZaposunForCausalLM(nn.Module):
         def result(y, hc):
             return dict(y if isinstance(y, dict) else dict(y=y), mix=hc.mix, out=hc.out, eps=cfg.norm_eps)
         for layer in self.layers:
-            h = to_next(layer.hc1, layer.norm1)
             if fused:
                 packed = bufs.packed(self.cols * len(layer.mixer.mixes)) if layer.mixer.mixes else bufs.stream
-                layer.shift(h, positions, step, packed=packed)
+                to_next(layer.hc1, layer.norm1, want_rows=False, shift=layer.shift.fused(positions, step, packed))
                 y = layer.mixer.decode(packed, rows, positions, step, bufs)
             else:
-                y = layer.mixer(layer.shift(h, positions, step), positions, step)
+                y = layer.mixer(layer.shift(to_next(layer.hc1, layer.norm1), positions, step), positions, step)
             update = result(y, layer.hc1)
             if layer.mlp is not None:
                 h = to_next(layer.hc2, layer.norm2, packed=bufs.stream if fused else None, want_rows=not fused)

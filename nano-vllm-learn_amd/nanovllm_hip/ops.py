@@ -1164,11 +1164,12 @@ def bigram_embed(tokens, positions, step, embed, bigram, mul_prev, mul_cur, last
     return x
 
 
-def stream_mix(x, streams, dtype, n, update=None, read=None, norm=None, packed=None, want_rows=True, out=None):
+def stream_mix(x, streams, dtype, n, update=None, read=None, norm=None, packed=None, want_rows=True, out=None, shift=None):
     """Hyper-connections between two sublayers.  x: [rows, streams, cols] (fp32), or [rows, cols] where all streams are alike.
     update = dict(y, mix [from, to], out [to]): x_t <- sum_s mix[s, t] x_s + out[t] y (into `out`, or in place); with post = (y2, w, w2, scale) y is
     scale (rms(y) w + rms(y2) w2) first, eps of the norm, as norm = (.., eps) or update["eps"].  Of the new streams u = sum_s read[s] x_s (None: plain sum);
-    norm = (weight, groups, eps): returns its RMS norm in `groups` equal parts of the n columns (in `dtype`; packed: in fragment order too); norm None: returns u (fp32)."""
+    norm = (weight, groups, eps): returns its RMS norm in `groups` equal parts of the n columns (in `dtype`; packed: in fragment order too); norm None: returns u (fp32).
+    shift = dict(positions, step, shift, ring, mu, packed), single tokens: token_shift of the normed rows with these arguments in the same launch."""
     alike = x.dim() == 2
     rows, cols = x.shape[0], x.shape[-1]
     _require_f32(x=x)
@@ -1210,6 +1211,21 @@ def stream_mix(x, streams, dtype, n, update=None, read=None, norm=None, packed=N
         if packed is not None:
             _packed_ok(packed, rows, cols)
             d.packed = packed.data_ptr()
+        if shift is not None:
+            ring, mu, dst, step, positions = (shift[k] for k in ("ring", "mu", "packed", "step", "positions"))
+            d.mixes, d.shifted_mix = 0 if mu is None else mu.shape[0], (rows + 15) // 16 * 16 * cols
+            _require_f32(shift=shift["shift"])
+            _require_gpu_bf16(ring=ring, packed=dst)
+            _require_i32(state_slots=step.state_slots)
+            assert shift["shift"].numel() == cols and ring.is_contiguous() and ring.shape[1:] == (3 if d.mixes else 2, cols)
+            assert dst.is_contiguous() and dst.numel() >= max(d.mixes, 1) * d.shifted_mix
+            assert step.num_decode == rows and step.state_slots.numel() >= rows and positions.dtype == torch.int64 and positions.is_contiguous() and positions.numel() == rows
+            if mu is not None:
+                _require_f32(mu=mu)
+                assert mu.shape[1] == cols
+                d.mu = mu.data_ptr()
+            d.shift, d.ring, d.depth, d.shifted = shift["shift"].data_ptr(), ring.data_ptr(), ring.shape[1], dst.data_ptr()
+            d.positions, d.state_slots = positions.data_ptr(), step.state_slots.data_ptr()
     _lib.check(_lib.load().nvh_stream_mix(ctypes.byref(d), _out_code(dtype), _stream()), "nvh_stream_mix")
     return res
 

@@ -44,7 +44,7 @@ def test_bigram_embed(buckets, mul_prev, mul_cur, dtype):
 
 # ------------------------------------------------------------------------------------------------ streams
 @pytest.mark.parametrize("dtype", [BF16, F32])
-@pytest.mark.parametrize("streams,n,cols,groups", [(1, 64, 64, 1), (2, 72, 128, 3), (3, 136, 192, 8), (4, 320, 320, 2), (4, 2048, 2048, 4), (5, 100, 128, 100), (8, 1000, 1024, 5), (16, 72, 72, 1),
+@pytest.mark.parametrize("streams,n,cols,groups", [(1, 64, 64, 1), (2, 72, 128, 3), (3, 136, 192, 8), (4, 352, 384, 2), (4, 2048, 2048, 4), (5, 100, 128, 100), (8, 1000, 1024, 5), (16, 72, 72, 1),
                                                    (4, 4160, 4160, 2), (2, 9000, 9024, 6)])
 def test_stream_mix(streams, n, cols, groups, dtype):
     rows, eps = 5, 1e-3
@@ -115,6 +115,28 @@ def test_token_shift_packed():
     assert ops().token_shift(h.cuda(), p.positions, p.meta(), shift.cuda(), ring, mu.cuda(), packed=packed) is None
     for k in range(5):
         assert torch.equal(ops().unpack_rows(packed[k * 32 * cols:(k + 1) * 32 * cols], rows, cols), want[k])
+
+
+@pytest.mark.parametrize("mixes", [0, 5])
+@pytest.mark.parametrize("streams,n,cols", [(1, 64, 64), (3, 100, 128), (4, 2048, 2048)])
+def test_shift_inside_the_stream_update(streams, n, cols, mixes):
+    """Single tokens: the norm and the shift in one launch give what the two launches give, rows, ring and all; first tokens and second ones too."""
+    rows = 19
+    x, y = padded(randn(rows, streams, n, dtype=F32), rows, streams, cols).cuda(), padded(randn(rows, n, seed=1), rows, cols).cuda()
+    w, shift = (padded(randn(n, seed=s, dtype=F32), cols).cuda() for s in (2, 4))
+    read = randn(streams, seed=5, dtype=F32).cuda()
+    update = dict(y=y, mix=randn(streams, streams, seed=6, dtype=F32).cuda(), out=randn(streams, seed=7, dtype=F32).cuda())
+    norm, mu = (w, 1, 1e-5), randn(mixes, cols, seed=8, dtype=F32).cuda() if mixes else None
+    p = Portions([(i % 4 if i < 12 else 700 + i, 1, 18 - i) for i in range(rows)])
+    rings = [randn(rows, 3 if mixes else 2, cols, seed=9).cuda() for _ in range(2)]
+    xs = [x.clone(), x.clone()]
+    packs = [torch.zeros(max(mixes, 1) * 32 * cols, dtype=BF16, device="cuda") for _ in range(2)]
+    h = ops().stream_mix(xs[0], streams, BF16, n, update, read, norm)
+    ops().token_shift(h, p.positions, p.meta(), shift, rings[0], mu, packed=packs[0])
+    assert ops().stream_mix(xs[1], streams, BF16, n, update, read, norm, want_rows=False,
+                            shift=dict(positions=p.positions, step=p.meta(), shift=shift, ring=rings[1], mu=mu, packed=packs[1])) is None
+    assert torch.equal(xs[0], xs[1]) and torch.equal(rings[0], rings[1])
+    close(packs[1], f64(packs[0]), BF16)
 
 
 @pytest.mark.parametrize("dtype", [BF16, F32])
@@ -466,7 +488,7 @@ def test_gelu_glu(dtype):
     close(ops().gelu_glu(gu.cuda()), Z.gelu_tanh(f64(gu)[:, :136]) * f64(gu)[:, 136:], dtype)
 
 
-@pytest.mark.parametrize("m,k,inter", [(1, 64, 16), (17, 320, 384), (33, 1280, 192), (64, 2048, 6144)])
+@pytest.mark.parametrize("m,k,inter", [(1, 64, 16), (17, 256, 448), (33, 1280, 192), (64, 2048, 6144)])
 def test_gelu_epilogue(m, k, inter):
     x, w = randn(m, k), randn(2 * inter, k, seed=1, scale=k ** -0.5)
     ws = torch.zeros(max(16, ops().linear_workspace_bytes(m, 2 * inter, k, "silu_mul")), dtype=torch.uint8, device="cuda")
@@ -477,7 +499,7 @@ def test_gelu_epilogue(m, k, inter):
     close(ops().fused_linear(x.cuda(), w.cuda(), epilogue="silu_mul", glu="gelu", workspace=ws), want, BF16, slack=2)
 
 
-@pytest.mark.parametrize("m,k,rows,tail", [(1, 64, 64, 16), (19, 320, 256, 64), (32, 2048, 2048, 64), (64, 1280, 128, 192), (5, 128, 16, 16)])
+@pytest.mark.parametrize("m,k,rows,tail", [(1, 64, 64, 16), (19, 192, 384, 64), (32, 2048, 2048, 64), (64, 1280, 128, 192), (5, 128, 16, 16)])
 def test_projection_of_several_inputs(m, k, rows, tail):
     """Groups of weight rows, each applied to its own activations; the last group of another size; contractions split over workgroups."""
     xs, w = [randn(m, k, seed=s) for s in range(5)], randn(4 * rows + tail, k, seed=9, scale=k ** -0.5)
