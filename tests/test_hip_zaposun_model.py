@@ -198,6 +198,23 @@ def test_long_contractions_decode(folder):
     check(torch.cat([torch.cat(r) for r in rows]), torch.cat([plain("long", r) for r in reqs]), BF16)
 
 
+@pytest.mark.parametrize("name,dtype", [("odd", F32), ("odd", BF16), ("wide", BF16)])
+def test_more_single_tokens_than_the_fused_path_takes(folder, name, dtype):
+    """Seventy sequences decoded together."""
+    vocab = CONFIGS[name]["vocab"]
+    reqs = [tokens(4 + i % 5, vocab, i) for i in range(70)]
+    eng = engine(folder, name, dtype, pool_tokens=70 * 64, max_num_seqs=70)
+    seqs = [eng.sequence(r[:-3]) for r in reqs]
+    eng.feed([(s, len(s)) for s in seqs], [[] for _ in seqs])
+    rows = []
+    for _ in range(3):
+        for s, r in zip(seqs, reqs):
+            s.append_token(r[len(s)])
+        rows.append(eng.feed([(s, 1) for s in seqs]).float().cpu())
+    want = torch.stack([Z.forward(CONFIGS[name], weights(name), r)[-3:] for r in reqs], dim=1)
+    check(torch.cat(rows), want.reshape(-1, vocab), dtype)
+
+
 # ------------------------------------------------------------------------------------------------ generation
 def follow(name, prompt, out, dtype):
     """Every generated token is the reference's arg-max after the same tokens, up to ties within rounding."""
